@@ -1,0 +1,80 @@
+// Shared helpers of the serving kernels (ragged batches, 32-bit residual).
+//
+// Every kernel here is written for an element type T of activations and
+// weights: `short` holds bf16 bits, `float` is the true 32-bit mode.
+#pragma once
+
+#include "../common.h"
+#include "../mfma.h"
+
+#define SV_PAGE 64  // tokens of one cache page
+#define SV_LOG2E 1.4426950408889634f
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef short s4v __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ float to_f(short v) { return bits2f(v); }
+__device__ __forceinline__ float to_f(float v) { return v; }
+__device__ __forceinline__ void from_f(short& o, float v) { o = f2bits(v); }
+__device__ __forceinline__ void from_f(float& o, float v) { o = v; }
+
+// 4 elements at p[0..3] (16 B / 8 B aligned)
+__device__ __forceinline__ void load4(const float* p, float* v) {
+  const f32x4 a = *(const f32x4*)p;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] = a[j];
+}
+__device__ __forceinline__ void load4(const short* p, float* v) {
+  const s4v a = *(const s4v*)p;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] = bits2f(a[j]);
+}
+__device__ __forceinline__ void store4(float* p, const float* v) {
+  f32x4 a;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) a[j] = v[j];
+  *(f32x4*)p = a;
+}
+__device__ __forceinline__ void store4(short* p, const float* v) {
+  s4v a;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) a[j] = f2bits(v[j]);
+  *(s4v*)p = a;
+}
+
+// 8 elements; `n` of them are inside the row, the rest read as zero.  VEC
+// promises 8-element alignment and a row length that is a multiple of 8.
+template <bool VEC, typename T>
+__device__ __forceinline__ void load8(const T* p, int n, float* v) {
+  if (VEC) {
+    if (n > 0) {
+      load4(p, v);
+      load4(p + 4, v + 4);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = 0.f;
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = j < n ? to_f(p[j]) : 0.f;
+  }
+}
+
+template <>
+__device__ __forceinline__ void load8<true, short>(const short* p, int n,
+                                                   float* v) {
+  const s8v a = n > 0 ? *(const s8v*)p : s8v{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = bits2f(a[j]);
+}
+
+__device__ __forceinline__ float silu_f(float x) {
+  return x / (1.f + __expf(-x));
+}
+__device__ __forceinline__ float sigmoid_f(float x) {
+  return 1.f / (1.f + __expf(-x));
+}
+// log(sigmoid(x)), stable on both sides
+__device__ __forceinline__ float log_sigmoid_f(float x) {
+  return fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
+}

@@ -1,0 +1,236 @@
+// Norms and pointwise steps of the serving path (32-bit residual stream).
+//
+// residual_norm: one pass that (1) adds a pending sublayer result to the
+// 32-bit residual, (2) stores the new residual, (3) writes the RMS-normed
+// row for the next projection and/or the concatenation [x; x0] that a
+// looped block projects.  The pending result is nothing, one tensor, or two
+// parallel branches that are RMS-normed on their own, scaled and summed.
+//
+// gated_norm: RMS norm over groups of a row, times a weight, times
+// sigmoid(gate) — the output stage of the gated recurrent mixers.
+
+#include "serving.h"
+
+struct ResidualNormArgs {
+  const float* x;        // [rows, W] residual, or null (starts from zero)
+  const void* delta;     // [rows, W] T (or f32), or null
+  const void* delta2;    // second branch, or null
+  const void* w1;        // branch norm weights [W] (dual mode)
+  const void* w2;
+  const void* vec;       // [W] added to every row, or null
+  float* x_out;          // [out_rows, W] or null
+  void* h;               // [out_rows, W] normed * w, or null
+  const void* w;         // [W] weight of the norm
+  void* cat;             // [out_rows, 2 W]: new x, then x0; or null
+  const void* x0;        // [rows, W]
+  const int* index;      // out row -> row, or null
+  int rows_out, W, delta_f32;
+  float eps, branch_scale;
+};
+
+template <typename T, int VEC>
+__device__ __forceinline__ void ld(const T* p, float* v) {
+  if (VEC == 4) load4(p, v); else v[0] = to_f(p[0]);
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void st(T* p, const float* v) {
+  if (VEC == 4) store4(p, v); else from_f(p[0], v[0]);
+}
+
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+residual_norm_kernel(ResidualNormArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float row[];  // [W]
+  __shared__ float red[16];
+  const int o = blockIdx.x;
+  const long r = a.index ? a.index[o] : o;
+  const int W = a.W, tid = threadIdx.x;
+  const T* d1 = (const T*)a.delta + r * W;
+  const float* d1f = (const float*)a.delta + r * W;
+  const T* d2 = (const T*)a.delta2 + r * W;
+
+  float s1 = 0.f, s2 = 0.f;
+  if (a.delta2) {
+    float q1 = 0.f, q2 = 0.f, v[VEC];
+    for (int i = tid * VEC; i < W; i += 256 * VEC) {
+      ld<T, VEC>(d1 + i, v);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) q1 += v[j] * v[j];
+      ld<T, VEC>(d2 + i, v);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) q2 += v[j] * v[j];
+    }
+    q1 = block_reduce_sum(q1, red);
+    __syncthreads();
+    q2 = block_reduce_sum(q2, red);
+    __syncthreads();
+    s1 = a.branch_scale / sqrtf(q1 / W + a.eps);
+    s2 = a.branch_scale / sqrtf(q2 / W + a.eps);
+  }
+
+  float sq = 0.f;
+  for (int i = tid * VEC; i < W; i += 256 * VEC) {
+    float v[VEC], t[VEC], u[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] = 0.f;
+    if (a.x) ld<float, VEC>(a.x + r * W + i, v);
+    if (a.delta2) {
+      ld<T, VEC>(d1 + i, t);
+      ld<T, VEC>((const T*)a.w1 + i, u);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) t[j] *= s1 * u[j];
+      float p[VEC];
+      ld<T, VEC>(d2 + i, p);
+      ld<T, VEC>((const T*)a.w2 + i, u);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] += t[j] + p[j] * s2 * u[j];
+    } else if (a.delta) {
+      if (a.delta_f32) ld<float, VEC>(d1f + i, t);
+      else ld<T, VEC>(d1 + i, t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] += t[j];
+    }
+    if (a.vec) {
+      ld<T, VEC>((const T*)a.vec + i, t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] += t[j];
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) sq += v[j] * v[j];
+    if (a.x_out) st<float, VEC>(a.x_out + (long)o * W + i, v);
+    if (a.cat) {
+      st<T, VEC>((T*)a.cat + 2L * o * W + i, v);
+      ld<T, VEC>((const T*)a.x0 + r * W + i, t);
+      st<T, VEC>((T*)a.cat + (2L * o + 1) * W + i, t);
+    }
+    if (a.h) st<float, VEC>(row + i, v);
+  }
+  if (!a.h) return;
+  sq = block_reduce_sum(sq, red);
+  const float rstd = 1.f / sqrtf(sq / W + a.eps);
+  for (int i = tid * VEC; i < W; i += 256 * VEC) {
+    float v[VEC], u[VEC];
+    ld<float, VEC>(row + i, v);  // written by this same thread
+    ld<T, VEC>((const T*)a.w + i, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] *= rstd * u[j];
+    st<T, VEC>((T*)a.h + (long)o * W + i, v);
+  }
+}
+
+extern "C" int sv_residual_norm(const ResidualNormArgs* a, int f32,
+                                hipStream_t stream) {
+  if (a->rows_out <= 0) return 0;
+  const size_t lds = a->h ? (size_t)a->W * sizeof(float) : 0;
+  if (lds > 160 * 1024 - 256) return 1;
+#define RN(T, V)                                                           \
+  residual_norm_kernel<T, V><<<a->rows_out, 256, lds, stream>>>(*a)
+  if (f32) { if (a->W % 4 == 0) RN(float, 4); else RN(float, 1); }
+  else     { if (a->W % 4 == 0) RN(short, 4); else RN(short, 1); }
+#undef RN
+  return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// o [rows, groups * gs] -> o / rms(group) * w * sigmoid(gate)
+// One wave per (row, group): NW waves of a block take neighbouring groups.
+// Long groups take the whole block.
+// ---------------------------------------------------------------------------
+template <typename T, int VEC, bool BLOCK>
+__global__ void __launch_bounds__(256)
+gated_norm_kernel(const T* __restrict__ o, const T* __restrict__ w,
+                  const T* __restrict__ gate, long gate_stride,
+                  T* __restrict__ out, int rows, int groups, int gs,
+                  float eps) {
+  __shared__ float red[16];
+  const int tid = BLOCK ? threadIdx.x : (threadIdx.x & 63);
+  const int step = (BLOCK ? 256 : 64) * VEC;
+  const long item = BLOCK ? (long)blockIdx.x
+                          : (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= (long)rows * groups) return;  // whole waves leave together
+  const long r = item / groups;
+  const int off = (int)(item % groups) * gs;
+  const T* src = o + item * gs;
+  const T* g = gate + r * gate_stride + off;
+  float sq = 0.f, v[VEC], u[VEC];
+  for (int i = tid * VEC; i < gs; i += step) {
+    ld<T, VEC>(src + i, v);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) sq += v[j] * v[j];
+  }
+  sq = BLOCK ? block_reduce_sum(sq, red) : wave_reduce(sq, SumOp());
+  const float rstd = 1.f / sqrtf(sq / gs + eps);
+  for (int i = tid * VEC; i < gs; i += step) {
+    ld<T, VEC>(src + i, v);
+    ld<T, VEC>(w + off + i, u);
+    float z[VEC];
+    ld<T, VEC>(g + i, z);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] *= rstd * u[j] * sigmoid_f(z[j]);
+    st<T, VEC>(out + item * gs + i, v);
+  }
+}
+
+extern "C" int sv_gated_norm(const void* o, const void* w, const void* gate,
+                             long gate_stride, void* out, int rows,
+                             int groups, int gs, float eps, int vec4, int f32,
+                             hipStream_t stream) {
+  if (rows <= 0) return 0;
+  const bool block = gs > 1024;
+  const long items = (long)rows * groups;
+  const int grid = (int)(block ? items : (items + 3) / 4);
+#define GN(T, V, B)                                                         \
+  gated_norm_kernel<T, V, B><<<grid, 256, 0, stream>>>(                     \
+      (const T*)o, (const T*)w, (const T*)gate, gate_stride, (T*)out, rows, \
+      groups, gs, eps)
+#define GNB(T, V) do { if (block) GN(T, V, true); else GN(T, V, false); } while (0)
+  if (f32) { if (vec4) GNB(float, 4); else GNB(float, 1); }
+  else     { if (vec4) GNB(short, 4); else GNB(short, 1); }
+#undef GNB
+#undef GN
+  return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// pointwise: max(x, 0)^2 in place; cap * tanh(x / cap) in place (f32)
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+relu_squared_kernel(T* __restrict__ x, long n) {
+  const long i = ((long)blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (i >= n) return;
+  float v[VEC];
+  ld<T, VEC>(x + i, v);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) {
+    const float p = fmaxf(v[j], 0.f);
+    v[j] = p * p;
+  }
+  st<T, VEC>(x + i, v);
+}
+
+extern "C" int sv_relu_squared(void* x, long n, int f32, hipStream_t stream) {
+  if (n <= 0) return 0;
+  const int vec = n % 4 == 0 ? 4 : 1;
+  const long blocks = (n / vec + 255) / 256;
+  if (f32) {
+    if (vec == 4) relu_squared_kernel<float, 4><<<blocks, 256, 0, stream>>>((float*)x, n);
+    else relu_squared_kernel<float, 1><<<blocks, 256, 0, stream>>>((float*)x, n);
+  } else {
+    if (vec == 4) relu_squared_kernel<short, 4><<<blocks, 256, 0, stream>>>((short*)x, n);
+    else relu_squared_kernel<short, 1><<<blocks, 256, 0, stream>>>((short*)x, n);
+  }
+  return (int)hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256)
+softcap_kernel(float* __restrict__ x, long n, float cap) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) x[i] = cap * tanhf(x[i] / cap);
+}
+
+extern "C" int sv_softcap(void* x, long n, float cap, hipStream_t stream) {
+  if (n <= 0) return 0;
+  softcap_kernel<<<(n + 255) / 256, 256, 0, stream>>>((float*)x, n, cap);
+  return (int)hipGetLastError();
+}
