@@ -4,6 +4,7 @@
 engine ranks with torchrun and put the server on rank 0's feed.
 
   python examples/inference/serve.py --model llama3-8b --port 8000
+  python examples/inference/serve.py --model /path/to/model_folder
   curl -X POST localhost:8000/generate -H 'Content-Type: application/json' \
        -d '{"token_ids": [[1, 2, 3]], "max_new_tokens": 16}'
 """
@@ -31,21 +32,22 @@ def build_app(model_name: str = "test-d128"):
                                 world_size=1)
 
     from neuronx_distributed_amd.parallel import parallel_state as ps
-    from neuronx_distributed_amd.models import get_config, LlamaForCausalLM
+    from neuronx_distributed_amd.models import (build_model, get_config,
+                                                load_pretrained)
     from neuronx_distributed_amd.inference.generation import generate
+    from neuronx_distributed_amd.inference.scheduler import generate_ragged
     from neuronx_distributed_amd.utils.sampling import Sampler
 
     if not ps.model_parallel_is_initialized():
         ps.initialize_model_parallel(tensor_model_parallel_size=1)
-    cfg = get_config(model_name)
     device = torch.device("cuda") if on_gpu else torch.device("cpu")
-    prev = torch.get_default_dtype()
-    if on_gpu:
-        torch.set_default_dtype(torch.bfloat16)
+    dtype = torch.bfloat16 if on_gpu else torch.float32
     torch.manual_seed(0)
-    with torch.device(device):
-        model = LlamaForCausalLM(cfg).eval()
-    torch.set_default_dtype(prev)
+    if os.path.isdir(model_name):  # config.json chooses the model class
+        model = load_pretrained(model_name, dtype, device)
+    else:
+        model = build_model("LlamaForCausalLM", get_config(model_name),
+                            dtype, device)
 
     app = FastAPI(title="neuronx-distributed-amd serving demo")
 
@@ -58,9 +60,12 @@ def build_app(model_name: str = "test-d128"):
 
     @app.post("/generate")
     def gen(req: GenRequest):
-        x = torch.tensor(req.token_ids, dtype=torch.long, device=device)
         sampler = Sampler(do_sample=req.do_sample, top_k=req.top_k,
                           temperature=req.temperature)
+        if getattr(model, "supports_ragged", False):  # unequal lengths
+            return {"token_ids": generate_ragged(
+                model, req.token_ids, req.max_new_tokens, sampler)}
+        x = torch.tensor(req.token_ids, dtype=torch.long, device=device)
         with torch.no_grad():
             out = generate(model, x, max_new_tokens=req.max_new_tokens,
                            sampler=sampler)

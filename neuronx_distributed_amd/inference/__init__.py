@@ -1,6 +1,6 @@
 from .model_builder import ModelBuilder
 from .nxd_model import NxDModel, StateInitializer
-from .parallel_context import NxDParallelState
+from .parallel_context import NxDParallelState, single_process_groups
 from .functions import (
     trace,
     compile,
@@ -12,3 +12,6 @@ from .functions import (
 from .kv_cache import (KVCache, RollingKVCache,
                        build_kv_caches)
 from .generation import generate
+from .paged_cache import CacheFull, CacheManager, MatrixState, PagedKV
+from .engine import InferenceEngine, StepEntry
+from .scheduler import Scheduler, generate_ragged

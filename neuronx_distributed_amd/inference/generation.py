@@ -19,11 +19,25 @@ def generate(model, input_ids: torch.Tensor, max_new_tokens: int = 32,
 
     On GPU the per-token decode step is captured in a hipGraph and
     replayed (launch-bound otherwise); pass ``use_cuda_graph=False`` for
-    the eager loop."""
+    the eager loop.
+
+    Models of the serving engine (``supports_ragged``) go through its
+    scheduler; rows that met ``eos_token_id`` early are filled with it."""
     from ..parallel import parallel_state as ps
     from .decode_graph import GraphDecoder
 
     sampler = sampler or Sampler(do_sample=False)
+    if getattr(model, "supports_ragged", False):
+        from .scheduler import generate_ragged
+
+        new = generate_ragged(model, input_ids.tolist(), max_new_tokens,
+                              sampler, eos_token_id,
+                              use_graphs=use_cuda_graph)
+        n = max(len(o) for o in new)
+        new = [o + [eos_token_id] * (n - len(o)) for o in new]
+        return torch.cat([input_ids, torch.tensor(
+            new, dtype=input_ids.dtype,
+            device=input_ids.device).reshape(len(new), n)], dim=1)
     cfg = model.config
     tp = ps.get_tensor_model_parallel_size()
     B, S = input_ids.shape

@@ -40,3 +40,15 @@ class NxDParallelState(contextlib.AbstractContextManager):
         ps.exit_aot_mode()
         ps._GROUPS = self._saved_groups
         return False
+
+
+def single_process_groups():
+    """Model-parallel groups of size one for a process that serves a model
+    alone: no network, the rendezvous store lives in this process."""
+    import torch.distributed as dist
+
+    if not dist.is_initialized():
+        dist.init_process_group("gloo", store=dist.HashStore(), rank=0,
+                                world_size=1)
+    if not ps.model_parallel_is_initialized():
+        ps.initialize_model_parallel(tensor_model_parallel_size=1)

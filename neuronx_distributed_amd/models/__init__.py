@@ -3,3 +3,7 @@ from .mixtral import (MixtralConfig, MixtralForCausalLM, MixtralModel,
                       get_moe_config, MOE_CONFIGS)
 from .gpt_neox import (GPTNeoXConfig, GPTNeoXForCausalLM, get_neox_config,
                        NEOX_CONFIGS)
+from .voletar import (VoletarConfig, VoletarForCausalLM, VOLETAR_CONFIGS,
+                      get_voletar_config)
+from .registry import (ModelEntry, build_model, load_pretrained,
+                       register_model, registered_models)

@@ -282,7 +282,10 @@ class LlamaAttention(nn.Module):
         # GEMM; casting K/V to fp32 would re-materialize the whole cache
         # every step) -> (B,Hkv,rep,Smax)
         qg = q.view(B, self.num_kv_local, rep, self.head_dim)
-        scores = (qg @ K.transpose(-1, -2)).float() * scale
+        # the cache is the LEFT operand: a transposed view on the right of a
+        # bf16 batched product is avoided
+        scores = (K @ qg.transpose(-1, -2).contiguous()).transpose(
+            -1, -2).float() * scale
         if hasattr(kv_cache, "position_index"):
             # rolling window cache: slots carry their GLOBAL position
             # (-1 = unwritten -> masked by idx > pos_t never holding...

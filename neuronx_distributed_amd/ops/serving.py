@@ -225,6 +225,14 @@ def _check_cache(q, k, v, kc, vc, H):
     return G, D, E
 
 
+def _out(out, rows, cols, like):
+    if out is None:
+        return torch.empty(rows, cols, dtype=like.dtype, device=like.device)
+    assert out.shape == (rows, cols) and out.is_contiguous() and \
+        out.dtype == like.dtype
+    return out
+
+
 def kv_append(k, v, kc, vc, pos, seq, block_table):
     """Write k (T, G*D) and v (T, G*E) at positions ``pos`` of the requests
     ``seq`` (int32, row of the block table)."""
@@ -242,7 +250,8 @@ def kv_append(k, v, kc, vc, pos, seq, block_table):
 
 def attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads: int,
               scale: float, window: int = 0, keep: int = 0,
-              append: bool = True, max_keys: int = 0) -> torch.Tensor:
+              append: bool = True, max_keys: int = 0,
+              out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """One query row per request row: decoding.  ``append`` also writes the
     row's own k/v into the cache (without it they must be there already).
     ``max_keys`` bounds the visible keys of any row (it only sets how many
@@ -254,7 +263,7 @@ def attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads: int,
         max_keys = min(max_keys, window + keep) if max_keys else window + keep
     want = max(1, 1024 // max(1, rows * G))
     splits = max(1, min(want, (max_keys + 127) // 128, 64))
-    out = torch.empty(rows, heads * E, dtype=q.dtype, device=q.device)
+    out = _out(out, rows, heads * E, q)
     part = torch.empty(rows * heads * splits * (E + 2), dtype=torch.float32,
                        device=q.device) if splits > 1 else None
     a = _RowsArgs(q=_p(q), k=_p(k), v=_p(v), qst=q.stride(0),
@@ -277,7 +286,8 @@ def attn_tiles_supported(q, kc, vc) -> bool:
 
 def attn_portions(q, k, v, kc, vc, pos, seq, block_table, tiles, heads: int,
                   scale: float, window: int = 0, keep: int = 0,
-                  max_keys: int = 0) -> torch.Tensor:
+                  max_keys: int = 0,
+                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Prompt portions: append k/v, then causal attention of every row over
     its request's cache.  ``tiles`` (n, 4) int32 lists (request, first row,
     rows <= 128, position of the first row)."""
@@ -286,8 +296,8 @@ def attn_portions(q, k, v, kc, vc, pos, seq, block_table, tiles, heads: int,
     if not attn_tiles_supported(q, kc, vc):
         return attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads,
                          scale, window, keep, append=False,
-                         max_keys=max_keys)
-    out = torch.empty(q.shape[0], heads * E, dtype=q.dtype, device=q.device)
+                         max_keys=max_keys, out=out)
+    out = _out(out, q.shape[0], heads * E, q)
     a = _TilesArgs(q=_p(q), qst=q.stride(0), kc=_p(kc), vc=_p(vc),
                    tiles=_p(tiles), bt=_p(block_table), out=_p(out),
                    MB=block_table.shape[1], H=heads, G=G, D=D, E=E,
@@ -319,11 +329,14 @@ class ExpGate:
 
 
 def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
-               chunked: bool) -> torch.Tensor:
+               chunked: bool,
+               out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Run a matrix memory over segments of a ragged batch.  q, k (T, H*D),
     v (T, H*E); S (slots, H, D, E) float32; n (slots, H, ceil(E/32), D) and
     m (slots, H, ceil(E/32)) float32 for an ExpGate.  ``seg`` (n, 4) int32
-    lists (slot, first row, rows, context).  ``chunked`` uses the 64-token
+    lists (slot, first row, rows, context); rows count from the start of
+    the tensors, so portions and single tokens of one batch can be run by
+    two calls into one ``out``.  ``chunked`` uses the 64-token
     MFMA kernel where it applies."""
     D, E = S.shape[2], S.shape[3]
     T = q.shape[0]
@@ -333,7 +346,7 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
     assert S.shape[1] == heads
     if D > MAX_HEAD_DIM:
         raise ValueError(f"key size {D} > {MAX_HEAD_DIM}")
-    out = torch.empty(T, heads * E, dtype=q.dtype, device=q.device)
+    out = _out(out, T, heads * E, q)
     a = _MemoryArgs(q=_p(q), k=_p(k), v=_p(v), qst=q.stride(0),
                     kst=k.stride(0), vst=v.stride(0), S=_p(S), seg=_p(seg),
                     out=_p(out), H=heads, D=D, E=E, gate_cap=1.0, qscale=1.0)
