@@ -35,11 +35,19 @@ def parse_args():
                    help="override layer count (debug only; overridden runs "
                         "are marked invalid in the output)")
     p.add_argument("--microbatch", type=int, default=8)
+    p.add_argument("--serving", nargs="?", const="all", default=None,
+                   choices=("all", "kernels", "models"),
+                   help="instead: the serving benchmark of the Voletar "
+                        "design beside Llama (bench_serving.py, 1 GPU)")
     return p.parse_args()
 
 
 def main():
     args = parse_args()
+    if args.serving:
+        import bench_serving
+
+        return bench_serving.main(args.serving)
     rank = int(os.environ.get("RANK", "0"))
     world = int(os.environ.get("WORLD_SIZE", str(args.gpus)))
     local_rank = int(os.environ.get("LOCAL_RANK", str(rank)))
