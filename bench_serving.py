@@ -150,8 +150,10 @@ def bench_kernels():
                                   b0 + 3, 15.0, D2 ** -0.5)
             else:
                 gate = sv.decay_gate([0.99] * H2, "cuda")
+            rows, first = sv.chunk_table(seg.tolist())
+            tab = (_i32(rows), _i32(first)) if T > 1 else ()
             (us,) = _time([_graphed(lambda: sv.memory_mix(
-                q, k, v, gate, S, nn, m, seg, H2, T > 1))])
+                q, k, v, gate, S, nn, m, seg, H2, *tab))])
             io = 2 * B * T * (n + H2 * E2) + \
                 (8 if ctx else 4) * B * H2 * D2 * E2
             # chunked: scores, weighted values, state in and out

@@ -44,7 +44,9 @@ class RaggedBatch:
     block_table: torch.Tensor  # (R, width)
     tiles: torch.Tensor        # (n, 4) query tiles of the portions
     portions: torch.Tensor     # (n, 4) slot, first row, rows, context
-    singles: torch.Tensor      # (n, 4) the same for single tokens
+    chunks: torch.Tensor       # (n, 4) chunks of the portions
+    chunk_first: torch.Tensor  # (portions + 1,) first chunk of each
+    singles: torch.Tensor      # (n, 4) like portions, for single tokens
     want: torch.Tensor         # (W,) rows whose logits are computed
     portion_tokens: int        # rows [0, portion_tokens) belong to portions
     max_keys: int              # no row sees more keys than this
@@ -53,13 +55,15 @@ class RaggedBatch:
 class _Layout:
     """Places of the batch's arrays in one int32 buffer (one upload)."""
 
-    def __init__(self, T, portion_tokens, R, n_tiles, n_portions, n_singles,
-                 n_want, width):
+    def __init__(self, T, portion_tokens, R, n_tiles, n_portions, n_chunks,
+                 n_singles, n_want, width):
         self.portion_tokens = portion_tokens
         self.at, n = {}, 0
         for name, shape in (("tokens", (T,)), ("pos", (T,)), ("seq", (T,)),
                             ("tiles", (n_tiles, 4)),
                             ("portions", (n_portions, 4)),
+                            ("chunks", (n_chunks, 4)),
+                            ("chunk_first", (n_portions + 1,)),
                             ("singles", (n_singles, 4)),
                             ("want", (n_want,)),
                             ("block_table", (R, width))):
@@ -154,12 +158,17 @@ class InferenceEngine:
         n_tiles = sum(-(-len(e.tokens) // TILE_ROWS) for e in entries
                       if len(e.tokens) > 1)
         want = [row_of[i] + w for i, e in enumerate(entries) for w in e.want]
+        chunks, first = sv.chunk_table(
+            [(states[i].slot, row_of[i], len(entries[i].tokens),
+              states[i].length) for i in order[:n_port]])
         lay = _Layout(T, portion_tokens, len(entries), n_tiles, n_port,
-                      len(entries) - n_port, len(want),
+                      len(chunks), len(entries) - n_port, len(want),
                       self.cache.table_width)
         host = np.zeros(lay.size, dtype=np.int32)
         v = lay.views(host)
         v["want"][:] = want
+        v["chunks"][:] = np.asarray(chunks, dtype=np.int32).reshape(-1, 4)
+        v["chunk_first"][:] = first
         tile = 0
         for s, i in enumerate(order):
             e, st, r0 = entries[i], states[i], row_of[i]
@@ -211,7 +220,7 @@ class InferenceEngine:
     def _capture(self, bucket: int):
         """Capture one decode step of ``bucket`` rows; the warm-up runs on
         padding rows only."""
-        lay = _Layout(bucket, 0, bucket, 0, 0, bucket, bucket,
+        lay = _Layout(bucket, 0, bucket, 0, 0, 0, bucket, bucket,
                       self.cache.table_width)
         host = np.zeros(lay.size, dtype=np.int32)
         self._fill_singles(lay.views(host), [], [], bucket)

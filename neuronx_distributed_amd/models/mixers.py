@@ -139,10 +139,12 @@ class _MatrixMemory(Mixer):
         gate = self.gate(h)
         out = torch.empty(h.shape[0], self.heads * self.vdim, dtype=h.dtype,
                           device=h.device)
-        for seg, chunked in ((batch.portions, True), (batch.singles, False)):
-            if seg.shape[0]:
-                sv.memory_mix(q, k, v, gate, S, n, m, seg, self.heads,
-                              chunked, out=out)
+        if batch.portions.shape[0]:
+            sv.memory_mix(q, k, v, gate, S, n, m, batch.portions, self.heads,
+                          batch.chunks, batch.chunk_first, out=out)
+        if batch.singles.shape[0]:
+            sv.memory_mix(q, k, v, gate, S, n, m, batch.singles, self.heads,
+                          out=out)
         return self.o(sv.gated_norm(out, self.norm, g, self.norm_group,
                                     self.eps))
 

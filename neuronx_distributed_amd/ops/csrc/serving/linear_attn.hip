@@ -15,8 +15,8 @@
 //          q is scaled by qscale.  S, n and m are zero at position 0.
 //
 //   sv_memory_steps   token after token; single-token decoding, the 32-bit
-//                     mode and sizes the chunk kernel does not take
-//   sv_memory_chunks  64-token chunks on MFMA for bf16 prompt portions
+//                     mode and sizes the chunk kernels do not take
+//   sv_memory_chunks  256-token chunks on MFMA for bf16 prompt portions
 //
 // Every group of 32 state columns keeps its own copy of n and m, so the
 // workgroups of a head never wait for each other.
@@ -226,30 +226,48 @@ extern "C" int sv_memory_steps(const MemoryArgs* a, int n_seg, int gated,
                : launch_steps<short, false>(*a, n_seg, stream);
 }
 
+
 // ---------------------------------------------------------------------------
-// 64-token chunks on MFMA (bf16 projections, 32-bit everything else)
+// Chunks on MFMA (bf16 projections, 32-bit everything else)
 //
-// A workgroup (4 waves) carries VT columns of one head's state through the
-// chunks of a segment; the state stays in MFMA accumulators.  With the local
-// cumulative log forget b_t and a_s = i_s - b_s, M_t = max(m, max_{s<=t} a_s):
+// A portion is cut into chunks of 256 tokens, and every chunk is computed in
+// parallel; only a scan over the chunks' states is sequential.  With local
+// inclusive sums b_t of the log forgets, c_t = max(f_t + c_(t-1), i_t) from
+// c = -inf, and m, S, n before the chunk:
 //
-//   o_t = e^(m - M_t) S^T q_t + sum_{s<=t} e^(a_s - M_t) (q_t . k_s) v_s
-//   S'  = e^(m - M_C) S + sum_s e^(a_s - M_C) k_s v_s^T,  m' = b_C + M_C
+//   gates    b_t, i_t, c_t of every token
+//   states   U = sum_s e^(b_L - b_s + i_s - c_L) k_s v_s^T   (and N with k_s)
+//   scan     m' = max(b_L + m, c_L)
+//            S' = e^(b_L + m - m') S + e^(c_L - m') U        (n' likewise)
+//   outputs  m_t = max(b_t + m, c_t)
+//            o_t ~ e^(b_t + m - m_t) S^T q_t
+//                  + sum_(s<=t) e^(b_t - b_s + i_s - m_t) (q_t . k_s) v_s
 //
-// (every exponent is <= 0).  The plain decay is the same with
-// e^(a_s - M_t) -> decay^(t-s).
+// every exponent is <= 0.  b is kept per 64 tokens (with the four totals of
+// a chunk), so near tokens never cancel large sums.  The plain decay has
+// e^(b_t - b_s + i_s - m_t) = decay^(t-s) and no m.
 //
 // 32-bit operands meet bf16 ones exactly: an f32 value is split into three
 // bf16 planes (8 + 8 + 8 bits) and each plane is multiplied on its own.
-// Products are 16x16x32; a wave owns 16 query rows.  Scores are produced
-// transposed (lane = query), so they feed the next product as its B operand
-// without leaving registers: the contraction order is the accumulator's row
-// order, and V^T is read from LDS in that same order.
+// Scores are produced transposed (lane = query), so they feed the next
+// product as its B operand from registers: the accumulator's row order is
+// the contraction order, and V^T is read from LDS in that same order.
 // ---------------------------------------------------------------------------
-__device__ __forceinline__ f32x4 mfma16(const frag_u& a, const frag_u& b,
-                                        f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.bf, b.bf, c, 0, 0, 0);
-}
+#define MC_L 256
+
+struct ChunkArgs {
+  MemoryArgs a;
+  const int* chunks;        // [n_chunks][4]: segment, first row, rows, ctx > 0
+                            //   or not the first chunk of its segment
+  const int* first;         // [n_seg + 1] first chunk of a segment
+  int n_chunks, n_seg, T;
+  float *b, *i, *c;         // [H][T] (gated)
+  float *tot, *cend;        // [n_chunks][H][4], [n_chunks][H] (gated)
+  float* U;                 // [n_chunks][H][E][D]
+  float* N;                 // [n_chunks][H][D] (gated): N, then n before
+  short* P;                 // [n_chunks][H][3][E][D] state before the chunk
+  float* mst;               // [n_chunks][H] m before the chunk (gated)
+};
 
 // split a pair of floats into three planes of packed bf16
 __device__ __forceinline__ void split3(float x, float y, uint* w) {
@@ -268,380 +286,585 @@ __device__ __forceinline__ void unpack8(uint4v u, float* v) {
     v[2 * j + 1] = __uint_as_float(u[j] & 0xffff0000u);
   }
 }
+template <bool ON>
 __device__ __forceinline__ uint4v silu8(uint4v u) {
-  float v[8];
-  unpack8(u, v);
+  if (ON) {
+    float v[8];
+    unpack8(u, v);
 #pragma unroll
-  for (int j = 0; j < 4; ++j)
-    u[j] = pack_bf16x2(silu_f(v[2 * j]), silu_f(v[2 * j + 1]));
+    for (int j = 0; j < 4; ++j)
+      u[j] = pack_bf16x2(silu_f(v[2 * j]), silu_f(v[2 * j + 1]));
+  }
   return u;
 }
 
+// ---- gates: one block per (chunk, head), one thread per token -------------
+__global__ void __launch_bounds__(MC_L)
+memory_gates_kernel(ChunkArgs x) {
+  const MemoryArgs& a = x.a;
+  const int h = blockIdx.x % a.H, ch = blockIdx.x / a.H;
+  const int row0 = x.chunks[4 * ch + 1], nrow = x.chunks[4 * ch + 2];
+  const int t = threadIdx.x, lane = t & 63, wid = t >> 6;
+  float i = -INFINITY, f = 0.f;
+  if (t < nrow)
+    log_gates(a, row0 + t, h, bits2f(((const short*)a.ib)[h]),
+              bits2f(((const short*)a.fb)[h]), i, f);
+  float F = f, I = i;                    // scan of (F, I) by (+, max)
+#pragma unroll
+  for (int off = 1; off < 64; off <<= 1) {
+    const float F0 = __shfl_up(F, off, 64), I0 = __shfl_up(I, off, 64);
+    if (lane >= off) {
+      I = fmaxf(I0 + F, I);
+      F += F0;
+    }
+  }
+  __shared__ float sF[4], sI[4];
+  if (lane == 63) {
+    sF[wid] = F;
+    sI[wid] = I;
+  }
+  __syncthreads();
+  float c = -INFINITY;
+  for (int w = 0; w < wid; ++w) c = fmaxf(c + sF[w], sI[w]);
+  c = fmaxf(c + F, I);
+  if (t < nrow) {
+    const long o = (long)h * x.T + row0 + t;
+    x.b[o] = F;
+    x.i[o] = i;
+    x.c[o] = c;
+  }
+  const long ci = (long)ch * a.H + h;
+  if (lane == 63) x.tot[ci * 4 + wid] = F;
+  if (t == MC_L - 1) x.cend[ci] = c;
+}
+
+// s-contiguous tile [rows][64] without padding: 16-byte slots are rotated so
+// that both the pairwise transposing writes (fixed row low bits) and the
+// fragment reads (consecutive rows) spread over the banks
+__device__ __forceinline__ int tslot(int row, int s) {
+  return row * 64 + ((((s >> 3) ^ (row >> 1) ^ (row >> 4)) & 7) << 3) +
+         (s & 7);
+}
+
+// ---- states: U of a chunk, 64 columns per workgroup ------------------------
 template <int DP, bool GATED>
 __global__ void __launch_bounds__(256)
-memory_chunks_kernel(MemoryArgs a) {
-  constexpr int VT = 32;
-  constexpr int NK = DP / 32;          // 32-deep steps over the key size
-  constexpr int MT = DP / 64;          // 16-row state tiles of a wave
-  constexpr int KB = DP * 2 + 16;      // K row pitch (bytes)
-  constexpr int TP = 72;               // pitch of s-contiguous rows
-  constexpr int SP = DP + 8;           // S^T plane pitch (elements)
-  constexpr int CPR = DP / 8;
-  constexpr int PAIRS = 32 * CPR / 256;
-  __shared__ __attribute__((aligned(16))) char kbuf[64 * KB];
-  __shared__ __attribute__((aligned(16))) short ktb[DP * TP];
-  __shared__ __attribute__((aligned(16))) short vtb[VT * TP];
-  __shared__ __attribute__((aligned(16))) short vwb[3][VT * TP];
-  __shared__ __attribute__((aligned(16))) short spl[3][VT * SP];
-  __shared__ float s_a[64], s_M[64], s_in[64], s_w[64], s_em[64];
-  __shared__ float s_n[DP];
-  __shared__ float s_m[2];             // m, and the state factor of a chunk
-
+memory_states_kernel(ChunkArgs x) {
+  constexpr int CPR = DP / 8, PAIRS = 32 * CPR / 256;
+  constexpr int MT = DP / 32, NT = DP / 64;   // m tiles; tiles of a wave
+  const MemoryArgs& a = x.a;
   const int D = a.D, E = a.E;
-  const int nt = (E + VT - 1) / VT;
-  const int vt = blockIdx.x % nt;
-  const int h = blockIdx.x / nt % a.H;
-  const int* sg = a.seg + 4 * (blockIdx.x / nt / a.H);
-  const long slot = sg[0];
-  const int row0 = sg[1], nrow = sg[2], ctx = sg[3];
+  const int nt = (E + 63) / 64;
+  const int et = blockIdx.x % nt, h = blockIdx.x / nt % a.H;
+  const int ch = blockIdx.x / nt / a.H;
+  const int row0 = x.chunks[4 * ch + 1], nrow = x.chunks[4 * ch + 2];
   const int tid = threadIdx.x, lane = tid & 63;
   const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int c16 = lane & 15, g = lane >> 4;
-  const int e0 = vt * VT;
-
-  const short* qp = (const short*)a.q + (long)h * D;
+  const int col = lane & 31, hi = lane >> 5;
+  const int e0 = et * 64;
+  const long ci = (long)ch * a.H + h;
+  __shared__ __attribute__((aligned(16))) short kt[DP * 64];
+  __shared__ __attribute__((aligned(16))) short vw[3][64 * 64];
+  __shared__ float s_w[MC_L];
+  {
+    float w = 0.f;
+    if (tid < nrow) {
+      if (GATED) {
+        const long o = (long)h * x.T + row0 + tid;
+        float d = x.tot[ci * 4 + wid] - x.b[o];
+        for (int j = wid + 1; j < 4; ++j) d += x.tot[ci * 4 + j];
+        w = expf(d + (x.i[o] - x.cend[ci]));
+      } else {
+        w = __builtin_amdgcn_exp2f((nrow - 1 - tid) * a.log2_decay[h]);
+      }
+    }
+    s_w[tid] = w;
+  }
   const short* kp = (const short*)a.k + (long)h * D;
   const short* vp = (const short*)a.v + (long)h * E + e0;
-  const float l2d = GATED ? 0.f : a.log2_decay[h];
-
-  // state: lane holds S[d = 16 (wid MT + i) + 4 g + r][e0 + 16 j + c16]
-  float* Sp = a.S + (slot * a.H + h) * D * E;
-  f32x4 S[MT][2] = {};
-  if (ctx > 0) {
-#pragma unroll
-    for (int i = 0; i < MT; ++i)
-#pragma unroll
-      for (int j = 0; j < 2; ++j)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int d = 16 * (wid * MT + i) + 4 * g + r;
-          const int e = e0 + 16 * j + c16;
-          if (d < D && e < E) S[i][j][r] = Sp[(long)d * E + e];
-        }
-  }
-  float ib = 0.f, fb = 0.f;
-  if (GATED) {
-    for (int d = tid; d < DP; d += 256)
-      s_n[d] = ctx > 0 && d < D ? a.n[((slot * a.H + h) * nt + vt) * D + d] : 0.f;
-    if (tid == 0) s_m[0] = ctx > 0 ? a.m[(slot * a.H + h) * nt + vt] : 0.f;
-    ib = bits2f(((const short*)a.ib)[h]);
-    fb = bits2f(((const short*)a.fb)[h]);
-  }
-
-  // the next chunk's rows travel in registers while this one is computed
+  const uint4v zero = {0, 0, 0, 0};
   uint4v kreg[2 * PAIRS], vreg[2];
-  frag_u qreg[NK];
-  float gi = 0.f, gf = 0.f;
-  const int v_r = tid >> 2 << 1, v_c = (tid & 3) * 8;  // tid < 128
+  const int v_r = tid >> 3 << 1, v_c = (tid & 7) * 8;
   auto issue = [&](int c0) {
-    const int L = min(64, nrow - c0);
-    const uint4v zero = {0, 0, 0, 0};
 #pragma unroll
     for (int p = 0; p < PAIRS; ++p) {
       const int it = p * 256 + tid;
       const int r = it / CPR * 2, c = it % CPR * 8;
 #pragma unroll
-      for (int x = 0; x < 2; ++x)
-        kreg[2 * p + x] = r + x < L && c < D
-            ? *(const uint4v*)(kp + (row0 + c0 + r + x) * a.kst + c) : zero;
-    }
-    if (tid < 128) {
-#pragma unroll
-      for (int x = 0; x < 2; ++x)
-        vreg[x] = v_r + x < L && e0 + v_c < E
-            ? *(const uint4v*)(vp + (row0 + c0 + v_r + x) * a.vst + v_c)
+      for (int y = 0; y < 2; ++y)
+        kreg[2 * p + y] = c0 + r + y < nrow && c < D
+            ? *(const uint4v*)(kp + (long)(row0 + c0 + r + y) * a.kst + c)
             : zero;
     }
-    const int t = 16 * wid + c16;
 #pragma unroll
-    for (int s = 0; s < NK; ++s) {
-      const int d = 32 * s + 8 * g;
-      qreg[s].u4 = t < L && d < D
-          ? *(const uint4v*)(qp + (row0 + c0 + t) * a.qst + d) : zero;
-    }
-    if (GATED && wid == 0) {
-      gi = gf = 0.f;
-      if (lane < L) {
-        const float* gr = a.gates + (long)(row0 + c0 + lane) * 2 * a.H;
-        gi = gr[h];
-        gf = gr[a.H + h];
-      }
-    }
+    for (int y = 0; y < 2; ++y)
+      vreg[y] = c0 + v_r + y < nrow && e0 + v_c < E
+          ? *(const uint4v*)(vp + (long)(row0 + c0 + v_r + y) * a.vst + v_c)
+          : zero;
   };
-
+  f32x16 acc[NT] = {};
+  float nacc = 0.f;
+  const bool with_n = GATED && et == 0;
   issue(0);
   for (int c0 = 0; c0 < nrow; c0 += 64) {
-    const int L = min(64, nrow - c0);
-    __syncthreads();                     // LDS of the previous chunk is free
-
-    // ---- gates / decay weights of the chunk (wave 0, lane = token) -------
-    if (wid == 0) {
-      if (GATED) {
-        float i = -INFINITY, f = 0.f;
-        if (lane < L) {
-          i = a.gate_cap * tanhf((gi + ib) / a.gate_cap);
-          f = log_sigmoid_f(a.gate_cap * tanhf((gf + fb) / a.gate_cap));
-        }
-        float b = f;
-#pragma unroll
-        for (int off = 1; off < 64; off <<= 1) {
-          const float o = __shfl_up(b, off, 64);
-          if (lane >= off) b += o;
-        }
-        const float as = i - b;
-        float M = as;
-#pragma unroll
-        for (int off = 1; off < 64; off <<= 1) {
-          const float o = __shfl_up(M, off, 64);
-          if (lane >= off) M = fmaxf(M, o);
-        }
-        const float m0 = s_m[0];
-        M = fmaxf(M, m0);
-        const float Mc = __shfl(M, 63, 64), bc = __shfl(b, 63, 64);
-        s_a[lane] = as;
-        s_M[lane] = M;
-        s_in[lane] = expf(m0 - M);
-        s_w[lane] = expf(as - Mc);       // 0 past the end (as = -inf)
-        s_em[lane] = expf(-(b + M));
-        if (lane == 63) {
-          s_m[1] = expf(m0 - Mc);
-          s_m[0] = bc + Mc;
-        }
-      } else {
-        s_in[lane] = __builtin_amdgcn_exp2f((lane + 1) * l2d);
-        s_w[lane] = lane < L ? (lane == L - 1 ? 1.f
-            : __builtin_amdgcn_exp2f((L - 1 - lane) * l2d)) : 0.f;
-        if (lane == 0) s_m[1] = __builtin_amdgcn_exp2f(L * l2d);
-      }
-    }
-    // ---- stage K, K^T, and the state's planes ----------------------------
-    frag_u qf[NK];
-#pragma unroll
-    for (int s = 0; s < NK; ++s)
-      qf[s].u4 = GATED ? qreg[s].u4 : silu8(qreg[s].u4);
+    __syncthreads();
 #pragma unroll
     for (int p = 0; p < PAIRS; ++p) {
       const int it = p * 256 + tid;
       const int r = it / CPR * 2, c = it % CPR * 8;
-      union { uint4v u; unsigned short s[8]; } x, y;
-      x.u = GATED ? kreg[2 * p] : silu8(kreg[2 * p]);
-      y.u = GATED ? kreg[2 * p + 1] : silu8(kreg[2 * p + 1]);
-      *(uint4v*)(kbuf + r * KB + c * 2) = x.u;
-      *(uint4v*)(kbuf + (r + 1) * KB + c * 2) = y.u;
+      union { uint4v u; unsigned short s[8]; } y0, y1;
+      y0.u = silu8<!GATED>(kreg[2 * p]);
+      y1.u = silu8<!GATED>(kreg[2 * p + 1]);
 #pragma unroll
       for (int j = 0; j < 8; ++j)
-        *(uint*)(ktb + (c + j) * TP + r) = (uint)x.s[j] | ((uint)y.s[j] << 16);
+        *(uint*)(kt + tslot(c + j, r)) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
     }
-#pragma unroll
-    for (int i = 0; i < MT; ++i)
-#pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        uint w0[3], w1[3];
-        split3(S[i][j][0], S[i][j][1], w0);
-        split3(S[i][j][2], S[i][j][3], w1);
-        const int off =
-            (16 * j + c16) * SP + 16 * (wid * MT + i) + 4 * g;
-#pragma unroll
-        for (int z = 0; z < 3; ++z)
-          *(uint2*)(&spl[z][off]) = uint2{w0[z], w1[z]};
-      }
-    __syncthreads();                     // weights are visible
-
-    // ---- stage V^T and the weighted V planes -----------------------------
-    if (tid < 128) {
-      const uint4v x = GATED ? vreg[0] : silu8(vreg[0]);
-      const uint4v y = GATED ? vreg[1] : silu8(vreg[1]);
-      float xf[8], yf[8];
-      unpack8(x, xf);
-      unpack8(y, yf);
-      const float wx = s_w[v_r], wy = s_w[v_r + 1];
+    {
+      float f0[8], f1[8];
+      unpack8(silu8<!GATED>(vreg[0]), f0);
+      unpack8(silu8<!GATED>(vreg[1]), f1);
+      const float w0 = s_w[c0 + v_r], w1 = s_w[c0 + v_r + 1];
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
         uint w[3];
-        split3(xf[j] * wx, yf[j] * wy, w);
-        const int off = (v_c + j) * TP + v_r;
-        *(uint*)(vtb + off) = pack_bf16x2(xf[j], yf[j]);
+        split3(f0[j] * w0, f1[j] * w1, w);
+        const int o = tslot(v_c + j, v_r);
 #pragma unroll
-        for (int z = 0; z < 3; ++z) *(uint*)(&vwb[z][off]) = w[z];
+        for (int z = 0; z < 3; ++z) *(uint*)(&vw[z][o]) = w[z];
       }
     }
+    __syncthreads();
     if (c0 + 64 < nrow) issue(c0 + 64);
-
-    // ---- scores^T of this wave's 16 queries against s <= t ---------------
-    const int t = 16 * wid + c16;
-    f32x4 P[4] = {};
 #pragma unroll
-    for (int st = 0; st < 4; ++st) {
-      if (st > wid) continue;            // wave-uniform
+    for (int kk = 0; kk < 4; ++kk) {
 #pragma unroll
-      for (int s = 0; s < NK; ++s) {
+      for (int y = 0; y < NT; ++y) {
+        const int tile = wid + 4 * y;
+        const int m = tile % MT, n = tile / MT;
         frag_u kf;
-        kf.u4 = *(const uint4v*)(kbuf + (16 * st + c16) * KB +
-                                 (32 * s + 8 * g) * 2);
-        P[st] = mfma16(kf, qf[s], P[st]);
+        kf.u4 = *(const uint4v*)(kt + tslot(32 * m + col, 16 * kk + 8 * hi));
+#pragma unroll
+        for (int z = 0; z < 3; ++z) {
+          frag_u vf;
+          vf.u4 = *(const uint4v*)(
+              &vw[z][tslot(32 * n + col, 16 * kk + 8 * hi)]);
+          acc[y] = mfma_bf16(kf.bf, vf.bf, acc[y]);
+        }
       }
     }
-    const float qs = GATED ? a.qscale : 1.f;
-    const float Mt = GATED ? s_M[t] : 0.f;
-    float rowsum = 0.f;
+    if (with_n && tid < DP) {
 #pragma unroll
-    for (int st = 0; st < 4; ++st)
+      for (int s = 0; s < 64; s += 8) {
+        float kv[8];
+        unpack8(*(const uint4v*)(kt + tslot(tid, s)), kv);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int s = 16 * st + 4 * g + r;
-        float w = 0.f;
-        if (s <= t && st <= wid) {
-          if (GATED) w = __expf(s_a[s] - Mt) * qs;
-          else w = s == t ? 1.f : __builtin_amdgcn_exp2f((t - s) * l2d);
-        }
-        P[st][r] *= w;
-        rowsum += P[st][r];
+        for (int j = 0; j < 8; ++j) nacc += s_w[c0 + s + j] * kv[j];
       }
-
-    // ---- the carried state's part ----------------------------------------
-    f32x4 O[2] = {};
+    }
+  }
+  float* U = x.U + ci * E * D;
 #pragma unroll
-    for (int j = 0; j < 2; ++j)
+  for (int y = 0; y < NT; ++y) {
+    const int tile = wid + 4 * y;
+    const int m = tile % MT, e = e0 + 32 * (tile / MT) + col;
+    if (e >= E) continue;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = 32 * m + 8 * r + 4 * hi;
+      if (d < D)
+        *(f32x4*)(U + (long)e * D + d) =
+            f32x4{acc[y][4 * r], acc[y][4 * r + 1], acc[y][4 * r + 2],
+                  acc[y][4 * r + 3]};
+    }
+  }
+  if (with_n && tid < D) x.N[ci * D + tid] = nacc;
+}
+
+// ---- scan over the chunks of a segment: tiles of 64 keys x 16 columns ------
+template <bool GATED>
+__global__ void __launch_bounds__(256)
+memory_scan_kernel(ChunkArgs x) {
+  const MemoryArgs& a = x.a;
+  const int D = a.D, E = a.E;
+  const int nd = (D + 63) / 64, ne = (E + 15) / 16;
+  const int dt = blockIdx.x % nd, et = blockIdx.x / nd % ne;
+  const int h = blockIdx.x / nd / ne % a.H;
+  const int sg = blockIdx.x / nd / ne / a.H;
+  const long slot = a.seg[4 * sg];
+  const int ctx = a.seg[4 * sg + 3];
+  const int tid = threadIdx.x;
+  const int d = dt * 64 + (tid & 15) * 4, e = et * 16 + (tid >> 4);
+  const bool live = d < D && e < E;
+  const int nt = (E + 31) / 32;
+  float* Sp = a.S + (slot * a.H + h) * D * E;
+  __shared__ float tr[64][17];
+  f32x4 S = {0.f, 0.f, 0.f, 0.f};
+  float m = 0.f;
+  if (ctx > 0) {
+    for (int i = tid; i < 64 * 16; i += 256) {
+      const int dd = dt * 64 + i / 16, ee = et * 16 + i % 16;
+      tr[i / 16][i % 16] = dd < D && ee < E ? Sp[(long)dd * E + ee] : 0.f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < 4; ++j) S[j] = tr[(tid & 15) * 4 + j][tid >> 4];
+    __syncthreads();
+    if (GATED) m = a.m[(slot * a.H + h) * nt];
+  }
+  // the first column tile also carries n
+  const bool with_n = GATED && et == 0 && tid < 64 && dt * 64 + tid < D;
+  float n = 0.f;
+  const long nat = (slot * a.H + h) * nt * D + dt * 64 + tid;
+  if (with_n && ctx > 0) n = a.n[nat];
+  const int c1 = x.first[sg + 1];
+  f32x4 Un = {0.f, 0.f, 0.f, 0.f};
+  int ch = x.first[sg];
+  if (live && ch < c1)
+    Un = *(const f32x4*)(x.U + ((long)ch * a.H + h) * E * D + (long)e * D + d);
+  for (; ch < c1; ++ch) {
+    const long ci = (long)ch * a.H + h;
+    const f32x4 U = Un;
+    if (live && ch + 1 < c1)
+      Un = *(const f32x4*)(x.U + (ci + a.H) * E * D + (long)e * D + d);
+    if (live && x.chunks[4 * ch + 3]) {
+      uint w0[3], w1[3];
+      split3(S[0], S[1], w0);
+      split3(S[2], S[3], w1);
+#pragma unroll
+      for (int z = 0; z < 3; ++z)
+        *(uint2*)(x.P + ((ci * 3 + z) * E + e) * D + d) = uint2{w0[z], w1[z]};
+    }
+    float fs, us = 1.f;
+    if (GATED) {
+      const float* tt = x.tot + ci * 4;
+      const float bm = tt[0] + tt[1] + tt[2] + tt[3] + m, ce = x.cend[ci];
+      const float mn = fmaxf(bm, ce);
+      fs = expf(bm - mn);
+      us = expf(ce - mn);
+      if (blockIdx.x % (nd * ne) == 0 && tid == 0) x.mst[ci] = m;
+      if (with_n) {
+        const long o = ci * D + dt * 64 + tid;
+        const float N = x.N[o];
+        x.N[o] = n;
+        n = fs * n + us * N;
+      }
+      m = mn;
+    } else {
+      fs = __builtin_amdgcn_exp2f(x.chunks[4 * ch + 2] * a.log2_decay[h]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) S[j] = fs * S[j] + us * U[j];
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) tr[(tid & 15) * 4 + j][tid >> 4] = S[j];
+  __syncthreads();
+  for (int i = tid; i < 64 * 16; i += 256) {
+    const int dd = dt * 64 + i / 16, ee = et * 16 + i % 16;
+    if (dd < D && ee < E) Sp[(long)dd * E + ee] = tr[i / 16][i % 16];
+  }
+  if (with_n)
+    for (int j = 0; j < nt; ++j) a.n[nat + (long)j * D] = n;
+}
+
+// m has one reader group per segment and head; it is stored last
+__global__ void __launch_bounds__(64)
+memory_last_m_kernel(ChunkArgs x) {
+  const MemoryArgs& a = x.a;
+  const int nt = (a.E + 31) / 32;
+  const int h = blockIdx.x % a.H, sg = blockIdx.x / a.H;
+  const int ch = x.first[sg + 1] - 1;
+  const long ci = (long)ch * a.H + h;
+  const float* tt = x.tot + ci * 4;
+  const float m = fmaxf(tt[0] + tt[1] + tt[2] + tt[3] + x.mst[ci], x.cend[ci]);
+  for (int j = threadIdx.x; j < nt; j += 64)
+    a.m[((long)a.seg[4 * sg] * a.H + h) * nt + j] = m;
+}
+
+// ---- outputs: 128 queries x VT columns per workgroup -----------------------
+template <int DP, int VT, bool GATED>
+__global__ void __launch_bounds__(256, DP <= 128 ? 2 : 1)
+memory_outputs_kernel(ChunkArgs x) {
+  constexpr int NC = DP / 16, NB = VT / 32;
+  constexpr int KP = DP * 2;             // K row pitch (bytes)
+  constexpr int CPR = DP / 8, PAIRS = 32 * CPR / 256;
+  constexpr int VC = VT / 8, VPAIRS = 32 * VC / 256;
+  constexpr int KV_B = 64 * KP + VT * 64 * 2;
+  constexpr int ST_B = 3 * 32 * KP;
+  const MemoryArgs& a = x.a;
+  const int D = a.D, E = a.E;
+  const int nt = (E + VT - 1) / VT;
+  const int et = blockIdx.x % nt, half = blockIdx.x / nt % 2;
+  const int h = blockIdx.x / nt / 2 % a.H, ch = blockIdx.x / nt / 2 / a.H;
+  const int row0 = x.chunks[4 * ch + 1], nrow = x.chunks[4 * ch + 2];
+  const bool carried = x.chunks[4 * ch + 3];
+  if (half * 128 >= nrow) return;        // the whole workgroup
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int col = lane & 31, hi = lane >> 5;
+  const int e0 = et * VT;
+  const long ci = (long)ch * a.H + h;
+  const int t = half * 128 + wid * 32 + col;   // place in the chunk
+  const int jt = half * 2 + (wid >> 1);        // its 64-token group
+  __shared__ __attribute__((aligned(16))) char
+      buf[KV_B > ST_B ? KV_B : ST_B];
+  char* kb = buf;
+  short* vb = (short*)(buf + 64 * KP);
+  __shared__ float s_col[64];
+  __shared__ float s_n[GATED ? DP : 1];
+  auto kswz = [](int row, int byte) {
+    return CPR >= 16 ? swz16(row, byte) : swz(row, byte);
+  };
+
+  frag_u qf[NC];
+  {
+    const short* src = (const short*)a.q + (long)(row0 + min(t, nrow - 1)) *
+                       a.qst + (long)h * D;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      const int d = c * 16 + hi * 8;
+      qf[c].u4 = d < D ? silu8<!GATED>(*(const uint4v*)(src + d))
+                       : uint4v{0, 0, 0, 0};
+    }
+  }
+  // row terms of the weights
+  float row = 0.f, inter, em = 0.f, l2d = 0.f;
+  const float qs = GATED ? a.qscale : 1.f;
+  float tot[4];
+  if (GATED) {
+    const long o = (long)h * x.T + row0 + min(t, nrow - 1);
+    float before = x.mst[ci];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      tot[j] = x.tot[ci * 4 + j];
+      if (j < jt) before += tot[j];
+    }
+    const float bt = x.b[o];
+    const float mt = fmaxf(bt + before, x.c[o]);
+    inter = __expf(bt + before - mt) * qs;
+    row = bt - mt;
+    em = expf(-mt);
+  } else {
+    l2d = a.log2_decay[h];
+    inter = __builtin_amdgcn_exp2f((t + 1) * l2d);
+  }
+
+  f32x16 ot[NB] = {};
+  float den = 0.f;
+  if (carried) {
+    // the carried state: its planes pass through LDS 32 columns at a time
+    if (GATED) {
+      for (int d = tid; d < DP; d += 256)
+        s_n[d] = d < D ? x.N[ci * D + d] : 0.f;
+    }
+    const short* P = x.P + ci * 3 * E * D;
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb) {
+      if (e0 + 32 * nb >= E) continue;   // uniform
+      __syncthreads();
+#pragma unroll
+      for (int i = 0; i < 3 * 32 * CPR / 256; ++i) {
+        const int it = i * 256 + tid;
+        const int c = it % CPR * 8, r = it / CPR;     // r: plane * 32 + row
+        const int e = e0 + 32 * nb + (r & 31);
+        *(uint4v*)(buf + r * KP + kswz(r & 31, c * 2)) = e < E && c < D
+            ? *(const uint4v*)(P + ((long)(r >> 5) * E + e) * D + c)
+            : uint4v{0, 0, 0, 0};
+      }
+      __syncthreads();
 #pragma unroll
       for (int z = 0; z < 3; ++z)
 #pragma unroll
-        for (int s = 0; s < NK; ++s) {
+        for (int c = 0; c < NC; ++c) {
           frag_u sf;
-          sf.u4 = *(const uint4v*)(&spl[z][(16 * j + c16) * SP + 32 * s +
-                                           8 * g]);
-          O[j] = mfma16(sf, qf[s], O[j]);
+          sf.u4 = *(const uint4v*)(buf + (z * 32 + col) * KP +
+                                   kswz(col, (c * 16 + hi * 8) * 2));
+          ot[nb] = mfma_bf16(sf.bf, qf[c].bf, ot[nb]);
         }
-    const float in = s_in[t] * qs;
-    O[0] *= in;
-    O[1] *= in;
-    float den = 1.f;
+      ot[nb] *= inter;
+    }
     if (GATED) {
-      float nq = 0.f;
 #pragma unroll
-      for (int s = 0; s < NK; ++s) {
+      for (int c = 0; c < NC; ++c) {
         float qv[8];
-        unpack8(qf[s].u4, qv);
+        unpack8(qf[c].u4, qv);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) nq += qv[j] * s_n[32 * s + 8 * g + j];
+        for (int j = 0; j < 8; ++j) den += qv[j] * s_n[c * 16 + hi * 8 + j];
       }
-      float d = rowsum + nq * in;
-      d += __shfl_xor(d, 16, 64);
-      d += __shfl_xor(d, 32, 64);
-      den = 1.f / (fmaxf(fabsf(d), s_em[t]) + GATED_EPS);
+      den *= inter;
     }
-    __syncthreads();                     // V^T is staged; s_n was read
+  }
 
-    // ---- the chunk's own part --------------------------------------------
+  // ---- keys of the chunk, 64 at a time, from the newest back ---------------
+  const short* kp = (const short*)a.k + (long)h * D;
+  const short* vp = (const short*)a.v + (long)h * E + e0;
+  const uint4v zero = {0, 0, 0, 0};
+  uint4v kreg[2 * PAIRS], vreg[2 * VPAIRS];
+  float colr = 0.f;
+  auto issue = [&](int J) {
+    const int c0 = 64 * J;
 #pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
-      if (2 * kk > wid) continue;
-      frag_u pf[3];
+    for (int p = 0; p < PAIRS; ++p) {
+      const int it = p * 256 + tid;
+      const int r = it / CPR * 2, c = it % CPR * 8;
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        const f32x4& p = P[2 * kk + (u >> 1)];
-        uint w[3];
-        split3(p[2 * (u & 1)], p[2 * (u & 1) + 1], w);
+      for (int y = 0; y < 2; ++y)
+        kreg[2 * p + y] = c0 + r + y < nrow && c < D
+            ? *(const uint4v*)(kp + (long)(row0 + c0 + r + y) * a.kst + c)
+            : zero;
+    }
 #pragma unroll
-        for (int z = 0; z < 3; ++z) pf[z].u[u] = w[z];
-      }
+    for (int p = 0; p < VPAIRS; ++p) {
+      const int it = p * 256 + tid;
+      const int r = it / VC * 2, c = it % VC * 8;
 #pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        const short* vr = vtb + (16 * j + c16) * TP + 32 * kk + 4 * g;
-        frag_u vf;
-        *(uint2*)&vf.u[0] = *(const uint2*)vr;
-        *(uint2*)&vf.u[2] = *(const uint2*)(vr + 16);
-#pragma unroll
-        for (int z = 0; z < 3; ++z) O[j] = mfma16(vf, pf[z], O[j]);
+      for (int y = 0; y < 2; ++y)
+        vreg[2 * p + y] = c0 + r + y < nrow && e0 + c < E
+            ? *(const uint4v*)(vp + (long)(row0 + c0 + r + y) * a.vst + c)
+            : zero;
+    }
+    if (GATED && tid < 64) {
+      colr = -INFINITY;
+      if (c0 + tid < nrow) {
+        const long o = (long)h * x.T + row0 + c0 + tid;
+        colr = x.i[o] - x.b[o];
       }
     }
-    if (t < L) {
-      short* dst = (short*)a.out + ((long)(row0 + c0 + t) * a.H + h) * E + e0;
+  };
+  const int J1 = min(half * 2 + 1, (nrow - 1) / 64);
+  issue(J1);
+  for (int J = J1; J >= 0; --J) {
+    __syncthreads();
 #pragma unroll
-      for (int j = 0; j < 2; ++j)
-        if (e0 + 16 * j + 4 * g < E)
-          *(uint2*)(dst + 16 * j + 4 * g) =
-              uint2{pack_bf16x2(O[j][0] * den, O[j][1] * den),
-                    pack_bf16x2(O[j][2] * den, O[j][3] * den)};
+    for (int p = 0; p < PAIRS; ++p) {
+      const int it = p * 256 + tid;
+      const int r = it / CPR * 2, c = it % CPR * 8;
+#pragma unroll
+      for (int y = 0; y < 2; ++y)
+        *(uint4v*)(kb + (r + y) * KP + kswz(r + y, c * 2)) =
+            silu8<!GATED>(kreg[2 * p + y]);
     }
+#pragma unroll
+    for (int p = 0; p < VPAIRS; ++p) {
+      const int it = p * 256 + tid;
+      const int r = it / VC * 2, c = it % VC * 8;
+      union { uint4v u; unsigned short s[8]; } y0, y1;
+      y0.u = silu8<!GATED>(vreg[2 * p]);
+      y1.u = silu8<!GATED>(vreg[2 * p + 1]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        *(uint*)(vb + tslot(c + j, r)) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
+    }
+    if (GATED && tid < 64) s_col[tid] = colr;
+    __syncthreads();
+    if (J > 0) issue(J - 1);
+    if (J > jt || half * 128 + wid * 32 >= nrow) continue;  // wave-uniform
 
-    // ---- advance the state -----------------------------------------------
-    const float fac = s_m[1];
+    // row part of the exponent for keys of group J
+    float base = row;
+    if (GATED && J < jt) {
 #pragma unroll
-    for (int i = 0; i < MT; ++i) {
-      frag_u kf[2];
+      for (int j = 0; j < 4; ++j)
+        if (j >= J && j < jt) base += tot[j];
+    }
+    f32x16 acc[2] = {};
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk)
-        kf[kk].u4 = *(const uint4v*)(ktb + (16 * (wid * MT + i) + c16) * TP +
-                                     32 * kk + 8 * g);
+    for (int k2 = 0; k2 < 2; ++k2) {
+      const int r = col + 32 * k2;
 #pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        S[i][j] *= fac;
-#pragma unroll
-        for (int z = 0; z < 3; ++z)
-#pragma unroll
-          for (int kk = 0; kk < 2; ++kk) {
-            frag_u vf;
-            vf.u4 = *(const uint4v*)(&vwb[z][(16 * j + c16) * TP + 32 * kk +
-                                             8 * g]);
-            S[i][j] = mfma16(kf[kk], vf, S[i][j]);
-          }
+      for (int c = 0; c < NC; ++c) {
+        frag_u kf;
+        kf.u4 = *(const uint4v*)(kb + r * KP + kswz(r, (c * 16 + hi * 8) * 2));
+        acc[k2] = mfma_bf16(kf.bf, qf[c].bf, acc[k2]);
       }
     }
-    if (GATED) {
-      for (int d = tid; d < DP; d += 256) {
-        float n = fac * s_n[d];
 #pragma unroll
-        for (int s = 0; s < 64; s += 8) {
-          float kv[8];
-          unpack8(*(const uint4v*)(ktb + d * TP + s), kv);
+    for (int k2 = 0; k2 < 2; ++k2)
 #pragma unroll
-          for (int j = 0; j < 8; ++j) n += s_w[s + j] * kv[j];
+      for (int r = 0; r < 16; ++r) {
+        const int s = 32 * k2 + acc_row(r, hi);
+        float w;
+        if (GATED) w = __expf(base + s_col[s]) * qs;
+        else w = __builtin_amdgcn_exp2f((float)(t - 64 * J - s) * l2d);
+        if (J == jt && 64 * J + s > t) w = 0.f;
+        acc[k2][r] *= w;
+        if (GATED) den += acc[k2][r];
+      }
+#pragma unroll
+    for (int k2 = 0; k2 < 2; ++k2)
+#pragma unroll
+      for (int cc = 0; cc < 2; ++cc) {
+        frag_u pf[3];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          uint w[3];
+          split3(acc[k2][8 * cc + 2 * u], acc[k2][8 * cc + 2 * u + 1], w);
+#pragma unroll
+          for (int z = 0; z < 3; ++z) pf[z].u[u] = w[z];
         }
-        s_n[d] = n;
+        const int s = 32 * k2 + 16 * cc + 4 * hi;
+#pragma unroll
+        for (int nb = 0; nb < NB; ++nb) {
+          frag_u vf;
+          *(uint2*)&vf.u[0] = *(const uint2*)(vb + tslot(32 * nb + col, s));
+          *(uint2*)&vf.u[2] =
+              *(const uint2*)(vb + tslot(32 * nb + col, s + 8));
+#pragma unroll
+          for (int z = 0; z < 3; ++z)
+            ot[nb] = mfma_bf16(vf.bf, pf[z].bf, ot[nb]);
+        }
       }
-    }
   }
 
-#pragma unroll
-  for (int i = 0; i < MT; ++i)
-#pragma unroll
-    for (int j = 0; j < 2; ++j)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = 16 * (wid * MT + i) + 4 * g + r;
-        const int e = e0 + 16 * j + c16;
-        if (d < D && e < E) Sp[(long)d * E + e] = S[i][j][r];
-      }
+  float inv = 1.f;
   if (GATED) {
-    for (int d = tid; d < D; d += 256)
-      a.n[((slot * a.H + h) * nt + vt) * D + d] = s_n[d];
-    if (tid == 0) a.m[(slot * a.H + h) * nt + vt] = s_m[0];
+    den += __shfl_xor(den, 32, 64);
+    inv = 1.f / (fmaxf(fabsf(den), em) + GATED_EPS);
   }
+  if (t >= nrow) return;
+  short* dst = (short*)a.out + ((long)(row0 + t) * a.H + h) * E + e0;
+#pragma unroll
+  for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+    for (int rg = 0; rg < 4; ++rg) {
+      const int e = 32 * nb + 8 * rg + 4 * hi;
+      if (e0 + e < E)
+        *(uint2*)(dst + e) =
+            uint2{pack_bf16x2(ot[nb][4 * rg] * inv, ot[nb][4 * rg + 1] * inv),
+                  pack_bf16x2(ot[nb][4 * rg + 2] * inv,
+                              ot[nb][4 * rg + 3] * inv)};
+    }
+}
+
+template <int DP, bool GATED>
+static void launch_chunks(const ChunkArgs& x, hipStream_t stream) {
+  const MemoryArgs& a = x.a;
+  const long ch = (long)x.n_chunks * a.H;
+  if (GATED) memory_gates_kernel<<<ch, MC_L, 0, stream>>>(x);
+  memory_states_kernel<DP, GATED>
+      <<<ch * ((a.E + 63) / 64), 256, 0, stream>>>(x);
+  memory_scan_kernel<GATED><<<(long)x.n_seg * a.H * ((a.D + 63) / 64) *
+                                  ((a.E + 15) / 16), 256, 0, stream>>>(x);
+  if (GATED)
+    memory_last_m_kernel<<<(long)x.n_seg * a.H, 64, 0, stream>>>(x);
+  if (a.E <= 64)
+    memory_outputs_kernel<DP, 64, GATED><<<ch * 2, 256, 0, stream>>>(x);
+  else
+    memory_outputs_kernel<DP, 128, GATED>
+        <<<ch * 2 * ((a.E + 127) / 128), 256, 0, stream>>>(x);
 }
 
 // bf16; D and E multiples of 8 with D <= 256; 16-byte aligned rows
-extern "C" int sv_memory_chunks(const MemoryArgs* a, int n_seg, int gated,
+extern "C" int sv_memory_chunks(const ChunkArgs* x, int gated,
                                 hipStream_t stream) {
-  if (n_seg <= 0) return 0;
-  const long grid = (long)n_seg * a->H * ((a->E + 31) / 32);
-#define MC(P)                                                              \
-  do {                                                                     \
-    if (gated) memory_chunks_kernel<P, true><<<grid, 256, 0, stream>>>(*a); \
-    else memory_chunks_kernel<P, false><<<grid, 256, 0, stream>>>(*a);      \
+  if (x->n_seg <= 0) return 0;
+#define MC(P)                                                     \
+  do {                                                            \
+    if (gated) launch_chunks<P, true>(*x, stream);                \
+    else launch_chunks<P, false>(*x, stream);                     \
   } while (0)
-  if (a->D <= 64) MC(64);
-  else if (a->D <= 128) MC(128);
-  else if (a->D <= 256) MC(256);
+  if (x->a.D <= 64) MC(64);
+  else if (x->a.D <= 128) MC(128);
+  else if (x->a.D <= 256) MC(256);
   else return 1;
 #undef MC
   return (int)hipGetLastError();

@@ -346,7 +346,7 @@ struct TilesArgs {
 };
 
 template <int DP, int NP>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, DP <= 128 ? 2 : 1)
 attn_tiles_kernel(TilesArgs a) {
   constexpr int NC = DP / 16;        // 16-wide chunks of the head size
   constexpr int NB = DP / 32;        // 32-row blocks of O^T
@@ -357,7 +357,8 @@ attn_tiles_kernel(TilesArgs a) {
   __shared__ __attribute__((aligned(16))) char kbuf[64 * KP];
   __shared__ __attribute__((aligned(16))) short vbuf[DP * VP];
 
-  const int* tl = a.tiles + 4 * blockIdx.y;
+  // later tiles of a portion see more keys: they start first
+  const int* tl = a.tiles + 4 * (gridDim.y - 1 - blockIdx.y);
   const int seq = tl[0], row0 = tl[1], nrow = tl[2], p0 = tl[3];
   const int h = blockIdx.x, g = h / (a.H / a.G);
   const int* bt = a.bt + (long)seq * a.MB;

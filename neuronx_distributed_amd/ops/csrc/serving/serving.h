@@ -68,12 +68,12 @@ __device__ __forceinline__ void load8<true, short>(const short* p, int n,
   for (int j = 0; j < 8; ++j) v[j] = bits2f(a[j]);
 }
 
-__device__ __forceinline__ float silu_f(float x) {
-  return x / (1.f + __expf(-x));
-}
+// v_rcp_f32 and v_exp_f32 are good to one unit in the last place
 __device__ __forceinline__ float sigmoid_f(float x) {
-  return 1.f / (1.f + __expf(-x));
+  return __builtin_amdgcn_rcpf(1.f +
+                               __builtin_amdgcn_exp2f(-x * SV_LOG2E));
 }
+__device__ __forceinline__ float silu_f(float x) { return x * sigmoid_f(x); }
 // log(sigmoid(x)), stable on both sides
 __device__ __forceinline__ float log_sigmoid_f(float x) {
   return fminf(x, 0.f) - log1pf(expf(-fabsf(x)));

@@ -17,7 +17,7 @@ import torch
 
 PAGE_SIZE = 64
 MAX_HEAD_DIM = 512          # attention q/k and v size, recurrent q/k size
-_TILE_ROWS = 128
+CHUNK = 256                 # tokens of one chunk of a matrix memory
 
 _LIB = None
 
@@ -99,6 +99,12 @@ class _MemoryArgs(ctypes.Structure):
                           ctypes.c_void_p)
                 + _fields("H D E", ctypes.c_int)
                 + _fields("gate_cap qscale", ctypes.c_float))
+
+
+class _ChunkArgs(ctypes.Structure):
+    _fields_ = ([("a", _MemoryArgs)] + _fields("chunks first", ctypes.c_void_p)
+                + _fields("n_chunks n_seg T", ctypes.c_int)
+                + _fields("b i c tot cend U N P mst", ctypes.c_void_p))
 
 
 # ---------------------------------------------------------------------------
@@ -328,16 +334,30 @@ class ExpGate:
     qscale: float
 
 
+def chunk_table(segments):
+    """Chunks of prompt portions: rows (segment, first row, rows, does a
+    state come in) and the first chunk of every segment, from rows (slot,
+    first row, rows, context)."""
+    rows, first = [], [0]
+    for i, (_, r0, n, ctx) in enumerate(segments):
+        for at in range(0, n, CHUNK):
+            rows.append((i, r0 + at, min(CHUNK, n - at),
+                         int(at > 0 or ctx > 0)))
+        first.append(len(rows))
+    return rows, first
+
+
 def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
-               chunked: bool,
+               chunks: Optional[torch.Tensor] = None,
+               chunk_first: Optional[torch.Tensor] = None,
                out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Run a matrix memory over segments of a ragged batch.  q, k (T, H*D),
     v (T, H*E); S (slots, H, D, E) float32; n (slots, H, ceil(E/32), D) and
     m (slots, H, ceil(E/32)) float32 for an ExpGate.  ``seg`` (n, 4) int32
     lists (slot, first row, rows, context); rows count from the start of
     the tensors, so portions and single tokens of one batch can be run by
-    two calls into one ``out``.  ``chunked`` uses the 64-token
-    MFMA kernel where it applies."""
+    two calls into one ``out``.  With the device form of
+    ``chunk_table`` the 256-token MFMA kernels run where they apply."""
     D, E = S.shape[2], S.shape[3]
     T = q.shape[0]
     assert q.shape[1] == k.shape[1] == heads * D and v.shape[1] == heads * E
@@ -364,10 +384,25 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
         assert gate.decay.shape == (heads,)
         a.decay, a.log2_decay = _p(gate.decay), _p(gate.log2_decay)
     lib = library()
-    if (chunked and q.dtype == torch.bfloat16 and D <= 256
+    if (chunks is not None and q.dtype == torch.bfloat16 and D <= 256
             and _aligned((D, E), q, k, v)):
-        st = lib.sv_memory_chunks(ctypes.byref(a), seg.shape[0], int(gated),
-                                  _stream())
+        nc = chunks.shape[0]
+        assert chunk_first.shape[0] == seg.shape[0] + 1
+        f32 = dict(dtype=torch.float32, device=q.device)
+        U = torch.empty(nc, heads, E, D, **f32)
+        P = torch.empty(nc, heads, 3, E, D, dtype=torch.bfloat16,
+                        device=q.device)
+        x = _ChunkArgs(a=a, chunks=_p(chunks), first=_p(chunk_first),
+                       n_chunks=nc, n_seg=seg.shape[0], T=T, U=_p(U),
+                       P=_p(P))
+        if gated:
+            bic = torch.empty(3, heads, T, **f32)
+            small = torch.empty(nc, heads, 6 + D, **f32)
+            x.b, x.i, x.c = (_p(t) for t in bic)
+            flat, nh = small.view(-1), nc * heads
+            x.tot, x.cend = _p(flat), _p(flat[4 * nh:])
+            x.mst, x.N = _p(flat[5 * nh:]), _p(flat[6 * nh:])
+        st = lib.sv_memory_chunks(ctypes.byref(x), int(gated), _stream())
     else:
         st = lib.sv_memory_steps(ctypes.byref(a), seg.shape[0], int(gated),
                                  _f32(q), _stream())
@@ -377,4 +412,6 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
 
 def decay_gate(decay, device) -> DecayGate:
     d = torch.tensor([float(x) for x in decay], dtype=torch.float64)
-    return DecayGate(d.float().to(device), torch.log2(d).float().to(device))
+    # finite for a decay of zero: 0 tokens apart must still weigh 2^0
+    log2 = torch.log2(d).clamp(min=-1e4)
+    return DecayGate(d.float().to(device), log2.float().to(device))

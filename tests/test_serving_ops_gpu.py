@@ -215,26 +215,35 @@ def _mem_inputs(H, D, E, T, dtype, seed=0):
     return p[:, :H * D], p[:, H * D:2 * H * D], p[:, 2 * H * D:][:, :H * E], p
 
 
+def _tables(sv, seg, chunked):
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32).cuda()
+    return (i32(seg), *map(i32, sv.chunk_table(seg))) if chunked \
+        else (i32(seg),)
+
+
 def _run_memory(sv, proj, sizes, cuts, H, gate_of, S, n, m, slot):
     outs, at = [], 0
     for c in cuts:
         part = proj[at:at + c].cuda()
         a, b, w = sizes
         q, k, v = part[:, :a], part[:, a:a + b], part[:, a + b:a + b + w]
-        seg = torch.tensor([[slot, 0, c, at]], dtype=torch.int32).cuda()
-        outs.append(sv.memory_mix(q, k, v, gate_of(at, c), S, n, m, seg, H,
-                                  chunked=c > 1))
+        seg = [(slot, 0, c, at)]
+        outs.append(sv.memory_mix(q, k, v, gate_of(at, c), S, n, m,
+                                  *_tables(sv, seg, c > 1)[:1], H,
+                                  *_tables(sv, seg, c > 1)[1:]))
         at += c
     return torch.cat(outs)
 
 
-CUTS = ([200], [64, 2, 62, 3, 65, 4], [100] + [1] * 100, [1, 1, 2, 128, 68])
+T_MEM = 600
+CUTS = ([T_MEM], [64, 2, 190, 3, 257, 84], [500] + [1] * 100,
+        [1, 1, 2, 256, 128, 212], [255, 256, 89])
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,D,E", MEM)
 def test_decayed_memory(sv, H, D, E, dtype):
-    T = 200
+    T = T_MEM
     decay = [0.0, 1.0, 0.97, 0.6, 0.999][:H] if H > 2 else [0.998, 0.5][:H]
     q, k, v, p = _mem_inputs(H, D, E, T, dtype, seed=7)
     d = lambda t, s: vo.silu(t.double()).view(T, H, s)
@@ -264,7 +273,7 @@ def _gates(H, T, i_scale, f_shift, seed=0):
                                              (3.0, -8.0), (0.1, 12.0)])
 @pytest.mark.parametrize("H,D,E", MEM)
 def test_gated_memory(sv, H, D, E, i_scale, f_shift, dtype):
-    T, cap = 200, 5.0 if H == 3 else 15.0
+    T, cap = T_MEM, 5.0 if H == 3 else 15.0
     q, k, v, p = _mem_inputs(H, D, E, T, dtype, seed=9)
     raw = _gates(H, T, i_scale, f_shift, seed=H)
     raw[37] = 40.0                 # one input stands out and is carried on
@@ -299,7 +308,7 @@ def test_gated_memory(sv, H, D, E, i_scale, f_shift, dtype):
                           m, slot=1)
         c = cond.unsqueeze(2)
         got = got.double().cpu().view(T, H, E)
-        _close(want + (got - want) / c, want, torch.float32, 6.0,
+        _close(want + (got - want) / c, want, torch.float32, 20.0,
                (H, D, E, cuts[:4])) if dtype == torch.float32 else \
             _close(got, want, dtype, 2.0, (H, D, E, cuts[:4]))
         assert (m[1].double().cpu() - m_w.view(H, 1)).abs().max() < 2e-3
@@ -314,7 +323,7 @@ def test_memory_batch_and_slots(sv, dtype, gated):
     """Segments of unequal length in one call equal each alone, whatever
     slots they use."""
     H, D, E = 2, 32, 48
-    lens, slots = [70, 2, 129, 64], [3, 0, 4, 1]
+    lens, slots = [70, 2, 529, 64], [3, 0, 4, 1]
     T = sum(lens)
     q, k, v, p = _mem_inputs(H, D, E, T, dtype, seed=11)
     raw = _gates(H, T, 1.0, 2.0).cuda()
@@ -332,15 +341,15 @@ def test_memory_batch_and_slots(sv, dtype, gated):
     pc = p.cuda()
     cut = lambda t: (t[:, :H * D], t[:, H * D:2 * H * D],
                      t[:, 2 * H * D:2 * H * D + H * E])
-    seg = torch.tensor([(s, a, n, 0) for s, a, n in
-                        zip(slots, starts, lens)], dtype=torch.int32).cuda()
+    seg, *tab = _tables(sv, [(s, a, n, 0) for s, a, n in
+                             zip(slots, starts, lens)], True)
     S, n, m = mk()
-    both = sv.memory_mix(*cut(pc), gate(0, T), S, n, m, seg, H, True)
+    both = sv.memory_mix(*cut(pc), gate(0, T), S, n, m, seg, H, *tab)
     for s, a, ln in zip(slots, starts, lens):
         S1, n1, m1 = mk()
-        one = torch.tensor([(0, 0, ln, 0)], dtype=torch.int32).cuda()
+        one, *tab = _tables(sv, [(0, 0, ln, 0)], True)
         alone = sv.memory_mix(*cut(pc[a:a + ln]), gate(a, a + ln), S1, n1,
-                              m1, one, H, True)
+                              m1, one, H, *tab)
         assert torch.equal(alone, both[a:a + ln])
         assert torch.equal(S1[0], S[s])
 
