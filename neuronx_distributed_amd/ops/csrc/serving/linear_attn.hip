@@ -267,6 +267,8 @@ struct ChunkArgs {
   float* N;                 // [n_chunks][H][D] (gated): N, then n before
   short* P;                 // [n_chunks][H][3][E][D] state before the chunk
   float* mst;               // [n_chunks][H] m before the chunk (gated)
+  short* VT;                // [n_chunks][H][E][256] V^T, activated
+  short* KA;                // [T][H][D] activated K (decay)
 };
 
 // split a pair of floats into three planes of packed bf16
@@ -338,14 +340,6 @@ memory_gates_kernel(ChunkArgs x) {
   if (t == MC_L - 1) x.cend[ci] = c;
 }
 
-// s-contiguous tile [rows][64] without padding: 16-byte slots are rotated so
-// that both the pairwise transposing writes (fixed row low bits) and the
-// fragment reads (consecutive rows) spread over the banks
-__device__ __forceinline__ int tslot(int row, int s) {
-  return row * 64 + ((((s >> 3) ^ (row >> 1) ^ (row >> 4)) & 7) << 3) +
-         (s & 7);
-}
-
 // ---- states: U of a chunk, 64 columns per workgroup ------------------------
 template <int DP, bool GATED>
 __global__ void __launch_bounds__(256)
@@ -365,6 +359,7 @@ memory_states_kernel(ChunkArgs x) {
   const long ci = (long)ch * a.H + h;
   __shared__ __attribute__((aligned(16))) short kt[DP * 64];
   __shared__ __attribute__((aligned(16))) short vw[3][64 * 64];
+  __shared__ __attribute__((aligned(16))) short vu[64 * 64];  // V^T as it is
   __shared__ float s_w[MC_L];
   {
     float w = 0.f;
@@ -385,6 +380,8 @@ memory_states_kernel(ChunkArgs x) {
   const uint4v zero = {0, 0, 0, 0};
   uint4v kreg[2 * PAIRS], vreg[2];
   const int v_r = tid >> 3 << 1, v_c = (tid & 7) * 8;
+  const TileWrite vtw(v_c, v_r);
+  const TileRead tr(col, 0);
   auto issue = [&](int c0) {
 #pragma unroll
     for (int p = 0; p < PAIRS; ++p) {
@@ -415,9 +412,15 @@ memory_states_kernel(ChunkArgs x) {
       union { uint4v u; unsigned short s[8]; } y0, y1;
       y0.u = silu8<!GATED>(kreg[2 * p]);
       y1.u = silu8<!GATED>(kreg[2 * p + 1]);
+      const TileWrite tw(c, r);
+      if (!GATED && et == 0 && c < D) {
+        short* ka = x.KA + ((long)(row0 + c0 + r) * a.H + h) * D + c;
+        if (c0 + r < nrow) *(uint4v*)ka = y0.u;
+        if (c0 + r + 1 < nrow) *(uint4v*)(ka + (long)a.H * D) = y1.u;
+      }
 #pragma unroll
       for (int j = 0; j < 8; ++j)
-        *(uint*)(kt + tslot(c + j, r)) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
+        *(uint*)(kt + tw.at(j)) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
     }
     {
       float f0[8], f1[8];
@@ -428,7 +431,8 @@ memory_states_kernel(ChunkArgs x) {
       for (int j = 0; j < 8; ++j) {
         uint w[3];
         split3(f0[j] * w0, f1[j] * w1, w);
-        const int o = tslot(v_c + j, v_r);
+        const int o = vtw.at(j);
+        *(uint*)(vu + o) = pack_bf16x2(f0[j], f1[j]);
 #pragma unroll
         for (int z = 0; z < 3; ++z) *(uint*)(&vw[z][o]) = w[z];
       }
@@ -436,18 +440,24 @@ memory_states_kernel(ChunkArgs x) {
     __syncthreads();
     if (c0 + 64 < nrow) issue(c0 + 64);
 #pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int e = (i * 256 + tid) >> 3, sl = tid & 7;
+      if (e0 + e < E)
+        *(uint4v*)(x.VT + (ci * E + e0 + e) * MC_L + c0 + 8 * sl) =
+            *(const uint4v*)(vu + tslot(e, 8 * sl));
+    }
+#pragma unroll
     for (int kk = 0; kk < 4; ++kk) {
 #pragma unroll
       for (int y = 0; y < NT; ++y) {
         const int tile = wid + 4 * y;
         const int m = tile % MT, n = tile / MT;
         frag_u kf;
-        kf.u4 = *(const uint4v*)(kt + tslot(32 * m + col, 16 * kk + 8 * hi));
+        kf.u4 = *(const uint4v*)(kt + tr.at(m, 2 * kk + hi));
 #pragma unroll
         for (int z = 0; z < 3; ++z) {
           frag_u vf;
-          vf.u4 = *(const uint4v*)(
-              &vw[z][tslot(32 * n + col, 16 * kk + 8 * hi)]);
+          vf.u4 = *(const uint4v*)(&vw[z][tr.at(n, 2 * kk + hi)]);
           acc[y] = mfma_bf16(kf.bf, vf.bf, acc[y]);
         }
       }
@@ -516,44 +526,70 @@ memory_scan_kernel(ChunkArgs x) {
   float n = 0.f;
   const long nat = (slot * a.H + h) * nt * D + dt * 64 + tid;
   if (with_n && ctx > 0) n = a.n[nat];
-  const int c1 = x.first[sg + 1];
-  f32x4 Un = {0.f, 0.f, 0.f, 0.f};
-  int ch = x.first[sg];
-  if (live && ch < c1)
-    Un = *(const f32x4*)(x.U + ((long)ch * a.H + h) * E * D + (long)e * D + d);
-  for (; ch < c1; ++ch) {
-    const long ci = (long)ch * a.H + h;
-    const f32x4 U = Un;
-    if (live && ch + 1 < c1)
-      Un = *(const f32x4*)(x.U + (ci + a.H) * E * D + (long)e * D + d);
-    if (live && x.chunks[4 * ch + 3]) {
-      uint w0[3], w1[3];
-      split3(S[0], S[1], w0);
-      split3(S[2], S[3], w1);
+  // the state factors of up to 64 chunks at a time, then the chunks with the
+  // next four U in flight
+  constexpr int PF = 4;
+  __shared__ float s_b[64], s_c[64];
+  const int c0 = x.first[sg], c1 = x.first[sg + 1];
+  const float l2d = GATED ? 0.f : a.log2_decay[h];
+  const long at = (long)e * D + d, step = (long)a.H * E * D;
+  const float* Up = x.U + ((long)c0 * a.H + h) * E * D + at;
+  f32x4 Un[PF] = {};
 #pragma unroll
-      for (int z = 0; z < 3; ++z)
-        *(uint2*)(x.P + ((ci * 3 + z) * E + e) * D + d) = uint2{w0[z], w1[z]};
-    }
-    float fs, us = 1.f;
-    if (GATED) {
-      const float* tt = x.tot + ci * 4;
-      const float bm = tt[0] + tt[1] + tt[2] + tt[3] + m, ce = x.cend[ci];
-      const float mn = fmaxf(bm, ce);
-      fs = expf(bm - mn);
-      us = expf(ce - mn);
-      if (blockIdx.x % (nd * ne) == 0 && tid == 0) x.mst[ci] = m;
-      if (with_n) {
-        const long o = ci * D + dt * 64 + tid;
-        const float N = x.N[o];
-        x.N[o] = n;
-        n = fs * n + us * N;
+  for (int j = 0; j < PF; ++j)
+    if (live && c0 + j < c1) Un[j] = *(const f32x4*)(Up + j * step);
+  for (int cb = c0; cb < c1; cb += 64) {
+    __syncthreads();
+    if (tid < 64 && cb + tid < c1) {
+      const long ci = (long)(cb + tid) * a.H + h;
+      if (GATED) {
+        const float* tt = x.tot + ci * 4;
+        s_b[tid] = tt[0] + tt[1] + tt[2] + tt[3];
+        s_c[tid] = x.cend[ci];
+      } else {
+        s_b[tid] = __builtin_amdgcn_exp2f(x.chunks[4 * (cb + tid) + 2] * l2d);
       }
-      m = mn;
-    } else {
-      fs = __builtin_amdgcn_exp2f(x.chunks[4 * ch + 2] * a.log2_decay[h]);
     }
+    __syncthreads();
+    const int ce = min(c1, cb + 64);
+    for (int ch0 = cb; ch0 < ce; ch0 += PF) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) S[j] = fs * S[j] + us * U[j];
+      for (int j = 0; j < PF; ++j) {
+        const int ch = ch0 + j;
+        if (ch >= ce) break;
+        const long ci = (long)ch * a.H + h;
+        const f32x4 U = Un[j];
+        if (live && ch + PF < c1)
+          Un[j] = *(const f32x4*)(Up + (long)(ch - c0 + PF) * step);
+        if (live && (ch > c0 || ctx > 0)) {
+          uint w0[3], w1[3];
+          split3(S[0], S[1], w0);
+          split3(S[2], S[3], w1);
+#pragma unroll
+          for (int z = 0; z < 3; ++z)
+            *(uint2*)(x.P + (ci * 3 + z) * E * D + at) = uint2{w0[z], w1[z]};
+        }
+        float fs, us = 1.f;
+        if (GATED) {
+          const float bm = s_b[ch - cb] + m;
+          const float mn = fmaxf(bm, s_c[ch - cb]);
+          fs = expf(bm - mn);
+          us = expf(s_c[ch - cb] - mn);
+          if (dt == 0 && et == 0 && tid == 0) x.mst[ci] = m;
+          if (with_n) {
+            const long o = ci * D + dt * 64 + tid;
+            const float N = x.N[o];
+            x.N[o] = n;
+            n = fs * n + us * N;
+          }
+          m = mn;
+        } else {
+          fs = s_b[ch - cb];
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) S[i] = fs * S[i] + us * U[i];
+      }
+    }
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j) tr[(tid & 15) * 4 + j][tid >> 4] = S[j];
@@ -566,28 +602,14 @@ memory_scan_kernel(ChunkArgs x) {
     for (int j = 0; j < nt; ++j) a.n[nat + (long)j * D] = n;
 }
 
-// m has one reader group per segment and head; it is stored last
-__global__ void __launch_bounds__(64)
-memory_last_m_kernel(ChunkArgs x) {
-  const MemoryArgs& a = x.a;
-  const int nt = (a.E + 31) / 32;
-  const int h = blockIdx.x % a.H, sg = blockIdx.x / a.H;
-  const int ch = x.first[sg + 1] - 1;
-  const long ci = (long)ch * a.H + h;
-  const float* tt = x.tot + ci * 4;
-  const float m = fmaxf(tt[0] + tt[1] + tt[2] + tt[3] + x.mst[ci], x.cend[ci]);
-  for (int j = threadIdx.x; j < nt; j += 64)
-    a.m[((long)a.seg[4 * sg] * a.H + h) * nt + j] = m;
-}
-
 // ---- outputs: 128 queries x VT columns per workgroup -----------------------
 template <int DP, int VT, bool GATED>
-__global__ void __launch_bounds__(256, DP <= 128 ? 2 : 1)
+__global__ void __launch_bounds__(256, DP <= 128 || VT <= 64 ? 2 : 1)
 memory_outputs_kernel(ChunkArgs x) {
   constexpr int NC = DP / 16, NB = VT / 32;
   constexpr int KP = DP * 2;             // K row pitch (bytes)
   constexpr int CPR = DP / 8, PAIRS = 32 * CPR / 256;
-  constexpr int VC = VT / 8, VPAIRS = 32 * VC / 256;
+  constexpr int VN = VT / 32;            // 16-byte pieces of V^T a thread
   constexpr int KV_B = 64 * KP + VT * 64 * 2;
   constexpr int ST_B = 3 * 32 * KP;
   const MemoryArgs& a = x.a;
@@ -597,6 +619,19 @@ memory_outputs_kernel(ChunkArgs x) {
   const int h = blockIdx.x / nt / 2 % a.H, ch = blockIdx.x / nt / 2 / a.H;
   const int row0 = x.chunks[4 * ch + 1], nrow = x.chunks[4 * ch + 2];
   const bool carried = x.chunks[4 * ch + 3];
+  if (GATED && et == 0 && half == 0) {
+    // m after the portion: nothing reads the slot's m any more
+    const int sg = x.chunks[4 * ch];
+    if (ch == x.first[sg + 1] - 1) {
+      const long ci = (long)ch * a.H + h;
+      const float* tt = x.tot + ci * 4;
+      const float m = fmaxf(tt[0] + tt[1] + tt[2] + tt[3] + x.mst[ci],
+                            x.cend[ci]);
+      const int mt = (E + 31) / 32;
+      for (int j = threadIdx.x; j < mt; j += 256)
+        a.m[((long)a.seg[4 * sg] * a.H + h) * mt + j] = m;
+    }
+  }
   if (half * 128 >= nrow) return;        // the whole workgroup
   const int tid = threadIdx.x, lane = tid & 63;
   const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -657,20 +692,32 @@ memory_outputs_kernel(ChunkArgs x) {
         s_n[d] = d < D ? x.N[ci * D + d] : 0.f;
     }
     const short* P = x.P + ci * 3 * E * D;
+    constexpr int NP = 3 * 32 * CPR / 256;
+    uint4v preg[NP];
+    auto fetch = [&](int nb) {
+#pragma unroll
+      for (int i = 0; i < NP; ++i) {
+        const int it = i * 256 + tid;
+        const int c = it % CPR * 8, r = it / CPR;     // r: plane * 32 + row
+        const int e = e0 + 32 * nb + (r & 31);
+        preg[i] = e < E && c < D
+            ? *(const uint4v*)(P + ((long)(r >> 5) * E + e) * D + c)
+            : uint4v{0, 0, 0, 0};
+      }
+    };
+    fetch(0);
 #pragma unroll
     for (int nb = 0; nb < NB; ++nb) {
       if (e0 + 32 * nb >= E) continue;   // uniform
       __syncthreads();
 #pragma unroll
-      for (int i = 0; i < 3 * 32 * CPR / 256; ++i) {
+      for (int i = 0; i < NP; ++i) {
         const int it = i * 256 + tid;
-        const int c = it % CPR * 8, r = it / CPR;     // r: plane * 32 + row
-        const int e = e0 + 32 * nb + (r & 31);
-        *(uint4v*)(buf + r * KP + kswz(r & 31, c * 2)) = e < E && c < D
-            ? *(const uint4v*)(P + ((long)(r >> 5) * E + e) * D + c)
-            : uint4v{0, 0, 0, 0};
+        const int c = it % CPR * 8, r = it / CPR;
+        *(uint4v*)(buf + r * KP + kswz(r & 31, c * 2)) = preg[i];
       }
       __syncthreads();
+      if (nb + 1 < NB) fetch(nb + 1);
 #pragma unroll
       for (int z = 0; z < 3; ++z)
 #pragma unroll
@@ -695,32 +742,26 @@ memory_outputs_kernel(ChunkArgs x) {
   }
 
   // ---- keys of the chunk, 64 at a time, from the newest back ---------------
-  const short* kp = (const short*)a.k + (long)h * D;
-  const short* vp = (const short*)a.v + (long)h * E + e0;
+  const short* kp = (GATED ? (const short*)a.k : x.KA) + (long)h * D;
+  const long kst = GATED ? a.kst : (long)a.H * D;
+  const short* vp = x.VT + (ci * E + e0) * MC_L;
   const uint4v zero = {0, 0, 0, 0};
-  uint4v kreg[2 * PAIRS], vreg[2 * VPAIRS];
+  uint4v kreg[2 * PAIRS], vreg[VN];
   float colr = 0.f;
   auto issue = [&](int J) {
     const int c0 = 64 * J;
 #pragma unroll
-    for (int p = 0; p < PAIRS; ++p) {
+    for (int p = 0; p < 2 * PAIRS; ++p) {
       const int it = p * 256 + tid;
-      const int r = it / CPR * 2, c = it % CPR * 8;
-#pragma unroll
-      for (int y = 0; y < 2; ++y)
-        kreg[2 * p + y] = c0 + r + y < nrow && c < D
-            ? *(const uint4v*)(kp + (long)(row0 + c0 + r + y) * a.kst + c)
-            : zero;
+      const int r = it / CPR, c = it % CPR * 8;
+      kreg[p] = c0 + r < nrow && c < D
+          ? *(const uint4v*)(kp + (long)(row0 + c0 + r) * kst + c) : zero;
     }
 #pragma unroll
-    for (int p = 0; p < VPAIRS; ++p) {
-      const int it = p * 256 + tid;
-      const int r = it / VC * 2, c = it % VC * 8;
-#pragma unroll
-      for (int y = 0; y < 2; ++y)
-        vreg[2 * p + y] = c0 + r + y < nrow && e0 + c < E
-            ? *(const uint4v*)(vp + (long)(row0 + c0 + r + y) * a.vst + c)
-            : zero;
+    for (int p = 0; p < VN; ++p) {
+      const int e = (p * 256 + tid) >> 3;
+      vreg[p] = e0 + e < E
+          ? *(const uint4v*)(vp + (long)e * MC_L + c0 + 8 * (tid & 7)) : zero;
     }
     if (GATED && tid < 64) {
       colr = -INFINITY;
@@ -730,30 +771,20 @@ memory_outputs_kernel(ChunkArgs x) {
       }
     }
   };
+  const TileRead vr(col, 4 * hi);
   const int J1 = min(half * 2 + 1, (nrow - 1) / 64);
   issue(J1);
   for (int J = J1; J >= 0; --J) {
     __syncthreads();
 #pragma unroll
-    for (int p = 0; p < PAIRS; ++p) {
+    for (int p = 0; p < 2 * PAIRS; ++p) {
       const int it = p * 256 + tid;
-      const int r = it / CPR * 2, c = it % CPR * 8;
-#pragma unroll
-      for (int y = 0; y < 2; ++y)
-        *(uint4v*)(kb + (r + y) * KP + kswz(r + y, c * 2)) =
-            silu8<!GATED>(kreg[2 * p + y]);
+      const int r = it / CPR, c = it % CPR * 8;
+      *(uint4v*)(kb + r * KP + kswz(r, c * 2)) = kreg[p];
     }
 #pragma unroll
-    for (int p = 0; p < VPAIRS; ++p) {
-      const int it = p * 256 + tid;
-      const int r = it / VC * 2, c = it % VC * 8;
-      union { uint4v u; unsigned short s[8]; } y0, y1;
-      y0.u = silu8<!GATED>(vreg[2 * p]);
-      y1.u = silu8<!GATED>(vreg[2 * p + 1]);
-#pragma unroll
-      for (int j = 0; j < 8; ++j)
-        *(uint*)(vb + tslot(c + j, r)) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
-    }
+    for (int p = 0; p < VN; ++p)
+      *(uint4v*)(vb + tslot((p * 256 + tid) >> 3, 8 * (tid & 7))) = vreg[p];
     if (GATED && tid < 64) s_col[tid] = colr;
     __syncthreads();
     if (J > 0) issue(J - 1);
@@ -766,19 +797,18 @@ memory_outputs_kernel(ChunkArgs x) {
       for (int j = 0; j < 4; ++j)
         if (j >= J && j < jt) base += tot[j];
     }
-    f32x16 acc[2] = {};
-#pragma unroll
+    // 32 keys at a time keeps the registers for two workgroups per CU
+#pragma unroll 1
     for (int k2 = 0; k2 < 2; ++k2) {
-      const int r = col + 32 * k2;
+      const int kr = col + 32 * k2;
+      f32x16 acc = {};
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
         frag_u kf;
-        kf.u4 = *(const uint4v*)(kb + r * KP + kswz(r, (c * 16 + hi * 8) * 2));
-        acc[k2] = mfma_bf16(kf.bf, qf[c].bf, acc[k2]);
+        kf.u4 =
+            *(const uint4v*)(kb + kr * KP + kswz(kr, (c * 16 + hi * 8) * 2));
+        acc = mfma_bf16(kf.bf, qf[c].bf, acc);
       }
-    }
-#pragma unroll
-    for (int k2 = 0; k2 < 2; ++k2)
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int s = 32 * k2 + acc_row(r, hi);
@@ -786,33 +816,31 @@ memory_outputs_kernel(ChunkArgs x) {
         if (GATED) w = __expf(base + s_col[s]) * qs;
         else w = __builtin_amdgcn_exp2f((float)(t - 64 * J - s) * l2d);
         if (J == jt && 64 * J + s > t) w = 0.f;
-        acc[k2][r] *= w;
-        if (GATED) den += acc[k2][r];
+        acc[r] *= w;
+        if (GATED) den += acc[r];
       }
-#pragma unroll
-    for (int k2 = 0; k2 < 2; ++k2)
 #pragma unroll
       for (int cc = 0; cc < 2; ++cc) {
         frag_u pf[3];
 #pragma unroll
         for (int u = 0; u < 4; ++u) {
           uint w[3];
-          split3(acc[k2][8 * cc + 2 * u], acc[k2][8 * cc + 2 * u + 1], w);
+          split3(acc[8 * cc + 2 * u], acc[8 * cc + 2 * u + 1], w);
 #pragma unroll
           for (int z = 0; z < 3; ++z) pf[z].u[u] = w[z];
         }
-        const int s = 32 * k2 + 16 * cc + 4 * hi;
+        const int slot = 4 * k2 + 2 * cc;
 #pragma unroll
         for (int nb = 0; nb < NB; ++nb) {
           frag_u vf;
-          *(uint2*)&vf.u[0] = *(const uint2*)(vb + tslot(32 * nb + col, s));
-          *(uint2*)&vf.u[2] =
-              *(const uint2*)(vb + tslot(32 * nb + col, s + 8));
+          *(uint2*)&vf.u[0] = *(const uint2*)(vb + vr.at(nb, slot));
+          *(uint2*)&vf.u[2] = *(const uint2*)(vb + vr.at(nb, slot + 1));
 #pragma unroll
           for (int z = 0; z < 3; ++z)
             ot[nb] = mfma_bf16(vf.bf, pf[z].bf, ot[nb]);
         }
       }
+    }
   }
 
   float inv = 1.f;
@@ -835,6 +863,8 @@ memory_outputs_kernel(ChunkArgs x) {
     }
 }
 
+// wider column tiles read the keys less often, as long as the accumulators
+// leave registers for two workgroups per CU
 template <int DP, bool GATED>
 static void launch_chunks(const ChunkArgs& x, hipStream_t stream) {
   const MemoryArgs& a = x.a;
@@ -844,12 +874,11 @@ static void launch_chunks(const ChunkArgs& x, hipStream_t stream) {
       <<<ch * ((a.E + 63) / 64), 256, 0, stream>>>(x);
   memory_scan_kernel<GATED><<<(long)x.n_seg * a.H * ((a.D + 63) / 64) *
                                   ((a.E + 15) / 16), 256, 0, stream>>>(x);
-  if (GATED)
-    memory_last_m_kernel<<<(long)x.n_seg * a.H, 64, 0, stream>>>(x);
-  if (a.E <= 64)
-    memory_outputs_kernel<DP, 64, GATED><<<ch * 2, 256, 0, stream>>>(x);
+  if (a.E <= 64 || DP > 128)
+    memory_outputs_kernel<DP, 64, GATED>
+        <<<ch * 2 * ((a.E + 63) / 64), 256, 0, stream>>>(x);
   else
-    memory_outputs_kernel<DP, 128, GATED>
+    memory_outputs_kernel<DP, (DP > 128 ? 64 : 128), GATED>
         <<<ch * 2 * ((a.E + 127) / 128), 256, 0, stream>>>(x);
 }
 

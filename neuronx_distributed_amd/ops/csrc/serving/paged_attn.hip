@@ -351,11 +351,10 @@ attn_tiles_kernel(TilesArgs a) {
   constexpr int NC = DP / 16;        // 16-wide chunks of the head size
   constexpr int NB = DP / 32;        // 32-row blocks of O^T
   constexpr int KP = DP * 2;         // K row pitch (bytes)
-  constexpr int VP = 72;             // V^T pitch (elements)
   constexpr int CPR = DP / 8;        // 16-byte slots of a row
   constexpr int PAIRS = 32 * CPR / 256;  // (row pair, slot) items a thread
   __shared__ __attribute__((aligned(16))) char kbuf[64 * KP];
-  __shared__ __attribute__((aligned(16))) short vbuf[DP * VP];
+  __shared__ __attribute__((aligned(16))) short vbuf[DP * 64];  // V^T
 
   // later tiles of a portion see more keys: they start first
   const int* tl = a.tiles + 4 * (gridDim.y - 1 - blockIdx.y);
@@ -425,12 +424,14 @@ attn_tiles_kernel(TilesArgs a) {
       union { uint4v u; unsigned short s[8]; } x, y;
       x.u = vreg[2 * p];
       y.u = vreg[2 * p + 1];
+      const TileWrite tw(c, r);
 #pragma unroll
       for (int j = 0; j < 8; ++j)
-        *(uint*)(vbuf + (c + j) * VP + r) = (uint)x.s[j] | ((uint)y.s[j] << 16);
+        *(uint*)(vbuf + tw.at(j)) = (uint)x.s[j] | ((uint)y.s[j] << 16);
     }
   };
 
+  const TileRead vt(col, 4 * hi);
   issue(0);
   for (int n = 0; n < ntiles; ++n) {
     __syncthreads();           // readers of the previous tile are done
@@ -510,13 +511,12 @@ attn_tiles_kernel(TilesArgs a) {
             y -= __uint_as_float(w & 0xffff0000u);
           }
         }
-        const int s = 32 * kb + 16 * cc + 4 * hi;
+        const int slot = 4 * kb + 2 * cc;
 #pragma unroll
         for (int nb = 0; nb < NB; ++nb) {
-          const short* vr = vbuf + (32 * nb + col) * VP + s;
           frag_u vf;
-          *(uint2*)&vf.u[0] = *(const uint2*)vr;
-          *(uint2*)&vf.u[2] = *(const uint2*)(vr + 8);
+          *(uint2*)&vf.u[0] = *(const uint2*)(vbuf + vt.at(nb, slot));
+          *(uint2*)&vf.u[2] = *(const uint2*)(vbuf + vt.at(nb, slot + 1));
 #pragma unroll
           for (int z = 0; z < NP; ++z)
             ot[nb] = mfma_bf16(vf.bf, pf[z].bf, ot[nb]);

@@ -78,3 +78,31 @@ __device__ __forceinline__ float silu_f(float x) { return x * sigmoid_f(x); }
 __device__ __forceinline__ float log_sigmoid_f(float x) {
   return fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
 }
+
+// s-contiguous tile [rows][64] without padding: 16-byte slots are rotated so
+// that both the pairwise transposing writes (fixed row low bits) and the
+// fragment reads (consecutive rows) spread over the banks
+__device__ __forceinline__ int tslot(int row, int s) {
+  return row * 64 + ((((s >> 3) ^ (row >> 1) ^ (row >> 4)) & 7) << 3) +
+         (s & 7);
+}
+
+// Lane part of the tile's addresses, so that an access costs one xor and an
+// immediate offset.
+struct TileRead {            // row = 32 nb + col, s = 8 slot + 4 hi (+ 0..7)
+  int base;                  // elements, slot bits xor-ed in later
+  __device__ __forceinline__ TileRead(int col, int low)
+      : base(col * 64 + ((((col >> 1) ^ (col >> 4)) & 7) << 3) + low) {}
+  __device__ __forceinline__ int at(int nb, int slot) const {
+    return (base ^ (((slot ^ (2 * nb)) & 7) << 3)) + nb * 2048;
+  }
+};
+struct TileWrite {           // row = c + j (c a multiple of 8), s = r
+  int base;
+  __device__ __forceinline__ TileWrite(int c, int r)
+      : base(c * 64 + ((((r >> 3) ^ ((c >> 1) & 4) ^ (c >> 4)) & 7) << 3) +
+             (r & 7)) {}
+  __device__ __forceinline__ int at(int j) const {
+    return (base ^ ((j >> 1) << 3)) + j * 64;
+  }
+};

@@ -104,7 +104,7 @@ class _MemoryArgs(ctypes.Structure):
 class _ChunkArgs(ctypes.Structure):
     _fields_ = ([("a", _MemoryArgs)] + _fields("chunks first", ctypes.c_void_p)
                 + _fields("n_chunks n_seg T", ctypes.c_int)
-                + _fields("b i c tot cend U N P mst", ctypes.c_void_p))
+                + _fields("b i c tot cend U N P mst VT KA", ctypes.c_void_p))
 
 
 # ---------------------------------------------------------------------------
@@ -392,9 +392,13 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
         U = torch.empty(nc, heads, E, D, **f32)
         P = torch.empty(nc, heads, 3, E, D, dtype=torch.bfloat16,
                         device=q.device)
+        VT = torch.empty(nc, heads, E, CHUNK, dtype=torch.bfloat16,
+                         device=q.device)
+        KA = None if gated else torch.empty(T, heads * D, dtype=q.dtype,
+                                            device=q.device)
         x = _ChunkArgs(a=a, chunks=_p(chunks), first=_p(chunk_first),
                        n_chunks=nc, n_seg=seg.shape[0], T=T, U=_p(U),
-                       P=_p(P))
+                       P=_p(P), VT=_p(VT), KA=_p(KA))
         if gated:
             bic = torch.empty(3, heads, T, **f32)
             small = torch.empty(nc, heads, 6 + D, **f32)
