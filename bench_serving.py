@@ -159,9 +159,15 @@ def bench_kernels():
             # chunked: scores, weighted values, state in and out
             C = 64 if T > 1 else 1
             fl = 2 * B * T * H2 * (C / 2 * (D2 + E2) + 2 * D2 * E2)
+            # the same with every product of a 32-bit operand at its MFMA
+            # cost, three bf16 products
+            f3 = 2 * B * T * H2 * (C / 2 * (D2 + 3 * E2) + 6 * D2 * E2)
+            extra = {"roofline_32bit_us": round(
+                max(f3 / PEAK_FLOPS, io / PEAK_BYTES) * 1e6, 2)} \
+                if T > 1 else {}
             _report("memory_" + ("chunks" if T > 1 else "steps"), us, fl, io,
                     gated=gated, heads=H2, dim=D2, vdim=E2, batch=B,
-                    tokens=T)
+                    tokens=T, **extra)
     # -- norms and pointwise ---------------------------------------------------
     for T in (32, 4096):
         Wd, F = 4096, 14336
