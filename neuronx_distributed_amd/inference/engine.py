@@ -8,20 +8,18 @@ own kernels.  Steps made of single tokens only replay a hipGraph captured
 per batch-size bucket.
 
 A model is served when it has ``cache_specs()`` and
-``forward_ragged(batch, pools)``.
+``forward_ragged(batch, pools)``; ``max_positions``, if it has one, bounds
+the context.
 """
 
-from dataclasses import dataclass, field
+from dataclasses import dataclass
 from typing import Dict, List, Optional, Sequence
 
 import numpy as np
 import torch
 
 from ..ops import serving as sv
-from ..utils.logger import get_logger
-from .paged_cache import CacheManager, RequestState
-
-logger = get_logger(__name__)
+from .paged_cache import PAGE_SIZE, CacheManager, RequestState
 
 TILE_ROWS = 128
 
@@ -90,6 +88,13 @@ class InferenceEngine:
         p = next(model.parameters())
         if not p.is_cuda:
             raise RuntimeError("the serving engine runs on the GPU only")
+        limit = getattr(model, "max_positions", None)
+        if limit is not None:
+            if max_context is not None and max_context > limit:
+                raise ValueError(f"a context of {max_context} tokens; the "
+                                 f"model has {limit} positions")
+            max_context = min(limit, max_context or
+                              CacheManager.pages_for(max_tokens) * PAGE_SIZE)
         self.model = model
         self.device = p.device
         self.cache = CacheManager(model.cache_specs(), max_tokens, max_seqs,

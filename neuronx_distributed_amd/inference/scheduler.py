@@ -10,10 +10,9 @@ from collections import deque
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional, Sequence
 
-import torch
-
 from ..utils.sampling import Sampler
 from .engine import InferenceEngine, StepEntry
+from .paged_cache import PAGE_SIZE, CacheManager
 
 
 @dataclass
@@ -129,9 +128,10 @@ def generate_ragged(model, prompts: Sequence[Sequence[int]],
                     use_graphs: bool = True) -> List[List[int]]:
     """Generate for prompts of unequal length; returns the new tokens of
     each, in order."""
-    max_seqs = max_seqs or max(1, min(len(prompts), 64))
-    page = 64
-    per = sorted((-(-(len(p) + max_new_tokens) // page) * page
+    if not prompts:
+        return []
+    max_seqs = max_seqs or min(len(prompts), 64)
+    per = sorted((CacheManager.pages_for(len(p) + max_new_tokens) * PAGE_SIZE
                   for p in prompts), reverse=True)
     engine = InferenceEngine(model, max_tokens=sum(per[:max_seqs]),
                              max_seqs=max_seqs, max_context=per[0],

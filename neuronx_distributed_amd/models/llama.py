@@ -232,6 +232,25 @@ class LlamaAttention(nn.Module):
             out = out.transpose(0, 1)
         return self.o_proj(out)
 
+    def cache_spec(self):
+        """What the serving engine keeps for this layer."""
+        from ..inference.paged_cache import PagedKV
+
+        return PagedKV(self.num_kv_local, self.head_dim, self.head_dim,
+                       self.sliding_window or 0)
+
+    def forward_ragged(self, h, cos, sin, batch, pool):
+        """Rows of a packed serving batch (portions and single tokens of
+        many requests) over the paged cache."""
+        from ..ops import serving as sv
+
+        q, k, v = self.qkv_proj(h)
+        sv.rope_rows_(q, k, cos, sin, batch.pos, self.head_dim,
+                      batch.max_keys)
+        return self.o_proj(sv.ragged_attention(
+            q, k, v, batch, pool, self.num_heads_local,
+            1.0 / math.sqrt(self.head_dim), self.sliding_window or 0))
+
     def _decode_step(self, q, k, v, cos, sin, pos_t, kv_cache, sp):
         """One-token decode with everything derived from the device tensor
         ``pos_t`` (shape (1,)) so the whole step can be captured in a
@@ -496,6 +515,34 @@ class LlamaForCausalLM(nn.Module):
             init_method=_init_method(config.initializer_range))
         if config.tie_word_embeddings:
             self.lm_head.weight = self.model.embed_tokens.weight
+
+    @property
+    def max_positions(self):
+        return self.model.rope_cos.shape[0]
+
+    def cache_specs(self):
+        return [[l.self_attn.cache_spec()] for l in self.model.layers]
+
+    def forward_ragged(self, batch, pools):
+        """One step of the serving engine: float32 logits (wanted, V/tp), or
+        None.  The residual stream is float32 here."""
+        from ..ops import serving as sv
+
+        m, eps = self.model, self.config.rms_norm_eps
+        x, pending = None, sv.Pending(m.embed_tokens(batch.tokens))
+        for layer, pool in zip(m.layers, pools):
+            x, h, _ = sv.residual_norm(x, pending, eps,
+                                       layer.input_layernorm.weight)
+            pending = sv.Pending(layer.self_attn.forward_ragged(
+                h, m.rope_cos, m.rope_sin, batch, pool[0]))
+            x, h, _ = sv.residual_norm(x, pending, eps,
+                                       layer.post_attention_layernorm.weight)
+            pending = sv.Pending(layer.mlp(h))
+        if not batch.want.shape[0]:
+            return None
+        _, h, _ = sv.residual_norm(x, pending, eps, m.norm.weight,
+                                   keep_x=False, index=batch.want)
+        return sv.linear_f32(h, self.lm_head.weight)
 
     def forward(self, input_ids, labels=None, pos_offset=0, kv_caches=None):
         hidden = self.model(input_ids, pos_offset, kv_caches)

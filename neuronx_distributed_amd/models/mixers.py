@@ -92,21 +92,9 @@ class SlidingAttention(Mixer):
 
     def forward(self, h, proj, batch, pools):
         q, k, v = self.split(proj)
-        kc, vc = pools[0]
-        out = torch.empty(h.shape[0], self.out_size, dtype=h.dtype,
-                          device=h.device)
-        n = batch.portion_tokens
-        args = dict(heads=self.heads, scale=self.scale, window=self.window,
-                    keep=self.keep_first, max_keys=batch.max_keys)
-        if n:
-            sv.attn_portions(q[:n], k[:n], v[:n], kc, vc, batch.pos[:n],
-                             batch.seq[:n], batch.block_table, batch.tiles,
-                             out=out[:n], **args)
-        if n < h.shape[0]:
-            sv.attn_rows(q[n:], k[n:], v[n:], kc, vc, batch.pos[n:],
-                         batch.seq[n:], batch.block_table, out=out[n:],
-                         **args)
-        return self.o(out)
+        return self.o(sv.ragged_attention(
+            q, k, v, batch, pools[0], self.heads, self.scale, self.window,
+            self.keep_first))
 
 
 class _MatrixMemory(Mixer):

@@ -13,7 +13,8 @@ engine only.
 """
 
 import dataclasses
-from dataclasses import dataclass, field
+import math
+from dataclasses import dataclass
 from typing import List, Optional
 
 import torch
@@ -79,8 +80,6 @@ MLPS = {"dense": lambda width, c: ReluSquaredMLP(width, c["ff"])}
 
 def _bench_layers(n, width, heads, kv_heads, dim, window, keep, m_heads,
                   m_dim, m_vdim, ff):
-    import math
-
     light = {"type": "lightning", "mlp": None, "mixer": {
         "heads": heads, "dim": dim, "vdim": dim,
         "decay": [math.exp(-2.0 ** (-8.0 * (h + 1) / heads))
@@ -98,7 +97,7 @@ VOLETAR_CONFIGS = {
     # layer shapes of a 7B-class decoder (random weights; for timing)
     "voletar-bench": VoletarConfig(
         vocab_size=32000, hidden_size=4096, norm_eps=1e-6,
-        logit_softcap=30.0, loop={"start": 0, "stop": 2, "times": 2},
+        logit_softcap=50.0, loop={"start": 0, "stop": 2, "times": 2},
         layers=_bench_layers(4, 4096, 32, 8, 128, 4096, 64, 16, 128, 256,
                              14336)),
     "voletar-tiny": VoletarConfig(

@@ -553,3 +553,39 @@ extern "C" int sv_attn_tiles(const TilesArgs* a, int n_tiles,
   else return 1;
   return (int)hipGetLastError();
 }
+
+// ---------------------------------------------------------------------------
+// rotary embedding (rotate-half) of the rows of a ragged batch, in place:
+// every row has its own position.  cos/sin [positions][D / 2] f32.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ void __launch_bounds__(256)
+rope_rows_kernel(T* __restrict__ q, long qst, int H, T* __restrict__ k,
+                 long kst, int G, const float* __restrict__ cosp,
+                 const float* __restrict__ sinp, const int* __restrict__ pos,
+                 int D) {
+  const int t = blockIdx.x, half = D / 2;
+  const long at = (long)pos[t] * half;
+  for (int i = threadIdx.x; i < (H + G) * half; i += 256) {
+    const int h = i / half, j = i % half;
+    T* p = h < H ? q + t * qst + (long)h * D : k + t * kst + (long)(h - H) * D;
+    const float c = cosp[at + j], s = sinp[at + j];
+    const float x = to_f(p[j]), y = to_f(p[j + half]);
+    from_f(p[j], x * c - y * s);
+    from_f(p[j + half], y * c + x * s);
+  }
+}
+
+extern "C" int sv_rope_rows(void* q, long qst, int H, void* k, long kst,
+                            int G, const float* cosp, const float* sinp,
+                            const int* pos, int T, int D, int f32,
+                            hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (f32)
+    rope_rows_kernel<float><<<T, 256, 0, stream>>>(
+        (float*)q, qst, H, (float*)k, kst, G, cosp, sinp, pos, D);
+  else
+    rope_rows_kernel<short><<<T, 256, 0, stream>>>(
+        (short*)q, qst, H, (short*)k, kst, G, cosp, sinp, pos, D);
+  return (int)hipGetLastError();
+}

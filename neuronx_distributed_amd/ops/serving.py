@@ -8,7 +8,6 @@ gates and recurrent state are 32-bit in both.
 """
 
 import ctypes
-import math
 import os
 from dataclasses import dataclass
 from typing import Optional
@@ -311,6 +310,41 @@ def attn_portions(q, k, v, kc, vc, pos, seq, block_table, tiles, heads: int,
     _check(library().sv_attn_tiles(ctypes.byref(a), tiles.shape[0],
                                    _stream()), "attn_tiles")
     return out
+
+
+def ragged_attention(q, k, v, batch, pool, heads: int, scale: float,
+                     window: int = 0, keep: int = 0) -> torch.Tensor:
+    """Attention of a packed batch over its cache pool: portions first, then
+    single tokens, into one (T, heads * E) tensor."""
+    kc, vc = pool
+    T, n = q.shape[0], batch.portion_tokens
+    out = torch.empty(T, heads * vc.shape[3], dtype=q.dtype, device=q.device)
+    args = dict(heads=heads, scale=scale, window=window, keep=keep,
+                max_keys=batch.max_keys)
+    if n:
+        attn_portions(q[:n], k[:n], v[:n], kc, vc, batch.pos[:n],
+                      batch.seq[:n], batch.block_table, batch.tiles,
+                      out=out[:n], **args)
+    if n < T:
+        attn_rows(q[n:], k[n:], v[n:], kc, vc, batch.pos[n:], batch.seq[n:],
+                  batch.block_table, out=out[n:], **args)
+    return out
+
+
+def rope_rows_(q, k, cos, sin, pos, dim: int, max_pos: int):
+    """Rotate the heads of q and k (rotate-half) in place, each row at its
+    own position; cos/sin (positions, dim / 2) float32."""
+    if max_pos > cos.shape[0]:
+        raise ValueError(f"position {max_pos - 1} is outside the rotary "
+                         f"table of {cos.shape[0]}")
+    assert cos.dtype == sin.dtype == torch.float32 and cos.is_contiguous()
+    assert sin.is_contiguous() and cos.shape[1] * 2 == dim
+    assert q.stride(1) == k.stride(1) == 1 and pos.shape[0] == q.shape[0]
+    vp, lg = ctypes.c_void_p, ctypes.c_long
+    _check(library().sv_rope_rows(
+        vp(_p(q)), lg(q.stride(0)), q.shape[1] // dim, vp(_p(k)),
+        lg(k.stride(0)), k.shape[1] // dim, vp(_p(cos)), vp(_p(sin)),
+        vp(_p(pos)), q.shape[0], dim, _f32(q), _stream()), "rope_rows")
 
 
 # ---------------------------------------------------------------------------

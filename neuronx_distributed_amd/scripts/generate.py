@@ -4,8 +4,8 @@
         --prompt 5,17,3 --prompt 9,9 --max-new-tokens 16
 
 Prompts are token ids; one JSON line per prompt is printed.  The model class
-is chosen by config.json.  Models of the serving engine run all prompts in
-one continuous batch; the others generate prompt by prompt.
+is chosen by config.json.  On a GPU, models of the serving engine run all
+prompts in one continuous batch; otherwise prompts are generated one by one.
 """
 
 import argparse
@@ -42,7 +42,7 @@ def main(argv=None):
     model = load_pretrained(a.model, getattr(torch, a.dtype), device)
     sampler = Sampler(do_sample=a.top_k > 0, top_k=a.top_k or 50,
                       temperature=a.temperature)
-    if getattr(model, "supports_ragged", False):
+    if device == "cuda" and hasattr(model, "forward_ragged"):
         outs = generate_ragged(model, prompts, a.max_new_tokens, sampler,
                                a.eos, a.max_seqs, a.max_step_tokens)
     else:

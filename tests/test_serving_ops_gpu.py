@@ -61,7 +61,7 @@ class Paged:
 
 ATTN = [
     # H, G, D, E, window, keep
-    (4, 2, 64, 64, 96, 20),
+    (4, 2, 56, 64, 90, 21),
     (6, 2, 40, 24, 70, 5),
     (3, 1, 20, 12, 33, 0),        # sizes that are no multiple of 8
     (8, 8, 128, 96, 130, 130),
@@ -120,7 +120,7 @@ def test_attention_prompt_portions_and_decoding(sv, case, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("window,keep", [(96, 20), (64, 64), (70, 3),
+@pytest.mark.parametrize("window,keep", [(92, 22), (64, 64), (70, 3),
                                          (33, 0), (128, 65)])
 def test_attention_edges_show(sv, window, keep, dtype):
     """One key stands out; queries just inside see it, just outside do not.
@@ -204,7 +204,7 @@ def test_attention_weights_keep_32_bits(sv):
 # matrix memories
 # ---------------------------------------------------------------------------
 
-MEM = [(4, 64, 32), (3, 48, 72), (2, 20, 12), (2, 128, 96), (1, 256, 40),
+MEM = [(4, 56, 40), (3, 48, 72), (2, 20, 12), (2, 128, 96), (1, 256, 40),
        (5, 8, 8), (1, 300, 34)]
 
 
