@@ -19,7 +19,8 @@ import numpy as np
 import torch
 
 from ..ops import serving as sv
-from .paged_cache import PAGE_SIZE, CacheManager, RequestState
+from .paged_cache import (PAGE_SIZE, CacheManager, PagedLatent,
+                          RequestState)
 
 TILE_ROWS = 128
 
@@ -48,16 +49,23 @@ class RaggedBatch:
     want: torch.Tensor         # (W,) rows whose logits are computed
     portion_tokens: int        # rows [0, portion_tokens) belong to portions
     max_keys: int              # no row sees more keys than this
+    # window -> keys of the portions, for latent attention; none when the
+    # portions are so short that they run like single tokens
+    spans: Dict[int, sv.KeySpans]
 
 
 class _Layout:
     """Places of the batch's arrays in one int32 buffer (one upload)."""
 
     def __init__(self, T, portion_tokens, R, n_tiles, n_portions, n_chunks,
-                 n_singles, n_want, width):
+                 n_singles, n_want, width, span_pages={}):
         self.portion_tokens = portion_tokens
+        self.windows = list(span_pages)
         self.at, n = {}, 0
-        for name, shape in (("tokens", (T,)), ("pos", (T,)), ("seq", (T,)),
+        spans = [a for w, pages in span_pages.items()
+                 for a in (((w, "pages"), (pages,)),
+                           ((w, "table"), (n_portions, width)))]
+        for name, shape in (*spans, ("tokens", (T,)), ("pos", (T,)), ("seq", (T,)),
                             ("tiles", (n_tiles, 4)),
                             ("portions", (n_portions, 4)),
                             ("chunks", (n_chunks, 4)),
@@ -75,8 +83,11 @@ class _Layout:
                 for k, (o, s, shape) in self.at.items()}
 
     def batch(self, buf, max_keys) -> RaggedBatch:
+        v = self.views(buf)
+        spans = {w: sv.KeySpans(v.pop((w, "pages")), v.pop((w, "table")))
+                 for w in self.windows}
         return RaggedBatch(portion_tokens=self.portion_tokens,
-                           max_keys=max_keys, **self.views(buf))
+                           max_keys=max_keys, spans=spans, **v)
 
 
 class InferenceEngine:
@@ -97,9 +108,12 @@ class InferenceEngine:
                               CacheManager.pages_for(max_tokens) * PAGE_SIZE)
         self.model = model
         self.device = p.device
-        self.cache = CacheManager(model.cache_specs(), max_tokens, max_seqs,
-                                  max_context, dtype=p.dtype,
-                                  device=self.device)
+        specs = model.cache_specs()
+        self.cache = CacheManager(specs, max_tokens, max_seqs, max_context,
+                                  dtype=p.dtype, device=self.device)
+        self._latent_windows = sorted({
+            s.window for run in specs for s in run
+            if isinstance(s, PagedLatent)})
         self.max_seqs = max_seqs
         self.use_graphs = use_graphs
         self._graphs: Dict[int, tuple] = {}
@@ -163,14 +177,19 @@ class InferenceEngine:
         n_tiles = sum(-(-len(e.tokens) // TILE_ROWS) for e in entries
                       if len(e.tokens) > 1)
         want = [row_of[i] + w for i, e in enumerate(entries) for w in e.want]
-        chunks, first = sv.chunk_table(
-            [(states[i].slot, row_of[i], len(entries[i].tokens),
-              states[i].length) for i in order[:n_port]])
+        portions = [(states[i].slot, row_of[i], len(entries[i].tokens),
+                     states[i].length) for i in order[:n_port]]
+        chunks, first = sv.chunk_table(portions)
+        spans = self._spans(portions, [states[i] for i in order[:n_port]])
         lay = _Layout(T, portion_tokens, len(entries), n_tiles, n_port,
                       len(chunks), len(entries) - n_port, len(want),
-                      self.cache.table_width)
+                      self.cache.table_width,
+                      {w: len(pages) for w, (pages, _) in spans.items()})
         host = np.zeros(lay.size, dtype=np.int32)
         v = lay.views(host)
+        for w, (pages, table) in spans.items():
+            v[w, "pages"][:] = pages
+            v[w, "table"][:] = table
         v["want"][:] = want
         v["chunks"][:] = np.asarray(chunks, dtype=np.int32).reshape(-1, 4)
         v["chunk_first"][:] = first
@@ -196,6 +215,17 @@ class InferenceEngine:
         buf = torch.from_numpy(host).to(self.device)
         return self.model.forward_ragged(lay.batch(buf, max_keys),
                                          self.cache.pools)
+
+    def _spans(self, portions, states):
+        """Host form of the portions' key spans for every latent window."""
+        if max((n for _, _, n, _ in portions), default=0) < \
+                sv.EXPAND_MIN_TOKENS or not self._latent_windows:
+            return {}
+        rows = np.zeros((len(states), self.cache.table_width), dtype=np.int32)
+        for st, row in zip(states, rows):
+            self.cache.table_row(st, row)
+        return {w: sv.key_spans(portions, rows, w)
+                for w in self._latent_windows}
 
     def _bucket(self, n: int) -> int:
         b = 1

@@ -3,6 +3,8 @@
 A model lists, for every layer run, what it keeps between steps:
 
 * ``PagedKV``      keys and values of an attention, in pages of 64 tokens,
+* ``PagedLatent``  latents and shared key columns of a latent attention, one
+                 row a token for all heads, in the same pages,
 * ``MatrixState``  the state of a recurrent matrix memory, one slot a request.
 
 All layers share one block table per request (page index -> the same page in
@@ -25,8 +27,25 @@ class CacheFull(RuntimeError):
     """No page or slot is free for what was asked."""
 
 
+class Paged:
+    """What is kept token by token: a ``window`` (0: every earlier token
+    stays visible) and ``keep_first`` tokens that stay visible behind it."""
+
+
 @dataclass(frozen=True)
-class PagedKV:
+class PagedLatent(Paged):
+    rank: int            # latent columns
+    shared: int          # rotated key columns, shared by all heads
+    window: int = 0
+    keep_first: int = 0
+
+    def allocate(self, pages, slots, dtype, device):
+        return torch.zeros(pages, PAGE_SIZE, self.rank + self.shared,
+                           dtype=dtype, device=device)
+
+
+@dataclass(frozen=True)
+class PagedKV(Paged):
     kv_heads: int
     dim: int
     vdim: int
@@ -76,7 +95,7 @@ class CacheManager:
         self.num_slots = max_seqs
         self.max_context = max_context or self.num_pages * PAGE_SIZE
         flat = [s for run in specs for s in run]
-        kv = [s for s in flat if isinstance(s, PagedKV)]
+        kv = [s for s in flat if isinstance(s, Paged)]
         self.paged = bool(kv)
         # a page may go once it is behind every layer's window
         self.window = max((s.window for s in kv), default=0) \

@@ -5,5 +5,7 @@ from .gpt_neox import (GPTNeoXConfig, GPTNeoXForCausalLM, get_neox_config,
                        NEOX_CONFIGS)
 from .voletar import (VoletarConfig, VoletarForCausalLM, VOLETAR_CONFIGS,
                       get_voletar_config)
+from .nesilorn import (NesilornConfig, NesilornForCausalLM, NESILORN_CONFIGS,
+                       get_nesilorn_config)
 from .registry import (ModelEntry, build_model, load_pretrained,
                        register_model, registered_models)

@@ -16,7 +16,7 @@ from typing import List, Sequence
 import torch
 import torch.nn as nn
 
-from ..inference.paged_cache import MatrixState, PagedKV
+from ..inference.paged_cache import MatrixState, PagedKV, PagedLatent
 from ..ops import serving as sv
 from ..parallel.layers import ColumnParallelLinear, RowParallelLinear
 
@@ -39,6 +39,26 @@ def copy_weight(param: torch.Tensor, value: torch.Tensor):
                          f"{tuple(param.shape)}")
     with torch.no_grad():
         param.copy_(value)
+
+
+class CheckpointReader:
+    """Hands out the tensors of a name -> tensor dictionary; a missing or
+    (``done``) an unused one is an error."""
+
+    def __init__(self, tensors: dict):
+        self.tensors, self.used = tensors, set()
+
+    def __call__(self, name: str) -> torch.Tensor:
+        if name not in self.tensors:
+            raise KeyError(f"checkpoint has no tensor {name!r}")
+        self.used.add(name)
+        return self.tensors[name]
+
+    def done(self):
+        extra = set(self.tensors) - self.used
+        if extra:
+            raise KeyError(f"checkpoint tensors without a place: "
+                           f"{sorted(extra)[:5]}")
 
 
 class Mixer(nn.Module):
@@ -95,6 +115,58 @@ class SlidingAttention(Mixer):
         return self.o(sv.ragged_attention(
             q, k, v, batch, pools[0], self.heads, self.scale, self.window,
             self.keep_first))
+
+
+class LatentAttention(Mixer):
+    """Softmax attention whose keys and values are projections of a small
+    latent, which alone is cached beside one rotated key part that all heads
+    share; a sliding window (0: plain causal) and a sigmoid gate on the
+    heads.  Every query head is [unrotated | rotated]."""
+    names = ("q", "dkv", "g")
+
+    def __init__(self, width, heads, dim, rot_dim, vdim, rank, scale,
+                 rot_base, rot_dims, eps, window=0):
+        super().__init__()
+        if rot_dims % 2 or not 0 <= rot_dims <= rot_dim:
+            raise ValueError(f"{rot_dims} of {rot_dim} dimensions turn")
+        if rank + rot_dim > sv.MAX_LATENT_ROW:
+            raise ValueError(f"latent row of {rank + rot_dim} > "
+                             f"{sv.MAX_LATENT_ROW}")
+        self.heads, self.dim, self.vdim = heads, dim, vdim
+        self.rank, self.scale, self.eps = rank, scale, eps
+        self.rot_base, self.rot_dims = rot_base, rot_dims
+        self.window = window
+        self.latent = PagedLatent(rank, rot_dim, window)
+        self.sizes = (heads * (dim + rot_dim), rank + rot_dim, heads * vdim)
+        self.norm = _vector(rank)
+        # W_uk twice: transposed per head for queries, with W_uv for keys
+        self.absorb = nn.Parameter(
+            torch.randn(heads, rank, dim) * rank ** -0.5)
+        self.expand = nn.Parameter(
+            torch.randn(heads * (dim + vdim), rank) * rank ** -0.5)
+        self._freq = None
+        self.o = _row(heads * vdim, width)
+
+    def cache_specs(self):
+        return [self.latent]
+
+    def load(self, get, prefix):
+        uk = get(prefix + "uk")
+        copy_weight(self.norm, get(prefix + "dkv.norm"))
+        copy_weight(self.expand, torch.cat([uk, get(prefix + "uv")]))
+        copy_weight(self.absorb, uk.view(self.heads, self.dim, self.rank)
+                    .transpose(1, 2))
+        copy_weight(self.o.weight, get(prefix + "o"))
+
+    def forward(self, h, proj, batch, pools):
+        q, kv, g = self.split(proj)
+        if self._freq is None or self._freq.device != h.device:
+            self._freq = sv.rotary_frequencies(self.rot_base, self.rot_dims,
+                                               h.device)
+        w = sv.LatentWeights(self.norm, self.absorb, self.expand, self._freq)
+        return self.o(sv.latent_attention(
+            q, kv, g, batch, pools[0], w, self.heads, self.dim, self.vdim,
+            self.scale, self.eps, self.window))
 
 
 class _MatrixMemory(Mixer):
@@ -235,8 +307,9 @@ class ParallelMixer(nn.Module):
             self.left_out, self.right_out, self.branch_scale)
 
 
-class ReluSquaredMLP(nn.Module):
-    """down(max(up x, 0)^2)"""
+class _PlainMLP(nn.Module):
+    """down(act(up x))"""
+    act = None
 
     def __init__(self, width, ff):
         super().__init__()
@@ -247,4 +320,46 @@ class ReluSquaredMLP(nn.Module):
         copy_weight(self.down.weight, get(prefix + "down"))
 
     def forward(self, h) -> sv.Pending:
-        return sv.Pending(self.down(sv.relu_squared_(self.up(h))))
+        return sv.Pending(self.down(self.act(self.up(h))))
+
+
+class ReluSquaredMLP(_PlainMLP):
+    act = staticmethod(sv.relu_squared_)
+
+
+class GeluMLP(_PlainMLP):
+    """The tanh form of gelu."""
+    act = staticmethod(sv.gelu_tanh_)
+
+
+class ExpertsMLP(nn.Module):
+    """A router with a bias and gated experts: min(g, limit) sigmoid(alpha g)
+    (clamp(u, limit) + shift); the ``top`` experts with the largest logits
+    are summed, weighted by a softmax over their logits.  The sum is left
+    pending, so it fuses into the next residual norm."""
+
+    def __init__(self, width, ff, experts, top, limit=math.inf, alpha=1.0,
+                 shift=0.0):
+        super().__init__()
+        if experts > sv.MAX_EXPERTS or not 1 <= top <= min(experts, 64):
+            raise ValueError(f"{top} of {experts} experts")
+        self.top, self.act = top, (alpha, limit, shift)
+        self.router = nn.Parameter(
+            torch.randn(experts, width) * width ** -0.5)
+        self.bias = nn.Parameter(torch.zeros(experts))
+        self.gate_up = nn.Parameter(torch.empty(experts, 2 * ff, width))
+        self.down = nn.Parameter(torch.empty(experts, width, ff))
+        nn.init.normal_(self.gate_up, std=width ** -0.5)
+        nn.init.normal_(self.down, std=ff ** -0.5)
+
+    def load(self, get, prefix):
+        copy_weight(self.router, get(prefix + "router"))
+        copy_weight(self.bias, get(prefix + "router.b"))
+        for e, (gu, down) in enumerate(zip(self.gate_up, self.down)):
+            p = f"{prefix}e{e}."
+            copy_weight(gu, torch.cat([get(p + "gate"), get(p + "up")]))
+            copy_weight(down, get(p + "down"))
+
+    def forward(self, h) -> sv.Pending:
+        return sv.moe_mlp(h, sv.linear_f32(h, self.router), self.bias,
+                          self.gate_up, self.down, self.top, *self.act)

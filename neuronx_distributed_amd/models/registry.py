@@ -142,3 +142,20 @@ def _voletar_build(config):
 register_model("Voletar", ModelEntry(
     _voletar_config, _voletar_build,
     lambda model, tensors: model.load_checkpoint(tensors)))
+
+
+def _nesilorn_config(d: dict):
+    from .nesilorn import NesilornConfig
+
+    return NesilornConfig.from_dict(d)
+
+
+def _nesilorn_build(config):
+    from .nesilorn import NesilornForCausalLM
+
+    return NesilornForCausalLM(config)
+
+
+register_model("Nesilorn", ModelEntry(
+    _nesilorn_config, _nesilorn_build,
+    lambda model, tensors: model.load_checkpoint(tensors)))

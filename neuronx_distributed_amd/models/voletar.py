@@ -23,8 +23,9 @@ import torch.nn as nn
 from ..ops import serving as sv
 from ..parallel import parallel_state as ps
 from ..parallel.layers import ColumnParallelLinear, ParallelEmbedding
-from .mixers import (DecayMemory, GatedMemory, ParallelMixer, ReluSquaredMLP,
-                     SingleMixer, SlidingAttention, copy_weight)
+from .mixers import (CheckpointReader, DecayMemory, GatedMemory, ParallelMixer,
+                     ReluSquaredMLP, SingleMixer, SlidingAttention,
+                     copy_weight)
 
 
 @dataclass
@@ -176,14 +177,7 @@ class VoletarForCausalLM(nn.Module):
     def load_checkpoint(self, tensors: dict):
         """Fill every parameter from a name -> tensor dictionary; a missing,
         unused or misshapen tensor is an error."""
-        used = set()
-
-        def get(name):
-            if name not in tensors:
-                raise KeyError(f"checkpoint has no tensor {name!r}")
-            used.add(name)
-            return tensors[name]
-
+        get = CheckpointReader(tensors)
         copy_weight(self.embed.weight, get("embed"))
         if self.config.loop:
             copy_weight(self.loop_in, get("loop.in"))
@@ -192,10 +186,7 @@ class VoletarForCausalLM(nn.Module):
             layer.load(get, f"l{i}.")
         copy_weight(self.final_norm, get("final.norm"))
         copy_weight(self.head.weight, get("head"))
-        extra = set(tensors) - used
-        if extra:
-            raise KeyError(f"checkpoint tensors without a place: "
-                           f"{sorted(extra)[:5]}")
+        get.done()
 
     def cache_specs(self):
         """What each layer run keeps; every pass of a looped layer has its

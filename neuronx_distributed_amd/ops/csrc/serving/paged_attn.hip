@@ -84,6 +84,7 @@ struct RowsArgs {
   const void *q, *k, *v;       // row 0 of the step's projections
   long qst, kst, vst;          // row strides (elements)
   void *kc, *vc;               // cache
+  long kcs, vcs;               // elements from one cached row to the next
   const int *pos, *seq, *bt;   // per row: position, sequence; block table
   float* part;                 // [rows][H][splits][E + 2] or null (1 split)
   void* out;                   // [rows][H * E]
@@ -91,12 +92,18 @@ struct RowsArgs {
   float scale;
 };
 
-// LPR lanes own one key row (8 dims each); RC query heads share the row.
-template <typename T, int LPR, int RC, bool VEC>
+// LPR lanes own one key row (DPL dims each); RC query heads share the row.
+template <bool VEC, int DPL, typename T>
+__device__ __forceinline__ void load_dims(const T* p, int n, float* v) {
+#pragma unroll
+  for (int j = 0; j < DPL; j += 8) load8<VEC>(p + j, n - j, v + j);
+}
+
+template <typename T, int LPR, int RC, bool VEC, int DPL = 8>
 __global__ void __launch_bounds__(256)
 attn_rows_kernel(RowsArgs a) {
   constexpr int NR = 64 / LPR;     // key rows of one wave step
-  constexpr int DV = LPR * 8;
+  constexpr int DV = LPR * DPL;
   const int rep = a.H / a.G;
   const int nrc = (rep + RC - 1) / RC;
   const int split = blockIdx.x % a.splits;
@@ -107,24 +114,25 @@ attn_rows_kernel(RowsArgs a) {
   const int lane = threadIdx.x & 63;
   const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int hl = lane % LPR, sub = lane / LPR;
-  const int d0 = 8 * hl;
-  const int nd = min(8, a.D - d0), ne = min(8, a.E - d0);  // <= 0: no dims
+  const int d0 = DPL * hl;
+  // dims of this lane; <= 0: none
+  const int nd = min(DPL, a.D - d0), ne = min(DPL, a.E - d0);
   const int D = a.D, E = a.E;
 
   const int i_pos = a.pos[row];
   const int* bt = a.bt + (long)a.seq[row] * a.MB;
 
-  float qv[RC][8];
+  float qv[RC][DPL];
 #pragma unroll
   for (int r = 0; r < RC; ++r) {
     const int h = g * rep + min(rc * RC + r, rep - 1);
-    load8<VEC>((const T*)a.q + row * a.qst + (long)h * D + d0, nd, qv[r]);
+    load_dims<VEC, DPL>((const T*)a.q + row * a.qst + (long)h * D + d0, nd, qv[r]);
   }
   const float s2 = a.scale * SV_LOG2E;
 #pragma unroll
   for (int r = 0; r < RC; ++r)
 #pragma unroll
-    for (int j = 0; j < 8; ++j) qv[r][j] *= s2;
+    for (int j = 0; j < DPL; ++j) qv[r][j] *= s2;
 
   const T* kn = (const T*)a.k + row * a.kst + (long)g * D;
   const T* vn = (const T*)a.v + row * a.vst + (long)g * E;
@@ -132,9 +140,9 @@ attn_rows_kernel(RowsArgs a) {
     const long page = bt[i_pos / SV_PAGE];
     const long base = (page * a.G + g) * SV_PAGE + i_pos % SV_PAGE;
     for (int i = threadIdx.x; i < D; i += 256)
-      ((T*)a.kc)[base * D + i] = kn[i];
+      ((T*)a.kc)[base * a.kcs + i] = kn[i];
     for (int i = threadIdx.x; i < E; i += 256)
-      ((T*)a.vc)[base * E + i] = vn[i];
+      ((T*)a.vc)[base * a.vcs + i] = vn[i];
   }
 
   // visible keys as one list: the kept first ones, then the window.  With
@@ -145,21 +153,21 @@ attn_rows_kernel(RowsArgs a) {
   const int per = (total + a.splits - 1) / a.splits;
   const int k0 = split * per, k1 = min(total, k0 + per);
 
-  float m[RC], l[RC], o[RC][8];
+  float m[RC], l[RC], o[RC][DPL];
 #pragma unroll
   for (int r = 0; r < RC; ++r) {
     m[r] = NEG_BIG;
     l[r] = 0.f;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) o[r][j] = 0.f;
+    for (int j = 0; j < DPL; ++j) o[r][j] = 0.f;
   }
 
   auto fetch = [&](int idx, float* kf, float* vf) {
     const int j = idx < nfirst ? idx : lo + idx - nfirst;
     const long base =
         ((long)bt[j / SV_PAGE] * a.G + g) * SV_PAGE + j % SV_PAGE;
-    load8<VEC>((const T*)a.kc + base * D + d0, nd, kf);
-    load8<VEC>((const T*)a.vc + base * E + d0, ne, vf);
+    load_dims<VEC, DPL>((const T*)a.kc + base * a.kcs + d0, nd, kf);
+    load_dims<VEC, DPL>((const T*)a.vc + base * a.vcs + d0, ne, vf);
   };
   auto absorb = [&](const float* kf, const float* vf, bool live) {
     float s[RC];
@@ -167,7 +175,7 @@ attn_rows_kernel(RowsArgs a) {
     for (int r = 0; r < RC; ++r) {
       s[r] = 0.f;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) s[r] += qv[r][j] * kf[j];
+      for (int j = 0; j < DPL; ++j) s[r] += qv[r][j] * kf[j];
     }
 #pragma unroll
     for (int off = LPR / 2; off > 0; off >>= 1)
@@ -181,30 +189,30 @@ attn_rows_kernel(RowsArgs a) {
       m[r] = mn;
       l[r] = l[r] * al + p;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) o[r][j] = o[r][j] * al + p * vf[j];
+      for (int j = 0; j < DPL; ++j) o[r][j] = o[r][j] * al + p * vf[j];
     }
   };
 
-  float kf[8], vf[8];
+  float kf[DPL], vf[DPL];
   int idx = k0 + wid * NR + sub;
 #pragma unroll
-  for (int j = 0; j < 8; ++j) kf[j] = vf[j] = 0.f;
+  for (int j = 0; j < DPL; ++j) kf[j] = vf[j] = 0.f;
   if (idx < k1) fetch(idx, kf, vf);
   for (int b = k0 + wid * NR; b < k1; b += 4 * NR, idx += 4 * NR) {
-    float kx[8], vx[8];
+    float kx[DPL], vx[DPL];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) kx[j] = vx[j] = 0.f;
+    for (int j = 0; j < DPL; ++j) kx[j] = vx[j] = 0.f;
     if (idx + 4 * NR < k1) fetch(idx + 4 * NR, kx, vx);
     absorb(kf, vf, idx < k1);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
+    for (int j = 0; j < DPL; ++j) {
       kf[j] = kx[j];
       vf[j] = vx[j];
     }
   }
   if (a.append && split == 0 && wid == 0) {
-    load8<VEC>(kn + d0, nd, kf);
-    load8<VEC>(vn + d0, ne, vf);
+    load_dims<VEC, DPL>(kn + d0, nd, kf);
+    load_dims<VEC, DPL>(vn + d0, ne, vf);
     absorb(kf, vf, sub == 0);
   }
 
@@ -221,7 +229,7 @@ attn_rows_kernel(RowsArgs a) {
       m[r] = mn;
       l[r] = l[r] * c1 + l2 * c2;
 #pragma unroll
-      for (int j = 0; j < 8; ++j)
+      for (int j = 0; j < DPL; ++j)
         o[r][j] = o[r][j] * c1 + __shfl_xor(o[r][j], off, 64) * c2;
     }
   __shared__ float so[4][RC][DV];
@@ -230,7 +238,7 @@ attn_rows_kernel(RowsArgs a) {
 #pragma unroll
     for (int r = 0; r < RC; ++r) {
 #pragma unroll
-      for (int j = 0; j < 8; ++j) so[wid][r][d0 + j] = o[r][j];
+      for (int j = 0; j < DPL; ++j) so[wid][r][d0 + j] = o[r][j];
       if (hl == 0) {
         sml[wid][r][0] = m[r];
         sml[wid][r][1] = l[r];
@@ -288,14 +296,27 @@ attn_rows_merge_kernel(const float* __restrict__ part, T* __restrict__ out,
   }
 }
 
+extern "C" int sv_attn_merge(const float* part, void* out, long rows,
+                             int splits, int E, int f32, hipStream_t stream) {
+  if (f32)
+    attn_rows_merge_kernel<float><<<rows, 64, 0, stream>>>(part, (float*)out,
+                                                           splits, E);
+  else
+    attn_rows_merge_kernel<short><<<rows, 64, 0, stream>>>(part, (short*)out,
+                                                           splits, E);
+  return (int)hipGetLastError();
+}
+
 template <typename T>
 static int launch_rows(const RowsArgs& a, int vec, hipStream_t stream) {
   const int rep = a.H / a.G;
   const int big = a.D > a.E ? a.D : a.E;
-  const int rcn = rep >= 8 ? 8 : rep > 2 ? 4 : rep;
+  const int rcn = big > 512 ? (rep > 1 ? 2 : 1)
+                            : rep >= 8 ? 8 : rep > 2 ? 4 : rep;
   const int nrc = (rep + rcn - 1) / rcn;
   const long grid = (long)a.rows * a.G * nrc * a.splits;
-#define AR(L, R, V) attn_rows_kernel<T, L, R, V><<<grid, 256, 0, stream>>>(a)
+#define AR(L, ...) \
+  attn_rows_kernel<T, L, __VA_ARGS__><<<grid, 256, 0, stream>>>(a)
 #define ARV(L, R) do { if (vec) AR(L, R, true); else AR(L, R, false); } while (0)
 #define ARR(L)                                                         \
   do {                                                                 \
@@ -306,13 +327,16 @@ static int launch_rows(const RowsArgs& a, int vec, hipStream_t stream) {
   else if (big <= 128) ARR(16);
   else if (big <= 256) ARR(32);
   else if (big <= 512) ARR(64);
-  else return 1;
+  else if (big <= 1024) {
+    if (rcn == 2) { if (vec) AR(64, 2, true, 16); else AR(64, 2, false, 16); }
+    else { if (vec) AR(64, 1, true, 16); else AR(64, 1, false, 16); }
+  } else return 1;
 #undef ARR
 #undef ARV
 #undef AR
   if (a.splits > 1)
-    attn_rows_merge_kernel<T><<<(long)a.rows * a.H, 64, 0, stream>>>(
-        a.part, (T*)a.out, a.splits, a.E);
+    return sv_attn_merge(a.part, a.out, (long)a.rows * a.H, a.splits, a.E,
+                         sizeof(T) == 4, stream);
   return (int)hipGetLastError();
 }
 
@@ -334,27 +358,45 @@ extern "C" int sv_attn_rows(const RowsArgs* a, int vec, int f32,
 // {4 hi + 0..3, 8 + 4 hi + 0..3} of a 16-key chunk is used as the
 // contraction order of P V, and V^T is read from LDS in the same order.
 // ---------------------------------------------------------------------------
+//
+// A key may end in columns that all heads share (kr): the rotated part of
+// latent attention, whose other columns are expanded into a workspace first.
+// The output may pass through sigmoid(gate).
 struct TilesArgs {
   const short* q;
   long qst;                 // row stride of q
-  const short *kc, *vc;
+  const short *kc, *vc, *kr;
+  long kpage, khead, krow;  // elements between pages, heads, rows
+  long vpage, vhead, vrow;
+  long rrow;                // between rows of kr (pages follow each other)
+  const short* gate;        // [T][H * E] or null
+  long gst;
   const int* tiles;         // [n_tiles][4]: seq, first row, rows, position
   const int* bt;
   short* out;               // [T][H * E]
-  int MB, H, G, D, E, window, keep;
+  int MB, H, G, D, E, DS;   // DS: columns of a key before the shared ones
+  int window, keep;
   float scale;
 };
 
-template <int DP, int NP>
-__global__ void __launch_bounds__(256, DP <= 128 ? 2 : 1)
+// 16-byte slots of a row of CPR slots, rotated so that consecutive rows of
+// one column spread over the banks
+template <int CPR>
+__device__ __forceinline__ int row_swz(int row, int byte) {
+  return byte ^ ((CPR % 16 == 0 ? row & 15
+                  : CPR % 8 == 0 ? (row >> 1) & 7 : (row >> 2) & 3) << 4);
+}
+
+template <int DK, int DE, int NP>
+__global__ void __launch_bounds__(256, DE <= 128 ? 2 : 1)
 attn_tiles_kernel(TilesArgs a) {
-  constexpr int NC = DP / 16;        // 16-wide chunks of the head size
-  constexpr int NB = DP / 32;        // 32-row blocks of O^T
-  constexpr int KP = DP * 2;         // K row pitch (bytes)
-  constexpr int CPR = DP / 8;        // 16-byte slots of a row
-  constexpr int PAIRS = 32 * CPR / 256;  // (row pair, slot) items a thread
+  constexpr int NC = DK / 16;        // 16-wide chunks of the key size
+  constexpr int NB = DE / 32;        // 32-row blocks of O^T
+  constexpr int KP = DK * 2;         // K row pitch (bytes)
+  constexpr int CK = DK / 8, CV = DE / 8;  // 16-byte slots of a row
+  constexpr int PK = 32 * CK / 256, PV = 32 * CV / 256;  // items a thread
   __shared__ __attribute__((aligned(16))) char kbuf[64 * KP];
-  __shared__ __attribute__((aligned(16))) short vbuf[DP * 64];  // V^T
+  __shared__ __attribute__((aligned(16))) short vbuf[DE * 64];  // V^T
 
   // later tiles of a portion see more keys: they start first
   const int* tl = a.tiles + 4 * (gridDim.y - 1 - blockIdx.y);
@@ -392,35 +434,50 @@ attn_tiles_kernel(TilesArgs a) {
   const int ntiles = nk + max(0, t_hi - t_lo + 1);
   const int w_lo = p0 + wid * 32, w_hi = min(w_lo + 31, q_hi);
 
-  uint4v kreg[2 * PAIRS], vreg[2 * PAIRS];
+  uint4v kreg[2 * PK], vreg[2 * PV];
   auto tile_of = [&](int n) { return n < nk ? n : t_lo + n - nk; };
+  // items are (row pair, slot) of the tile
   auto issue = [&](int n) {
-    const long base = ((long)bt[tile_of(n)] * a.G + g) * SV_PAGE;
+    const long page = bt[tile_of(n)];
+    const short* kb = a.kc + page * a.kpage + g * a.khead;
+    const short* vb = a.vc + page * a.vpage + g * a.vhead;
+    const short* rb = a.kr + page * SV_PAGE * a.rrow - a.DS;
 #pragma unroll
-    for (int p = 0; p < PAIRS; ++p) {
+    for (int p = 0; p < PK; ++p) {
       const int it = p * 256 + tid;
-      const int r = it / CPR * 2, c = it % CPR * 8;
+      const int r = it / CK * 2, c = it % CK * 8;
 #pragma unroll
-      for (int x = 0; x < 2; ++x) {
+      for (int x = 0; x < 2; ++x)
         kreg[2 * p + x] = c < D
-            ? *(const uint4v*)(a.kc + (base + r + x) * D + c)
+            ? *(const uint4v*)(c < a.DS ? kb + (r + x) * a.krow + c
+                                        : rb + (r + x) * a.rrow + c)
             : uint4v{0, 0, 0, 0};
-        vreg[2 * p + x] = c < E
-            ? *(const uint4v*)(a.vc + (base + r + x) * E + c)
-            : uint4v{0, 0, 0, 0};
-      }
     }
-  };
-  auto kswz = [](int row, int byte) {
-    return CPR >= 16 ? swz16(row, byte) : swz(row, byte);
+#pragma unroll
+    for (int p = 0; p < PV; ++p) {
+      const int it = p * 256 + tid;
+      const int r = it / CV * 2, c = it % CV * 8;
+#pragma unroll
+      for (int x = 0; x < 2; ++x)
+        vreg[2 * p + x] = c < E
+            ? *(const uint4v*)(vb + (r + x) * a.vrow + c)
+            : uint4v{0, 0, 0, 0};
+    }
   };
   auto commit = [&]() {
 #pragma unroll
-    for (int p = 0; p < PAIRS; ++p) {
+    for (int p = 0; p < PK; ++p) {
       const int it = p * 256 + tid;
-      const int r = it / CPR * 2, c = it % CPR * 8;
-      *(uint4v*)(kbuf + r * KP + kswz(r, c * 2)) = kreg[2 * p];
-      *(uint4v*)(kbuf + (r + 1) * KP + kswz(r + 1, c * 2)) = kreg[2 * p + 1];
+      const int r = it / CK * 2, c = it % CK * 16;
+#pragma unroll
+      for (int x = 0; x < 2; ++x)
+        *(uint4v*)(kbuf + (r + x) * KP + row_swz<CK>(r + x, c)) =
+            kreg[2 * p + x];
+    }
+#pragma unroll
+    for (int p = 0; p < PV; ++p) {
+      const int it = p * 256 + tid;
+      const int r = it / CV * 2, c = it % CV * 8;
       union { uint4v u; unsigned short s[8]; } x, y;
       x.u = vreg[2 * p];
       y.u = vreg[2 * p + 1];
@@ -452,7 +509,7 @@ attn_tiles_kernel(TilesArgs a) {
       for (int c = 0; c < NC; ++c) {
         frag_u kf;
         kf.u4 = *(const uint4v*)(kbuf + row * KP +
-                                 kswz(row, (c * 16 + hi * 8) * 2));
+                                 row_swz<CK>(row, (c * 16 + hi * 8) * 2));
         acc[kb] = mfma_bf16(kf.bf, qf[c].bf, acc[kb]);
       }
     }
@@ -533,24 +590,33 @@ attn_tiles_kernel(TilesArgs a) {
     for (int rg = 0; rg < 4; ++rg) {
       const int d = 32 * nb + 8 * rg + 4 * hi;
       if (d < E) {
-        uint2 w = {pack_bf16x2(ot[nb][4 * rg] * inv, ot[nb][4 * rg + 1] * inv),
-                   pack_bf16x2(ot[nb][4 * rg + 2] * inv,
-                               ot[nb][4 * rg + 3] * inv)};
+        float o[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[j] = ot[nb][4 * rg + j] * inv;
+        if (a.gate) {
+          float z[4];
+          load4(a.gate + (long)(row0 + my) * a.gst + (long)h * E + d, z);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) o[j] *= sigmoid_f(z[j]);
+        }
+        uint2 w = {pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
         *(uint2*)(dst + d) = w;
       }
     }
 }
 
-// D and E multiples of 8, at most 256; q rows 16-byte aligned
+// D, DS and E multiples of 8, at most 256; every row 16-byte aligned
 extern "C" int sv_attn_tiles(const TilesArgs* a, int n_tiles,
                              hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  const int big = a->D > a->E ? a->D : a->E;
   const dim3 grid(a->H, n_tiles);
-  if (big <= 64) attn_tiles_kernel<64, 3><<<grid, 256, 0, stream>>>(*a);
-  else if (big <= 128) attn_tiles_kernel<128, 3><<<grid, 256, 0, stream>>>(*a);
-  else if (big <= 256) attn_tiles_kernel<256, 3><<<grid, 256, 0, stream>>>(*a);
+#define AT(K, V) attn_tiles_kernel<K, V, 3><<<grid, 256, 0, stream>>>(*a)
+  if (a->D <= 64 && a->E <= 64) AT(64, 64);
+  else if (a->D <= 128 && a->E <= 128) AT(128, 128);
+  else if (a->D <= 192 && a->E <= 128) AT(192, 128);
+  else if (a->D <= 256 && a->E <= 256) AT(256, 256);
   else return 1;
+#undef AT
   return (int)hipGetLastError();
 }
 

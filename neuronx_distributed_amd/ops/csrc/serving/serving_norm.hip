@@ -1,10 +1,12 @@
 // Norms and pointwise steps of the serving path (32-bit residual stream).
 //
 // residual_norm: one pass that (1) adds a pending sublayer result to the
-// 32-bit residual, (2) stores the new residual, (3) writes the RMS-normed
-// row for the next projection and/or the concatenation [x; x0] that a
-// looped block projects.  The pending result is nothing, one tensor, or two
-// parallel branches that are RMS-normed on their own, scaled and summed.
+// 32-bit residual, (2) stores the new residual, (3) writes the row for the
+// next projection (RMS-normed, or just rounded) and/or the concatenation
+// [x; x0] that a looped block projects.  The pending result is nothing, one
+// tensor, a weighted sum of several rows a token (expert outputs), or two
+// parallel branches.  One tensor or sum may be RMS-normed before it is added,
+// two branches always are; the result is scaled.
 //
 // gated_norm: RMS norm over groups of a row, times a weight, times
 // sigmoid(gate) — the output stage of the gated recurrent mixers.
@@ -15,17 +17,19 @@ struct ResidualNormArgs {
   const float* x;        // [rows, W] residual, or null (starts from zero)
   const void* delta;     // [rows, W] T (or f32), or null
   const void* delta2;    // second branch, or null
-  const void* w1;        // branch norm weights [W] (dual mode)
-  const void* w2;
+  const void* w1;        // norm weights [W] of the pending result, or null
+  const void* w2;        // of the second branch
+  const float* coef;     // [rows, parts]: delta is [rows * parts, W]; or null
   const void* vec;       // [W] added to every row, or null
   float* x_out;          // [out_rows, W] or null
   void* h;               // [out_rows, W] normed * w, or null
-  const void* w;         // [W] weight of the norm
+  const void* w;         // [W] weight of the norm; null: h is x, rounded
   void* cat;             // [out_rows, 2 W]: new x, then x0; or null
   const void* x0;        // [rows, W]
   const int* index;      // out row -> row, or null
-  int rows_out, W, delta_f32;
-  float eps, branch_scale;
+  int rows_out, W, delta_f32, parts;
+  float eps, scale;
+  float w_base, p_base;  // added to w, and to w1 and w2
 };
 
 template <typename T, int VEC>
@@ -49,7 +53,27 @@ residual_norm_kernel(ResidualNormArgs a) {
   const float* d1f = (const float*)a.delta + r * W;
   const T* d2 = (const T*)a.delta2 + r * W;
 
-  float s1 = 0.f, s2 = 0.f;
+  // the pending result when it is one tensor or a weighted sum of rows
+  auto single = [&](int i, float* v) {
+    if (a.coef) {
+      float t[VEC];
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] = 0.f;
+      const T* d = (const T*)a.delta + r * a.parts * W;
+      for (int p = 0; p < a.parts; ++p) {
+        const float c = a.coef[r * a.parts + p];
+        ld<T, VEC>(d + (long)p * W + i, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[j] += c * t[j];
+      }
+    } else if (a.delta_f32) {
+      ld<float, VEC>(d1f + i, v);
+    } else {
+      ld<T, VEC>(d1 + i, v);
+    }
+  };
+
+  float s1 = a.scale, s2 = 0.f;
   if (a.delta2) {
     float q1 = 0.f, q2 = 0.f, v[VEC];
     for (int i = tid * VEC; i < W; i += 256 * VEC) {
@@ -64,8 +88,19 @@ residual_norm_kernel(ResidualNormArgs a) {
     __syncthreads();
     q2 = block_reduce_sum(q2, red);
     __syncthreads();
-    s1 = a.branch_scale / sqrtf(q1 / W + a.eps);
-    s2 = a.branch_scale / sqrtf(q2 / W + a.eps);
+    s1 = a.scale / sqrtf(q1 / W + a.eps);
+    s2 = a.scale / sqrtf(q2 / W + a.eps);
+  } else if (a.w1) {
+    float q1 = 0.f, v[VEC];
+    for (int i = tid * VEC; i < W; i += 256 * VEC) {
+      single(i, v);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) q1 += v[j] * v[j];
+      st<float, VEC>(row + i, v);
+    }
+    q1 = block_reduce_sum(q1, red);
+    __syncthreads();
+    s1 = a.scale / sqrtf(q1 / W + a.eps);
   }
 
   float sq = 0.f;
@@ -78,17 +113,21 @@ residual_norm_kernel(ResidualNormArgs a) {
       ld<T, VEC>(d1 + i, t);
       ld<T, VEC>((const T*)a.w1 + i, u);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) t[j] *= s1 * u[j];
+      for (int j = 0; j < VEC; ++j) t[j] *= s1 * (a.p_base + u[j]);
       float p[VEC];
       ld<T, VEC>(d2 + i, p);
       ld<T, VEC>((const T*)a.w2 + i, u);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) v[j] += t[j] + p[j] * s2 * u[j];
-    } else if (a.delta) {
-      if (a.delta_f32) ld<float, VEC>(d1f + i, t);
-      else ld<T, VEC>(d1 + i, t);
+      for (int j = 0; j < VEC; ++j) v[j] += t[j] + p[j] * s2 * (a.p_base + u[j]);
+    } else if (a.w1) {
+      ld<float, VEC>(row + i, t);  // written by this same thread
+      ld<T, VEC>((const T*)a.w1 + i, u);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) v[j] += t[j];
+      for (int j = 0; j < VEC; ++j) v[j] += t[j] * s1 * (a.p_base + u[j]);
+    } else if (a.delta) {
+      single(i, t);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] += s1 * t[j];
     }
     if (a.vec) {
       ld<T, VEC>((const T*)a.vec + i, t);
@@ -103,9 +142,12 @@ residual_norm_kernel(ResidualNormArgs a) {
       ld<T, VEC>((const T*)a.x0 + r * W + i, t);
       st<T, VEC>((T*)a.cat + (2L * o + 1) * W + i, t);
     }
-    if (a.h) st<float, VEC>(row + i, v);
+    if (a.h) {
+      if (a.w) st<float, VEC>(row + i, v);
+      else st<T, VEC>((T*)a.h + (long)o * W + i, v);
+    }
   }
-  if (!a.h) return;
+  if (!a.h || !a.w) return;
   sq = block_reduce_sum(sq, red);
   const float rstd = 1.f / sqrtf(sq / W + a.eps);
   for (int i = tid * VEC; i < W; i += 256 * VEC) {
@@ -113,7 +155,7 @@ residual_norm_kernel(ResidualNormArgs a) {
     ld<float, VEC>(row + i, v);  // written by this same thread
     ld<T, VEC>((const T*)a.w + i, u);
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) v[j] *= rstd * u[j];
+    for (int j = 0; j < VEC; ++j) v[j] *= rstd * (a.w_base + u[j]);
     st<T, VEC>((T*)a.h + (long)o * W + i, v);
   }
 }
@@ -121,7 +163,8 @@ residual_norm_kernel(ResidualNormArgs a) {
 extern "C" int sv_residual_norm(const ResidualNormArgs* a, int f32,
                                 hipStream_t stream) {
   if (a->rows_out <= 0) return 0;
-  const size_t lds = a->h ? (size_t)a->W * sizeof(float) : 0;
+  const bool staged = (a->h && a->w) || (a->w1 && !a->delta2);
+  const size_t lds = staged ? (size_t)a->W * sizeof(float) : 0;
   if (lds > 160 * 1024 - 256) return 1;
 #define RN(T, V)                                                           \
   residual_norm_kernel<T, V><<<a->rows_out, 256, lds, stream>>>(*a)
@@ -192,35 +235,53 @@ extern "C" int sv_gated_norm(const void* o, const void* w, const void* gate,
 }
 
 // ---------------------------------------------------------------------------
-// pointwise: max(x, 0)^2 in place; cap * tanh(x / cap) in place (f32)
+// pointwise, in place: max(x, 0)^2, the tanh form of gelu;
+// cap * tanh(x / cap) (f32)
 // ---------------------------------------------------------------------------
-template <typename T, int VEC>
+struct ReluSquared {
+  __device__ static float at(float x) {
+    const float p = fmaxf(x, 0.f);
+    return p * p;
+  }
+};
+// 0.5 x (1 + tanh(u)) = x sigmoid(2 u)
+struct GeluTanh {
+  __device__ static float at(float x) {
+    const float u = 0.7978845608028654f * (x + 0.044715f * x * x * x);
+    return x * sigmoid_f(2.f * u);
+  }
+};
+
+template <typename T, int VEC, typename F>
 __global__ void __launch_bounds__(256)
-relu_squared_kernel(T* __restrict__ x, long n) {
+pointwise_kernel(T* __restrict__ x, long n) {
   const long i = ((long)blockIdx.x * 256 + threadIdx.x) * VEC;
   if (i >= n) return;
   float v[VEC];
   ld<T, VEC>(x + i, v);
 #pragma unroll
-  for (int j = 0; j < VEC; ++j) {
-    const float p = fmaxf(v[j], 0.f);
-    v[j] = p * p;
-  }
+  for (int j = 0; j < VEC; ++j) v[j] = F::at(v[j]);
   st<T, VEC>(x + i, v);
 }
 
-extern "C" int sv_relu_squared(void* x, long n, int f32, hipStream_t stream) {
+template <typename F>
+static int launch_pointwise(void* x, long n, int f32, hipStream_t stream) {
   if (n <= 0) return 0;
   const int vec = n % 4 == 0 ? 4 : 1;
   const long blocks = (n / vec + 255) / 256;
-  if (f32) {
-    if (vec == 4) relu_squared_kernel<float, 4><<<blocks, 256, 0, stream>>>((float*)x, n);
-    else relu_squared_kernel<float, 1><<<blocks, 256, 0, stream>>>((float*)x, n);
-  } else {
-    if (vec == 4) relu_squared_kernel<short, 4><<<blocks, 256, 0, stream>>>((short*)x, n);
-    else relu_squared_kernel<short, 1><<<blocks, 256, 0, stream>>>((short*)x, n);
-  }
+#define PW(T, V) pointwise_kernel<T, V, F><<<blocks, 256, 0, stream>>>((T*)x, n)
+  if (f32) { if (vec == 4) PW(float, 4); else PW(float, 1); }
+  else     { if (vec == 4) PW(short, 4); else PW(short, 1); }
+#undef PW
   return (int)hipGetLastError();
+}
+
+extern "C" int sv_relu_squared(void* x, long n, int f32, hipStream_t stream) {
+  return launch_pointwise<ReluSquared>(x, n, f32, stream);
+}
+
+extern "C" int sv_gelu_tanh(void* x, long n, int f32, hipStream_t stream) {
+  return launch_pointwise<GeluTanh>(x, n, f32, stream);
 }
 
 __global__ void __launch_bounds__(256)

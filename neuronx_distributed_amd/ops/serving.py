@@ -16,6 +16,9 @@ import torch
 
 PAGE_SIZE = 64
 MAX_HEAD_DIM = 512          # attention q/k and v size, recurrent q/k size
+MAX_LATENT_ROW = 1024       # latents and shared key columns of a cached row
+MAX_EXPERTS = 512
+EXPAND_MIN_TOKENS = 32      # shorter portions attend in the latent space
 CHUNK = 256                 # tokens of one chunk of a matrix memory
 
 _LIB = None
@@ -69,16 +72,18 @@ def _fields(names, ctype):
 
 
 class _ResidualNormArgs(ctypes.Structure):
-    _fields_ = (_fields("x delta delta2 w1 w2 vec x_out h w cat x0 index",
-                        ctypes.c_void_p)
-                + _fields("rows_out W delta_f32", ctypes.c_int)
-                + _fields("eps branch_scale", ctypes.c_float))
+    _fields_ = (_fields("x delta delta2 w1 w2 coef vec x_out h w cat x0 "
+                        "index", ctypes.c_void_p)
+                + _fields("rows_out W delta_f32 parts", ctypes.c_int)
+                + _fields("eps scale w_base p_base", ctypes.c_float))
 
 
 class _RowsArgs(ctypes.Structure):
     _fields_ = (_fields("q k v", ctypes.c_void_p)
                 + _fields("qst kst vst", ctypes.c_long)
-                + _fields("kc vc pos seq bt part out", ctypes.c_void_p)
+                + _fields("kc vc", ctypes.c_void_p)
+                + _fields("kcs vcs", ctypes.c_long)
+                + _fields("pos seq bt part out", ctypes.c_void_p)
                 + _fields("MB rows H G D E splits append window keep",
                           ctypes.c_int)
                 + _fields("scale", ctypes.c_float))
@@ -86,9 +91,54 @@ class _RowsArgs(ctypes.Structure):
 
 class _TilesArgs(ctypes.Structure):
     _fields_ = (_fields("q", ctypes.c_void_p) + _fields("qst", ctypes.c_long)
-                + _fields("kc vc tiles bt out", ctypes.c_void_p)
-                + _fields("MB H G D E window keep", ctypes.c_int)
+                + _fields("kc vc kr", ctypes.c_void_p)
+                + _fields("kpage khead krow vpage vhead vrow rrow",
+                          ctypes.c_long)
+                + _fields("gate", ctypes.c_void_p)
+                + _fields("gst", ctypes.c_long)
+                + _fields("tiles bt out", ctypes.c_void_p)
+                + _fields("MB H G D E DS window keep", ctypes.c_int)
                 + _fields("scale", ctypes.c_float))
+
+
+class _LatentAppendArgs(ctypes.Structure):
+    _fields_ = (_fields("q", ctypes.c_void_p)
+                + _fields("qst qh", ctypes.c_long)
+                + _fields("qr", ctypes.c_void_p)
+                + _fields("qrst qrh", ctypes.c_long)
+                + _fields("kv", ctypes.c_void_p)
+                + _fields("kvst", ctypes.c_long)
+                + _fields("w freq cache pos seq bt", ctypes.c_void_p)
+                + _fields("MB H R P rot", ctypes.c_int)
+                + _fields("eps", ctypes.c_float))
+
+
+class _HeadLinearArgs(ctypes.Structure):
+    _fields_ = (_fields("x", ctypes.c_void_p)
+                + _fields("xst xh", ctypes.c_long)
+                + _fields("w out", ctypes.c_void_p)
+                + _fields("ost oh", ctypes.c_long)
+                + _fields("gate", ctypes.c_void_p)
+                + _fields("gst gh", ctypes.c_long)
+                + _fields("T H N K", ctypes.c_int))
+
+
+class _LatentRowsArgs(ctypes.Structure):
+    _fields_ = (_fields("q cache pos seq bt part out", ctypes.c_void_p)
+                + _fields("MB rows H R P splits window", ctypes.c_int)
+                + _fields("scale", ctypes.c_float))
+
+
+class _MoePlanArgs(ctypes.Structure):
+    _fields_ = (_fields("z bias idx coef order tiles", ctypes.c_void_p)
+                + _fields("T E top tile_rows max_tiles", ctypes.c_int))
+
+
+class _MoeGemmArgs(ctypes.Structure):
+    _fields_ = (_fields("x", ctypes.c_void_p) + _fields("xst", ctypes.c_long)
+                + _fields("w out order tiles", ctypes.c_void_p)
+                + _fields("top N K max_tiles", ctypes.c_int)
+                + _fields("alpha limit shift", ctypes.c_float))
 
 
 class _MemoryArgs(ctypes.Structure):
@@ -125,24 +175,38 @@ def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 @dataclass
 class Pending:
     """A sublayer result that has not been added to the residual yet: one
-    tensor, or two branches that are RMS-normed with their own weights,
-    scaled and summed.  ``vec`` is a row added to every token."""
+    tensor, or two branches that are RMS-normed with their own weights and
+    summed; ``scale`` times that.  One tensor is RMS-normed when ``w1`` is
+    given.  ``coef`` (rows, parts) makes a row the weighted sum of ``parts``
+    rows of ``delta`` (rows * parts, W).  ``centred``: w1 and w2 are stored as
+    their distance from one.  ``vec`` is a row added to every token."""
     delta: torch.Tensor
     delta2: Optional[torch.Tensor] = None
     w1: Optional[torch.Tensor] = None
     w2: Optional[torch.Tensor] = None
-    branch_scale: float = 1.0
+    scale: float = 1.0
     vec: Optional[torch.Tensor] = None
+    coef: Optional[torch.Tensor] = None
+    centred: bool = False
 
 
 def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
                   eps: float, weight: Optional[torch.Tensor] = None,
                   x0: Optional[torch.Tensor] = None, keep_x: bool = True,
-                  index: Optional[torch.Tensor] = None, dtype=None):
+                  index: Optional[torch.Tensor] = None, dtype=None,
+                  centred: bool = False, copy: bool = False):
     """Add ``pending`` to the float32 residual ``x`` (None: zero) and return
-    (new x or None, RMS-normed row * weight or None, [new x; x0] or None)."""
+    (new x or None, RMS-normed row * weight or None, [new x; x0] or None).
+    ``centred``: the weight is stored as its distance from one.  ``copy``: the
+    second result is the new x itself, rounded to ``dtype``."""
     src = x if pending is None else pending.delta
     rows, W = src.shape
+    if pending is not None and pending.coef is not None:
+        assert pending.coef.is_contiguous() and \
+            pending.coef.dtype == torch.float32
+        assert pending.delta2 is None and \
+            pending.coef.numel() == rows
+        rows = pending.coef.shape[0]
     dtype = dtype or (weight if weight is not None else x0).dtype
     f32 = _f32(src) if dtype == torch.float32 else 0
     out_rows = rows if index is None else index.shape[0]
@@ -150,12 +214,13 @@ def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
     x_new = torch.empty(out_rows, W, dtype=torch.float32, device=dev) \
         if keep_x else None
     h = torch.empty(out_rows, W, dtype=dtype, device=dev) \
-        if weight is not None else None
+        if weight is not None or copy else None
     cat = torch.empty(out_rows, 2 * W, dtype=dtype, device=dev) \
         if x0 is not None else None
     a = _ResidualNormArgs(rows_out=out_rows, W=W, eps=eps)
     a.x, a.x_out, a.h, a.w = _p(x), _p(x_new), _p(h), _p(weight)
     a.cat, a.x0, a.index = _p(cat), _p(x0), _p(index)
+    a.w_base, a.scale = float(centred), 1.0
     if pending is not None:
         d = pending.delta
         assert d.is_contiguous() and d.dtype in (dtype, torch.float32)
@@ -164,7 +229,11 @@ def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
             and pending.delta2.shape == d.shape)
         a.delta, a.delta2 = _p(d), _p(pending.delta2)
         a.w1, a.w2, a.vec = _p(pending.w1), _p(pending.w2), _p(pending.vec)
-        a.branch_scale = pending.branch_scale
+        a.coef, a.scale = _p(pending.coef), pending.scale
+        if pending.coef is not None:
+            a.parts = pending.coef.shape[1]
+            assert d.dtype == dtype
+        a.p_base = float(pending.centred)
         a.delta_f32 = int(d.dtype == torch.float32 and
                           dtype != torch.float32)
     _check(library().sv_residual_norm(ctypes.byref(a), f32, _stream()),
@@ -195,6 +264,14 @@ def relu_squared_(x: torch.Tensor) -> torch.Tensor:
     _check(library().sv_relu_squared(ctypes.c_void_p(_p(x)),
                                      ctypes.c_long(x.numel()), _f32(x),
                                      _stream()), "relu_squared")
+    return x
+
+
+def gelu_tanh_(x: torch.Tensor) -> torch.Tensor:
+    assert x.is_contiguous()
+    _check(library().sv_gelu_tanh(ctypes.c_void_p(_p(x)),
+                                  ctypes.c_long(x.numel()), _f32(x),
+                                  _stream()), "gelu_tanh")
     return x
 
 
@@ -253,6 +330,12 @@ def kv_append(k, v, kc, vc, pos, seq, block_table):
         int(_aligned((D, E), k, v)), _f32(k), _stream()), "kv_append")
 
 
+def _row_splits(target: int, units: int, max_keys: int, per: int) -> int:
+    """Workgroups that share a row: enough for ``target`` of them, each with
+    about ``per`` keys or more."""
+    return max(1, min(target // max(1, units), -(-max_keys // per), 64))
+
+
 def attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads: int,
               scale: float, window: int = 0, keep: int = 0,
               append: bool = True, max_keys: int = 0,
@@ -266,13 +349,13 @@ def attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads: int,
     assert pos.shape[0] == rows and seq.shape[0] == rows
     if window > 0:
         max_keys = min(max_keys, window + keep) if max_keys else window + keep
-    want = max(1, 1024 // max(1, rows * G))
-    splits = max(1, min(want, (max_keys + 127) // 128, 64))
+    splits = _row_splits(1024, rows * G, max_keys, 128)
     out = _out(out, rows, heads * E, q)
     part = torch.empty(rows * heads * splits * (E + 2), dtype=torch.float32,
                        device=q.device) if splits > 1 else None
     a = _RowsArgs(q=_p(q), k=_p(k), v=_p(v), qst=q.stride(0),
                   kst=k.stride(0), vst=v.stride(0), kc=_p(kc), vc=_p(vc),
+                  kcs=D, vcs=E,
                   pos=_p(pos), seq=_p(seq), bt=_p(block_table),
                   part=_p(part), out=_p(out), MB=block_table.shape[1],
                   rows=rows, H=heads, G=G, D=D, E=E, splits=splits,
@@ -304,8 +387,10 @@ def attn_portions(q, k, v, kc, vc, pos, seq, block_table, tiles, heads: int,
                          max_keys=max_keys, out=out)
     out = _out(out, q.shape[0], heads * E, q)
     a = _TilesArgs(q=_p(q), qst=q.stride(0), kc=_p(kc), vc=_p(vc),
+                   kpage=G * PAGE_SIZE * D, khead=PAGE_SIZE * D, krow=D,
+                   vpage=G * PAGE_SIZE * E, vhead=PAGE_SIZE * E, vrow=E,
                    tiles=_p(tiles), bt=_p(block_table), out=_p(out),
-                   MB=block_table.shape[1], H=heads, G=G, D=D, E=E,
+                   MB=block_table.shape[1], H=heads, G=G, D=D, E=E, DS=D,
                    window=window, keep=keep, scale=scale)
     _check(library().sv_attn_tiles(ctypes.byref(a), tiles.shape[0],
                                    _stream()), "attn_tiles")
@@ -453,3 +538,299 @@ def decay_gate(decay, device) -> DecayGate:
     # finite for a decay of zero: 0 tokens apart must still weigh 2^0
     log2 = torch.log2(d).clamp(min=-1e4)
     return DecayGate(d.float().to(device), log2.float().to(device))
+
+
+# ---------------------------------------------------------------------------
+# latent attention
+# ---------------------------------------------------------------------------
+
+@dataclass
+class KeySpans:
+    """The keys that the prompt portions of a step see, gathered page after
+    page into a workspace."""
+    pages: torch.Tensor        # (n,) cache page of every workspace page
+    table: torch.Tensor        # (portions, width) position / 64 -> its page
+
+
+def key_spans(portions, block_table, window: int):
+    """Host form of KeySpans: (pages, table) as lists of int from portions
+    (slot, first row, rows, context) and their block-table rows."""
+    pages, table = [], []
+    for (_, _, n, ctx), row in zip(portions, block_table):
+        a = max(0, ctx - window + 1) // PAGE_SIZE if window > 0 else 0
+        b = (ctx + n - 1) // PAGE_SIZE
+        places = [0] * len(row)
+        for p in range(a, b + 1):
+            places[p] = len(pages)
+            pages.append(int(row[p]))
+        table.append(places)
+    return pages, table
+
+
+def rotary_frequencies(base: float, dims: int, device) -> torch.Tensor:
+    """Radians a position of every rotated pair, float64."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    return torch.pow(torch.tensor(base, dtype=torch.float64),
+                     -2.0 * i / dims).to(device)
+
+
+@dataclass
+class LatentWeights:
+    norm: torch.Tensor         # (rank,) of the latents
+    absorb: torch.Tensor       # (H, rank, dim): query -> latent space
+    expand: torch.Tensor       # (H * dim + H * vdim, rank): keys, values
+    freq: torch.Tensor         # (rot / 2,) float64, from rotary_frequencies
+
+
+def latent_append(q, rot_at: int, q_step: int, qr, qr_at: int, qr_step: int,
+                  kv, w: LatentWeights, cache, pos, seq, block_table,
+                  heads: int, eps: float):
+    """Norm the latents of kv (T, rank + P), rotate the shared key, write
+    both into the cache (pages, 64, rank + P); rotate columns [rot_at, + P) of
+    every head of q (heads ``q_step`` apart) into those at ``qr_at`` of qr."""
+    T, R = q.shape[0], w.norm.shape[0]
+    P = cache.shape[2] - R
+    half = w.freq.shape[0]
+    assert kv.shape == (T, R + P) and cache.shape[1] == PAGE_SIZE
+    assert cache.is_contiguous() and 2 * half <= P
+    assert w.freq.dtype == torch.float64 and w.freq.is_cuda
+    assert q.stride(1) == qr.stride(1) == kv.stride(1) == 1
+    assert q.dtype == qr.dtype == kv.dtype == cache.dtype == w.norm.dtype
+    assert (heads - 1) * q_step + rot_at + P <= q.shape[1]
+    assert (heads - 1) * qr_step + qr_at + P <= qr.shape[1]
+    assert pos.shape[0] == seq.shape[0] == T == qr.shape[0]
+    size = q.element_size()
+    a = _LatentAppendArgs(
+        q=_p(q) + rot_at * size, qst=q.stride(0), qh=q_step,
+        qr=_p(qr) + qr_at * size, qrst=qr.stride(0), qrh=qr_step, kv=_p(kv),
+        kvst=kv.stride(0), w=_p(w.norm), freq=_p(w.freq), cache=_p(cache),
+        pos=_p(pos), seq=_p(seq), bt=_p(block_table),
+        MB=block_table.shape[1], H=heads, R=R, P=P, rot=2 * half, eps=eps)
+    _check(library().sv_latent_append(ctypes.byref(a), T, _f32(q),
+                                      _stream()), "latent_append")
+
+
+def head_linear(x, x_step: int, w, out, out_step: int,
+                gate: Optional[torch.Tensor] = None):
+    """out[t, h * out_step + n] = sum_k x[t, h * x_step + k] w[h, n, k], times
+    sigmoid(gate[t, h * N + n])."""
+    H, N, K = w.shape
+    T = x.shape[0]
+    assert w.is_contiguous() and x.stride(1) == out.stride(1) == 1
+    assert x.dtype == w.dtype == out.dtype and out.shape[0] == T
+    assert (H - 1) * x_step + K <= x.shape[1]
+    assert (H - 1) * out_step + N <= out.shape[1]
+    a = _HeadLinearArgs(x=_p(x), xst=x.stride(0), xh=x_step, w=_p(w),
+                        out=_p(out), ost=out.stride(0), oh=out_step,
+                        T=T, H=H, N=N, K=K)
+    mfma = x.dtype == torch.bfloat16 and K >= 8 and N >= 4 and N % 4 == 0 \
+        and _aligned((K, x_step, out_step), x, out)
+    if gate is not None:
+        assert gate.shape == (T, H * N) and gate.stride(1) == 1
+        assert gate.dtype == x.dtype
+        a.gate, a.gst, a.gh = _p(gate), gate.stride(0), N
+        mfma = mfma and _aligned((), gate)
+    _check(library().sv_head_linear(ctypes.byref(a), int(mfma), _f32(x),
+                                    _stream()), "head_linear")
+    return out
+
+
+def latent_rows_supported(dtype, rank: int, shared: int) -> bool:
+    return (dtype == torch.bfloat16 and rank % 8 == 0 and shared % 8 == 0
+            and rank <= 512 and shared <= 64)
+
+
+def latent_rows(q, cache, rank: int, pos, seq, block_table, heads: int,
+                scale: float, window: int = 0, max_keys: int = 0):
+    """Absorbed queries q (rows, H * (rank + P)) over the cached rows, which
+    hold the rows' own keys already -> (rows, H * rank) sums of latents."""
+    rows, D = q.shape[0], cache.shape[2]
+    assert q.is_contiguous() and q.shape[1] == heads * D
+    assert cache.is_contiguous() and cache.shape[1] == PAGE_SIZE
+    assert q.dtype == cache.dtype and pos.shape[0] == seq.shape[0] == rows
+    if D > MAX_LATENT_ROW:
+        raise ValueError(f"latent row of {D} > {MAX_LATENT_ROW}")
+    if window > 0:
+        max_keys = min(max_keys, window) if max_keys else window
+    out = torch.empty(rows, heads * rank, dtype=q.dtype, device=q.device)
+    fast = latent_rows_supported(q.dtype, rank, D - rank)
+    splits = _row_splits(512, rows * -(-heads // 32), max_keys, 64) if fast \
+        else _row_splits(1024, rows, max_keys, 128)
+    part = torch.empty(rows * heads * splits * (rank + 2),
+                       dtype=torch.float32, device=q.device) \
+        if splits > 1 else None
+    if fast:
+        a = _LatentRowsArgs(
+            q=_p(q), cache=_p(cache), pos=_p(pos), seq=_p(seq),
+            bt=_p(block_table), part=_p(part), out=_p(out),
+            MB=block_table.shape[1], rows=rows, H=heads, R=rank, P=D - rank,
+            splits=splits, window=window, scale=scale)
+        _check(library().sv_latent_rows(ctypes.byref(a), _stream()),
+               "latent_rows")
+        return out
+    # one key/value head whose value is the front of its key
+    a = _RowsArgs(q=_p(q), k=_p(q), v=_p(q), qst=q.stride(0),
+                  kst=q.stride(0), vst=q.stride(0), kc=_p(cache),
+                  vc=_p(cache), kcs=D, vcs=D, pos=_p(pos), seq=_p(seq),
+                  bt=_p(block_table), part=_p(part), out=_p(out),
+                  MB=block_table.shape[1], rows=rows, H=heads, G=1, D=D,
+                  E=rank, splits=splits, append=0, window=window, keep=0,
+                  scale=scale)
+    _check(library().sv_attn_rows(ctypes.byref(a),
+                                  int(_aligned((D, rank), q)), _f32(q),
+                                  _stream()), "attn_rows")
+    return out
+
+
+def latent_tiles_supported(q, gate, dim, vdim, rank, shared) -> bool:
+    return (q.dtype == torch.bfloat16 and dim + shared <= 256
+            and vdim <= 256
+            and _aligned((dim, vdim, rank, shared), q)
+            and (gate is None or _aligned((), gate)))
+
+
+def latent_portions(q, gate, cache, w: LatentWeights, batch,
+                    spans: KeySpans, heads: int, dim: int, vdim: int,
+                    scale: float, window: int, out):
+    """Prompt portions with rotated queries q (T, H * (dim + P)): gather the
+    visible rows, make all heads' keys and values with one product, attend."""
+    R = w.norm.shape[0]
+    P = cache.shape[2] - R
+    n = spans.pages.shape[0]
+    ws = torch.empty(n * PAGE_SIZE, R + P, dtype=q.dtype, device=q.device)
+    _check(library().sv_latent_gather(
+        ctypes.c_void_p(_p(cache)), ctypes.c_void_p(_p(ws)),
+        ctypes.c_void_p(_p(spans.pages)), n,
+        PAGE_SIZE * (R + P) * q.element_size(), _stream()), "latent_gather")
+    kv = torch.mm(ws[:, :R], w.expand.t())
+    assert q.shape[1] == heads * (dim + P) and q.stride(1) == 1
+    assert kv.shape[1] == heads * (dim + vdim) and kv.is_contiguous()
+    assert out.shape == (q.shape[0], heads * vdim) and out.is_contiguous()
+    row, size = kv.shape[1], q.element_size()
+    a = _TilesArgs(q=_p(q), qst=q.stride(0), kc=_p(kv),
+                   vc=_p(kv) + heads * dim * size, kr=_p(ws) + R * size,
+                   kpage=PAGE_SIZE * row, khead=dim, krow=row,
+                   vpage=PAGE_SIZE * row, vhead=vdim, vrow=row, rrow=R + P,
+                   tiles=_p(batch.tiles), bt=_p(spans.table), out=_p(out),
+                   MB=spans.table.shape[1], H=heads, G=heads, D=dim + P,
+                   E=vdim, DS=dim, window=window, keep=0, scale=scale)
+    if gate is not None:
+        assert gate.shape == out.shape and gate.stride(1) == 1
+        a.gate, a.gst = _p(gate), gate.stride(0)
+    _check(library().sv_attn_tiles(ctypes.byref(a), batch.tiles.shape[0],
+                                   _stream()), "attn_tiles")
+    return out
+
+
+def latent_attention(q, kv, gate, batch, cache, w: LatentWeights, heads: int,
+                     dim: int, vdim: int, scale: float, eps: float,
+                     window: int = 0) -> torch.Tensor:
+    """Latent attention of a packed batch.  q (T, H * (dim + P)) head by head
+    [unrotated | rotated], kv (T, rank + P), gate (T, H * vdim) or None ->
+    (T, H * vdim), times sigmoid(gate)."""
+    T, R = q.shape[0], w.norm.shape[0]
+    D = cache.shape[2]
+    P = D - R
+    out = torch.empty(T, heads * vdim, dtype=q.dtype, device=q.device)
+    n = batch.portion_tokens
+    spans = batch.spans.get(window)
+    if spans is None or not latent_tiles_supported(q, gate, dim, vdim, R, P):
+        n = 0
+    if n:
+        g = None if gate is None else gate[:n]
+        latent_append(q[:n], dim, dim + P, q[:n], dim, dim + P, kv[:n], w,
+                      cache, batch.pos[:n], batch.seq[:n], batch.block_table,
+                      heads, eps)
+        latent_portions(q[:n], g, cache, w, batch, spans, heads, dim, vdim,
+                        scale, window, out[:n])
+    if n < T:
+        at = (batch.pos[n:], batch.seq[n:], batch.block_table)
+        ql = torch.empty(T - n, heads * D, dtype=q.dtype, device=q.device)
+        latent_append(q[n:], dim, dim + P, ql, R, D, kv[n:], w, cache, *at,
+                      heads, eps)
+        head_linear(q[n:], dim + P, w.absorb, ql, D)
+        lat = latent_rows(ql, cache, R, *at, heads, scale, window,
+                          batch.max_keys)
+        head_linear(lat, R, w.expand[heads * dim:].view(heads, vdim, R),
+                    out[n:], vdim, None if gate is None else gate[n:])
+    return out
+
+
+# ---------------------------------------------------------------------------
+# mixture of experts
+# ---------------------------------------------------------------------------
+
+MOE_PLAIN, MOE_STREAM, MOE_TILES = 0, 1, 2
+MOE_TILE_ROWS = {MOE_PLAIN: 32, MOE_STREAM: 32, MOE_TILES: 128}
+MOE_STREAM_ROWS = 64        # rows an expert, up to which weights are streamed
+
+
+@dataclass
+class MoePlan:
+    coef: torch.Tensor         # (T, top) float32 weights of the chosen
+    idx: torch.Tensor          # (T, top) int32 chosen experts
+    order: torch.Tensor        # (T * top,) pairs, expert by expert
+    tiles: torch.Tensor        # (n, 4) expert, first slot, slots
+    how: int                   # kernel of the grouped products
+
+
+def moe_plan(z: torch.Tensor, bias: Optional[torch.Tensor], top: int,
+             how: int) -> MoePlan:
+    """Choose the ``top`` experts with the largest logits z + bias of every
+    row, their weights a softmax over the chosen, and group the pairs."""
+    T, E = z.shape
+    assert z.dtype == torch.float32 and z.is_contiguous() and z.is_cuda
+    if E > MAX_EXPERTS or not 1 <= top <= min(64, E):
+        raise ValueError(f"{top} of {E} experts")
+    pairs, rows = T * top, MOE_TILE_ROWS[how]
+    n = min(pairs, pairs // rows + E)
+    ints = torch.empty(2 * pairs + 4 * n, dtype=torch.int32, device=z.device)
+    p = MoePlan(torch.empty(T, top, dtype=torch.float32, device=z.device),
+                ints[4 * n:4 * n + pairs].view(T, top), ints[4 * n + pairs:],
+                ints[:4 * n].view(n, 4), how)
+    a = _MoePlanArgs(z=_p(z), bias=_p(bias), idx=_p(p.idx), coef=_p(p.coef),
+                     order=_p(p.order), tiles=_p(p.tiles), T=T, E=E, top=top,
+                     tile_rows=rows, max_tiles=n)
+    _check(library().sv_moe_plan(
+        ctypes.byref(a), 0 if bias is None else _f32(bias), _stream()),
+        "moe_plan")
+    return p
+
+
+def moe_gemm(x: torch.Tensor, w: torch.Tensor, plan: MoePlan, gated: bool,
+             alpha: float = 1.0, limit: float = float("inf"),
+             shift: float = 0.0) -> torch.Tensor:
+    """Grouped product over w (E, rows, K).  ``gated``: rows of x (T, K) ->
+    min(g, limit) sigmoid(alpha g) (clamp(u, limit) + shift) of w = [gate;
+    up], in slot order.  Else: slots x (T * top, K) -> pairs."""
+    pairs = plan.order.shape[0]
+    N, K = w.shape[1] // (2 if gated else 1), w.shape[2]
+    assert x.stride(1) == 1 and x.shape[1] == K and w.is_contiguous()
+    assert x.dtype == w.dtype and w.shape[1] == N * (2 if gated else 1)
+    assert x.shape[0] == (plan.coef.shape[0] if gated else pairs)
+    out = torch.empty(pairs, N, dtype=x.dtype, device=x.device)
+    a = _MoeGemmArgs(x=_p(x), xst=x.stride(0), w=_p(w), out=_p(out),
+                     order=_p(plan.order), tiles=_p(plan.tiles),
+                     top=plan.coef.shape[1] if gated else 0, N=N, K=K,
+                     max_tiles=plan.tiles.shape[0], alpha=alpha, limit=limit,
+                     shift=shift)
+    assert plan.how == MOE_PLAIN or (x.dtype == torch.bfloat16
+                                     and _aligned((N, K), x))
+    _check(library().sv_moe_gemm(ctypes.byref(a), plan.how, int(gated),
+                                 _f32(x), _stream()), "moe_gemm")
+    return out
+
+
+def moe_mlp(h, z, bias, gate_up, down, top: int, alpha: float, limit: float,
+            shift: float) -> Pending:
+    """Gated experts on h (T, W) with router logits z (T, E): a pending sum
+    of the chosen experts' outputs."""
+    E, W, ff = down.shape
+    pairs = h.shape[0] * top
+    if h.dtype != torch.bfloat16 or not _aligned((W, ff), h):
+        how = MOE_PLAIN
+    else:
+        how = MOE_STREAM if pairs <= MOE_STREAM_ROWS * E else MOE_TILES
+    plan = moe_plan(z, bias, top, how)
+    act = moe_gemm(h, gate_up, plan, True, alpha, limit, shift)
+    return Pending(moe_gemm(act, down, plan, False), coef=plan.coef)
