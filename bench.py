@@ -37,8 +37,12 @@ def parse_args():
     p.add_argument("--microbatch", type=int, default=8)
     p.add_argument("--serving", nargs="?", const="all", default=None,
                    choices=("all", "kernels", "models"),
-                   help="instead: the serving benchmark of the Voletar "
-                        "design beside Llama (bench_serving.py, 1 GPU)")
+                   help="instead: the serving benchmark of a design beside "
+                        "its closest relative (bench_serving.py, 1 GPU)")
+    p.add_argument("--design", default="all",
+                   choices=("all", "voletar", "nesilorn"),
+                   help="with --serving: Voletar beside Llama, Nesilorn "
+                        "beside Mixtral, or both")
     return p.parse_args()
 
 
@@ -47,7 +51,7 @@ def main():
     if args.serving:
         import bench_serving
 
-        return bench_serving.main(args.serving)
+        return bench_serving.main(args.serving, args.design)
     rank = int(os.environ.get("RANK", "0"))
     world = int(os.environ.get("WORLD_SIZE", str(args.gpus)))
     local_rank = int(os.environ.get("LOCAL_RANK", str(rank)))

@@ -1,14 +1,16 @@
 #!/usr/bin/env python3
-"""Serving benchmark of the Voletar design beside Llama at equal layer sizes
-(random weights, one MI355X):
+"""Serving benchmark of a design beside its closest relative at equal layer
+sizes (random weights, one MI355X): Voletar beside Llama, Nesilorn beside
+Mixtral.
 
-    python bench.py --serving            kernels and whole models
-    python bench.py --serving kernels    (or: models)
+    python bench.py --serving                          all of it
+    python bench.py --serving kernels                  (or: models)
+    python bench.py --serving kernels --design nesilorn
 
 Kernels: time, roofline time (the larger of MFMA flops at 2.5 PFLOP/s and
 bytes at 8 TB/s) and how far from it, for each serving kernel and the like
-kernel that Llama runs.  Models: prefill and decode tokens/s.  Both sides are
-timed in turn in one process; one JSON line per result.
+kernel that the relative runs.  Models: prefill and decode tokens/s.  Both
+sides are timed in turn in one process; one JSON line per result.
 """
 
 import json
@@ -299,15 +301,340 @@ def bench_models(layers=None):
         torch.cuda.empty_cache()
 
 
-def main(what="all"):
+# ---------------------------------------------------------------------------
+# Nesilorn beside Mixtral
+# ---------------------------------------------------------------------------
+
+def _kernel_us(f, name, reps=10):
+    """Device microseconds a call of f spends in kernels called ``name``: for
+    calls that read the device from the host and cannot be captured."""
+    from torch.profiler import ProfilerActivity, profile
+
+    f()
+    torch.cuda.synchronize()
+    with profile(activities=[ProfilerActivity.CUDA,
+                             ProfilerActivity.CPU]) as prof:
+        for _ in range(reps):
+            f()
+        torch.cuda.synchronize()
+    return sum(e.self_device_time_total for e in prof.key_averages()
+               if name in e.key) / reps
+
+
+def _latent_case(sv, B, T, ctx, H, D, P, E, R):
+    """A packed step of B requests with T new tokens each at context ctx."""
+    from types import SimpleNamespace
+
+    n = -(-(ctx + T) // 64)
+    bt = torch.randperm(B * n).int().view(B, n)
+    b = SimpleNamespace(
+        block_table=bt.cuda(), max_keys=ctx + T,
+        pos=_i32(list(range(ctx, ctx + T)) * B),
+        seq=_i32([r for r in range(B) for _ in range(T)]),
+        portion_tokens=B * T if T > 1 else 0, spans={})
+    if T > 1:
+        b.tiles = _i32([(r, r * T + s, 128, ctx + s) for r in range(B)
+                        for s in range(0, T, 128)])
+    w = sv.LatentWeights(
+        _bf(R), (torch.randn(H, R, D, device="cuda") * R ** -0.5).bfloat16(),
+        (torch.randn(H * (D + E), R, device="cuda") * R ** -0.5).bfloat16(),
+        sv.rotary_frequencies(1e4, P, "cuda"))
+    cache = _bf(B * n, 64, R + P)
+    sizes = (H * (D + P), R + P, H * E)
+    p = _bf(B * T, sum(sizes))
+    q, kv, g = p.split(sizes, 1)
+    return b, w, cache, q, kv, g
+
+
+def bench_latent_kernels():
+    from neuronx_distributed_amd import ops
+    from neuronx_distributed_amd.ops import serving as sv
+
+    dev = dict(device="cuda")
+    H, D, P, E, R, G, LD = 32, 128, 64, 128, 512, 8, 128
+    scale = (D + P) ** -0.5
+    # -- prompts -------------------------------------------------------------
+    for T, W in ((4096, 4096), (8192, 4096), (8192, 1024)):
+        b, w, cache, q, kv, g = _latent_case(sv, 1, T, 0, H, D, P, E, R)
+        pages, table = sv.key_spans([(0, 0, T, 0)], b.block_table.tolist(), W)
+        b.spans = {W: sv.KeySpans(_i32(pages), _i32(table))}
+        out = torch.empty(T, H * E, dtype=torch.bfloat16, **dev)
+        fq, fk, fv = (_bf(1, h, T, LD) for h in (H, G, G))
+        win = W if W < T else 0
+        kve = _bf(T, H * (D + E))
+        ws = _bf(T, R + P)
+        us, tus, lus = _time([
+            _graphed(lambda: sv.latent_attention(
+                q, kv, g, b, cache, w, H, D, E, scale, 1e-5, W)),
+            _graphed(lambda: sv.expanded_attention(
+                q, g, kve, ws, b.tiles, b.spans[W], H, D, E, scale, W, out)),
+            _graphed(lambda: ops.flash_attn(fq, fk, fv, True, None, win))])
+        pairs = sum(min(i + 1, W) for i in range(T))
+        lio = 2 * T * (2 * H + 2 * G) * LD
+        like = ("flash_attn", lus, 4 * pairs * H * LD, lio)
+        fl = 2 * pairs * H * (D + P + E)
+        io = 2 * T * (H * (D + P + 2 * E) + R + P)
+        _report("latent_attention (append, gather, expand, tiles)", us,
+                fl + 2 * T * R * H * (D + E), io, like, tokens=T, window=W)
+        _report("attn_tiles on expanded keys", tus, fl,
+                io + 2 * T * H * (D + E), like, tokens=T, window=W)
+    # -- single tokens ---------------------------------------------------------
+    for B, ctx in ((1, 4096), (32, 1024), (32, 4096), (128, 4096)):
+        b, w, cache, q, kv, g = _latent_case(sv, B, 1, ctx, H, D, P, E, R)
+        ql = _bf(B, H * (R + P))
+        Smax = ctx + 64
+        lq, lk, lv = _bf(B, H * LD), _bf(B, G * LD), _bf(B, G * LD)
+        kc = torch.zeros(B, G, Smax, LD, dtype=torch.bfloat16, **dev)
+        vc = torch.zeros_like(kc)
+        cos = torch.ones(Smax, LD // 2, **dev)
+        pt = torch.tensor([ctx], dtype=torch.int64, **dev)
+        lat = _bf(B, H * R)
+        out = _bf(B, H * E)
+        wv = w.expand[H * D:].view(H, E, R)
+        wl = _bf(E * H, R)
+        t = _time([
+            _graphed(lambda: sv.latent_attention(
+                q, kv, g, b, cache, w, H, D, E, scale, 1e-5, 4096)),
+            _graphed(lambda: sv.latent_rows(
+                ql, cache, R, b.pos, b.seq, b.block_table, H, scale, 4096,
+                ctx + 1)),
+            _graphed(lambda: ops.decode_attn_step(
+                lq, lk, lv, kc, vc, cos, cos, pt, H, G, LD ** -0.5)),
+            _graphed(lambda: sv.head_linear(q, D + P, w.absorb, ql, R + P)),
+            _graphed(lambda: sv.head_linear(lat, R, wv, out, E, g)),
+            _graphed(lambda: torch.mm(lat[:, :R], wl.t())),
+            _graphed(lambda: sv.latent_append(
+                q, D, D + P, ql, R, R + P, kv, w, cache, b.pos, b.seq,
+                b.block_table, H, 1e-5))])
+        lb = 4 * B * G * (ctx + 1) * LD + 4 * B * H * LD
+        like = ("decode_attn_step", t[2], 4 * B * H * (ctx + 1) * LD, lb)
+        cb = 2 * B * min(ctx + 1, 4096) * (R + P)
+        fl = 2 * B * H * min(ctx + 1, 4096) * (2 * R + P)
+        wb = 2 * H * (D + E) * R
+        _report("latent_attention (append, absorb, rows, values)", t[0],
+                fl + 2 * B * H * R * (D + E),
+                cb + wb + 2 * B * H * (D + P + 2 * E), like, batch=B,
+                context=ctx)
+        _report("latent_rows", t[1], fl, cb + 2 * B * H * (2 * R + P), like,
+                batch=B, context=ctx)
+        mm = ("mm of the same weights", t[5], 2 * B * H * E * R,
+              2 * H * E * R + 2 * B * (R + H * E))
+        _report("head_linear (absorb)", t[3], 2 * B * H * D * R,
+                2 * H * D * R + 2 * B * H * (D + R), mm, batch=B)
+        _report("head_linear (values, gate)", t[4], 2 * B * H * E * R,
+                2 * H * E * R + 2 * B * H * (2 * E + R), mm, batch=B)
+        _report("latent_append", t[6], 0, 4 * B * (H * P + R + P), batch=B)
+    # -- experts ---------------------------------------------------------------
+    for (Wd, ff, n, top) in ((4096, 14336, 8, 2), (2048, 1408, 64, 6)):
+        gu, down = (torch.randn(n, a, c, device="cuda",
+                                dtype=torch.bfloat16) * c ** -0.5
+                    for a, c in ((2 * ff, Wd), (Wd, ff)))
+        bias = _bf(n)
+        lgu = gu.transpose(1, 2).contiguous()
+        ldn = down.transpose(1, 2).contiguous()
+        for T in (1, 32, 128, 512, 4096, 16384):
+            x, z = _bf(T, Wd), torch.randn(T, n, **dev)
+            how = sv.MOE_STREAM if T * top <= sv.MOE_STREAM_ROWS * n \
+                else sv.MOE_TILES
+            plan = sv.moe_plan(z, bias, top, how)
+            act = sv.moe_gemm(x, gu, plan, True, 1.702, 7.0, 1.0)
+            hit = int(plan.idx.unique().numel())
+            idx = plan.idx.long()
+            fns = [_graphed(lambda: sv.moe_mlp(x, z, bias, gu, down, top,
+                                               1.702, 7.0, 1.0)),
+                   _graphed(lambda: sv.moe_plan(z, bias, top, how)),
+                   _graphed(lambda: sv.moe_gemm(x, gu, plan, True, 1.702,
+                                                7.0, 1.0)),
+                   _graphed(lambda: sv.moe_gemm(act, down, plan, False))]
+            if T <= 512:
+                aff = torch.zeros(T, n, **dev).scatter_(1, idx, 0.5)
+                t = _time(fns)
+                lus = _kernel_us(lambda: ops.moe_decode_glu(
+                    x, lgu, ldn, aff, idx), "moe_")
+                name = "moe_decode_glu, its kernels"
+            else:
+                rows = plan.order.long() // top
+                xs = x[rows].contiguous()
+                offs = torch.bincount(idx.flatten(), minlength=n).cumsum(
+                    0).int()
+
+                def grouped():
+                    a = ops.swiglu(torch._grouped_mm(xs, lgu, offs=offs))
+                    return torch._grouped_mm(a, ldn, offs=offs)
+                try:
+                    t = _time(fns + [grouped])
+                    lus = t[4]
+                except RuntimeError as e:
+                    print(json.dumps({"skipped": "_grouped_mm",
+                                      "why": str(e)[:100]}), flush=True)
+                    t, lus = _time(fns), None
+                name = "grouped_mm, swiglu, grouped_mm"
+            fl = 6 * T * top * Wd * ff
+            io = 6 * hit * Wd * ff + 2 * T * Wd * (1 + top)
+            kw = dict(tokens=T, width=Wd, ff=ff, experts=n, top=top)
+            _report("moe_mlp (plan, gate/up, down)", t[0], fl, io,
+                    lus and (name, lus, fl, io), **kw)
+            _report("moe_gemm (gate/up)", t[2], fl * 2 / 3,
+                    4 * hit * Wd * ff + 2 * T * (Wd + top * ff), **kw)
+            _report("moe_gemm (down)", t[3], fl / 3,
+                    2 * hit * Wd * ff + 2 * T * top * (Wd + ff), **kw)
+            _report("moe_plan", t[1], 0, 4 * T * n + 12 * T * top, **kw)
+        del gu, down, lgu, ldn
+        torch.cuda.empty_cache()
+    # -- norms and pointwise -----------------------------------------------------
+    for T in (32, 4096):
+        Wd, F, top = 4096, 14336, 2
+        x, xb, d = torch.randn(T, Wd, **dev), _bf(T, Wd), _bf(T, Wd)
+        d2, coef, w = _bf(T * top, Wd), torch.rand(T, top, **dev), _bf(Wd)
+        u, gu = _bf(T, F), _bf(T, 2 * F)
+        kw = dict(w1=w, centred=True)
+        t = _time([
+            _graphed(lambda: sv.residual_norm(
+                x, sv.Pending(d, **kw), 1e-6, copy=True,
+                dtype=torch.bfloat16)),
+            _graphed(lambda: sv.residual_norm(
+                x, sv.Pending(d2, coef=coef, **kw), 1e-6, copy=True,
+                dtype=torch.bfloat16)),
+            _graphed(lambda: ops.add_rmsnorm(xb, d, w, 1e-6)),
+            _graphed(lambda: sv.gelu_tanh_(u)),
+            _graphed(lambda: ops.swiglu(gu))])
+        n = T * Wd
+        like = ("add_rmsnorm", t[2], 0, 8 * n)
+        _report("residual_norm (output norm)", t[0], 0, 12 * n, like, rows=T)
+        _report("residual_norm (experts' sum, output norm)", t[1], 0,
+                (10 + 2 * top) * n, like, rows=T)
+        _report("gelu_tanh", t[3], 0, 4 * T * F,
+                ("swiglu", t[4], 0, 6 * T * F), rows=T)
+
+
+def bench_latent_models():
+    import os
+
+    from neuronx_distributed_amd.inference import (InferenceEngine, StepEntry,
+                                                   single_process_groups)
+    from neuronx_distributed_amd.inference.kv_cache import build_kv_caches
+    from neuronx_distributed_amd.models import (build_model,
+                                                get_nesilorn_config)
+    from neuronx_distributed_amd.models.mixtral import (MixtralForCausalLM,
+                                                        get_moe_config)
+
+    single_process_groups()
+    torch.manual_seed(0)
+    cfg = get_nesilorn_config("nesilorn-bench")
+    n = len(cfg.layers)
+    nes = build_model("Nesilorn", cfg, torch.bfloat16, "cuda")
+    mcfg = get_moe_config("mixtral-8x7b", num_hidden_layers=n,
+                          max_position_embeddings=16384, capacity_factor=0.0)
+    os.environ["NXDA_FAST_INIT"] = "1"
+    torch.set_default_dtype(torch.bfloat16)
+    try:
+        with torch.device("cuda"):
+            mix = MixtralForCausalLM(mcfg).eval()
+    finally:
+        torch.set_default_dtype(torch.float32)
+        del os.environ["NXDA_FAST_INIT"]
+    size = lambda m: sum(p.numel() for p in m.parameters()) / 1e9
+    print(json.dumps({"nesilorn_b_params": round(size(nes), 2),
+                      "mixtral_b_params": round(size(mix), 2),
+                      "layers": n, "data": "random weights"}), flush=True)
+
+    def caches_for(B, T):
+        return build_kv_caches(n, B, mcfg.num_key_value_heads, T,
+                               mcfg.head_dim, device=torch.device("cuda"))
+
+    # logits of the last token on both sides
+    for B, T in ((1, 2048), (1, 4096), (4, 4096)):
+        toks = torch.randint(0, 32000, (B, T))
+        x, rows = toks.cuda(), toks.tolist()
+        eng = InferenceEngine(nes, max_tokens=B * T, max_seqs=B)
+        caches = caches_for(B, T)
+
+        def run_n():
+            eng.step([StepEntry(b, rows[b], [T - 1]) for b in range(B)])
+            for b in range(B):
+                eng.finish(b)
+
+        def run_m():
+            with torch.no_grad():
+                h, _ = mix.model(x, 0, caches)
+                mix.lm_head(h[:, -1])
+
+        best = [math.inf, math.inf]
+        for _ in range(4):
+            for i, f in enumerate((run_n, run_m)):
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                f()
+                torch.cuda.synchronize()
+                best[i] = min(best[i], time.perf_counter() - t0)
+        print(json.dumps({
+            "prefill": {"batch": B, "tokens": T},
+            "nesilorn_tokens_per_s": round(B * T / best[0]),
+            "mixtral_tokens_per_s": round(B * T / best[1])}), flush=True)
+        del eng, caches
+        torch.cuda.empty_cache()
+
+    # decode with greedy feedback: the engine replays a graph; Mixtral runs
+    # step by step, since its routing reads counts on the host
+    for B, ctx in ((1, 2048), (32, 2048), (128, 2048)):
+        steps = 8
+        rows = torch.randint(0, 32000, (B, ctx)).tolist()
+        eng = InferenceEngine(nes, max_tokens=B * (ctx + 64), max_seqs=B,
+                              max_context=ctx + 64)
+        for b in range(B):
+            eng.step([StepEntry(b, rows[b])])
+        tok = [1] * B
+
+        def step_n(tok):
+            lg = eng.step([StepEntry(b, [tok[b]], [0]) for b in range(B)])
+            return lg.argmax(-1).tolist()
+
+        caches = caches_for(B, ctx + 64)
+        tl, at = torch.ones(B, 1, dtype=torch.long, device="cuda"), ctx
+        tok = step_n(tok)
+        best = [math.inf, math.inf]
+        for _ in range(3):
+            for side in (0, 1):
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                for _ in range(steps):
+                    if side == 0:
+                        tok = step_n(tok)
+                    else:
+                        with torch.no_grad():
+                            lg = mix(tl, pos_offset=torch.tensor(
+                                [at], device="cuda"), kv_caches=caches)
+                        tl = lg[:, -1].argmax(-1, keepdim=True)
+                        tl.tolist()
+                        at += 1
+                torch.cuda.synchronize()
+                best[side] = min(best[side],
+                                 (time.perf_counter() - t0) / steps)
+        print(json.dumps({
+            "decode": {"batch": B, "context": ctx},
+            "nesilorn_ms": round(best[0] * 1e3, 3),
+            "mixtral_ms": round(best[1] * 1e3, 3),
+            "nesilorn_tokens_per_s": round(B / best[0]),
+            "mixtral_tokens_per_s": round(B / best[1])}), flush=True)
+        del eng, caches
+        torch.cuda.empty_cache()
+
+
+DESIGNS = {"voletar": (bench_kernels, bench_models),
+           "nesilorn": (bench_latent_kernels, bench_latent_models)}
+
+
+def main(what="all", design="all"):
     torch.cuda.set_device(0)
-    if what in ("all", "kernels"):
-        bench_kernels()
-    if what in ("all", "models"):
-        bench_models()
+    for name, (kernels, models) in DESIGNS.items():
+        if design in ("all", name):
+            if what in ("all", "kernels"):
+                kernels()
+            if what in ("all", "models"):
+                models()
 
 
 if __name__ == "__main__":
     import sys
 
-    main(*sys.argv[1:2])
+    main(*sys.argv[1:3])

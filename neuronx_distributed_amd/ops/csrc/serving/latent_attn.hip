@@ -200,8 +200,8 @@ head_linear_mfma_kernel(HeadLinearArgs a) {
 template <typename T>
 __global__ void __launch_bounds__(256)
 head_linear_kernel(HeadLinearArgs a) {
-  const int n = blockIdx.x * 256 + threadIdx.x, h = blockIdx.y;
-  const long t = blockIdx.z;
+  const int n = blockIdx.y * 256 + threadIdx.x, h = blockIdx.z;
+  const long t = blockIdx.x;
   if (n >= a.N) return;
   const T* x = (const T*)a.x + t * a.xst + h * a.xh;
   const T* w = (const T*)a.w + ((long)h * a.N + n) * a.K;
@@ -222,7 +222,7 @@ extern "C" int sv_head_linear(const HeadLinearArgs* a, int mfma, int f32,
       head_linear_mfma_kernel<false><<<dim3((nt + 3) / 4, a->H, tt), 256, 0,
                                        stream>>>(*a);
   } else {
-    const dim3 grid((a->N + 255) / 256, a->H, a->T);
+    const dim3 grid(a->T, (a->N + 255) / 256, a->H);
     if (f32) head_linear_kernel<float><<<grid, 256, 0, stream>>>(*a);
     else head_linear_kernel<short><<<grid, 256, 0, stream>>>(*a);
   }

@@ -703,21 +703,33 @@ def latent_portions(q, gate, cache, w: LatentWeights, batch,
         ctypes.c_void_p(_p(spans.pages)), n,
         PAGE_SIZE * (R + P) * q.element_size(), _stream()), "latent_gather")
     kv = torch.mm(ws[:, :R], w.expand.t())
+    return expanded_attention(q, gate, kv, ws, batch.tiles, spans, heads,
+                              dim, vdim, scale, window, out)
+
+
+def expanded_attention(q, gate, kv, ws, tiles, spans: KeySpans, heads: int,
+                       dim: int, vdim: int, scale: float, window: int, out):
+    """Query tiles over keys and values kv (rows, H * dim + H * vdim) of the
+    workspace rows ws (rows, rank + P), whose last columns end every key."""
+    P = q.shape[1] // heads - dim
+    R = ws.shape[1] - P
     assert q.shape[1] == heads * (dim + P) and q.stride(1) == 1
-    assert kv.shape[1] == heads * (dim + vdim) and kv.is_contiguous()
+    assert kv.shape == (spans.pages.shape[0] * PAGE_SIZE,
+                        heads * (dim + vdim)) and kv.is_contiguous()
+    assert ws.shape[0] == kv.shape[0] and ws.is_contiguous()
     assert out.shape == (q.shape[0], heads * vdim) and out.is_contiguous()
     row, size = kv.shape[1], q.element_size()
     a = _TilesArgs(q=_p(q), qst=q.stride(0), kc=_p(kv),
                    vc=_p(kv) + heads * dim * size, kr=_p(ws) + R * size,
                    kpage=PAGE_SIZE * row, khead=dim, krow=row,
                    vpage=PAGE_SIZE * row, vhead=vdim, vrow=row, rrow=R + P,
-                   tiles=_p(batch.tiles), bt=_p(spans.table), out=_p(out),
+                   tiles=_p(tiles), bt=_p(spans.table), out=_p(out),
                    MB=spans.table.shape[1], H=heads, G=heads, D=dim + P,
                    E=vdim, DS=dim, window=window, keep=0, scale=scale)
     if gate is not None:
         assert gate.shape == out.shape and gate.stride(1) == 1
         a.gate, a.gst = _p(gate), gate.stride(0)
-    _check(library().sv_attn_tiles(ctypes.byref(a), batch.tiles.shape[0],
+    _check(library().sv_attn_tiles(ctypes.byref(a), tiles.shape[0],
                                    _stream()), "attn_tiles")
     return out
 
