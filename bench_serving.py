@@ -434,8 +434,7 @@ def bench_latent_kernels():
         ldn = down.transpose(1, 2).contiguous()
         for T in (1, 32, 128, 512, 4096, 16384):
             x, z = _bf(T, Wd), torch.randn(T, n, **dev)
-            how = sv.MOE_STREAM if T * top <= sv.MOE_STREAM_ROWS * n \
-                else sv.MOE_TILES
+            how = sv.moe_kernel(T * top, n)
             plan = sv.moe_plan(z, bias, top, how)
             act = sv.moe_gemm(x, gu, plan, True, 1.702, 7.0, 1.0)
             hit = int(plan.idx.unique().numel())

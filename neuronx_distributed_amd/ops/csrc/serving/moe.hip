@@ -169,12 +169,16 @@ __device__ __forceinline__ float glu(const MoeGemmArgs& a, float g, float u) {
   return g * sigmoid_f(a.alpha * g) * (u + a.shift);
 }
 
-// -- many rows per expert: MFMA tiles ---------------------------------------
+// -- MFMA tiles ---------------------------------------
 // BM slots x BN weight rows, K in steps of 64 through two LDS buffers; the
-// next step's words travel in registers while this one is multiplied.  With
-// a gated activation the weight rows of a tile alternate 32 gate, 32 up, so a
-// lane holds both of a column.
-template <int BM, int BN, int WM, int WN, bool GLU>
+// next step's words travel while this one is multiplied: straight into LDS
+// (DMA, K a multiple of 64) or through registers.  With a gated activation
+// the weight rows of a tile alternate 32 gate, 32 up, so a lane holds both of
+// a column.
+typedef __attribute__((address_space(1))) const void* global_ptr;
+typedef __attribute__((address_space(3))) void* lds_ptr;
+
+template <int BM, int BN, int WM, int WN, bool GLU, bool DMA>
 __global__ void __launch_bounds__(BM / WM * BN / WN * 64)
 moe_tiles_kernel(MoeGemmArgs a) {
   constexpr int NT = BM / WM * BN / WN * 64;
@@ -182,8 +186,10 @@ moe_tiles_kernel(MoeGemmArgs a) {
   constexpr int LX = BM * 8 / NT, LW = BN * 8 / NT;
   constexpr int GROUP = 8;
   constexpr int NOUT = GLU ? BN / 2 : BN;    // columns of a tile's result
-  __shared__ __attribute__((aligned(16))) short xs[2][BM * 64];
-  __shared__ __attribute__((aligned(16))) short ws[2][BN * 64];
+  // apart by name, so that a read of one buffer need not wait for the words
+  // on their way into the other
+  __shared__ __attribute__((aligned(16))) short xs0[BM * 64], xs1[BM * 64];
+  __shared__ __attribute__((aligned(16))) short ws0[BN * 64], ws1[BN * 64];
 
   // neighbours in the list of tiles run on one XCD: groups of GROUP slot
   // tiles by all column tiles, slot tiles fastest
@@ -207,8 +213,10 @@ moe_tiles_kernel(MoeGemmArgs a) {
   const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int col = lane & 31, hi = lane >> 5;
   const int wm = wid % (BM / WM) * WM, wn = wid / (BM / WM) * WN;
-  const int K = a.K, N = a.N, kc = tid % 8 * 8;
-  const int NW = GLU ? 2 * N : N;
+  const int K = a.K, N = a.N;
+  // 16-byte slot (r, s) of a tile lies at place s ^ (r >> 1); thread tid
+  // fills places tid, tid + NT, ... of a buffer, NT / 8 rows apart
+  const int kc = ((tid ^ (tid >> 4)) & 7) * 8;
 
   const short* px[LX];
   const short* pw[LW];
@@ -224,11 +232,25 @@ moe_tiles_kernel(MoeGemmArgs a) {
     int n = GLU ? tn * NOUT + (r >> 6) * 32 + (r & 31) : tn * NOUT + r;
     n = min(n, N - 1);
     if (GLU && (r & 32)) n += N;
-    pw[i] = (const short*)a.w + ((long)e * NW + n) * K + kc;
+    pw[i] = (const short*)a.w + ((long)e * (GLU ? 2 * N : N) + n) * K + kc;
   }
 
   uint4v rx[LX], rw[LW];
-  auto issue = [&](int k0) {
+  auto issue = [&](int k0, short* xs, short* ws) {
+    if (DMA) {
+      // a wave's 64 places follow each other
+#pragma unroll
+      for (int i = 0; i < LX; ++i)
+        __builtin_amdgcn_global_load_lds(
+            (global_ptr)(px[i] + k0), (lds_ptr)(xs + (i * NT + wid * 64) * 8),
+            16, 0, 0);
+#pragma unroll
+      for (int i = 0; i < LW; ++i)
+        __builtin_amdgcn_global_load_lds(
+            (global_ptr)(pw[i] + k0), (lds_ptr)(ws + (i * NT + wid * 64) * 8),
+            16, 0, 0);
+      return;
+    }
     const bool in_k = k0 + kc < K;
     const uint4v zero = {0, 0, 0, 0};
 #pragma unroll
@@ -236,42 +258,62 @@ moe_tiles_kernel(MoeGemmArgs a) {
 #pragma unroll
     for (int i = 0; i < LW; ++i) rw[i] = in_k ? *(const uint4v*)(pw[i] + k0) : zero;
   };
-  auto at = [](int r, int slot) { return r * 64 + ((slot ^ (r >> 1)) & 7) * 8; };
-  auto commit = [&](int b) {
+  auto commit = [&](short* xs, short* ws) {
+    if (DMA) return;
 #pragma unroll
-    for (int i = 0; i < LX; ++i)
-      *(uint4v*)(xs[b] + at((i * NT + tid) / 8, tid % 8)) = rx[i];
+    for (int i = 0; i < LX; ++i) *(uint4v*)(xs + (i * NT + tid) * 8) = rx[i];
 #pragma unroll
-    for (int i = 0; i < LW; ++i)
-      *(uint4v*)(ws[b] + at((i * NT + tid) / 8, tid % 8)) = rw[i];
+    for (int i = 0; i < LW; ++i) *(uint4v*)(ws + (i * NT + tid) * 8) = rw[i];
   };
 
+  // A step has four chunks of 16 columns.  The fragments of a chunk are read
+  // while the one before is multiplied; the last chunk of a step is
+  // multiplied after the barrier, while the next step's first is read.
   f32x16 acc[CN][CM] = {};
-  issue(0);
-  commit(0);
-  __syncthreads();
-  int b = 0;
-  for (int k0 = 0; k0 < K; k0 += 64, b ^= 1) {
-    const bool more = k0 + 64 < K;
-    if (more) issue(k0 + 64);
+  frag_u fx[2][CM] = {}, fw[2][CN] = {};
+  auto multiply = [&](int c) {
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
-      frag_u fx[CM], fw[CN];
+    for (int n = 0; n < CN; ++n)
 #pragma unroll
       for (int m = 0; m < CM; ++m)
-        fx[m].u4 = *(const uint4v*)(xs[b] + at(wm + 32 * m + col, 2 * c + hi));
+        acc[n][m] = mfma_bf16(fw[c & 1][n].bf, fx[c & 1][m].bf, acc[n][m]);
+  };
+  auto step = [&](const short* xs, const short* ws) {
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      // row 32 m + col, slot 2 c + hi
+      const int at = col * 64 + (((2 * c + hi) ^ (col >> 1)) & 7) * 8;
+#pragma unroll
+      for (int m = 0; m < CM; ++m)
+        fx[c & 1][m].u4 = *(const uint4v*)(xs + wm * 64 + at + m * 2048);
 #pragma unroll
       for (int n = 0; n < CN; ++n)
-        fw[n].u4 = *(const uint4v*)(ws[b] + at(wn + 32 * n + col, 2 * c + hi));
-#pragma unroll
-      for (int n = 0; n < CN; ++n)
-#pragma unroll
-        for (int m = 0; m < CM; ++m)
-          acc[n][m] = mfma_bf16(fw[n].bf, fx[m].bf, acc[n][m]);
+        fw[c & 1][n].u4 = *(const uint4v*)(ws + wn * 64 + at + n * 2048);
+      multiply(c - 1);             // of the step before, if c is 0
+      // two products, the reads, the other products
+      __builtin_amdgcn_sched_group_barrier(0x8, CM * CN < 2 ? 1 : 2, 0);
+      __builtin_amdgcn_sched_group_barrier(0x100, CM + CN, 0);
+      if (CM * CN > 2) __builtin_amdgcn_sched_group_barrier(0x8, CM * CN - 2, 0);
     }
-    if (more) commit(b ^ 1);
+    __builtin_amdgcn_sched_barrier(0);
+  };
+  const int steps = (K + 63) / 64;
+  issue(0, xs0, ws0);
+  commit(xs0, ws0);
+  __syncthreads();                 // also waits for the words on their way
+  for (int i = 0; i + 1 < steps; i += 2) {
+    issue(i * 64 + 64, xs1, ws1);
+    step(xs0, ws0);
+    commit(xs1, ws1);
+    __syncthreads();
+    issue(min(i + 2, steps - 1) * 64, xs0, ws0);   // the last one is not read
+    step(xs1, ws1);
+    commit(xs0, ws0);
     __syncthreads();
   }
+  if (steps & 1) step(xs0, ws0);
+  multiply(3);
 
 #pragma unroll
   for (int m = 0; m < CM; ++m) {
@@ -298,7 +340,7 @@ moe_tiles_kernel(MoeGemmArgs a) {
   }
 }
 
-// -- few rows per expert: stream the weights --------------------------------
+// -- a few rows per expert: stream the weights --------------------------------
 // One workgroup = 32 weight rows (16 gate and their 16 up rows) by up to 32
 // slots; its four waves take every fourth 64-column block of K and meet in
 // LDS.  Weights go straight from memory to registers, once per tile.
@@ -415,19 +457,31 @@ __global__ void __launch_bounds__(256) moe_plain_kernel(MoeGemmArgs a) {
 template <int BM, int BN, int WM, int WN, bool GLU>
 static void launch_tiles(const MoeGemmArgs& a, hipStream_t stream) {
   constexpr int NOUT = GLU ? BN / 2 : BN;
+  constexpr int NT = BM / WM * BN / WN * 64;
   const long grid = (long)a.max_tiles * ((a.N + NOUT - 1) / NOUT);
-  moe_tiles_kernel<BM, BN, WM, WN, GLU>
-      <<<grid, BM / WM * BN / WN * 64, 0, stream>>>(a);
+  if (a.K % 64 == 0)
+    moe_tiles_kernel<BM, BN, WM, WN, GLU, true><<<grid, NT, 0, stream>>>(a);
+  else
+    moe_tiles_kernel<BM, BN, WM, WN, GLU, false><<<grid, NT, 0, stream>>>(a);
 }
 
-// how: 0 any size and type, 1 stream, 2 tiles (1 and 2: bf16, N, K, xst and
-// bases in 8 elements).  The plan's tile_rows: 32, 32, 128.
+// how: 0 any size and type, 1 stream, 2 to 5 tiles (1 to 5: bf16, N, K, xst
+// and bases in 8 elements).  The plan's tile_rows: 32, 32, 32, 64, 128, 256.
 extern "C" int sv_moe_gemm(const MoeGemmArgs* a, int how, int gated, int f32,
                            hipStream_t stream) {
   if (a->max_tiles <= 0) return 0;
-  if (how == 2) {
+  if (how == 5) {
+    if (gated) launch_tiles<256, 256, 128, 64, true>(*a, stream);
+    else launch_tiles<256, 256, 128, 64, false>(*a, stream);
+  } else if (how == 4) {
     if (gated) launch_tiles<128, 256, 64, 64, true>(*a, stream);
     else launch_tiles<128, 256, 64, 64, false>(*a, stream);
+  } else if (how == 3) {
+    if (gated) launch_tiles<64, 256, 64, 64, true>(*a, stream);
+    else launch_tiles<64, 128, 64, 32, false>(*a, stream);
+  } else if (how == 2) {
+    if (gated) launch_tiles<32, 256, 32, 64, true>(*a, stream);
+    else launch_tiles<32, 128, 32, 32, false>(*a, stream);
   } else if (how == 1) {
     const dim3 grid((a->N + (gated ? 15 : 31)) / (gated ? 16 : 32), a->max_tiles);
     if (gated) moe_stream_kernel<true><<<grid, 256, 0, stream>>>(*a);

@@ -274,36 +274,64 @@ attn_rows_kernel(RowsArgs a) {
   }
 }
 
-template <typename T>
-__global__ void __launch_bounds__(64)
+// One workgroup = one query row and head, 64 V columns; its four waves take
+// every fourth split.  At most 64 splits.
+template <typename T, int V>
+__global__ void __launch_bounds__(256)
 attn_rows_merge_kernel(const float* __restrict__ part, T* __restrict__ out,
                        int splits, int E) {
+  __shared__ float coef[64], sum[4][64][V];
   const long rh = blockIdx.x;
+  const int lane = threadIdx.x & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const float* p = part + rh * splits * (E + 2);
-  float mm = NEG_BIG;
-  for (int s = 0; s < splits; ++s) mm = fmaxf(mm, p[s * (E + 2) + E]);
-  float ll = 0.f;
-  for (int s = 0; s < splits; ++s)
-    ll += p[s * (E + 2) + E + 1] *
-          __builtin_amdgcn_exp2f(p[s * (E + 2) + E] - mm);
-  const float inv = 1.f / ll;
-  for (int e = threadIdx.x; e < E; e += 64) {
-    float acc = 0.f;
-    for (int s = 0; s < splits; ++s)
-      acc += p[s * (E + 2) + e] *
-             __builtin_amdgcn_exp2f(p[s * (E + 2) + E] - mm);
-    from_f(out[rh * E + e], acc * inv);
+  if (wid == 0) {
+    float m = NEG_BIG, l = 0.f;
+    if (lane < splits) {
+      m = p[(long)lane * (E + 2) + E];
+      l = p[(long)lane * (E + 2) + E + 1];
+    }
+    float mm = m;
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) mm = fmaxf(mm, __shfl_xor(mm, off, 64));
+    const float w = __builtin_amdgcn_exp2f(m - mm);
+    l *= w;
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) l += __shfl_xor(l, off, 64);
+    coef[lane] = w / l;
   }
+  __syncthreads();
+  const int e = (blockIdx.y * 64 + lane) * V;
+  float acc[V] = {};
+  if (e < E) {
+    const float* src = p + e;
+#pragma unroll 8
+    for (int s = wid; s < splits; s += 4) {
+      const float c = coef[s];
+#pragma unroll
+      for (int j = 0; j < V; ++j) acc[j] += c * src[(long)s * (E + 2) + j];
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) sum[wid][lane][j] = acc[j];
+  __syncthreads();
+  if (wid > 0 || e >= E) return;
+#pragma unroll
+  for (int j = 0; j < V; ++j)
+    from_f(out[rh * E + e + j], sum[0][lane][j] + sum[1][lane][j] +
+                                    sum[2][lane][j] + sum[3][lane][j]);
 }
 
 extern "C" int sv_attn_merge(const float* part, void* out, long rows,
                              int splits, int E, int f32, hipStream_t stream) {
-  if (f32)
-    attn_rows_merge_kernel<float><<<rows, 64, 0, stream>>>(part, (float*)out,
-                                                           splits, E);
-  else
-    attn_rows_merge_kernel<short><<<rows, 64, 0, stream>>>(part, (short*)out,
-                                                           splits, E);
+  if (splits > 64) return 1;
+  const int v = E % 2 ? 1 : 2;
+  const dim3 grid(rows, (E + 64 * v - 1) / (64 * v));
+#define AM(T, V) attn_rows_merge_kernel<T, V><<<grid, 256, 0, stream>>>( \
+      part, (T*)out, splits, E)
+  if (f32) { if (v == 2) AM(float, 2); else AM(float, 1); }
+  else     { if (v == 2) AM(short, 2); else AM(short, 1); }
+#undef AM
   return (int)hipGetLastError();
 }
 

@@ -654,7 +654,7 @@ def latent_rows(q, cache, rank: int, pos, seq, block_table, heads: int,
         max_keys = min(max_keys, window) if max_keys else window
     out = torch.empty(rows, heads * rank, dtype=q.dtype, device=q.device)
     fast = latent_rows_supported(q.dtype, rank, D - rank)
-    splits = _row_splits(512, rows * -(-heads // 32), max_keys, 64) if fast \
+    splits = _row_splits(512, rows * -(-heads // 32), max_keys, 128) if fast \
         else _row_splits(1024, rows, max_keys, 128)
     part = torch.empty(rows * heads * splits * (rank + 2),
                        dtype=torch.float32, device=q.device) \
@@ -772,9 +772,18 @@ def latent_attention(q, kv, gate, batch, cache, w: LatentWeights, heads: int,
 # mixture of experts
 # ---------------------------------------------------------------------------
 
-MOE_PLAIN, MOE_STREAM, MOE_TILES = 0, 1, 2
-MOE_TILE_ROWS = {MOE_PLAIN: 32, MOE_STREAM: 32, MOE_TILES: 128}
-MOE_STREAM_ROWS = 64        # rows an expert, up to which weights are streamed
+# kernels of the grouped products, and the most slots of their tiles
+MOE_PLAIN, MOE_STREAM = 0, 1
+MOE_TILES = (2, 3, 4, 5)
+MOE_TILE_ROWS = (32, 32, 32, 64, 128, 256)
+
+
+def moe_kernel(pairs: int, experts: int) -> int:
+    """The fastest kernel for ``pairs`` spread over ``experts`` (measured)."""
+    rows = pairs / experts
+    if rows < 4:
+        return MOE_STREAM
+    return MOE_TILES[sum(rows >= r for r in (24, 112, 160))]
 
 
 @dataclass
@@ -839,10 +848,8 @@ def moe_mlp(h, z, bias, gate_up, down, top: int, alpha: float, limit: float,
     of the chosen experts' outputs."""
     E, W, ff = down.shape
     pairs = h.shape[0] * top
-    if h.dtype != torch.bfloat16 or not _aligned((W, ff), h):
-        how = MOE_PLAIN
-    else:
-        how = MOE_STREAM if pairs <= MOE_STREAM_ROWS * E else MOE_TILES
-    plan = moe_plan(z, bias, top, how)
+    fast = h.dtype == torch.bfloat16 and _aligned((W, ff), h)
+    plan = moe_plan(z, bias, top,
+                    moe_kernel(pairs, E) if fast else MOE_PLAIN)
     act = moe_gemm(h, gate_up, plan, True, alpha, limit, shift)
     return Pending(moe_gemm(act, down, plan, False), coef=plan.coef)

@@ -290,7 +290,7 @@ def test_head_linear(sv, H, N, K, T, dtype):
 @pytest.mark.parametrize("T,E,top", [(1, 3, 1), (5, 8, 8), (64, 65, 6),
                                      (65, 130, 4), (300, 512, 20),
                                      (700, 8, 2)])
-@pytest.mark.parametrize("how", [0, 2])
+@pytest.mark.parametrize("how", [0, 3, 4, 5])
 def test_plan_routes_and_groups(sv, T, E, top, how):
     z = _rand(T, E, dtype=torch.float32)
     bias = _rand(E, dtype=torch.float32, seed=1)
@@ -309,13 +309,21 @@ def test_plan_routes_and_groups(sv, T, E, top, how):
     assert seen == list(range(T * top))
 
 
+def test_kernel_of_the_grouped_products_fits_the_load():
+    from neuronx_distributed_amd.ops import serving as sv
+
+    rows = [sv.MOE_TILE_ROWS[sv.moe_kernel(n, 8)]
+            for n in (1, 40, 64, 300, 1000, 5000)]
+    assert rows == [32, 32, 32, 64, 128, 256]
+
+
 def test_plan_breaks_ties_by_index_and_takes_uneven_loads(sv):
     z = torch.zeros(70, 9)
     p = sv.moe_plan(z.cuda(), None, 3, 0)
     assert (p.idx.cpu() == torch.tensor([0, 1, 2])).all()
     _close(p.coef, torch.full((70, 3), 1 / 3), torch.float32)
     z[:, 7] = 5.0                  # every row to one expert
-    p = sv.moe_plan(z.cuda(), None, 1, 2)
+    p = sv.moe_plan(z.cuda(), None, 1, 4)
     assert (p.idx.cpu() == 7).all()
     assert [t[:3] for t in p.tiles.cpu().tolist() if t[2]] == [[7, 0, 70]]
 
@@ -352,7 +360,7 @@ def test_experts(sv, case, dtype):
     gu = torch.cat([gate, up], 1).cuda()
     hows = [sv.MOE_PLAIN]
     if dtype == torch.bfloat16 and W % 8 == 0 and ff % 8 == 0:
-        hows += [sv.MOE_STREAM, sv.MOE_TILES]
+        hows += [sv.MOE_STREAM, *sv.MOE_TILES]
     for how in hows:
         p = sv.moe_plan(z.cuda(), bias.cuda(), top, how)
         act = sv.moe_gemm(h.cuda(), gu, p, True, 1.702, limit, 1.0)
