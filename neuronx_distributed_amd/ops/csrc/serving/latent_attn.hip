@@ -251,9 +251,6 @@ struct LatentRowsArgs {
   float scale;
 };
 
-typedef short tr4 __attribute__((ext_vector_type(4)));
-typedef __attribute__((address_space(3))) tr4* lds_tr4;
-
 template <int EP>
 __global__ void __launch_bounds__(256, 2)
 latent_rows_kernel(LatentRowsArgs a) {

@@ -175,9 +175,6 @@ __device__ __forceinline__ float glu(const MoeGemmArgs& a, float g, float u) {
 // (DMA, K a multiple of 64) or through registers.  With a gated activation
 // the weight rows of a tile alternate 32 gate, 32 up, so a lane holds both of
 // a column.
-typedef __attribute__((address_space(1))) const void* global_ptr;
-typedef __attribute__((address_space(3))) void* lds_ptr;
-
 template <int BM, int BN, int WM, int WN, bool GLU, bool DMA>
 __global__ void __launch_bounds__(BM / WM * BN / WN * 64)
 moe_tiles_kernel(MoeGemmArgs a) {

@@ -384,7 +384,8 @@ extern "C" int sv_attn_rows(const RowsArgs* a, int vec, int f32,
 // NP bf16 planes (3 planes carry the full 24-bit significand) and V enters
 // once per plane.  P never leaves registers: the accumulator's row order
 // {4 hi + 0..3, 8 + 4 hi + 0..3} of a 16-key chunk is used as the
-// contraction order of P V, and V^T is read from LDS in the same order.
+// contraction order of P V, and V^T is read from LDS in the same order
+// (transposing loads).
 // ---------------------------------------------------------------------------
 //
 // A key may end in columns that all heads share (kr): the rotated part of
@@ -407,24 +408,29 @@ struct TilesArgs {
   float scale;
 };
 
-// 16-byte slots of a row of CPR slots, rotated so that consecutive rows of
-// one column spread over the banks
-template <int CPR>
-__device__ __forceinline__ int row_swz(int row, int byte) {
-  return byte ^ ((CPR % 16 == 0 ? row & 15
-                  : CPR % 8 == 0 ? (row >> 1) & 7 : (row >> 2) & 3) << 4);
+// The 16-byte slots of a key row are rotated within groups of eight, so that
+// consecutive rows of one column spread over the banks; those of a value row
+// in pieces of four, which a transposing read takes from four rows at once.
+template <int SLOTS>
+__device__ __forceinline__ int key_turn(int row) {
+  return (SLOTS % 16 == 0 ? row : row >> 1) & 7;
+}
+template <int SLOTS>
+__device__ __forceinline__ int value_turn(int row) {
+  return (SLOTS % 16 == 0 ? row & 3 : (row >> 1) & 1) << 2;
 }
 
-template <int DK, int DE, int NP>
+template <int DK, int DE, int NP, bool SHARED>
 __global__ void __launch_bounds__(256, DE <= 128 ? 2 : 1)
 attn_tiles_kernel(TilesArgs a) {
   constexpr int NC = DK / 16;        // 16-wide chunks of the key size
   constexpr int NB = DE / 32;        // 32-row blocks of O^T
   constexpr int KP = DK * 2;         // K row pitch (bytes)
   constexpr int CK = DK / 8, CV = DE / 8;  // 16-byte slots of a row
-  constexpr int PK = 32 * CK / 256, PV = 32 * CV / 256;  // items a thread
-  __shared__ __attribute__((aligned(16))) char kbuf[64 * KP];
-  __shared__ __attribute__((aligned(16))) short vbuf[DE * 64];  // V^T
+  // two key tiles, rows as in the cache; apart by name, so that a read of one
+  // need not wait for the words on their way into the other
+  __shared__ __attribute__((aligned(16))) char k0[64 * KP], k1[64 * KP];
+  __shared__ __attribute__((aligned(16))) char v0[128 * DE], v1[128 * DE];
 
   // later tiles of a portion see more keys: they start first
   const int* tl = a.tiles + 4 * (gridDim.y - 1 - blockIdx.y);
@@ -462,104 +468,93 @@ attn_tiles_kernel(TilesArgs a) {
   const int ntiles = nk + max(0, t_hi - t_lo + 1);
   const int w_lo = p0 + wid * 32, w_hi = min(w_lo + 31, q_hi);
 
-  uint4v kreg[2 * PK], vreg[2 * PV];
+  // 32-bit within a page
+  const int krow = (int)a.krow, vrow = (int)a.vrow, rrow = (int)a.rrow;
   auto tile_of = [&](int n) { return n < nk ? n : t_lo + n - nk; };
-  // items are (row pair, slot) of the tile
-  auto issue = [&](int n) {
+  // Ask for the rows of a tile: a wave's 64 slots of 16 bytes follow each
+  // other in LDS, so the rotation of a row's slots is done on the source.
+  auto issue = [&](int n, char* kd, char* vd) {
     const long page = bt[tile_of(n)];
     const short* kb = a.kc + page * a.kpage + g * a.khead;
     const short* vb = a.vc + page * a.vpage + g * a.vhead;
-    const short* rb = a.kr + page * SV_PAGE * a.rrow - a.DS;
+    const short* rb = SHARED ? a.kr + page * SV_PAGE * rrow - a.DS : nullptr;
 #pragma unroll
-    for (int p = 0; p < PK; ++p) {
-      const int it = p * 256 + tid;
-      const int r = it / CK * 2, c = it % CK * 8;
-#pragma unroll
-      for (int x = 0; x < 2; ++x)
-        kreg[2 * p + x] = c < D
-            ? *(const uint4v*)(c < a.DS ? kb + (r + x) * a.krow + c
-                                        : rb + (r + x) * a.rrow + c)
-            : uint4v{0, 0, 0, 0};
+    for (int p = 0; p < CK / 4; ++p) {
+      const int it = p * 256 + tid, r = it / CK;
+      const int c = (it % CK ^ key_turn<CK>(r)) * 8;
+      if (c >= D) continue;
+      __builtin_amdgcn_global_load_lds(
+          (global_ptr)(SHARED && c >= a.DS ? rb + (r * rrow + c)
+                                           : kb + (r * krow + c)),
+          (lds_ptr)(kd + (p * 256 + wid * 64) * 16), 16, 0, 0);
     }
 #pragma unroll
-    for (int p = 0; p < PV; ++p) {
-      const int it = p * 256 + tid;
-      const int r = it / CV * 2, c = it % CV * 8;
-#pragma unroll
-      for (int x = 0; x < 2; ++x)
-        vreg[2 * p + x] = c < E
-            ? *(const uint4v*)(vb + (r + x) * a.vrow + c)
-            : uint4v{0, 0, 0, 0};
+    for (int p = 0; p < CV / 4; ++p) {
+      const int it = p * 256 + tid, r = it / CV;
+      const int c = (it % CV ^ value_turn<CV>(r)) * 8;
+      if (c >= E) continue;
+      __builtin_amdgcn_global_load_lds(
+          (global_ptr)(vb + (r * vrow + c)),
+          (lds_ptr)(vd + (p * 256 + wid * 64) * 16), 16, 0, 0);
     }
   };
-  auto commit = [&]() {
+  // this lane's part of the addresses in a tile (bytes): slot 2 c + hi of key
+  // row col; a transposing read, where 16 lanes turn 4 keys by 16 columns
+  int kx[4];
 #pragma unroll
-    for (int p = 0; p < PK; ++p) {
-      const int it = p * 256 + tid;
-      const int r = it / CK * 2, c = it % CK * 16;
-#pragma unroll
-      for (int x = 0; x < 2; ++x)
-        *(uint4v*)(kbuf + (r + x) * KP + row_swz<CK>(r + x, c)) =
-            kreg[2 * p + x];
-    }
-#pragma unroll
-    for (int p = 0; p < PV; ++p) {
-      const int it = p * 256 + tid;
-      const int r = it / CV * 2, c = it % CV * 8;
-      union { uint4v u; unsigned short s[8]; } x, y;
-      x.u = vreg[2 * p];
-      y.u = vreg[2 * p + 1];
-      const TileWrite tw(c, r);
-#pragma unroll
-      for (int j = 0; j < 8; ++j)
-        *(uint*)(vbuf + tw.at(j)) = (uint)x.s[j] | ((uint)y.s[j] << 16);
-    }
-  };
+  for (int c = 0; c < 4; ++c)
+    kx[c] = col * KP + ((2 * c + hi) ^ key_turn<CK>(col)) * 16;
+  const int tr_key = 4 * hi + ((lane & 15) >> 2);
+  const int vx = (tr_key * DE + ((lane >> 4) & 1) * 16 + (lane & 3) * 4 +
+                  value_turn<CV>(tr_key) * 8) * 2;
 
-  const TileRead vt(col, 4 * hi);
-  issue(0);
-  for (int n = 0; n < ntiles; ++n) {
-    __syncthreads();           // readers of the previous tile are done
-    commit();
-    __syncthreads();
-    if (n + 1 < ntiles) issue(n + 1);
-
+  auto attend = [&](int n, const char* kbuf, char* vbuf) {
     const int kv0 = tile_of(n) * SV_PAGE;
     const bool active = wid * 32 < nrow && kv0 <= w_hi &&
         (a.window <= 0 || kv0 < a.keep || kv0 + SV_PAGE - 1 > w_lo - a.window);
-    if (!active) continue;
+    if (!active) return;
 
     f32x16 acc[2] = {};
 #pragma unroll
-    for (int kb = 0; kb < 2; ++kb) {
-      const int row = col + 32 * kb;
+    for (int c = 0; c < NC; ++c)
 #pragma unroll
-      for (int c = 0; c < NC; ++c) {
+      for (int kb = 0; kb < 2; ++kb) {
         frag_u kf;
-        kf.u4 = *(const uint4v*)(kbuf + row * KP +
-                                 row_swz<CK>(row, (c * 16 + hi * 8) * 2));
+        kf.u4 = *(const uint4v*)(kbuf + kx[c & 3] + (c >> 2) * 128 +
+                                 kb * 32 * KP);
         acc[kb] = mfma_bf16(kf.bf, qf[c].bf, acc[kb]);
       }
+    // the reads run two chunks ahead
+    __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
+#pragma unroll
+    for (int c = 0; c < NC - 2; ++c) {
+      __builtin_amdgcn_sched_group_barrier(0x8, 2, 0);
+      __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);
     }
+    __builtin_amdgcn_sched_group_barrier(0x8, 4, 0);
 
     const bool masked = kv0 + SV_PAGE - 1 > w_lo ||
         (a.window > 0 && w_hi - kv0 >= a.window &&
          kv0 + SV_PAGE > a.keep);
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) acc[kb] *= s2;
+    if (masked) {
+      const int i0 = my_pos - kv0;             // keys up to i0 are not ahead
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          const int j = 32 * kb + acc_row(r, hi);
+          const bool gone = j > i0 || (a.window > 0 && i0 - j >= a.window &&
+                                       kv0 + j >= a.keep);
+          acc[kb][r] = gone ? NEG_BIG : acc[kb][r];
+        }
+    }
     float mt = NEG_BIG;
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
-      for (int r = 0; r < 16; ++r) {
-        float s = acc[kb][r] * s2;
-        if (masked) {
-          const int j = kv0 + 32 * kb + acc_row(r, hi);
-          if (j > my_pos ||
-              (a.window > 0 && my_pos - j >= a.window && j >= a.keep))
-            s = NEG_BIG;
-        }
-        acc[kb][r] = s;
-        mt = fmaxf(mt, s);
-      }
+      for (int r = 0; r < 16; ++r) mt = fmaxf(mt, acc[kb][r]);
     mt = fmaxf(mt, __shfl_xor(mt, 32, 64));
     const float m_new = fmaxf(m_run, mt);
     const float m_eff = fmaxf(m_new, -1e28f);  // an all-masked row stays 0
@@ -596,17 +591,46 @@ attn_tiles_kernel(TilesArgs a) {
             y -= __uint_as_float(w & 0xffff0000u);
           }
         }
-        const int slot = 4 * kb + 2 * cc;
 #pragma unroll
         for (int nb = 0; nb < NB; ++nb) {
-          frag_u vf;
-          *(uint2*)&vf.u[0] = *(const uint2*)(vbuf + vt.at(nb, slot));
-          *(uint2*)&vf.u[2] = *(const uint2*)(vbuf + vt.at(nb, slot + 1));
+          union { tr4 t[2]; bf16x8 bf; } vf;
+#pragma unroll
+          for (int u = 0; u < 2; ++u)
+            vf.t[u] = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                (lds_tr4)(vbuf + (vx ^ (nb * 64)) +
+                          (32 * kb + 16 * cc + 8 * u) * DE * 2));
 #pragma unroll
           for (int z = 0; z < NP; ++z)
             ot[nb] = mfma_bf16(vf.bf, pf[z].bf, ot[nb]);
         }
+        __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
+#pragma unroll
+        for (int nb = 0; nb < NB - 2; ++nb) {
+          __builtin_amdgcn_sched_group_barrier(0x8, NP, 0);
+          __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);
+        }
+        __builtin_amdgcn_sched_group_barrier(0x8, 2 * NP, 0);
       }
+  };
+
+  if (D < DK) {                // columns that no tile writes
+    for (int i = tid; i < 64 * CK; i += 256) {
+      *(uint4v*)(k0 + i * 16) = uint4v{0, 0, 0, 0};
+      *(uint4v*)(k1 + i * 16) = uint4v{0, 0, 0, 0};
+    }
+    __syncthreads();
+  }
+  issue(0, k0, v0);
+  __syncthreads();             // also waits for the words on their way
+  for (int n = 0; n < ntiles; n += 2) {
+    const bool more = n + 1 < ntiles;
+    if (more) issue(n + 1, k1, v1);
+    attend(n, k0, v0);
+    __syncthreads();
+    if (!more) break;
+    if (n + 2 < ntiles) issue(n + 2, k0, v0);
+    attend(n + 1, k1, v1);
+    __syncthreads();
   }
 
   if (my >= nrow) return;
@@ -638,7 +662,11 @@ extern "C" int sv_attn_tiles(const TilesArgs* a, int n_tiles,
                              hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   const dim3 grid(a->H, n_tiles);
-#define AT(K, V) attn_tiles_kernel<K, V, 3><<<grid, 256, 0, stream>>>(*a)
+#define AT(K, V)                                                          \
+  do {                                                                    \
+    if (a->kr) attn_tiles_kernel<K, V, 3, true><<<grid, 256, 0, stream>>>(*a); \
+    else attn_tiles_kernel<K, V, 3, false><<<grid, 256, 0, stream>>>(*a); \
+  } while (0)
   if (a->D <= 64 && a->E <= 64) AT(64, 64);
   else if (a->D <= 128 && a->E <= 128) AT(128, 128);
   else if (a->D <= 192 && a->E <= 128) AT(192, 128);

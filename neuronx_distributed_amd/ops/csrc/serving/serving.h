@@ -13,6 +13,12 @@
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef short s4v __attribute__((ext_vector_type(4)));
 
+// operands of direct loads into LDS and of transposing LDS loads
+typedef __attribute__((address_space(1))) const void* global_ptr;
+typedef __attribute__((address_space(3))) void* lds_ptr;
+typedef short tr4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) tr4* lds_tr4;
+
 __device__ __forceinline__ float to_f(short v) { return bits2f(v); }
 __device__ __forceinline__ float to_f(float v) { return v; }
 __device__ __forceinline__ void from_f(short& o, float v) { o = f2bits(v); }
