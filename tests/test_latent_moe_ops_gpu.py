@@ -87,6 +87,7 @@ LATENT = [
     (33, 8, 64, 8, 320, 1),
     (3, 10, 6, 7, 21, 70),          # sizes that are no multiple of 8
     (2, 40, 80, 200, 600, 65),      # too large for the MFMA row kernel
+    (2, 112, 48, 96, 64, 90),       # key and value tiles with empty columns
     (2, 6, 2, 3, 9, 0),             # odd sums from several key ranges
 ]
 
