@@ -12,7 +12,7 @@ from .functions import (
 from .kv_cache import (KVCache, RollingKVCache,
                        build_kv_caches)
 from .generation import generate
-from .paged_cache import (CacheFull, CacheManager, MatrixState, PagedKV,
-                          PagedLatent)
+from .paged_cache import (CacheFull, CacheManager, ConvRing, MatrixState,
+                          PagedKV, PagedLatent)
 from .engine import InferenceEngine, StepEntry
 from .scheduler import Scheduler, generate_ragged

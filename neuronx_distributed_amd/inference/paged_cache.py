@@ -5,7 +5,9 @@ A model lists, for every layer run, what it keeps between steps:
 * ``PagedKV``      keys and values of an attention, in pages of 64 tokens,
 * ``PagedLatent``  latents and shared key columns of a latent attention, one
                  row a token for all heads, in the same pages,
-* ``MatrixState``  the state of a recurrent matrix memory, one slot a request.
+* ``MatrixState``  the state of a recurrent matrix memory, one slot a request,
+* ``ConvRing``     the last inputs of a short convolution over time, one slot a
+                 request.
 
 All layers share one block table per request (page index -> the same page in
 every layer's pool), so the host tracks pages once.  Pages behind every
@@ -74,6 +76,18 @@ class MatrixState:
         nt = (self.vdim + 31) // 32
         return (S, torch.zeros(slots, self.heads, nt, self.dim, **f32),
                 torch.zeros(slots, self.heads, nt, **f32))
+
+
+@dataclass(frozen=True)
+class ConvRing:
+    """The input at position p is in place p % taps; a place is read only if
+    its request has been there, so a slot needs no clearing."""
+    channels: int
+    taps: int
+
+    def allocate(self, pages, slots, dtype, device):
+        return torch.zeros(slots, self.taps, self.channels, dtype=dtype,
+                           device=device)
 
 
 @dataclass

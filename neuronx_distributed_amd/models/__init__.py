@@ -7,5 +7,7 @@ from .voletar import (VoletarConfig, VoletarForCausalLM, VOLETAR_CONFIGS,
                       get_voletar_config)
 from .nesilorn import (NesilornConfig, NesilornForCausalLM, NESILORN_CONFIGS,
                        get_nesilorn_config)
+from .sutuvik import (SutuvikConfig, SutuvikForCausalLM, SUTUVIK_CONFIGS,
+                      get_sutuvik_config)
 from .registry import (ModelEntry, build_model, load_pretrained,
                        register_model, registered_models)

@@ -11,12 +11,13 @@ kernels read as strided slices.
 """
 
 import math
-from typing import List, Sequence
+from typing import List, Optional, Sequence
 
 import torch
 import torch.nn as nn
 
-from ..inference.paged_cache import MatrixState, PagedKV, PagedLatent
+from ..inference.paged_cache import (ConvRing, MatrixState, PagedKV,
+                                     PagedLatent)
 from ..ops import serving as sv
 from ..parallel.layers import ColumnParallelLinear, RowParallelLinear
 
@@ -54,6 +55,10 @@ class CheckpointReader:
         self.used.add(name)
         return self.tensors[name]
 
+    def skip(self, name: str):
+        """This tensor may be there, and has no place."""
+        self.used.add(name)
+
     def done(self):
         extra = set(self.tensors) - self.used
         if extra:
@@ -66,6 +71,7 @@ class Mixer(nn.Module):
     which they are stacked, ``sizes`` their widths."""
     names: Sequence[str]
     sizes: Sequence[int]
+    padding = 0         # rows of zeros behind the projections
 
     def cache_specs(self) -> list:
         raise NotImplementedError
@@ -76,6 +82,8 @@ class Mixer(nn.Module):
             if p.shape[0] != s:
                 raise ValueError(f"{prefix}{n} has {p.shape[0]} rows, "
                                  f"expected {s}")
+        if self.padding:
+            parts.append(parts[0].new_zeros(self.padding, parts[0].shape[1]))
         return torch.cat(parts)
 
     def split(self, proj):
@@ -115,6 +123,114 @@ class SlidingAttention(Mixer):
         return self.o(sv.ragged_attention(
             q, k, v, batch, pools[0], self.heads, self.scale, self.window,
             self.keep_first))
+
+
+class ScoredAttention(Mixer):
+    """Causal softmax attention with grouped key/value heads and modified
+    scores; what is None or zero is left out.
+
+    rot        rotation of neighbouring pairs: base, dims, scaling
+    qk_norm    RMS norm of queries and keys, a head: "plain" or "weighted"
+    q_temp     queries grow with their position: coef, every
+    slopes     distance bias, a number a head
+    head_temp  a learned factor of the scores, a head
+    softcap    cap of the scores
+    sink       a score of the denominator alone: "zero" or "learned"
+    gate       a sigmoid gate a head
+    v_mix      values take a share of those of the first layer that has it
+    """
+
+    def __init__(self, width, heads, kv_heads, dim, vdim, scale, eps,
+                 rot=None, qk_norm=None, q_temp=None, slopes=None,
+                 head_temp=False, softcap=0.0, sink=None, gate=False,
+                 v_mix=False):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if rot and (rot["dims"] % 2 or not 0 <= rot["dims"] <= dim):
+            raise ValueError(f"{rot['dims']} of {dim} dimensions turn")
+        if qk_norm not in (None, "plain", "weighted") or \
+                sink not in (None, "zero", "learned"):
+            raise ValueError(f"norm {qk_norm!r}, sink {sink!r}")
+        if slopes is not None and len(slopes) != heads:
+            raise ValueError("one slope per head")
+        if max(dim, vdim) > sv.MAX_HEAD_DIM:
+            raise ValueError(f"head size {max(dim, vdim)} > "
+                             f"{sv.MAX_HEAD_DIM}")
+        self.heads, self.scale, self.eps = heads, scale, eps
+        self.rot, self.qk_norm = rot, qk_norm
+        self.q_temp = (q_temp["coef"], q_temp["every"]) if q_temp else (0., 0)
+        self.slopes, self.softcap = slopes, softcap or 0.0
+        self.v_mix, self.gated = v_mix, gate
+        self.kv = PagedKV(kv_heads, dim, vdim)
+        self.names = ("q", "k", "v") + (("g",) if gate else ())
+        self.sizes = (heads * dim, kv_heads * dim, kv_heads * vdim) + \
+            ((heads,) if gate else ())
+        # a whole number of 16-byte words a row
+        self.padding = -sum(self.sizes) % 8
+        self.loads = []
+        if qk_norm == "weighted":
+            self.q_norm, self.k_norm = _vector(dim), _vector(dim)
+            self.loads += [("q_norm", "q.norm"), ("k_norm", "k.norm")]
+        if head_temp:
+            self.temp = _vector(heads)
+            self.loads.append(("temp", "temp"))
+        if sink == "learned":
+            self.sink = nn.Parameter(torch.zeros(heads))
+            self.loads.append(("sink", "sink"))
+        elif sink == "zero":
+            self.register_buffer("sink", torch.zeros(heads),
+                                 persistent=False)
+        if v_mix:
+            self.mix = nn.Parameter(torch.full((), 0.5))
+            self.loads.append(("mix", "vmix"))
+        self.o = _row(heads * vdim, width)
+        self._const = None
+
+    def cache_specs(self):
+        return [self.kv]
+
+    def load(self, get, prefix):
+        for name, key in self.loads:
+            copy_weight(getattr(self, name), get(prefix + key))
+        if not self.v_mix:
+            get.skip(prefix + "vmix")
+        copy_weight(self.o.weight, get(prefix + "o"))
+
+    def _constants(self, device):
+        if self._const is None or self._const[0] != device:
+            freq = sv.rotary_frequencies(
+                self.rot["base"], self.rot["dims"], device,
+                self.rot.get("scaling")) if self.rot else None
+            slope = None if self.slopes is None else torch.tensor(
+                self.slopes, dtype=torch.float64).float().to(device)
+            self._const = device, freq, slope
+        return self._const[1:]
+
+    def forward(self, h, proj, batch, pools, values: Optional[list] = None):
+        """``values`` is a step's list of the values that layers share: the
+        first layer that mixes puts its own there."""
+        q, k, v, *g = self.split(proj)
+        freq, slope = self._constants(h.device)
+        prep = sv.QkvPrep(freq=freq, norm=self.qk_norm is not None,
+                          q_norm=getattr(self, "q_norm", None),
+                          k_norm=getattr(self, "k_norm", None), eps=self.eps,
+                          temp_coef=self.q_temp[0], temp_every=self.q_temp[1])
+        if self.v_mix:
+            if values:
+                prep.first, prep.mix = values[0], self.mix
+            else:
+                values.append(v)
+        mod = sv.ScoreMod(temp=getattr(self, "temp", None), cap=self.softcap,
+                          slope=slope, sink=getattr(self, "sink", None),
+                          gate=g[0] if g else None)
+        return self.o(sv.ragged_attention(q, k, v, batch, pools[0],
+                                          self.heads, self.scale, prep=prep,
+                                          mod=mod))
+
+
+def alibi_slopes(heads: int) -> List[float]:
+    return [2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)]
 
 
 class LatentAttention(Mixer):
@@ -252,13 +368,93 @@ class GatedMemory(_MatrixMemory):
                           1.0 / math.sqrt(self.dim))
 
 
+class StateSpaceMemory(Mixer):
+    """State-space duality (Mamba-2): a matrix state per head whose decay and
+    input weight come from a projected time step; x, B and C pass a short causal
+    convolution and silu, heads share B and C in groups; a skip of x, a silu
+    gate, then a norm over ``norm_groups`` equal parts."""
+    names = ("in",)
+
+    def __init__(self, width, heads, vdim, state, groups, taps, norm_groups,
+                 eps):
+        super().__init__()
+        inner = heads * vdim
+        if heads % groups or inner % norm_groups:
+            raise ValueError(f"{heads} heads in {groups} groups, {inner} "
+                             f"columns in {norm_groups}")
+        if state > sv.MAX_HEAD_DIM or not 1 <= taps <= sv.MAX_TAPS:
+            raise ValueError(f"state of {state}, {taps} taps")
+        self.heads, self.eps, self.norm_group = heads, eps, \
+            inner // norm_groups
+        self.parts = (inner, groups * state, groups * state)   # x, B, C
+        channels = sum(self.parts)
+        self.sizes = (inner, channels)
+        self.padding = -sum(self.sizes) % 8
+        self.memory = MatrixState(heads, state, vdim)
+        self.ring = ConvRing(channels, taps)
+        self.step_proj = nn.Parameter(
+            torch.randn(heads, width) * width ** -0.5)
+        self.step_bias = nn.Parameter(torch.zeros(heads))
+        self.A_log = nn.Parameter(torch.zeros(heads))
+        self.skip = _vector(heads)
+        self.conv = nn.Parameter(torch.full((taps, channels), 1.0 / taps))
+        self.conv_bias = nn.Parameter(torch.zeros(channels))
+        self.norm = _vector(inner)
+        self.o = _row(inner, width)
+
+    def cache_specs(self):
+        return [self.memory, self.ring]
+
+    def stacked(self, get, prefix):
+        w = get(prefix + "in")
+        n = sum(self.sizes)
+        if w.shape[0] != n + self.heads:
+            raise ValueError(f"{prefix}in has {w.shape[0]} rows, expected "
+                             f"{n + self.heads}")
+        return torch.cat([w[:n], w.new_zeros(self.padding, w.shape[1])])
+
+    def load(self, get, prefix):
+        copy_weight(self.step_proj, get(prefix + "in")[-self.heads:])
+        copy_weight(self.conv, get(prefix + "conv").t())
+        for name, key in (("step_bias", "dt_bias"), ("A_log", "A_log"),
+                          ("skip", "D"), ("conv_bias", "conv.b"),
+                          ("norm", "norm")):
+            copy_weight(getattr(self, name), get(prefix + key))
+        copy_weight(self.o.weight, get(prefix + "o"))
+
+    def forward(self, h, proj, batch, pools):
+        (S, _, _), ring = pools
+        z, xbc = self.split(proj)
+        step = sv.linear_f32(h, self.step_proj)
+        conv = sv.ShortConv(self.conv, ring, self.conv_bias)
+        n, T = batch.portion_tokens, h.shape[0]
+        out = torch.empty_like(z, memory_format=torch.contiguous_format)
+
+        def mix(a, b, x, seg, **kw):
+            v, k, q = x.split(self.parts, dim=1)
+            gate = sv.TimeGate(step[a:b], self.step_bias, self.A_log,
+                               self.skip, z[a:b], kw.pop("conv", None))
+            sv.memory_mix(q, k, v, gate, S, None, None, seg, self.heads,
+                          out=out[a:b], **kw)
+
+        if n:
+            x = sv.short_conv(xbc[:n], conv, batch.portions, batch.chunks,
+                              silu=True)
+            mix(0, n, x, batch.portions, chunks=batch.chunks,
+                chunk_first=batch.chunk_first)
+        if n < T:      # the rows of a segment count from the whole batch
+            mix(0, T, xbc, batch.singles, conv=conv)
+        return self.o(sv.gated_norm(out, self.norm, None, self.norm_group,
+                                    self.eps))
+
+
 class SingleMixer(nn.Module):
     """One mixer with its projection."""
 
     def __init__(self, width, mixer: Mixer):
         super().__init__()
         self.mixer = mixer
-        self.proj = _column(width, sum(mixer.sizes))
+        self.proj = _column(width, sum(mixer.sizes) + mixer.padding)
 
     def cache_specs(self) -> List:
         return self.mixer.cache_specs()
@@ -267,8 +463,9 @@ class SingleMixer(nn.Module):
         copy_weight(self.proj.weight, self.mixer.stacked(get, prefix))
         self.mixer.load(get, prefix)
 
-    def forward(self, h, batch, pools) -> sv.Pending:
-        return sv.Pending(self.mixer(h, self.proj(h), batch, pools))
+    def forward(self, h, batch, pools, **shared) -> sv.Pending:
+        return sv.Pending(self.mixer(h, self.proj(h), batch, pools,
+                                     **shared))
 
 
 class ParallelMixer(nn.Module):
@@ -334,16 +531,17 @@ class GeluMLP(_PlainMLP):
 
 class ExpertsMLP(nn.Module):
     """A router with a bias and gated experts: min(g, limit) sigmoid(alpha g)
-    (clamp(u, limit) + shift); the ``top`` experts with the largest logits
-    are summed, weighted by a softmax over their logits.  The sum is left
-    pending, so it fuses into the next residual norm."""
+    (clamp(u, limit) + shift); the chosen experts are summed, weighted as
+    ``routing`` (or the plain routing, if it is a number of experts) says.  The
+    sum is left pending, so it fuses into the next residual norm."""
 
-    def __init__(self, width, ff, experts, top, limit=math.inf, alpha=1.0,
-                 shift=0.0):
+    def __init__(self, width, ff, experts, routing, limit=math.inf, alpha=1.0,
+                 shift=0.0, bias_name="router.b"):
         super().__init__()
-        if experts > sv.MAX_EXPERTS or not 1 <= top <= min(experts, 64):
-            raise ValueError(f"{top} of {experts} experts")
-        self.top, self.act = top, (alpha, limit, shift)
+        self.routing = sv.Routing(routing) if isinstance(routing, int) \
+            else routing
+        self.routing.check(experts)
+        self.act, self.bias_name = (alpha, limit, shift), bias_name
         self.router = nn.Parameter(
             torch.randn(experts, width) * width ** -0.5)
         self.bias = nn.Parameter(torch.zeros(experts))
@@ -354,7 +552,7 @@ class ExpertsMLP(nn.Module):
 
     def load(self, get, prefix):
         copy_weight(self.router, get(prefix + "router"))
-        copy_weight(self.bias, get(prefix + "router.b"))
+        copy_weight(self.bias, get(prefix + self.bias_name))
         for e, (gu, down) in enumerate(zip(self.gate_up, self.down)):
             p = f"{prefix}e{e}."
             copy_weight(gu, torch.cat([get(p + "gate"), get(p + "up")]))
@@ -362,4 +560,25 @@ class ExpertsMLP(nn.Module):
 
     def forward(self, h) -> sv.Pending:
         return sv.moe_mlp(h, sv.linear_f32(h, self.router), self.bias,
-                          self.gate_up, self.down, self.top, *self.act)
+                          self.gate_up, self.down, self.routing, *self.act)
+
+
+class TokenSide(nn.Module):
+    """A vector of the token, of this layer's columns of a table, gated by the
+    stream: proj(gelu(gate x) * table[token]), normed on its way into the
+    stream.  The table belongs to the model."""
+
+    def __init__(self, width, dim, layer):
+        super().__init__()
+        self.at = layer * dim
+        self.gate, self.proj = _column(width, dim), _row(dim, width)
+        self.norm = _vector(width)
+
+    def load(self, get, prefix):
+        copy_weight(self.gate.weight, get(prefix + "gate"))
+        copy_weight(self.proj.weight, get(prefix + "proj"))
+        copy_weight(self.norm, get(prefix + "norm"))
+
+    def forward(self, x, table, tokens) -> sv.Pending:
+        g = sv.gelu_rows_(self.gate(x), table, tokens, self.at)
+        return sv.Pending(self.proj(g), w1=self.norm)

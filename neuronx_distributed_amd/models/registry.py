@@ -159,3 +159,20 @@ def _nesilorn_build(config):
 register_model("Nesilorn", ModelEntry(
     _nesilorn_config, _nesilorn_build,
     lambda model, tensors: model.load_checkpoint(tensors)))
+
+
+def _sutuvik_config(d: dict):
+    from .sutuvik import SutuvikConfig
+
+    return SutuvikConfig.from_dict(d)
+
+
+def _sutuvik_build(config):
+    from .sutuvik import SutuvikForCausalLM
+
+    return SutuvikForCausalLM(config)
+
+
+register_model("Sutuvik", ModelEntry(
+    _sutuvik_config, _sutuvik_build,
+    lambda model, tensors: model.load_checkpoint(tensors)))

@@ -37,14 +37,6 @@ struct LatentAppendArgs {
   float eps;
 };
 
-// The angle is reduced in double, so its error does not grow with the
-// position.
-__device__ __forceinline__ void turn(double f, int p, float* c, float* s) {
-  const double a = f * p;
-  const double r = a - rint(a * 0.15915494309189535) * 6.283185307179586;
-  sincosf((float)r, s, c);
-}
-
 template <typename T>
 __global__ void __launch_bounds__(256)
 latent_append_kernel(LatentAppendArgs a) {

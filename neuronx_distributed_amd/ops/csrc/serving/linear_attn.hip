@@ -3,7 +3,7 @@
 //   S_t = a_t S_(t-1) + b_t k_t v_t^T,    o_t = S_t^T q_t
 //
 // per head, with a 32-bit state S [D][E] per (slot, head) that lives across
-// steps.  Two gatings share the kernels:
+// steps.  Three gatings share the kernels:
 //
 //   decay  a_t = decay_h, b_t = 1; q, k and v pass through silu.
 //   gated  log gates i, f from a projection, soft-capped:
@@ -13,6 +13,10 @@
 //            b_t = exp(i - m_t), n_t = a_t n_(t-1) + b_t k_t,
 //            o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6);
 //          q is scaled by qscale.  S, n and m are zero at position 0.
+//   timed  a time step from a projection (state-space duality):
+//            b_t = softplus(x + bias), a_t = exp(-exp(A_log) b_t),
+//          heads share q and k in groups, o_t + skip v_t is multiplied by
+//          silu(z).
 //
 //   sv_memory_steps   token after token; single-token decoding, the 32-bit
 //                     mode and sizes the chunk kernels do not take
@@ -28,11 +32,14 @@
 
 #define GATED_EPS 1e-6f
 
+enum Gating { DECAY = 0, GATED = 1, TIMED = 2 };
+
 struct MemoryArgs {
   const void *q, *k, *v;    // first row of the step's projections
   long qst, kst, vst;       // row strides (elements)
-  const float* gates;       // [T][2 H] raw i then f (gated)
-  const void *ib, *fb;      // [H] gate biases, T (gated)
+  const float* gates;       // [T][2 H] raw i then f (gated); [T][H] (timed)
+  const void *ib, *fb;      // [H] biases, T: of i and f (gated); of the time
+                            //   step, and A_log (timed)
   const float* decay;       // [H] (decay)
   const float* log2_decay;  // [H] (decay)
   float* S;                 // [slots][H][D][E]
@@ -42,7 +49,20 @@ struct MemoryArgs {
   void* out;                // [T][H * E]
   int H, D, E;
   float gate_cap, qscale;
+  // timed only
+  int G;                    // heads of q and k
+  const void* skip;         // [H], T
+  const void* z;            // [T][H * E] rows
+  long zst;
+  // q, k and v of single tokens before their causal convolution (steps only)
+  const void *cw, *cb;      // [taps][C], [C]; cw null: they have passed it
+  void* ring;               // [slots][taps][C]: position p in place p % taps
+  int taps, C, kch, qch;    // channels of v, k, q start at 0, kch, qch
 };
+
+__device__ __forceinline__ float softplus_f(float x) {
+  return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
+}
 
 __device__ __forceinline__ void log_gates(const MemoryArgs& a, long row,
                                           int h, float ib, float fb,
@@ -55,7 +75,7 @@ __device__ __forceinline__ void log_gates(const MemoryArgs& a, long row,
 // ---------------------------------------------------------------------------
 // token after token: a workgroup owns 32 columns of one head's state
 // ---------------------------------------------------------------------------
-template <typename T, int NI, bool GATED, bool VEC>
+template <typename T, int NI, int GATE, bool VEC>
 __global__ void __launch_bounds__(256)
 memory_steps_kernel(MemoryArgs a) {
   const int D = a.D, E = a.E;
@@ -92,17 +112,34 @@ memory_steps_kernel(MemoryArgs a) {
   // n: dim d belongs to thread d (and d + 256)
   constexpr int NN = (NI * 32 + 255) / 256;
   float n[NN], m = 0.f, ib = 0.f, fb = 0.f;
-  if (GATED) {
+  if (GATE == GATED) {
 #pragma unroll
     for (int i = 0; i < NN; ++i) {
       const int d = tid + 256 * i;
       n[i] = ctx > 0 && d < D ? a.n[((slot * a.H + h) * nt + vt) * D + d] : 0.f;
     }
     if (ctx > 0) m = a.m[(slot * a.H + h) * nt + vt];
+  }
+  if (GATE != DECAY) {
     ib = to_f(((const T*)a.ib)[h]);
     fb = to_f(((const T*)a.fb)[h]);
   }
-  const float decay = GATED ? 0.f : a.decay[h];
+  const float decay = GATE == DECAY ? a.decay[h] : 0.f;
+  const int hk = GATE == TIMED ? h / (a.H / a.G) : h;   // head of q and k
+  const bool conv = GATE == TIMED && a.cw;
+  // channel c of a single token after its convolution; `keep` writes the
+  // token's own input into the ring
+  auto convolve = [&](float x, int c, bool keep) {
+    const int last = a.taps - 1;
+    T* ring = (T*)a.ring + slot * a.taps * a.C + c;
+    const T* w = (const T*)a.cw + c;
+    float y = to_f(((const T*)a.cb)[c]) + to_f(w[(long)last * a.C]) * x;
+    for (int k = max(0, last - ctx); k < last; ++k)
+      y += to_f(w[(long)k * a.C]) *
+           to_f(ring[(long)((ctx - last + k) % a.taps) * a.C]);
+    if (keep) from_f(ring[(long)(ctx % a.taps) * a.C], x);
+    return silu_f(y);
+  };
 
   for (int t = 0; t < nrow; ++t) {
     const long row = row0 + t;
@@ -110,10 +147,15 @@ memory_steps_kernel(MemoryArgs a) {
     for (int d = tid; d < NI * 32; d += 256) {
       float x = 0.f, y = 0.f;
       if (d < D) {
-        x = to_f(((const T*)a.q)[row * a.qst + (long)h * D + d]);
-        y = to_f(((const T*)a.k)[row * a.kst + (long)h * D + d]);
-        if (GATED) x *= a.qscale;
-        else { x = silu_f(x); y = silu_f(y); }
+        x = to_f(((const T*)a.q)[row * a.qst + (long)hk * D + d]);
+        y = to_f(((const T*)a.k)[row * a.kst + (long)hk * D + d]);
+        if (GATE == GATED) x *= a.qscale;
+        if (GATE == DECAY) { x = silu_f(x); y = silu_f(y); }
+        if (conv) {
+          const bool keep = vt == 0 && h % (a.H / a.G) == 0;
+          x = convolve(x, a.qch + hk * D + d, keep);
+          y = convolve(y, a.kch + hk * D + d, keep);
+        }
       }
       sq[b][d] = x;
       sk[b][d] = y;
@@ -122,10 +164,16 @@ memory_steps_kernel(MemoryArgs a) {
       const int e = vt * 32 + tid;
       float x = e < E ? to_f(((const T*)a.v)[row * a.vst + (long)h * E + e])
                       : 0.f;
-      sv[b][tid] = GATED ? x : silu_f(x);
+      if (GATE == DECAY) x = silu_f(x);
+      if (conv && e < E) x = convolve(x, h * E + e, true);
+      sv[b][tid] = x;
     }
     float fs = decay, is = 1.f;
-    if (GATED) {
+    if (GATE == TIMED) {
+      is = softplus_f(a.gates[row * a.H + h] + ib);
+      fs = expf(-expf(fb) * is);
+    }
+    if (GATE == GATED) {
       float gi, gf;
       log_gates(a, row, h, ib, fb, gi, gf);
       const float mn = fmaxf(gf + m, gi);
@@ -153,7 +201,7 @@ memory_steps_kernel(MemoryArgs a) {
     if (lane < 8)
 #pragma unroll
       for (int j = 0; j < 4; ++j) red[b][wid][4 * vq + j] = o[j];
-    if (GATED) {
+    if (GATE == GATED) {
       float nq = 0.f;
 #pragma unroll
       for (int i = 0; i < NN; ++i) {
@@ -170,9 +218,14 @@ memory_steps_kernel(MemoryArgs a) {
     if (tid < 32 && vt * 32 + tid < E) {
       float r = red[b][0][tid] + red[b][1][tid] + red[b][2][tid] +
                 red[b][3][tid];
-      if (GATED) {
+      if (GATE == GATED) {
         const float nq = redn[b][0] + redn[b][1] + redn[b][2] + redn[b][3];
         r /= fmaxf(fabsf(nq), expf(-m)) + GATED_EPS;
+      }
+      if (GATE == TIMED) {
+        const long at = (long)h * E + vt * 32 + tid;
+        r += to_f(((const T*)a.skip)[h]) * sv[b][tid];
+        r *= silu_f(to_f(((const T*)a.z)[row * a.zst + at]));
       }
       from_f(((T*)a.out)[row * a.H * E + (long)h * E + vt * 32 + tid], r);
     }
@@ -190,7 +243,7 @@ memory_steps_kernel(MemoryArgs a) {
         if (e0 + j < E) Sp[(long)d * E + e0 + j] = S[i][j];
     }
   }
-  if (GATED) {
+  if (GATE == GATED) {
 #pragma unroll
     for (int i = 0; i < NN; ++i) {
       const int d = tid + 256 * i;
@@ -200,11 +253,11 @@ memory_steps_kernel(MemoryArgs a) {
   }
 }
 
-template <typename T, bool GATED>
+template <typename T, int GATE>
 static int launch_steps(const MemoryArgs& a, int n_seg, hipStream_t stream) {
   const long grid = (long)n_seg * a.H * ((a.E + 31) / 32);
   const bool vec = a.E % 4 == 0;
-#define MS(N, V) memory_steps_kernel<T, N, GATED, V><<<grid, 256, 0, stream>>>(a)
+#define MS(N, V) memory_steps_kernel<T, N, GATE, V><<<grid, 256, 0, stream>>>(a)
 #define MSV(N) do { if (vec) MS(N, true); else MS(N, false); } while (0)
   if (a.D <= 64) MSV(2);
   else if (a.D <= 128) MSV(4);
@@ -216,14 +269,15 @@ static int launch_steps(const MemoryArgs& a, int n_seg, hipStream_t stream) {
   return (int)hipGetLastError();
 }
 
-extern "C" int sv_memory_steps(const MemoryArgs* a, int n_seg, int gated,
+extern "C" int sv_memory_steps(const MemoryArgs* a, int n_seg, int gating,
                                int f32, hipStream_t stream) {
   if (n_seg <= 0) return 0;
-  if (f32)
-    return gated ? launch_steps<float, true>(*a, n_seg, stream)
-                 : launch_steps<float, false>(*a, n_seg, stream);
-  return gated ? launch_steps<short, true>(*a, n_seg, stream)
-               : launch_steps<short, false>(*a, n_seg, stream);
+#define MS(T)                                                          \
+  (gating == GATED   ? launch_steps<T, GATED>(*a, n_seg, stream)       \
+   : gating == TIMED ? launch_steps<T, TIMED>(*a, n_seg, stream)       \
+                     : launch_steps<T, DECAY>(*a, n_seg, stream))
+  return f32 ? MS(float) : MS(short);
+#undef MS
 }
 
 
@@ -245,7 +299,8 @@ extern "C" int sv_memory_steps(const MemoryArgs* a, int n_seg, int gated,
 //
 // every exponent is <= 0.  b is kept per 64 tokens (with the four totals of
 // a chunk), so near tokens never cancel large sums.  The plain decay has
-// e^(b_t - b_s + i_s - m_t) = decay^(t-s) and no m.
+// e^(b_t - b_s + i_s - m_t) = decay^(t-s) and no m; the timed gating has
+// e^(b_t - b_s) times the time step of s, and no m.
 //
 // 32-bit operands meet bf16 ones exactly: an f32 value is split into three
 // bf16 planes (8 + 8 + 8 bits) and each plane is multiplied on its own.
@@ -261,8 +316,9 @@ struct ChunkArgs {
                             //   or not the first chunk of its segment
   const int* first;         // [n_seg + 1] first chunk of a segment
   int n_chunks, n_seg, T;
-  float *b, *i, *c;         // [H][T] (gated)
-  float *tot, *cend;        // [n_chunks][H][4], [n_chunks][H] (gated)
+  float *b, *i, *c;         // [H][T] (gated; timed: i is the step, no c)
+  float *tot, *cend;        // [n_chunks][H][4], [n_chunks][H] (gated; timed:
+                            //   no cend)
   float* U;                 // [n_chunks][H][E][D]
   float* N;                 // [n_chunks][H][D] (gated): N, then n before
   short* P;                 // [n_chunks][H][3][E][D] state before the chunk
@@ -301,6 +357,7 @@ __device__ __forceinline__ uint4v silu8(uint4v u) {
 }
 
 // ---- gates: one block per (chunk, head), one thread per token -------------
+template <int GATE>
 __global__ void __launch_bounds__(MC_L)
 memory_gates_kernel(ChunkArgs x) {
   const MemoryArgs& a = x.a;
@@ -308,9 +365,16 @@ memory_gates_kernel(ChunkArgs x) {
   const int row0 = x.chunks[4 * ch + 1], nrow = x.chunks[4 * ch + 2];
   const int t = threadIdx.x, lane = t & 63, wid = t >> 6;
   float i = -INFINITY, f = 0.f;
-  if (t < nrow)
-    log_gates(a, row0 + t, h, bits2f(((const short*)a.ib)[h]),
-              bits2f(((const short*)a.fb)[h]), i, f);
+  const float ib = bits2f(((const short*)a.ib)[h]);
+  const float fb = bits2f(((const short*)a.fb)[h]);
+  if (t < nrow) {
+    if (GATE == TIMED) {
+      i = softplus_f(a.gates[(long)(row0 + t) * a.H + h] + ib);
+      f = -expf(fb) * i;
+    } else {
+      log_gates(a, row0 + t, h, ib, fb, i, f);
+    }
+  }
   float F = f, I = i;                    // scan of (F, I) by (+, max)
 #pragma unroll
   for (int off = 1; off < 64; off <<= 1) {
@@ -333,15 +397,15 @@ memory_gates_kernel(ChunkArgs x) {
     const long o = (long)h * x.T + row0 + t;
     x.b[o] = F;
     x.i[o] = i;
-    x.c[o] = c;
+    if (GATE == GATED) x.c[o] = c;
   }
   const long ci = (long)ch * a.H + h;
   if (lane == 63) x.tot[ci * 4 + wid] = F;
-  if (t == MC_L - 1) x.cend[ci] = c;
+  if (GATE == GATED && t == MC_L - 1) x.cend[ci] = c;
 }
 
 // ---- states: U of a chunk, 64 columns per workgroup ------------------------
-template <int DP, bool GATED>
+template <int DP, int GATE>
 __global__ void __launch_bounds__(256)
 memory_states_kernel(ChunkArgs x) {
   constexpr int CPR = DP / 8, PAIRS = 32 * CPR / 256;
@@ -364,18 +428,20 @@ memory_states_kernel(ChunkArgs x) {
   {
     float w = 0.f;
     if (tid < nrow) {
-      if (GATED) {
+      if (GATE != DECAY) {
         const long o = (long)h * x.T + row0 + tid;
         float d = x.tot[ci * 4 + wid] - x.b[o];
         for (int j = wid + 1; j < 4; ++j) d += x.tot[ci * 4 + j];
-        w = expf(d + (x.i[o] - x.cend[ci]));
+        w = GATE == TIMED ? expf(d) * x.i[o]
+                          : expf(d + (x.i[o] - x.cend[ci]));
       } else {
         w = __builtin_amdgcn_exp2f((nrow - 1 - tid) * a.log2_decay[h]);
       }
     }
     s_w[tid] = w;
   }
-  const short* kp = (const short*)a.k + (long)h * D;
+  const int hk = GATE == TIMED ? h / (a.H / a.G) : h;
+  const short* kp = (const short*)a.k + (long)hk * D;
   const short* vp = (const short*)a.v + (long)h * E + e0;
   const uint4v zero = {0, 0, 0, 0};
   uint4v kreg[2 * PAIRS], vreg[2];
@@ -401,7 +467,7 @@ memory_states_kernel(ChunkArgs x) {
   };
   f32x16 acc[NT] = {};
   float nacc = 0.f;
-  const bool with_n = GATED && et == 0;
+  const bool with_n = GATE == GATED && et == 0;
   issue(0);
   for (int c0 = 0; c0 < nrow; c0 += 64) {
     __syncthreads();
@@ -410,10 +476,10 @@ memory_states_kernel(ChunkArgs x) {
       const int it = p * 256 + tid;
       const int r = it / CPR * 2, c = it % CPR * 8;
       union { uint4v u; unsigned short s[8]; } y0, y1;
-      y0.u = silu8<!GATED>(kreg[2 * p]);
-      y1.u = silu8<!GATED>(kreg[2 * p + 1]);
+      y0.u = silu8<GATE == DECAY>(kreg[2 * p]);
+      y1.u = silu8<GATE == DECAY>(kreg[2 * p + 1]);
       const TileWrite tw(c, r);
-      if (!GATED && et == 0 && c < D) {
+      if (GATE == DECAY && et == 0 && c < D) {
         short* ka = x.KA + ((long)(row0 + c0 + r) * a.H + h) * D + c;
         if (c0 + r < nrow) *(uint4v*)ka = y0.u;
         if (c0 + r + 1 < nrow) *(uint4v*)(ka + (long)a.H * D) = y1.u;
@@ -424,8 +490,8 @@ memory_states_kernel(ChunkArgs x) {
     }
     {
       float f0[8], f1[8];
-      unpack8(silu8<!GATED>(vreg[0]), f0);
-      unpack8(silu8<!GATED>(vreg[1]), f1);
+      unpack8(silu8<GATE == DECAY>(vreg[0]), f0);
+      unpack8(silu8<GATE == DECAY>(vreg[1]), f1);
       const float w0 = s_w[c0 + v_r], w1 = s_w[c0 + v_r + 1];
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
@@ -491,7 +557,7 @@ memory_states_kernel(ChunkArgs x) {
 }
 
 // ---- scan over the chunks of a segment: tiles of 64 keys x 16 columns ------
-template <bool GATED>
+template <int GATE>
 __global__ void __launch_bounds__(256)
 memory_scan_kernel(ChunkArgs x) {
   const MemoryArgs& a = x.a;
@@ -519,10 +585,10 @@ memory_scan_kernel(ChunkArgs x) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) S[j] = tr[(tid & 15) * 4 + j][tid >> 4];
     __syncthreads();
-    if (GATED) m = a.m[(slot * a.H + h) * nt];
+    if (GATE == GATED) m = a.m[(slot * a.H + h) * nt];
   }
   // the first column tile also carries n
-  const bool with_n = GATED && et == 0 && tid < 64 && dt * 64 + tid < D;
+  const bool with_n = GATE == GATED && et == 0 && tid < 64 && dt * 64 + tid < D;
   float n = 0.f;
   const long nat = (slot * a.H + h) * nt * D + dt * 64 + tid;
   if (with_n && ctx > 0) n = a.n[nat];
@@ -531,7 +597,7 @@ memory_scan_kernel(ChunkArgs x) {
   constexpr int PF = 4;
   __shared__ float s_b[64], s_c[64];
   const int c0 = x.first[sg], c1 = x.first[sg + 1];
-  const float l2d = GATED ? 0.f : a.log2_decay[h];
+  const float l2d = GATE == DECAY ? a.log2_decay[h] : 0.f;
   const long at = (long)e * D + d, step = (long)a.H * E * D;
   const float* Up = x.U + ((long)c0 * a.H + h) * E * D + at;
   f32x4 Un[PF] = {};
@@ -542,10 +608,11 @@ memory_scan_kernel(ChunkArgs x) {
     __syncthreads();
     if (tid < 64 && cb + tid < c1) {
       const long ci = (long)(cb + tid) * a.H + h;
-      if (GATED) {
+      if (GATE != DECAY) {
         const float* tt = x.tot + ci * 4;
-        s_b[tid] = tt[0] + tt[1] + tt[2] + tt[3];
-        s_c[tid] = x.cend[ci];
+        const float b = tt[0] + tt[1] + tt[2] + tt[3];
+        s_b[tid] = GATE == TIMED ? expf(b) : b;
+        if (GATE == GATED) s_c[tid] = x.cend[ci];
       } else {
         s_b[tid] = __builtin_amdgcn_exp2f(x.chunks[4 * (cb + tid) + 2] * l2d);
       }
@@ -570,7 +637,7 @@ memory_scan_kernel(ChunkArgs x) {
             *(uint2*)(x.P + (ci * 3 + z) * E * D + at) = uint2{w0[z], w1[z]};
         }
         float fs, us = 1.f;
-        if (GATED) {
+        if (GATE == GATED) {
           const float bm = s_b[ch - cb] + m;
           const float mn = fmaxf(bm, s_c[ch - cb]);
           fs = expf(bm - mn);
@@ -603,7 +670,7 @@ memory_scan_kernel(ChunkArgs x) {
 }
 
 // ---- outputs: 128 queries x VT columns per workgroup -----------------------
-template <int DP, int VT, bool GATED>
+template <int DP, int VT, int GATE>
 __global__ void __launch_bounds__(256, DP <= 128 || VT <= 64 ? 2 : 1)
 memory_outputs_kernel(ChunkArgs x) {
   constexpr int NC = DP / 16, NB = VT / 32;
@@ -619,7 +686,7 @@ memory_outputs_kernel(ChunkArgs x) {
   const int h = blockIdx.x / nt / 2 % a.H, ch = blockIdx.x / nt / 2 / a.H;
   const int row0 = x.chunks[4 * ch + 1], nrow = x.chunks[4 * ch + 2];
   const bool carried = x.chunks[4 * ch + 3];
-  if (GATED && et == 0 && half == 0) {
+  if (GATE == GATED && et == 0 && half == 0) {
     // m after the portion: nothing reads the slot's m any more
     const int sg = x.chunks[4 * ch];
     if (ch == x.first[sg + 1] - 1) {
@@ -644,40 +711,41 @@ memory_outputs_kernel(ChunkArgs x) {
       buf[KV_B > ST_B ? KV_B : ST_B];
   char* kb = buf;
   short* vb = (short*)(buf + 64 * KP);
-  __shared__ float s_col[64];
-  __shared__ float s_n[GATED ? DP : 1];
+  __shared__ float s_col[64], s_step[GATE == TIMED ? 64 : 1];
+  __shared__ float s_n[GATE == GATED ? DP : 1];
   auto kswz = [](int row, int byte) {
     return CPR >= 16 ? swz16(row, byte) : swz(row, byte);
   };
 
+  const int hk = GATE == TIMED ? h / (a.H / a.G) : h;
   frag_u qf[NC];
   {
     const short* src = (const short*)a.q + (long)(row0 + min(t, nrow - 1)) *
-                       a.qst + (long)h * D;
+                       a.qst + (long)hk * D;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       const int d = c * 16 + hi * 8;
-      qf[c].u4 = d < D ? silu8<!GATED>(*(const uint4v*)(src + d))
+      qf[c].u4 = d < D ? silu8<GATE == DECAY>(*(const uint4v*)(src + d))
                        : uint4v{0, 0, 0, 0};
     }
   }
   // row terms of the weights
   float row = 0.f, inter, em = 0.f, l2d = 0.f;
-  const float qs = GATED ? a.qscale : 1.f;
+  const float qs = GATE == GATED ? a.qscale : 1.f;
   float tot[4];
-  if (GATED) {
+  if (GATE != DECAY) {
     const long o = (long)h * x.T + row0 + min(t, nrow - 1);
-    float before = x.mst[ci];
+    float before = GATE == GATED ? x.mst[ci] : 0.f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       tot[j] = x.tot[ci * 4 + j];
       if (j < jt) before += tot[j];
     }
     const float bt = x.b[o];
-    const float mt = fmaxf(bt + before, x.c[o]);
+    const float mt = GATE == GATED ? fmaxf(bt + before, x.c[o]) : 0.f;
     inter = __expf(bt + before - mt) * qs;
     row = bt - mt;
-    em = expf(-mt);
+    if (GATE == GATED) em = expf(-mt);
   } else {
     l2d = a.log2_decay[h];
     inter = __builtin_amdgcn_exp2f((t + 1) * l2d);
@@ -687,7 +755,7 @@ memory_outputs_kernel(ChunkArgs x) {
   float den = 0.f;
   if (carried) {
     // the carried state: its planes pass through LDS 32 columns at a time
-    if (GATED) {
+    if (GATE == GATED) {
       for (int d = tid; d < DP; d += 256)
         s_n[d] = d < D ? x.N[ci * D + d] : 0.f;
     }
@@ -729,7 +797,7 @@ memory_outputs_kernel(ChunkArgs x) {
         }
       ot[nb] *= inter;
     }
-    if (GATED) {
+    if (GATE == GATED) {
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
         float qv[8];
@@ -742,12 +810,12 @@ memory_outputs_kernel(ChunkArgs x) {
   }
 
   // ---- keys of the chunk, 64 at a time, from the newest back ---------------
-  const short* kp = (GATED ? (const short*)a.k : x.KA) + (long)h * D;
-  const long kst = GATED ? a.kst : (long)a.H * D;
+  const short* kp = (GATE == DECAY ? x.KA : (const short*)a.k) + (long)hk * D;
+  const long kst = GATE == DECAY ? (long)a.H * D : a.kst;
   const short* vp = x.VT + (ci * E + e0) * MC_L;
   const uint4v zero = {0, 0, 0, 0};
   uint4v kreg[2 * PAIRS], vreg[VN];
-  float colr = 0.f;
+  float colr = 0.f, stepr = 0.f;
   auto issue = [&](int J) {
     const int c0 = 64 * J;
 #pragma unroll
@@ -763,11 +831,13 @@ memory_outputs_kernel(ChunkArgs x) {
       vreg[p] = e0 + e < E
           ? *(const uint4v*)(vp + (long)e * MC_L + c0 + 8 * (tid & 7)) : zero;
     }
-    if (GATED && tid < 64) {
+    if (GATE != DECAY && tid < 64) {
       colr = -INFINITY;
+      stepr = 0.f;
       if (c0 + tid < nrow) {
         const long o = (long)h * x.T + row0 + c0 + tid;
-        colr = x.i[o] - x.b[o];
+        stepr = x.i[o];
+        colr = GATE == TIMED ? -x.b[o] : stepr - x.b[o];
       }
     }
   };
@@ -785,14 +855,15 @@ memory_outputs_kernel(ChunkArgs x) {
 #pragma unroll
     for (int p = 0; p < VN; ++p)
       *(uint4v*)(vb + tslot((p * 256 + tid) >> 3, 8 * (tid & 7))) = vreg[p];
-    if (GATED && tid < 64) s_col[tid] = colr;
+    if (GATE != DECAY && tid < 64) s_col[tid] = colr;
+    if (GATE == TIMED && tid < 64) s_step[tid] = stepr;
     __syncthreads();
     if (J > 0) issue(J - 1);
     if (J > jt || half * 128 + wid * 32 >= nrow) continue;  // wave-uniform
 
     // row part of the exponent for keys of group J
     float base = row;
-    if (GATED && J < jt) {
+    if (GATE != DECAY && J < jt) {
 #pragma unroll
       for (int j = 0; j < 4; ++j)
         if (j >= J && j < jt) base += tot[j];
@@ -813,11 +884,12 @@ memory_outputs_kernel(ChunkArgs x) {
       for (int r = 0; r < 16; ++r) {
         const int s = 32 * k2 + acc_row(r, hi);
         float w;
-        if (GATED) w = __expf(base + s_col[s]) * qs;
+        if (GATE == TIMED) w = __expf(base + s_col[s]) * s_step[s];
+        else if (GATE == GATED) w = __expf(base + s_col[s]) * qs;
         else w = __builtin_amdgcn_exp2f((float)(t - 64 * J - s) * l2d);
         if (J == jt && 64 * J + s > t) w = 0.f;
         acc[r] *= w;
-        if (GATED) den += acc[r];
+        if (GATE == GATED) den += acc[r];
       }
 #pragma unroll
       for (int cc = 0; cc < 2; ++cc) {
@@ -844,52 +916,63 @@ memory_outputs_kernel(ChunkArgs x) {
   }
 
   float inv = 1.f;
-  if (GATED) {
+  if (GATE == GATED) {
     den += __shfl_xor(den, 32, 64);
     inv = 1.f / (fmaxf(fabsf(den), em) + GATED_EPS);
   }
   if (t >= nrow) return;
+  const float skip = GATE == TIMED ? bits2f(((const short*)a.skip)[h]) : 0.f;
   short* dst = (short*)a.out + ((long)(row0 + t) * a.H + h) * E + e0;
 #pragma unroll
   for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
     for (int rg = 0; rg < 4; ++rg) {
       const int e = 32 * nb + 8 * rg + 4 * hi;
-      if (e0 + e < E)
-        *(uint2*)(dst + e) =
-            uint2{pack_bf16x2(ot[nb][4 * rg] * inv, ot[nb][4 * rg + 1] * inv),
-                  pack_bf16x2(ot[nb][4 * rg + 2] * inv,
-                              ot[nb][4 * rg + 3] * inv)};
+      if (e0 + e >= E) continue;
+      float o[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) o[j] = ot[nb][4 * rg + j] * inv;
+      if (GATE == TIMED) {
+        float v[4], z[4];
+        const long at = (long)h * E + e0 + e;
+        load4((const short*)a.v + (long)(row0 + t) * a.vst + at, v);
+        load4((const short*)a.z + (long)(row0 + t) * a.zst + at, z);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[j] = (o[j] + skip * v[j]) * silu_f(z[j]);
+      }
+      *(uint2*)(dst + e) = uint2{pack_bf16x2(o[0], o[1]),
+                                 pack_bf16x2(o[2], o[3])};
     }
 }
 
 // wider column tiles read the keys less often, as long as the accumulators
 // leave registers for two workgroups per CU
-template <int DP, bool GATED>
+template <int DP, int GATE>
 static void launch_chunks(const ChunkArgs& x, hipStream_t stream) {
   const MemoryArgs& a = x.a;
   const long ch = (long)x.n_chunks * a.H;
-  if (GATED) memory_gates_kernel<<<ch, MC_L, 0, stream>>>(x);
-  memory_states_kernel<DP, GATED>
+  if (GATE != DECAY) memory_gates_kernel<GATE><<<ch, MC_L, 0, stream>>>(x);
+  memory_states_kernel<DP, GATE>
       <<<ch * ((a.E + 63) / 64), 256, 0, stream>>>(x);
-  memory_scan_kernel<GATED><<<(long)x.n_seg * a.H * ((a.D + 63) / 64) *
-                                  ((a.E + 15) / 16), 256, 0, stream>>>(x);
+  memory_scan_kernel<GATE><<<(long)x.n_seg * a.H * ((a.D + 63) / 64) *
+                                 ((a.E + 15) / 16), 256, 0, stream>>>(x);
   if (a.E <= 64 || DP > 128)
-    memory_outputs_kernel<DP, 64, GATED>
+    memory_outputs_kernel<DP, 64, GATE>
         <<<ch * 2 * ((a.E + 63) / 64), 256, 0, stream>>>(x);
   else
-    memory_outputs_kernel<DP, (DP > 128 ? 64 : 128), GATED>
+    memory_outputs_kernel<DP, (DP > 128 ? 64 : 128), GATE>
         <<<ch * 2 * ((a.E + 127) / 128), 256, 0, stream>>>(x);
 }
 
 // bf16; D and E multiples of 8 with D <= 256; 16-byte aligned rows
-extern "C" int sv_memory_chunks(const ChunkArgs* x, int gated,
+extern "C" int sv_memory_chunks(const ChunkArgs* x, int gating,
                                 hipStream_t stream) {
   if (x->n_seg <= 0) return 0;
 #define MC(P)                                                     \
   do {                                                            \
-    if (gated) launch_chunks<P, true>(*x, stream);                \
-    else launch_chunks<P, false>(*x, stream);                     \
+    if (gating == GATED) launch_chunks<P, GATED>(*x, stream);     \
+    else if (gating == TIMED) launch_chunks<P, TIMED>(*x, stream); \
+    else launch_chunks<P, DECAY>(*x, stream);                     \
   } while (0)
   if (x->a.D <= 64) MC(64);
   else if (x->a.D <= 128) MC(128);

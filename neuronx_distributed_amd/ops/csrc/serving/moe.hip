@@ -2,8 +2,8 @@
 // matrix products.  Every launch has a size that the host knows from the
 // number of rows alone, so a decode step can be captured in a graph.
 //
-//   sv_moe_route   logits -> chosen experts and softmax weights of each row
-//   sv_moe_plan    (row, choice) pairs grouped by expert: order and tiles
+//   sv_moe_plan    logits -> chosen experts and weights of each row; (row,
+//                  choice) pairs grouped by expert: order and tiles
 //   sv_moe_gemm    one grouped product: gate/up with the gated activation in
 //                  its epilogue, or down
 //
@@ -27,12 +27,61 @@ struct MoePlanArgs {
   int* order;               // [T * top] slot -> pair
   int* tiles;               // [max_tiles][4]: expert, first slot, slots, 0
   int T, E, top, tile_rows, max_tiles;
+  int sigmoid;              // scores sigmoid(z), chosen by score + bias
+  int groups, keep;         // experts of the best groups only (groups > 1)
 };
 
-// One wave, one row: the largest logits in descending order, the lower index
-// first among equals; softmax over the chosen.
+// Keep the choice scores v of the best groups, drop the others.  A group of
+// neighbours counts the sum of its two largest.  `mem` is the wave's own.
+template <int NV>
+__device__ __forceinline__ void best_groups(const MoePlanArgs& a, float* v,
+                                            float* mem) {
+  const int lane = threadIdx.x & 63, size = a.E / a.groups;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) mem[i * 64 + lane] = v[i];
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  float score = -INFINITY;
+  if (lane < a.groups) {
+    float m1 = -INFINITY, m2 = -INFINITY;
+    for (int j = 0; j < size; ++j) {
+      const float x = mem[lane * size + j];
+      m2 = fmaxf(m2, fminf(m1, x));
+      m1 = fmaxf(m1, x);
+    }
+    score = size > 1 ? m1 + m2 : m1;
+  }
+  __builtin_amdgcn_wave_barrier();
+  unsigned long long kept = 0;
+  for (int k = 0; k < a.keep; ++k) {
+    const bool open = lane < a.groups && !(kept >> lane & 1);
+    float best = open ? score : -INFINITY;
+    int at = open ? lane : 64;
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+      const float ob = __shfl_xor(best, off, 64);
+      const int oa = __shfl_xor(at, off, 64);
+      if (ob > best || (ob == best && oa < at)) {
+        best = ob;
+        at = oa;
+      }
+    }
+    kept |= 1ull << (at & 63);
+  }
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int e = i * 64 + lane;
+    if (e < a.E && !(kept >> (e / size) & 1)) v[i] = -INFINITY;
+  }
+}
+
+// One wave, one row: the largest choice scores in descending order, the lower
+// index first among equals.  Choice scores are the logits with their bias, the
+// weights a softmax over the chosen; or sigmoids with a bias, the weights the
+// chosen sigmoids over their sum.
 template <typename T>
-__device__ __forceinline__ void route_row(const MoePlanArgs& a, int t) {
+__device__ __forceinline__ void route_row(const MoePlanArgs& a, int t,
+                                          float* mem) {
   const int lane = threadIdx.x & 63;
   constexpr int NV = MOE_MAX_EXPERTS / 64;
   const T* bias = (const T*)a.bias;
@@ -41,8 +90,13 @@ __device__ __forceinline__ void route_row(const MoePlanArgs& a, int t) {
   for (int i = 0; i < NV; ++i) {
     const int e = i * 64 + lane;
     v[i] = -INFINITY;
-    if (e < a.E) v[i] = a.z[(long)t * a.E + e] + (bias ? to_f(bias[e]) : 0.f);
+    if (e < a.E) {
+      const float z = a.z[(long)t * a.E + e];
+      v[i] = (a.sigmoid ? 1.f / (1.f + expf(-z)) : z) +
+             (bias ? to_f(bias[e]) : 0.f);
+    }
   }
+  if (a.groups > 1) best_groups<NV>(a, v, mem);
   float mine = 0.f, first = 0.f, sum = 0.f;
   int mine_e = 0;
   for (int k = 0; k < a.top; ++k) {
@@ -68,13 +122,15 @@ __device__ __forceinline__ void route_row(const MoePlanArgs& a, int t) {
     for (int i = 0; i < NV; ++i)
       if (at == i * 64 + lane) v[i] = -INFINITY;
     if (k == 0) first = best;
-    const float w = expf(best - first);
+    const float w = a.sigmoid ? 1.f / (1.f + expf(-a.z[(long)t * a.E + at]))
+                              : expf(best - first);
     sum += w;
     if (lane == k) {
       mine = w;
       mine_e = at;
     }
   }
+  if (a.sigmoid) sum += 1e-20f;
   if (lane < a.top) {
     a.idx[(long)t * a.top + lane] = mine_e;
     a.coef[(long)t * a.top + lane] = mine / sum;
@@ -83,8 +139,9 @@ __device__ __forceinline__ void route_row(const MoePlanArgs& a, int t) {
 
 template <typename T>
 __global__ void __launch_bounds__(256) moe_route_kernel(MoePlanArgs a) {
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (t < a.T) route_row<T>(a, t);
+  __shared__ float mem[4][MOE_MAX_EXPERTS];
+  const int wid = threadIdx.x >> 6, t = blockIdx.x * 4 + wid;
+  if (t < a.T) route_row<T>(a, t, mem[wid]);
 }
 
 // One workgroup.  ROUTE: it also routes the (few) rows first.
@@ -92,8 +149,9 @@ template <typename T, bool ROUTE>
 __global__ void __launch_bounds__(1024) moe_plan_kernel(MoePlanArgs a) {
   __shared__ int count[MOE_MAX_EXPERTS], slots[1024], tile_at[1024];
   const int tid = threadIdx.x, E = a.E, pairs = a.T * a.top;
+  __shared__ float mem[ROUTE ? 16 : 1][MOE_MAX_EXPERTS];
   if (ROUTE)
-    for (int t = tid >> 6; t < a.T; t += 16) route_row<T>(a, t);
+    for (int t = tid >> 6; t < a.T; t += 16) route_row<T>(a, t, mem[tid >> 6]);
   for (int e = tid; e < E; e += 1024) count[e] = 0;
   __syncthreads();               // orders the block's own global writes too
   for (int p = tid; p < pairs; p += 1024) atomicAdd(&count[a.idx[p]], 1);
@@ -133,6 +191,9 @@ extern "C" int sv_moe_plan(const MoePlanArgs* a, int f32,
                            hipStream_t stream) {
   if (a->T <= 0) return 0;
   if (a->E > MOE_MAX_EXPERTS || a->top > 64 || a->top > a->E) return 1;
+  if (a->groups < 1 || a->groups > 64 || a->E % a->groups || a->keep < 1 ||
+      a->keep > a->groups || a->keep * (a->E / a->groups) < a->top)
+    return 1;
   const bool fused = a->T <= 64;
   if (!fused) {
     const int grid = (a->T + 3) / 4;

@@ -5,7 +5,13 @@
 // for the query at position i:  j <= i and (i - j < window or j < keep).
 // window <= 0 means plain causal.  Sizes D and E need not be equal.
 //
+// Scores and the softmax may be modified (ScoreArgs): a factor a head, a soft
+// cap, a bias that falls with the distance, a sink in the denominator; the
+// output may pass through one gate a head.
+//
 //   sv_kv_append   writes the K/V rows of a step into their pages
+//   sv_qkv_append  the same with rotation and norm of queries and keys and with
+//                  values mixed with another layer's
 //   sv_attn_rows   one query row per workgroup group: single-token decoding
 //                  (the row's own K/V is appended here) and the 32-bit mode
 //   sv_attn_tiles  MFMA flash kernel over 128-row tiles for prompt portions
@@ -78,6 +84,138 @@ extern "C" int sv_kv_append(const void* k, const void* v, long kst, long vst,
 }
 
 // ---------------------------------------------------------------------------
+// append with what comes before the attention.  LPH lanes own a head of a row
+// (8 elements each).  Queries are changed in place, keys and values go into
+// their pages only.
+// ---------------------------------------------------------------------------
+struct QkvArgs {
+  void* q;
+  const void *k, *v;
+  long qst, kst, vst;
+  const double* freq;       // [rot / 2] radians a position: elements 2i and
+                            //   2i + 1 turn; or null
+  const void *qw, *kw;      // [D] weights of the norm, or null
+  const void* first;        // values to mix in, or null
+  long fst;
+  const void* mix;          // their share (one number)
+  void *kc, *vc;
+  const int *pos, *seq, *bt;
+  int MB, T, H, G, D, E, rot;
+  int norm;                 // queries and keys over their root mean square
+  int temp_every;           // > 0: queries times 1 + coef ln(floor((p + 1) /
+  float temp_coef, eps;     //   every) + 1)
+};
+
+template <typename T, int LPH, bool VEC>
+__global__ void __launch_bounds__(256) qkv_append_kernel(QkvArgs a) {
+  constexpr int PER = 256 / LPH;         // heads of a workgroup
+  const int heads = a.H + 2 * a.G;
+  const long item = (long)blockIdx.x * PER + threadIdx.x / LPH;
+  const long row = min(item / heads, (long)a.T - 1);
+  const bool live = item < (long)a.T * heads;
+  const int hh = item % heads, d0 = threadIdx.x % LPH * 8;
+  const int p = a.pos[row];
+  const long page = a.bt[(long)a.seq[row] * a.MB + p / SV_PAGE];
+  const bool is_q = hh < a.H, is_v = hh >= a.H + a.G;
+  const int g = is_q ? 0 : is_v ? hh - a.H - a.G : hh - a.H;
+  const int size = is_v ? a.E : a.D;
+  const int n = min(8, size - d0);       // elements of this lane; <= 0: none
+  const T* src = is_q   ? (const T*)a.q + row * a.qst + (long)hh * a.D
+                 : is_v ? (const T*)a.v + row * a.vst + (long)g * a.E
+                        : (const T*)a.k + row * a.kst + (long)g * a.D;
+  float x[8];
+  load8<VEC>(src + d0, n, x);
+  if (is_v && a.first) {
+    const float m = to_f(((const T*)a.mix)[0]);
+    float f[8];
+    load8<VEC>((const T*)a.first + row * a.fst + (long)g * a.E + d0, n, f);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = (1.f - m) * x[j] + m * f[j];
+  }
+  if (!is_v && a.freq) {
+#pragma unroll
+    for (int j = 0; j < 8; j += 2) {
+      if (d0 + j >= a.rot) continue;
+      float c, s;
+      turn(a.freq[(d0 + j) / 2], p, &c, &s);
+      const float u = x[j], w = x[j + 1];
+      x[j] = u * c - w * s;
+      x[j + 1] = w * c + u * s;
+    }
+  }
+  if (a.norm) {                          // all lanes: values join the shuffles
+    float sq = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) sq += x[j] * x[j];
+#pragma unroll
+    for (int off = LPH / 2; off > 0; off >>= 1) sq += __shfl_xor(sq, off, 64);
+    if (!is_v) {
+      const float rstd = 1.f / sqrtf(sq / a.D + a.eps);
+      const T* w = (const T*)(is_q ? a.qw : a.kw);
+      float u[8];
+      if (w) load8<VEC>(w + d0, n, u);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] *= w ? rstd * u[j] : rstd;
+    }
+  }
+  if (is_q && a.temp_every > 0) {
+    const float t = 1.f + a.temp_coef * logf((float)((p + 1) / a.temp_every + 1));
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] *= t;
+  }
+  if (!live || n <= 0) return;
+  const long at = (page * a.G + g) * SV_PAGE + p % SV_PAGE;
+  T* dst = is_q   ? (T*)a.q + row * a.qst + (long)hh * a.D
+           : is_v ? (T*)a.vc + at * a.E : (T*)a.kc + at * a.D;
+  if (VEC) {
+    store4(dst + d0, x);
+    store4(dst + d0 + 4, x + 4);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (j < n) from_f(dst[d0 + j], x[j]);
+  }
+}
+
+// D and E at most 512; vec: D, E, strides and bases in 8 elements
+extern "C" int sv_qkv_append(const QkvArgs* a, int vec, int f32,
+                             hipStream_t stream) {
+  if (a->T <= 0) return 0;
+  if (a->rot % 2 || a->rot > a->D) return 1;
+  const int big = a->D > a->E ? a->D : a->E;
+  const long items = (long)a->T * (a->H + 2 * a->G);
+#define QA(T, L, V)                                              \
+  qkv_append_kernel<T, L, V>                                     \
+      <<<(items + 256 / L - 1) / (256 / L), 256, 0, stream>>>(*a)
+#define QAV(L)                                                   \
+  do {                                                           \
+    if (f32) { if (vec) QA(float, L, true); else QA(float, L, false); } \
+    else     { if (vec) QA(short, L, true); else QA(short, L, false); } \
+  } while (0)
+  if (big <= 64) QAV(8);
+  else if (big <= 128) QAV(16);
+  else if (big <= 256) QAV(32);
+  else if (big <= 512) QAV(64);
+  else return 1;
+#undef QAV
+#undef QA
+  return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// scores: s = q.k scale temp_h; s <- cap tanh(s / cap); s <- s - slope_h
+// (i - j); the denominator also holds exp(sink_h); the output of head h is
+// multiplied by sigmoid(gate[row][h]).  What is null or zero is left out.
+// ---------------------------------------------------------------------------
+struct ScoreArgs {
+  const void *temp, *sink;  // [H], T
+  const float* slope;       // [H]
+  const void* gate;         // [rows][H], T
+  long gst;
+  float cap;
+};
+
+// ---------------------------------------------------------------------------
 // rows
 // ---------------------------------------------------------------------------
 struct RowsArgs {
@@ -90,6 +228,7 @@ struct RowsArgs {
   void* out;                   // [rows][H * E]
   int MB, rows, H, G, D, E, splits, append, window, keep;
   float scale;
+  ScoreArgs mod;
 };
 
 // LPR lanes own one key row (DPL dims each); RC query heads share the row.
@@ -128,11 +267,18 @@ attn_rows_kernel(RowsArgs a) {
     const int h = g * rep + min(rc * RC + r, rep - 1);
     load_dims<VEC, DPL>((const T*)a.q + row * a.qst + (long)h * D + d0, nd, qv[r]);
   }
-  const float s2 = a.scale * SV_LOG2E;
+  // scores in units of log 2, of the cap if there is one
+  const float cap = a.mod.cap;
+  const float s2 = cap > 0.f ? a.scale / cap : a.scale * SV_LOG2E;
+  float slope[RC];
 #pragma unroll
-  for (int r = 0; r < RC; ++r)
+  for (int r = 0; r < RC; ++r) {
+    const int h = g * rep + min(rc * RC + r, rep - 1);
+    const float t = a.mod.temp ? s2 * to_f(((const T*)a.mod.temp)[h]) : s2;
+    slope[r] = a.mod.slope ? a.mod.slope[h] * SV_LOG2E : 0.f;
 #pragma unroll
-    for (int j = 0; j < DPL; ++j) qv[r][j] *= s2;
+    for (int j = 0; j < DPL; ++j) qv[r][j] *= t;
+  }
 
   const T* kn = (const T*)a.k + row * a.kst + (long)g * D;
   const T* vn = (const T*)a.v + row * a.vst + (long)g * E;
@@ -169,7 +315,7 @@ attn_rows_kernel(RowsArgs a) {
     load_dims<VEC, DPL>((const T*)a.kc + base * a.kcs + d0, nd, kf);
     load_dims<VEC, DPL>((const T*)a.vc + base * a.vcs + d0, ne, vf);
   };
-  auto absorb = [&](const float* kf, const float* vf, bool live) {
+  auto absorb = [&](const float* kf, const float* vf, bool live, int away) {
     float s[RC];
 #pragma unroll
     for (int r = 0; r < RC; ++r) {
@@ -181,8 +327,12 @@ attn_rows_kernel(RowsArgs a) {
     for (int off = LPR / 2; off > 0; off >>= 1)
 #pragma unroll
       for (int r = 0; r < RC; ++r) s[r] += __shfl_xor(s[r], off, 64);
+    if (cap > 0.f)
+#pragma unroll
+      for (int r = 0; r < RC; ++r) s[r] = cap * SV_LOG2E * tanhf(s[r]);
 #pragma unroll
     for (int r = 0; r < RC; ++r) {
+      s[r] -= slope[r] * away;
       const float mn = live ? fmaxf(m[r], s[r]) : m[r];
       const float al = __builtin_amdgcn_exp2f(m[r] - mn);
       const float p = live ? __builtin_amdgcn_exp2f(s[r] - mn) : 0.f;
@@ -203,7 +353,7 @@ attn_rows_kernel(RowsArgs a) {
 #pragma unroll
     for (int j = 0; j < DPL; ++j) kx[j] = vx[j] = 0.f;
     if (idx + 4 * NR < k1) fetch(idx + 4 * NR, kx, vx);
-    absorb(kf, vf, idx < k1);
+    absorb(kf, vf, idx < k1, i_pos - (idx < nfirst ? idx : lo + idx - nfirst));
 #pragma unroll
     for (int j = 0; j < DPL; ++j) {
       kf[j] = kx[j];
@@ -213,7 +363,7 @@ attn_rows_kernel(RowsArgs a) {
   if (a.append && split == 0 && wid == 0) {
     load_dims<VEC, DPL>(kn + d0, nd, kf);
     load_dims<VEC, DPL>(vn + d0, ne, vf);
-    absorb(kf, vf, sub == 0);
+    absorb(kf, vf, sub == 0, 0);
   }
 
   // fold the NR row groups of the wave, then the 4 waves
@@ -260,6 +410,16 @@ attn_rows_kernel(RowsArgs a) {
       oo += so[w][r][e] * c;
     }
     const int h = g * rep + rc * RC + r;
+    if (a.mod.sink && split == 0) {      // once for all splits
+      const float sink = to_f(((const T*)a.mod.sink)[h]) * SV_LOG2E;
+      const float mn = fmaxf(mm, sink);
+      const float c = __builtin_amdgcn_exp2f(mm - mn);
+      ll = ll * c + __builtin_amdgcn_exp2f(sink - mn);
+      oo *= c;
+      mm = mn;
+    }
+    if (a.mod.gate)
+      oo *= sigmoid_f(to_f(((const T*)a.mod.gate)[row * a.mod.gst + h]));
     if (a.splits == 1) {
       from_f(((T*)a.out)[((long)row * a.H + h) * E + e], oo / ll);
     } else {
@@ -406,6 +566,7 @@ struct TilesArgs {
   int MB, H, G, D, E, DS;   // DS: columns of a key before the shared ones
   int window, keep;
   float scale;
+  ScoreArgs mod;            // its gate is one number a head
 };
 
 // The 16-byte slots of a key row are rotated within groups of eight, so that
@@ -420,7 +581,9 @@ __device__ __forceinline__ int value_turn(int row) {
   return (SLOTS % 16 == 0 ? row & 3 : (row >> 1) & 1) << 2;
 }
 
-template <int DK, int DE, int NP, bool SHARED>
+// MOD: 0 plain scores, 1 with a distance bias, 2 with a soft cap (and the bias,
+// if there is one); a sink and the gates are handled in all.
+template <int DK, int DE, int NP, bool SHARED, int MOD>
 __global__ void __launch_bounds__(256, DE <= 128 ? 2 : 1)
 attn_tiles_kernel(TilesArgs a) {
   constexpr int NC = DK / 16;        // 16-wide chunks of the key size
@@ -457,7 +620,12 @@ attn_tiles_kernel(TilesArgs a) {
 
   f32x16 ot[NB] = {};
   float m_run = NEG_BIG, l_run = 0.f;
-  const float s2 = a.scale * SV_LOG2E;
+  const float s2 = a.scale * SV_LOG2E *
+      (a.mod.temp ? bits2f(((const short*)a.mod.temp)[h]) : 1.f);
+  const float slope = MOD && a.mod.slope ? a.mod.slope[h] * SV_LOG2E : 0.f;
+  // tanh(x) = 1 - 2 / (1 + e^2x), with x in units of log 2 / cap
+  const float cap2 = MOD == 2 ? a.mod.cap * SV_LOG2E : 0.f;
+  const float in_cap = MOD == 2 ? 2.f / a.mod.cap : 0.f;
 
   const int q_hi = p0 + nrow - 1;
   const int t_hi = q_hi / SV_PAGE;
@@ -538,8 +706,21 @@ attn_tiles_kernel(TilesArgs a) {
          kv0 + SV_PAGE > a.keep);
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) acc[kb] *= s2;
+    const int i0 = my_pos - kv0;               // keys up to i0 are not ahead
+    if (MOD == 2)
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int r = 0; r < 16; ++r)
+          acc[kb][r] = cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(
+              1.f + __builtin_amdgcn_exp2f(acc[kb][r] * in_cap));
+    if (MOD == 1 || (MOD == 2 && slope != 0.f))
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int r = 0; r < 16; ++r)
+          acc[kb][r] -= slope * (float)(i0 - 32 * kb - acc_row(r, hi));
     if (masked) {
-      const int i0 = my_pos - kv0;             // keys up to i0 are not ahead
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
@@ -634,7 +815,16 @@ attn_tiles_kernel(TilesArgs a) {
   }
 
   if (my >= nrow) return;
-  const float inv = 1.f / l_run;
+  float inv = 1.f / l_run;
+  if (a.mod.sink) {
+    const float sink = bits2f(((const short*)a.mod.sink)[h]) * SV_LOG2E;
+    const float mn = fmaxf(m_run, sink);
+    const float c = __builtin_amdgcn_exp2f(m_run - mn);
+    inv = c / (l_run * c + __builtin_amdgcn_exp2f(sink - mn));
+  }
+  if (a.mod.gate)
+    inv *= sigmoid_f(bits2f(
+        ((const short*)a.mod.gate)[(long)(row0 + my) * a.mod.gst + h]));
   short* dst = a.out + ((long)(row0 + my) * a.H + h) * E;
 #pragma unroll
   for (int nb = 0; nb < NB; ++nb)
@@ -662,10 +852,16 @@ extern "C" int sv_attn_tiles(const TilesArgs* a, int n_tiles,
                              hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   const dim3 grid(a->H, n_tiles);
-#define AT(K, V)                                                          \
-  do {                                                                    \
-    if (a->kr) attn_tiles_kernel<K, V, 3, true><<<grid, 256, 0, stream>>>(*a); \
-    else attn_tiles_kernel<K, V, 3, false><<<grid, 256, 0, stream>>>(*a); \
+  const int mod = a->mod.cap > 0.f ? 2 : a->mod.slope ? 1 : 0;
+  if (a->kr && mod) return 1;
+#define ATK(K, V, S, M) \
+  attn_tiles_kernel<K, V, 3, S, M><<<grid, 256, 0, stream>>>(*a)
+#define AT(K, V)                          \
+  do {                                    \
+    if (a->kr) ATK(K, V, true, 0);        \
+    else if (mod == 2) ATK(K, V, false, 2); \
+    else if (mod == 1) ATK(K, V, false, 1); \
+    else ATK(K, V, false, 0);             \
   } while (0)
   if (a->D <= 64 && a->E <= 64) AT(64, 64);
   else if (a->D <= 128 && a->E <= 128) AT(128, 128);
@@ -673,6 +869,7 @@ extern "C" int sv_attn_tiles(const TilesArgs* a, int n_tiles,
   else if (a->D <= 256 && a->E <= 256) AT(256, 256);
   else return 1;
 #undef AT
+#undef ATK
   return (int)hipGetLastError();
 }
 

@@ -85,6 +85,15 @@ __device__ __forceinline__ float log_sigmoid_f(float x) {
   return fminf(x, 0.f) - log1pf(expf(-fabsf(x)));
 }
 
+// cos and sin of position p of a pair that turns f radians a position.  The
+// angle is reduced in double, so its error does not grow with the
+// position.
+__device__ __forceinline__ void turn(double f, int p, float* c, float* s) {
+  const double a = f * p;
+  const double r = a - rint(a * 0.15915494309189535) * 6.283185307179586;
+  sincosf((float)r, s, c);
+}
+
 // s-contiguous tile [rows][64] without padding: 16-byte slots are rotated so
 // that both the pairwise transposing writes (fixed row low bits) and the
 // fragment reads (consecutive rows) spread over the banks

@@ -6,10 +6,15 @@
 // [x; x0] that a looped block projects.  The pending result is nothing, one
 // tensor, a weighted sum of several rows a token (expert outputs), or two
 // parallel branches.  One tensor or sum may be RMS-normed before it is added,
-// two branches always are; the result is scaled.
+// two branches always are; the result is scaled.  A norm may run in groups:
+// equal consecutive parts of the row, each over its own root mean square.
+//
+// The normed rows of single tokens may pass a causal convolution over time on
+// their way out (h + conv(h)): the last inputs of their request come from a
+// ring, which takes the new one.
 //
 // gated_norm: RMS norm over groups of a row, times a weight, times
-// sigmoid(gate) — the output stage of the gated recurrent mixers.
+// sigmoid(gate) if there is one — the output stage of the recurrent mixers.
 
 #include "serving.h"
 
@@ -27,9 +32,18 @@ struct ResidualNormArgs {
   void* cat;             // [out_rows, 2 W]: new x, then x0; or null
   const void* x0;        // [rows, W]
   const int* index;      // out row -> row, or null
+  // convolution of the rows from conv_row on, which are single tokens
+  const void* conv;      // [taps][W] weights, or null
+  void* ring;            // [slots][taps][W]: the input at position p is in
+                         //   place p % taps
+  const int* singles;    // [][4]: slot, row, 1, position
+  void* hc;              // [out_rows, W] convolved rows
   int rows_out, W, delta_f32, parts;
+  int groups, p_groups;  // parts of the norm and of the pending result's norm
+  int taps, conv_row;
   float eps, scale;
   float w_base, p_base;  // added to w, and to w1 and w2
+  float h_scale;         // multiplies h
 };
 
 template <typename T, int VEC>
@@ -45,6 +59,7 @@ template <typename T, int VEC>
 __global__ void __launch_bounds__(256)
 residual_norm_kernel(ResidualNormArgs a) {
   extern __shared__ __attribute__((aligned(16))) float row[];  // [W]
+  float* part_rstd = row + a.W;    // [groups], if a norm has several
   __shared__ float red[16];
   const int o = blockIdx.x;
   const long r = a.index ? a.index[o] : o;
@@ -73,6 +88,19 @@ residual_norm_kernel(ResidualNormArgs a) {
     }
   };
 
+  // 1 / rms of each of n parts of the row in LDS
+  auto norm_parts = [&](int n) {
+    const int size = W / n, lane = tid & 63;
+    __syncthreads();
+    for (int g = tid >> 6; g < n; g += 4) {
+      float q = 0.f;
+      for (int i = lane; i < size; i += 64) q += row[g * size + i] * row[g * size + i];
+      q = wave_reduce(q, SumOp());
+      if (lane == 0) part_rstd[g] = 1.f / sqrtf(q / size + a.eps);
+    }
+    __syncthreads();
+  };
+
   float s1 = a.scale, s2 = 0.f;
   if (a.delta2) {
     float q1 = 0.f, q2 = 0.f, v[VEC];
@@ -98,10 +126,15 @@ residual_norm_kernel(ResidualNormArgs a) {
       for (int j = 0; j < VEC; ++j) q1 += v[j] * v[j];
       st<float, VEC>(row + i, v);
     }
-    q1 = block_reduce_sum(q1, red);
-    __syncthreads();
-    s1 = a.scale / sqrtf(q1 / W + a.eps);
+    if (a.p_groups > 1) {
+      norm_parts(a.p_groups);
+    } else {
+      q1 = block_reduce_sum(q1, red);
+      __syncthreads();
+      s1 = a.scale / sqrtf(q1 / W + a.eps);
+    }
   }
+  const int p_size = a.p_groups > 1 ? W / a.p_groups : W;
 
   float sq = 0.f;
   for (int i = tid * VEC; i < W; i += 256 * VEC) {
@@ -122,6 +155,7 @@ residual_norm_kernel(ResidualNormArgs a) {
     } else if (a.w1) {
       ld<float, VEC>(row + i, t);  // written by this same thread
       ld<T, VEC>((const T*)a.w1 + i, u);
+      if (a.p_groups > 1) s1 = a.scale * part_rstd[i / p_size];
 #pragma unroll
       for (int j = 0; j < VEC; ++j) v[j] += t[j] * s1 * (a.p_base + u[j]);
     } else if (a.delta) {
@@ -148,15 +182,50 @@ residual_norm_kernel(ResidualNormArgs a) {
     }
   }
   if (!a.h || !a.w) return;
-  sq = block_reduce_sum(sq, red);
-  const float rstd = 1.f / sqrtf(sq / W + a.eps);
+  float rstd = 0.f;
+  if (a.groups > 1) {
+    norm_parts(a.groups);
+  } else {
+    sq = block_reduce_sum(sq, red);
+    rstd = 1.f / sqrtf(sq / W + a.eps);
+  }
+  const int size = a.groups > 1 ? W / a.groups : W;
+  const bool conv = a.conv && o >= a.conv_row;
+  const int* sg = a.singles + 4L * (o - a.conv_row);
   for (int i = tid * VEC; i < W; i += 256 * VEC) {
     float v[VEC], u[VEC];
     ld<float, VEC>(row + i, v);  // written by this same thread
     ld<T, VEC>((const T*)a.w + i, u);
+    if (a.groups > 1) rstd = part_rstd[i / size];
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) v[j] *= rstd * (a.w_base + u[j]);
-    st<T, VEC>((T*)a.h + (long)o * W + i, v);
+    for (int j = 0; j < VEC; ++j) v[j] *= rstd * (a.w_base + u[j]) * a.h_scale;
+    if (!conv) {
+      st<T, VEC>((T*)a.h + (long)o * W + i, v);
+      continue;
+    }
+    // the ring holds inputs as T, and so enters the row itself
+    const int p = sg[3], last = a.taps - 1;
+    T* ring = (T*)a.ring + (long)sg[0] * a.taps * W + i;
+    const T* cw = (const T*)a.conv + i;
+    T h[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      from_f(h[j], v[j]);
+      v[j] = to_f(h[j]);
+    }
+    float acc[VEC];
+    ld<T, VEC>(cw + (long)last * W, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) acc[j] = v[j] + u[j] * v[j];
+    for (int k = max(0, last - p); k < last; ++k) {
+      float c[VEC];
+      ld<T, VEC>(cw + (long)k * W, u);
+      ld<T, VEC>(ring + (long)((p - last + k) % a.taps) * W, c);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) acc[j] += u[j] * c[j];
+    }
+    st<T, VEC>(ring + (long)(p % a.taps) * W, v);
+    st<T, VEC>((T*)a.hc + (long)o * W + i, acc);
   }
 }
 
@@ -164,12 +233,19 @@ extern "C" int sv_residual_norm(const ResidualNormArgs* a, int f32,
                                 hipStream_t stream) {
   if (a->rows_out <= 0) return 0;
   const bool staged = (a->h && a->w) || (a->w1 && !a->delta2);
-  const size_t lds = staged ? (size_t)a->W * sizeof(float) : 0;
+  const int parts = a->groups > a->p_groups ? a->groups : a->p_groups;
+  const size_t lds =
+      staged ? ((size_t)a->W + (parts > 1 ? parts : 0)) * sizeof(float) : 0;
   if (lds > 160 * 1024 - 256) return 1;
+  if (a->W % a->groups || a->W % a->p_groups) return 1;
+  if (a->conv && (!a->h || !a->w)) return 1;
+  // four elements of a thread lie in one part
+  const bool vec = a->W % 4 == 0 && (a->W / a->groups) % 4 == 0 &&
+                   (a->W / a->p_groups) % 4 == 0;
 #define RN(T, V)                                                           \
   residual_norm_kernel<T, V><<<a->rows_out, 256, lds, stream>>>(*a)
-  if (f32) { if (a->W % 4 == 0) RN(float, 4); else RN(float, 1); }
-  else     { if (a->W % 4 == 0) RN(short, 4); else RN(short, 1); }
+  if (f32) { if (vec) RN(float, 4); else RN(float, 1); }
+  else     { if (vec) RN(short, 4); else RN(short, 1); }
 #undef RN
   return (int)hipGetLastError();
 }
@@ -194,7 +270,7 @@ gated_norm_kernel(const T* __restrict__ o, const T* __restrict__ w,
   const long r = item / groups;
   const int off = (int)(item % groups) * gs;
   const T* src = o + item * gs;
-  const T* g = gate + r * gate_stride + off;
+  const T* g = gate ? gate + r * gate_stride + off : nullptr;
   float sq = 0.f, v[VEC], u[VEC];
   for (int i = tid * VEC; i < gs; i += step) {
     ld<T, VEC>(src + i, v);
@@ -206,10 +282,14 @@ gated_norm_kernel(const T* __restrict__ o, const T* __restrict__ w,
   for (int i = tid * VEC; i < gs; i += step) {
     ld<T, VEC>(src + i, v);
     ld<T, VEC>(w + off + i, u);
-    float z[VEC];
-    ld<T, VEC>(g + i, z);
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) v[j] *= rstd * u[j] * sigmoid_f(z[j]);
+    for (int j = 0; j < VEC; ++j) v[j] *= rstd * u[j];
+    if (g) {
+      float z[VEC];
+      ld<T, VEC>(g + i, z);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[j] *= sigmoid_f(z[j]);
+    }
     st<T, VEC>(out + item * gs + i, v);
   }
 }
@@ -282,6 +362,32 @@ extern "C" int sv_relu_squared(void* x, long n, int f32, hipStream_t stream) {
 
 extern "C" int sv_gelu_tanh(void* x, long n, int f32, hipStream_t stream) {
   return launch_pointwise<GeluTanh>(x, n, f32, stream);
+}
+
+// x [rows][n] -> gelu(x) * (columns [at, at + n) of table[token])
+template <typename T>
+__global__ void __launch_bounds__(256)
+gelu_rows_kernel(T* __restrict__ x, const T* __restrict__ table, long tst,
+                 const int* __restrict__ tokens, long rows, int n, int at) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= rows * n) return;
+  const long r = i / n;
+  from_f(x[i], GeluTanh::at(to_f(x[i])) *
+                   to_f(table[tokens[r] * tst + at + (int)(i - r * n)]));
+}
+
+extern "C" int sv_gelu_rows(void* x, const void* table, long tst,
+                            const int* tokens, long rows, int n, int at,
+                            int f32, hipStream_t stream) {
+  if (rows <= 0) return 0;
+  const long blocks = (rows * n + 255) / 256;
+  if (f32)
+    gelu_rows_kernel<float><<<blocks, 256, 0, stream>>>(
+        (float*)x, (const float*)table, tst, tokens, rows, n, at);
+  else
+    gelu_rows_kernel<short><<<blocks, 256, 0, stream>>>(
+        (short*)x, (const short*)table, tst, tokens, rows, n, at);
+  return (int)hipGetLastError();
 }
 
 __global__ void __launch_bounds__(256)

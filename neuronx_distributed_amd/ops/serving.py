@@ -8,9 +8,10 @@ gates and recurrent state are 32-bit in both.
 """
 
 import ctypes
+import math
 import os
-from dataclasses import dataclass
-from typing import Optional
+from dataclasses import dataclass, replace
+from typing import Optional, Union
 
 import torch
 
@@ -18,6 +19,7 @@ PAGE_SIZE = 64
 MAX_HEAD_DIM = 512          # attention q/k and v size, recurrent q/k size
 MAX_LATENT_ROW = 1024       # latents and shared key columns of a cached row
 MAX_EXPERTS = 512
+MAX_TAPS = 65               # of a short convolution
 EXPAND_MIN_TOKENS = 32      # shorter portions attend in the latent space
 CHUNK = 256                 # tokens of one chunk of a matrix memory
 
@@ -73,9 +75,34 @@ def _fields(names, ctype):
 
 class _ResidualNormArgs(ctypes.Structure):
     _fields_ = (_fields("x delta delta2 w1 w2 coef vec x_out h w cat x0 "
-                        "index", ctypes.c_void_p)
-                + _fields("rows_out W delta_f32 parts", ctypes.c_int)
-                + _fields("eps scale w_base p_base", ctypes.c_float))
+                        "index conv ring singles hc", ctypes.c_void_p)
+                + _fields("rows_out W delta_f32 parts groups p_groups taps "
+                          "conv_row", ctypes.c_int)
+                + _fields("eps scale w_base p_base h_scale", ctypes.c_float))
+
+
+class _ConvArgs(ctypes.Structure):
+    _fields_ = (_fields("x", ctypes.c_void_p) + _fields("xst", ctypes.c_long)
+                + _fields("w bias out", ctypes.c_void_p)
+                + _fields("ost", ctypes.c_long)
+                + _fields("ring seg chunks", ctypes.c_void_p)
+                + _fields("n_chunks chunk C taps silu add", ctypes.c_int))
+
+
+class _QkvArgs(ctypes.Structure):
+    _fields_ = (_fields("q k v", ctypes.c_void_p)
+                + _fields("qst kst vst", ctypes.c_long)
+                + _fields("freq qw kw first", ctypes.c_void_p)
+                + _fields("fst", ctypes.c_long)
+                + _fields("mix kc vc pos seq bt", ctypes.c_void_p)
+                + _fields("MB T H G D E rot norm temp_every", ctypes.c_int)
+                + _fields("temp_coef eps", ctypes.c_float))
+
+
+class _ScoreArgs(ctypes.Structure):
+    _fields_ = (_fields("temp sink slope gate", ctypes.c_void_p)
+                + _fields("gst", ctypes.c_long)
+                + _fields("cap", ctypes.c_float))
 
 
 class _RowsArgs(ctypes.Structure):
@@ -86,7 +113,7 @@ class _RowsArgs(ctypes.Structure):
                 + _fields("pos seq bt part out", ctypes.c_void_p)
                 + _fields("MB rows H G D E splits append window keep",
                           ctypes.c_int)
-                + _fields("scale", ctypes.c_float))
+                + _fields("scale", ctypes.c_float) + [("mod", _ScoreArgs)])
 
 
 class _TilesArgs(ctypes.Structure):
@@ -98,7 +125,7 @@ class _TilesArgs(ctypes.Structure):
                 + _fields("gst", ctypes.c_long)
                 + _fields("tiles bt out", ctypes.c_void_p)
                 + _fields("MB H G D E DS window keep", ctypes.c_int)
-                + _fields("scale", ctypes.c_float))
+                + _fields("scale", ctypes.c_float) + [("mod", _ScoreArgs)])
 
 
 class _LatentAppendArgs(ctypes.Structure):
@@ -131,7 +158,8 @@ class _LatentRowsArgs(ctypes.Structure):
 
 class _MoePlanArgs(ctypes.Structure):
     _fields_ = (_fields("z bias idx coef order tiles", ctypes.c_void_p)
-                + _fields("T E top tile_rows max_tiles", ctypes.c_int))
+                + _fields("T E top tile_rows max_tiles sigmoid groups keep",
+                          ctypes.c_int))
 
 
 class _MoeGemmArgs(ctypes.Structure):
@@ -147,7 +175,12 @@ class _MemoryArgs(ctypes.Structure):
                 + _fields("gates ib fb decay log2_decay S n m seg out",
                           ctypes.c_void_p)
                 + _fields("H D E", ctypes.c_int)
-                + _fields("gate_cap qscale", ctypes.c_float))
+                + _fields("gate_cap qscale", ctypes.c_float)
+                + _fields("G", ctypes.c_int)
+                + _fields("skip z", ctypes.c_void_p)
+                + _fields("zst", ctypes.c_long)
+                + _fields("cw cb ring", ctypes.c_void_p)
+                + _fields("taps C kch qch", ctypes.c_int))
 
 
 class _ChunkArgs(ctypes.Structure):
@@ -177,7 +210,7 @@ class Pending:
     """A sublayer result that has not been added to the residual yet: one
     tensor, or two branches that are RMS-normed with their own weights and
     summed; ``scale`` times that.  One tensor is RMS-normed when ``w1`` is
-    given.  ``coef`` (rows, parts) makes a row the weighted sum of ``parts``
+    given, over ``groups`` equal parts each.  ``coef`` (rows, parts) makes a row the weighted sum of ``parts``
     rows of ``delta`` (rows * parts, W).  ``centred``: w1 and w2 are stored as
     their distance from one.  ``vec`` is a row added to every token."""
     delta: torch.Tensor
@@ -188,17 +221,62 @@ class Pending:
     vec: Optional[torch.Tensor] = None
     coef: Optional[torch.Tensor] = None
     centred: bool = False
+    groups: int = 1
+
+
+@dataclass
+class ShortConv:
+    """A causal convolution over time, one filter a channel, with the last
+    inputs of every request: ``ring`` (slots, taps, C) holds the input at
+    position p in place p % taps."""
+    w: torch.Tensor            # (taps, C); the last row weighs the token itself
+    ring: torch.Tensor
+    bias: Optional[torch.Tensor] = None
+
+    def check(self, C, dtype):
+        assert self.w.shape[1] == C and self.w.is_contiguous()
+        assert self.ring.shape[1:] == self.w.shape
+        assert self.ring.is_contiguous() and self.w.shape[0] <= MAX_TAPS
+        assert self.w.dtype == self.ring.dtype == dtype
+        assert self.bias is None or (self.bias.shape == (C,)
+                                     and self.bias.dtype == dtype)
+
+
+def short_conv(x, conv: ShortConv, seg, chunks, silu: bool = False,
+               add: bool = False,
+               out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Convolve the rows of prompt portions x (T, C) and keep their last
+    inputs: silu(y), or x + y, of y = bias + conv(x).  ``seg`` lists the
+    portions (slot, first row, rows, context), ``chunks`` is the device form of
+    ``chunk_table``."""
+    T, C = x.shape
+    conv.check(C, x.dtype)
+    assert x.stride(1) == 1
+    out = _out(out, T, C, x)
+    a = _ConvArgs(x=_p(x), xst=x.stride(0), w=_p(conv.w), bias=_p(conv.bias),
+                  out=_p(out), ost=C, ring=_p(conv.ring), seg=_p(seg),
+                  chunks=_p(chunks), n_chunks=chunks.shape[0], chunk=CHUNK,
+                  C=C, taps=conv.w.shape[0], silu=int(silu), add=int(add))
+    _check(library().sv_short_conv(ctypes.byref(a),
+                                   int(_aligned((C,), x, out)), _f32(x),
+                                   _stream()), "short_conv")
+    return out
 
 
 def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
                   eps: float, weight: Optional[torch.Tensor] = None,
                   x0: Optional[torch.Tensor] = None, keep_x: bool = True,
                   index: Optional[torch.Tensor] = None, dtype=None,
-                  centred: bool = False, copy: bool = False):
+                  centred: bool = False, copy: bool = False, groups: int = 1,
+                  scale: float = 1.0, conv: Optional[ShortConv] = None,
+                  batch=None):
     """Add ``pending`` to the float32 residual ``x`` (None: zero) and return
     (new x or None, RMS-normed row * weight or None, [new x; x0] or None).
     ``centred``: the weight is stored as its distance from one.  ``copy``: the
-    second result is the new x itself, rounded to ``dtype``."""
+    second result is the new x itself, rounded to ``dtype``.  ``groups``: every
+    one of so many equal parts is normed on its own.  ``scale`` multiplies the
+    second result.  ``conv``: the second result is h + conv(h) of the rows h of
+    ``batch``."""
     src = x if pending is None else pending.delta
     rows, W = src.shape
     if pending is not None and pending.coef is not None:
@@ -217,7 +295,8 @@ def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
         if weight is not None or copy else None
     cat = torch.empty(out_rows, 2 * W, dtype=dtype, device=dev) \
         if x0 is not None else None
-    a = _ResidualNormArgs(rows_out=out_rows, W=W, eps=eps)
+    a = _ResidualNormArgs(rows_out=out_rows, W=W, eps=eps, groups=groups,
+                          p_groups=1, h_scale=scale)
     a.x, a.x_out, a.h, a.w = _p(x), _p(x_new), _p(h), _p(weight)
     a.cat, a.x0, a.index = _p(cat), _p(x0), _p(index)
     a.w_base, a.scale = float(centred), 1.0
@@ -230,30 +309,51 @@ def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
         a.delta, a.delta2 = _p(d), _p(pending.delta2)
         a.w1, a.w2, a.vec = _p(pending.w1), _p(pending.w2), _p(pending.vec)
         a.coef, a.scale = _p(pending.coef), pending.scale
+        a.p_groups = pending.groups
+        assert pending.groups == 1 or (pending.w1 is not None
+                                       and pending.delta2 is None)
         if pending.coef is not None:
             a.parts = pending.coef.shape[1]
             assert d.dtype == dtype
         a.p_base = float(pending.centred)
         a.delta_f32 = int(d.dtype == torch.float32 and
                           dtype != torch.float32)
+    hc = None
+    if conv is not None:
+        assert weight is not None and index is None
+        conv.check(W, dtype)
+        hc = torch.empty_like(h)
+        n = batch.portion_tokens
+        assert out_rows - n == batch.singles.shape[0] and conv.bias is None
+        a.conv, a.ring, a.hc = _p(conv.w), _p(conv.ring), _p(hc)
+        a.singles, a.taps, a.conv_row = _p(batch.singles), conv.w.shape[0], n
     _check(library().sv_residual_norm(ctypes.byref(a), f32, _stream()),
            "residual_norm")
+    if hc is not None:
+        if n:
+            short_conv(h[:n], conv, batch.portions, batch.chunks, add=True,
+                       out=hc[:n])
+        h = hc
     return x_new, h, cat
 
 
-def gated_norm(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor,
-               group: int, eps: float) -> torch.Tensor:
+def gated_norm(o: torch.Tensor, weight: torch.Tensor,
+               gate: Optional[torch.Tensor], group: int,
+               eps: float) -> torch.Tensor:
     """o (T, N): every ``group`` elements divided by their root mean square,
-    times weight (N,), times sigmoid(gate (T, N))."""
+    times weight (N,), times sigmoid(gate (T, N)) if there is a gate."""
     T, N = o.shape
-    assert N % group == 0 and gate.shape == o.shape
-    assert gate.stride(1) == 1 and o.is_contiguous()
+    assert N % group == 0 and o.is_contiguous()
     out = torch.empty_like(o)
-    vec4 = int(group % 4 == 0 and gate.stride(0) % 4 == 0
-               and gate.storage_offset() % 4 == 0)
+    vec4 = int(group % 4 == 0)
+    if gate is not None:
+        assert gate.shape == o.shape and gate.stride(1) == 1
+        vec4 = int(vec4 and gate.stride(0) % 4 == 0
+                   and gate.storage_offset() % 4 == 0)
     _check(library().sv_gated_norm(
         ctypes.c_void_p(_p(o)), ctypes.c_void_p(_p(weight)),
-        ctypes.c_void_p(_p(gate)), ctypes.c_long(gate.stride(0)),
+        ctypes.c_void_p(_p(gate)),
+        ctypes.c_long(0 if gate is None else gate.stride(0)),
         ctypes.c_void_p(_p(out)), T, N // group, group, ctypes.c_float(eps),
         vec4, _f32(o), _stream()), "gated_norm")
     return out
@@ -272,6 +372,21 @@ def gelu_tanh_(x: torch.Tensor) -> torch.Tensor:
     _check(library().sv_gelu_tanh(ctypes.c_void_p(_p(x)),
                                   ctypes.c_long(x.numel()), _f32(x),
                                   _stream()), "gelu_tanh")
+    return x
+
+
+def gelu_rows_(x: torch.Tensor, table: torch.Tensor, tokens: torch.Tensor,
+               at: int) -> torch.Tensor:
+    """x (T, n) <- gelu(x), in its tanh form, times the columns [at, at + n)
+    of table (vocab, columns) in the rows ``tokens`` (T,) int32."""
+    T, n = x.shape
+    assert x.is_contiguous() and table.stride(1) == 1
+    assert x.dtype == table.dtype and 0 <= at <= table.shape[1] - n
+    assert tokens.dtype == torch.int32 and tokens.shape == (T,)
+    _check(library().sv_gelu_rows(
+        ctypes.c_void_p(_p(x)), ctypes.c_void_p(_p(table)),
+        ctypes.c_long(table.stride(0)), ctypes.c_void_p(_p(tokens)),
+        ctypes.c_long(T), n, at, _f32(x), _stream()), "gelu_rows")
     return x
 
 
@@ -330,6 +445,89 @@ def kv_append(k, v, kc, vc, pos, seq, block_table):
         int(_aligned((D, E), k, v)), _f32(k), _stream()), "kv_append")
 
 
+@dataclass
+class QkvPrep:
+    """What happens to queries, keys and values before they are attended and
+    cached: the first elements of a head turn in neighbouring pairs, queries
+    and keys are RMS-normed a head, queries grow with their position, values
+    take a share of another layer's."""
+    freq: Optional[torch.Tensor] = None    # (dims / 2,) float64 rad a position
+    norm: bool = False
+    q_norm: Optional[torch.Tensor] = None  # (D,) weights of the norm
+    k_norm: Optional[torch.Tensor] = None
+    eps: float = 0.0
+    temp_coef: float = 0.0                 # q *= 1 + coef ln(floor((p + 1) /
+    temp_every: int = 0                    #   every) + 1), if every > 0
+    first: Optional[torch.Tensor] = None   # (T, G * E)
+    mix: Optional[torch.Tensor] = None     # one number: v + mix (first - v)
+
+
+@dataclass
+class ScoreMod:
+    """Of the scores s = q.k scale and their softmax: s *= temp[h];
+    s = cap tanh(s / cap); s -= slope[h] distance; exp(sink[h]) joins the
+    denominator; the output is multiplied by sigmoid(gate[row, h])."""
+    temp: Optional[torch.Tensor] = None    # (H,)
+    cap: float = 0.0
+    slope: Optional[torch.Tensor] = None   # (H,) float32
+    sink: Optional[torch.Tensor] = None    # (H,)
+    gate: Optional[torch.Tensor] = None    # (T, H)
+
+    def rows(self, a, b):
+        """The same for rows [a, b) of the batch."""
+        return self if self.gate is None else replace(self,
+                                                      gate=self.gate[a:b])
+
+
+def _score_args(mod: Optional[ScoreMod], q, H) -> _ScoreArgs:
+    if mod is None:
+        return _ScoreArgs()
+    for t in (mod.temp, mod.sink):
+        assert t is None or (t.shape == (H,) and t.dtype == q.dtype
+                             and t.is_cuda and t.is_contiguous())
+    assert mod.slope is None or (mod.slope.shape == (H,) and mod.slope.is_cuda
+                                 and mod.slope.dtype == torch.float32)
+    a = _ScoreArgs(temp=_p(mod.temp), sink=_p(mod.sink), slope=_p(mod.slope),
+                   cap=mod.cap)
+    if mod.gate is not None:
+        assert mod.gate.shape == (q.shape[0], H) and mod.gate.stride(1) == 1
+        assert mod.gate.dtype == q.dtype
+        a.gate, a.gst = _p(mod.gate), mod.gate.stride(0)
+    return a
+
+
+def qkv_append(q, k, v, kc, vc, pos, seq, block_table, heads: int,
+               prep: QkvPrep):
+    """Prepare q (T, H*D) in place and write the prepared k and v at positions
+    ``pos`` of the requests ``seq``."""
+    G, D, E = _check_cache(q, k, v, kc, vc, heads)
+    T = q.shape[0]
+    assert pos.shape[0] == seq.shape[0] == T
+    a = _QkvArgs(q=_p(q), k=_p(k), v=_p(v), qst=q.stride(0), kst=k.stride(0),
+                 vst=v.stride(0), kc=_p(kc), vc=_p(vc), pos=_p(pos),
+                 seq=_p(seq), bt=_p(block_table), MB=block_table.shape[1],
+                 T=T, H=heads, G=G, D=D, E=E, norm=int(prep.norm),
+                 temp_every=prep.temp_every, temp_coef=prep.temp_coef,
+                 eps=prep.eps)
+    tensors = [q, k, v]
+    if prep.freq is not None:
+        assert prep.freq.dtype == torch.float64 and prep.freq.is_cuda
+        a.freq, a.rot = _p(prep.freq), 2 * prep.freq.shape[0]
+    for name, w in (("qw", prep.q_norm), ("kw", prep.k_norm)):
+        if w is not None:
+            assert w.shape == (D,) and w.dtype == q.dtype and prep.norm
+            setattr(a, name, _p(w))
+    if prep.first is not None:
+        f = prep.first
+        assert f.shape == v.shape and f.stride(1) == 1 and f.dtype == v.dtype
+        assert prep.mix.numel() == 1 and prep.mix.dtype == v.dtype
+        a.first, a.fst, a.mix = _p(f), f.stride(0), _p(prep.mix)
+        tensors.append(f)
+    _check(library().sv_qkv_append(
+        ctypes.byref(a), int(_aligned((D, E), *tensors)), _f32(q), _stream()),
+        "qkv_append")
+
+
 def _row_splits(target: int, units: int, max_keys: int, per: int) -> int:
     """Workgroups that share a row: enough for ``target`` of them, each with
     about ``per`` keys or more."""
@@ -339,7 +537,8 @@ def _row_splits(target: int, units: int, max_keys: int, per: int) -> int:
 def attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads: int,
               scale: float, window: int = 0, keep: int = 0,
               append: bool = True, max_keys: int = 0,
-              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+              out: Optional[torch.Tensor] = None,
+              mod: Optional[ScoreMod] = None) -> torch.Tensor:
     """One query row per request row: decoding.  ``append`` also writes the
     row's own k/v into the cache (without it they must be there already).
     ``max_keys`` bounds the visible keys of any row (it only sets how many
@@ -359,7 +558,8 @@ def attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads: int,
                   pos=_p(pos), seq=_p(seq), bt=_p(block_table),
                   part=_p(part), out=_p(out), MB=block_table.shape[1],
                   rows=rows, H=heads, G=G, D=D, E=E, splits=splits,
-                  append=int(append), window=window, keep=keep, scale=scale)
+                  append=int(append), window=window, keep=keep, scale=scale,
+                  mod=_score_args(mod, q, heads))
     _check(library().sv_attn_rows(ctypes.byref(a),
                                   int(_aligned((D, E), q, k, v)), _f32(q),
                                   _stream()), "attn_rows")
@@ -374,45 +574,55 @@ def attn_tiles_supported(q, kc, vc) -> bool:
 
 def attn_portions(q, k, v, kc, vc, pos, seq, block_table, tiles, heads: int,
                   scale: float, window: int = 0, keep: int = 0,
-                  max_keys: int = 0,
-                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """Prompt portions: append k/v, then causal attention of every row over
-    its request's cache.  ``tiles`` (n, 4) int32 lists (request, first row,
-    rows <= 128, position of the first row)."""
+                  append: bool = True, max_keys: int = 0,
+                  out: Optional[torch.Tensor] = None,
+                  mod: Optional[ScoreMod] = None) -> torch.Tensor:
+    """Prompt portions: append k/v (unless they are there), then causal
+    attention of every row over its request's cache.  ``tiles`` (n, 4) int32
+    lists (request, first row, rows <= 128, position of the first row)."""
     G, D, E = _check_cache(q, k, v, kc, vc, heads)
-    kv_append(k, v, kc, vc, pos, seq, block_table)
+    if append:
+        kv_append(k, v, kc, vc, pos, seq, block_table)
     if not attn_tiles_supported(q, kc, vc):
         return attn_rows(q, k, v, kc, vc, pos, seq, block_table, heads,
                          scale, window, keep, append=False,
-                         max_keys=max_keys, out=out)
+                         max_keys=max_keys, out=out, mod=mod)
     out = _out(out, q.shape[0], heads * E, q)
     a = _TilesArgs(q=_p(q), qst=q.stride(0), kc=_p(kc), vc=_p(vc),
                    kpage=G * PAGE_SIZE * D, khead=PAGE_SIZE * D, krow=D,
                    vpage=G * PAGE_SIZE * E, vhead=PAGE_SIZE * E, vrow=E,
                    tiles=_p(tiles), bt=_p(block_table), out=_p(out),
                    MB=block_table.shape[1], H=heads, G=G, D=D, E=E, DS=D,
-                   window=window, keep=keep, scale=scale)
+                   window=window, keep=keep, scale=scale,
+                   mod=_score_args(mod, q, heads))
     _check(library().sv_attn_tiles(ctypes.byref(a), tiles.shape[0],
                                    _stream()), "attn_tiles")
     return out
 
 
 def ragged_attention(q, k, v, batch, pool, heads: int, scale: float,
-                     window: int = 0, keep: int = 0) -> torch.Tensor:
+                     window: int = 0, keep: int = 0,
+                     prep: Optional[QkvPrep] = None,
+                     mod: Optional[ScoreMod] = None) -> torch.Tensor:
     """Attention of a packed batch over its cache pool: portions first, then
-    single tokens, into one (T, heads * E) tensor."""
+    single tokens, into one (T, heads * E) tensor.  ``prep`` changes q in
+    place."""
     kc, vc = pool
     T, n = q.shape[0], batch.portion_tokens
     out = torch.empty(T, heads * vc.shape[3], dtype=q.dtype, device=q.device)
     args = dict(heads=heads, scale=scale, window=window, keep=keep,
-                max_keys=batch.max_keys)
+                max_keys=batch.max_keys, append=prep is None)
+    if prep is not None:
+        qkv_append(q, k, v, kc, vc, batch.pos, batch.seq, batch.block_table,
+                   heads, prep)
     if n:
         attn_portions(q[:n], k[:n], v[:n], kc, vc, batch.pos[:n],
                       batch.seq[:n], batch.block_table, batch.tiles,
-                      out=out[:n], **args)
+                      out=out[:n], mod=mod and mod.rows(0, n), **args)
     if n < T:
         attn_rows(q[n:], k[n:], v[n:], kc, vc, batch.pos[n:], batch.seq[n:],
-                  batch.block_table, out=out[n:], **args)
+                  batch.block_table, out=out[n:], mod=mod and mod.rows(n, T),
+                  **args)
     return out
 
 
@@ -453,6 +663,23 @@ class ExpGate:
     qscale: float
 
 
+@dataclass
+class TimeGate:
+    """A time step from a projection: dt = softplus(raw + bias), S <-
+    exp(-exp(A_log) dt) S + dt k v^T; o = (S^T q + skip v) silu(z).  Heads share
+    q and k in groups.  ``conv``: q, k and v of single tokens have not passed
+    their convolution and silu yet; its channels are v's, then k's, then q's."""
+    raw: torch.Tensor          # (T, H) float32
+    bias: torch.Tensor         # (H,)
+    A_log: torch.Tensor        # (H,)
+    skip: torch.Tensor         # (H,)
+    z: torch.Tensor            # (T, H * E)
+    conv: Optional[ShortConv] = None
+
+
+_GATINGS = {DecayGate: 0, ExpGate: 1, TimeGate: 2}
+
+
 def chunk_table(segments):
     """Chunks of prompt portions: rows (segment, first row, rows, does a
     state come in) and the first chunk of every segment, from rows (slot,
@@ -471,7 +698,7 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
                chunk_first: Optional[torch.Tensor] = None,
                out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Run a matrix memory over segments of a ragged batch.  q, k (T, H*D),
-    v (T, H*E); S (slots, H, D, E) float32; n (slots, H, ceil(E/32), D) and
+    v (T, H*E) — q, k (T, G*D) for a TimeGate; S (slots, H, D, E) float32; n (slots, H, ceil(E/32), D) and
     m (slots, H, ceil(E/32)) float32 for an ExpGate.  ``seg`` (n, 4) int32
     lists (slot, first row, rows, context); rows count from the start of
     the tensors, so portions and single tokens of one batch can be run by
@@ -479,7 +706,7 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
     ``chunk_table`` the 256-token MFMA kernels run where they apply."""
     D, E = S.shape[2], S.shape[3]
     T = q.shape[0]
-    assert q.shape[1] == k.shape[1] == heads * D and v.shape[1] == heads * E
+    assert q.shape[1] == k.shape[1] and v.shape[1] == heads * E
     assert q.stride(1) == k.stride(1) == v.stride(1) == 1
     assert S.is_contiguous() and S.dtype == torch.float32
     assert S.shape[1] == heads
@@ -488,9 +715,31 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
     out = _out(out, T, heads * E, q)
     a = _MemoryArgs(q=_p(q), k=_p(k), v=_p(v), qst=q.stride(0),
                     kst=k.stride(0), vst=v.stride(0), S=_p(S), seg=_p(seg),
-                    out=_p(out), H=heads, D=D, E=E, gate_cap=1.0, qscale=1.0)
-    gated = isinstance(gate, ExpGate)
-    if gated:
+                    out=_p(out), H=heads, D=D, E=E, gate_cap=1.0, qscale=1.0,
+                    G=q.shape[1] // D)
+    assert q.shape[1] == a.G * D and heads % a.G == 0
+    gating = _GATINGS[type(gate)]
+    gated, timed = isinstance(gate, ExpGate), isinstance(gate, TimeGate)
+    assert timed or a.G == heads
+    strided = [q, k, v]
+    if timed:
+        for t in (gate.bias, gate.A_log, gate.skip):
+            assert t.shape == (heads,) and t.dtype == q.dtype
+        assert gate.raw.shape == (T, heads) and gate.raw.is_contiguous() \
+            and gate.raw.dtype == torch.float32
+        assert gate.z.shape == v.shape and gate.z.stride(1) == 1 \
+            and gate.z.dtype == v.dtype
+        a.gates, a.ib, a.fb = _p(gate.raw), _p(gate.bias), _p(gate.A_log)
+        a.skip, a.z, a.zst = _p(gate.skip), _p(gate.z), gate.z.stride(0)
+        strided.append(gate.z)
+        if gate.conv is not None:
+            assert chunks is None      # one token a segment
+            a.kch, a.qch = heads * E, heads * E + k.shape[1]
+            a.C, a.taps = a.qch + q.shape[1], gate.conv.w.shape[0]
+            gate.conv.check(a.C, q.dtype)
+            a.cw, a.cb = _p(gate.conv.w), _p(gate.conv.bias)
+            a.ring = _p(gate.conv.ring)
+    elif gated:
         nt = (E + 31) // 32
         assert n.shape[1:] == (heads, nt, D) and m.shape[1:] == (heads, nt)
         assert gate.raw.shape == (T, 2 * heads) and \
@@ -504,7 +753,7 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
         a.decay, a.log2_decay = _p(gate.decay), _p(gate.log2_decay)
     lib = library()
     if (chunks is not None and q.dtype == torch.bfloat16 and D <= 256
-            and _aligned((D, E), q, k, v)):
+            and _aligned((D, E), *strided)):
         nc = chunks.shape[0]
         assert chunk_first.shape[0] == seg.shape[0] + 1
         f32 = dict(dtype=torch.float32, device=q.device)
@@ -513,21 +762,25 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
                         device=q.device)
         VT = torch.empty(nc, heads, E, CHUNK, dtype=torch.bfloat16,
                          device=q.device)
-        KA = None if gated else torch.empty(T, heads * D, dtype=q.dtype,
-                                            device=q.device)
+        KA = torch.empty(T, heads * D, dtype=q.dtype, device=q.device) \
+            if isinstance(gate, DecayGate) else None
         x = _ChunkArgs(a=a, chunks=_p(chunks), first=_p(chunk_first),
                        n_chunks=nc, n_seg=seg.shape[0], T=T, U=_p(U),
                        P=_p(P), VT=_p(VT), KA=_p(KA))
-        if gated:
+        if timed:
+            bic = torch.empty(2, heads, T, **f32)
+            small = torch.empty(nc, heads, 4, **f32)
+            x.b, x.i, x.tot = _p(bic[0]), _p(bic[1]), _p(small)
+        elif gated:
             bic = torch.empty(3, heads, T, **f32)
             small = torch.empty(nc, heads, 6 + D, **f32)
             x.b, x.i, x.c = (_p(t) for t in bic)
             flat, nh = small.view(-1), nc * heads
             x.tot, x.cend = _p(flat), _p(flat[4 * nh:])
             x.mst, x.N = _p(flat[5 * nh:]), _p(flat[6 * nh:])
-        st = lib.sv_memory_chunks(ctypes.byref(x), int(gated), _stream())
+        st = lib.sv_memory_chunks(ctypes.byref(x), gating, _stream())
     else:
-        st = lib.sv_memory_steps(ctypes.byref(a), seg.shape[0], int(gated),
+        st = lib.sv_memory_steps(ctypes.byref(a), seg.shape[0], gating,
                                  _f32(q), _stream())
     _check(st, "memory_mix")
     return out
@@ -567,11 +820,21 @@ def key_spans(portions, block_table, window: int):
     return pages, table
 
 
-def rotary_frequencies(base: float, dims: int, device) -> torch.Tensor:
-    """Radians a position of every rotated pair, float64."""
+def rotary_frequencies(base: float, dims: int, device,
+                       scaling: Optional[dict] = None) -> torch.Tensor:
+    """Radians a position of every rotated pair, float64.  ``scaling`` (factor,
+    low, high, original): a pair that turns less than ``low`` times in
+    ``original`` positions is slowed by ``factor``, one that turns more than
+    ``high`` times is kept, those between are interpolated."""
     i = torch.arange(dims // 2, dtype=torch.float64)
-    return torch.pow(torch.tensor(base, dtype=torch.float64),
-                     -2.0 * i / dims).to(device)
+    f = torch.pow(torch.tensor(base, dtype=torch.float64), -2.0 * i / dims)
+    if scaling:
+        low, high = scaling["low"], scaling["high"]
+        turns = scaling["original"] * f / (2.0 * math.pi)
+        keep = ((turns - low) / (high - low)).clamp(0.0, 1.0) \
+            if high > low else (turns > low).double()
+        f = f * (keep + (1.0 - keep) / scaling["factor"])
+    return f.to(device)
 
 
 @dataclass
@@ -787,6 +1050,28 @@ def moe_kernel(pairs: int, experts: int) -> int:
 
 
 @dataclass
+class Routing:
+    """How logits choose experts.  Plain: the largest z + bias, weights a
+    softmax over the chosen.  ``sigmoid``: the largest sigmoid(z) + bias,
+    weights the chosen sigmoids over their sum.  With several ``groups`` of
+    neighbours only the experts of the ``keep`` best can be chosen; a group
+    counts the sum of its two largest."""
+    top: int
+    sigmoid: bool = False
+    groups: int = 1
+    keep: int = 1
+
+    def check(self, experts: int):
+        g = self.groups
+        if experts > MAX_EXPERTS or not 1 <= self.top <= min(64, experts):
+            raise ValueError(f"{self.top} of {experts} experts")
+        if not 1 <= g <= 64 or experts % g or not 1 <= self.keep <= g or \
+                self.keep * (experts // g) < self.top:
+            raise ValueError(f"{self.top} experts from {self.keep} of {g} "
+                             f"groups of {experts}")
+
+
+@dataclass
 class MoePlan:
     coef: torch.Tensor         # (T, top) float32 weights of the chosen
     idx: torch.Tensor          # (T, top) int32 chosen experts
@@ -795,14 +1080,16 @@ class MoePlan:
     how: int                   # kernel of the grouped products
 
 
-def moe_plan(z: torch.Tensor, bias: Optional[torch.Tensor], top: int,
-             how: int) -> MoePlan:
-    """Choose the ``top`` experts with the largest logits z + bias of every
-    row, their weights a softmax over the chosen, and group the pairs."""
+def moe_plan(z: torch.Tensor, bias: Optional[torch.Tensor],
+             routing: Union[int, Routing], how: int) -> MoePlan:
+    """Choose the experts of every row from its logits z (plainly, if
+    ``routing`` is just their number), and group the pairs."""
     T, E = z.shape
+    if isinstance(routing, int):
+        routing = Routing(routing)
     assert z.dtype == torch.float32 and z.is_contiguous() and z.is_cuda
-    if E > MAX_EXPERTS or not 1 <= top <= min(64, E):
-        raise ValueError(f"{top} of {E} experts")
+    routing.check(E)
+    top = routing.top
     pairs, rows = T * top, MOE_TILE_ROWS[how]
     n = min(pairs, pairs // rows + E)
     ints = torch.empty(2 * pairs + 4 * n, dtype=torch.int32, device=z.device)
@@ -811,7 +1098,9 @@ def moe_plan(z: torch.Tensor, bias: Optional[torch.Tensor], top: int,
                 ints[:4 * n].view(n, 4), how)
     a = _MoePlanArgs(z=_p(z), bias=_p(bias), idx=_p(p.idx), coef=_p(p.coef),
                      order=_p(p.order), tiles=_p(p.tiles), T=T, E=E, top=top,
-                     tile_rows=rows, max_tiles=n)
+                     tile_rows=rows, max_tiles=n,
+                     sigmoid=int(routing.sigmoid), groups=routing.groups,
+                     keep=routing.keep)
     _check(library().sv_moe_plan(
         ctypes.byref(a), 0 if bias is None else _f32(bias), _stream()),
         "moe_plan")
@@ -842,14 +1131,16 @@ def moe_gemm(x: torch.Tensor, w: torch.Tensor, plan: MoePlan, gated: bool,
     return out
 
 
-def moe_mlp(h, z, bias, gate_up, down, top: int, alpha: float, limit: float,
-            shift: float) -> Pending:
+def moe_mlp(h, z, bias, gate_up, down, routing: Union[int, Routing],
+            alpha: float, limit: float, shift: float) -> Pending:
     """Gated experts on h (T, W) with router logits z (T, E): a pending sum
     of the chosen experts' outputs."""
+    if isinstance(routing, int):
+        routing = Routing(routing)
     E, W, ff = down.shape
-    pairs = h.shape[0] * top
+    pairs = h.shape[0] * routing.top
     fast = h.dtype == torch.bfloat16 and _aligned((W, ff), h)
-    plan = moe_plan(z, bias, top,
+    plan = moe_plan(z, bias, routing,
                     moe_kernel(pairs, E) if fast else MOE_PLAIN)
     act = moe_gemm(h, gate_up, plan, True, alpha, limit, shift)
     return Pending(moe_gemm(act, down, plan, False), coef=plan.coef)
