@@ -47,7 +47,7 @@ class SutuvikConfig:
                    norm_groups=d["norm"]["groups"],
                    conv_taps=d["canon"]["taps"],
                    side_dim=d["token_side"]["dim"],
-                   logit_scale=d["logit_scale"])
+                   logit_scale=d.get("logit_scale", 1.0))
 
 
 def _mamba2(width, c, eps):
@@ -59,7 +59,7 @@ def _mamba2(width, c, eps):
 def _attention(width, c, eps):
     return SingleMixer(width, ScoredAttention(
         width, c["heads"], c["kv_heads"], c["dim"], c["vdim"], c["scale"],
-        eps, qk_norm="weighted", q_temp=c["q_temp"],
+        eps, qk_norm="weighted", q_temp=c.get("q_temp"),
         slopes=alibi_slopes(c["heads"]), sink="learned", gate=True,
         v_mix=bool(c.get("v_mix"))))
 
@@ -67,8 +67,8 @@ def _attention(width, c, eps):
 def _attention_2(width, c, eps):
     return SingleMixer(width, ScoredAttention(
         width, c["heads"], c["kv_heads"], c["dim"], c["vdim"], c["scale"],
-        eps, rot=c["rot"], qk_norm="plain", head_temp=True,
-        softcap=c["softcap"], sink="zero", v_mix=bool(c.get("v_mix"))))
+        eps, rot=c.get("rot"), qk_norm="plain", head_temp=True,
+        softcap=c.get("softcap"), sink="zero", v_mix=bool(c.get("v_mix"))))
 
 
 def _experts(width, c):

@@ -195,8 +195,31 @@ def route(z, correction, groups, keep, top):
     return idx, w / (w.sum(dim=1, keepdim=True) + 1e-20)
 
 
-def experts_mlp(W, p, h, cfg):
+def route_margin(z, correction, groups, keep, top):
+    """How far every row is from choosing otherwise: the smaller gap between
+    the last kept and the first dropped group, or expert."""
+    s = sigmoid(z) + correction
+    parts = s.view(len(s), groups, -1)
+    n = min(2, parts.shape[2])
+    score = parts.sort(dim=2, descending=True).values[..., :n].sum(dim=2)
+    best, order = score.sort(dim=1, descending=True)
+    gap = torch.full((len(s),), math.inf, dtype=s.dtype)
+    if keep < groups:
+        gap = best[:, keep - 1] - best[:, keep]
+    open_ = torch.zeros_like(score, dtype=torch.bool).scatter_(
+        1, order[:, :keep], True).repeat_interleave(parts.shape[2], dim=1)
+    v = s.masked_fill(~open_, -math.inf).sort(dim=1, descending=True).values
+    if top < s.shape[1]:
+        gap = torch.minimum(gap, v[:, top - 1] - v[:, top])
+    return gap
+
+
+def experts_mlp(W, p, h, cfg, margins=None):
     r = cfg["router"]
+    if margins is not None:
+        margins.append(route_margin(
+            h @ W[p + "router"].T, W[p + "correction"], r["groups"]["count"],
+            r["groups"]["keep"], r["top"]))
     idx, w = route(h @ W[p + "router"].T, W[p + "correction"],
                    r["groups"]["count"], r["groups"]["keep"], r["top"])
     out = torch.zeros_like(h)
@@ -213,9 +236,10 @@ def token_side(W, p, x, e, eps):
     return rms(y, eps) * W[p + "norm"]
 
 
-def forward(cfg, weights, tokens, dtype=torch.float64, layers=None):
+def forward(cfg, weights, tokens, dtype=torch.float64, layers=None,
+            margins=None):
     """Logits (T, vocab) of one sequence; ``layers`` collects the residual
-    stream after every layer."""
+    stream after every layer, ``margins`` the routers' margins."""
     W = {n: w.to(dtype) for n, w in weights.items()}
     eps, groups = cfg["norm"]["eps"], cfg["norm"]["groups"]
     dim = cfg["token_side"]["dim"]
@@ -237,7 +261,7 @@ def forward(cfg, weights, tokens, dtype=torch.float64, layers=None):
         x = x + y
         if L["mlp"] is not None:
             h = group_norm(x, W[p + "norm2"], groups, eps)
-            x = x + experts_mlp(W, p + "mlp.", h, L["mlp"])
+            x = x + experts_mlp(W, p + "mlp.", h, L["mlp"], margins)
         e = W["side.embed"][toks][:, i * dim:(i + 1) * dim]
         x = x + token_side(W, p + "side.", x, e, eps)
         if layers is not None:
