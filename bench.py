@@ -40,9 +40,9 @@ def parse_args():
                    help="instead: the serving benchmark of a design beside "
                         "its closest relative (bench_serving.py, 1 GPU)")
     p.add_argument("--design", default="all",
-                   choices=("all", "voletar", "nesilorn"),
+                   choices=("all", "voletar", "nesilorn", "sutuvik"),
                    help="with --serving: Voletar beside Llama, Nesilorn "
-                        "beside Mixtral, or both")
+                        "beside Mixtral, Sutuvik beside Nesilorn, or all")
     return p.parse_args()
 
 

@@ -1,7 +1,8 @@
 #!/usr/bin/env python3
 """Serving benchmark of a design beside its closest relative at equal layer
 sizes (random weights, one MI355X): Voletar beside Llama, Nesilorn beside
-Mixtral.
+Mixtral, Sutuvik beside Nesilorn (its kernels beside those of Voletar and
+Nesilorn).
 
     python bench.py --serving                          all of it
     python bench.py --serving kernels                  (or: models)
@@ -619,8 +620,257 @@ def bench_latent_models():
         torch.cuda.empty_cache()
 
 
+# ---------------------------------------------------------------------------
+# Sutuvik beside Nesilorn and Voletar
+# ---------------------------------------------------------------------------
+
+def bench_state_kernels():
+    from types import SimpleNamespace
+
+    from neuronx_distributed_amd.models.mixers import alibi_slopes
+    from neuronx_distributed_amd.ops import serving as sv
+
+    dev = dict(device="cuda")
+    bf = torch.bfloat16
+    # -- timed memories beside decayed ones of half the state ----------------
+    H, G, N, P, taps = 128, 8, 128, 64, 4
+    LH, LD = 32, 128
+    inner, gn = H * P, G * N
+    C = inner + 2 * gn
+    w, b = _bf(taps, C), _bf(C)
+    small = [_bf(H) for _ in range(3)]
+    like_gate = sv.decay_gate([0.99] * LH, "cuda")
+    for B, T in ((1, 4096), (4, 4096), (1, 1), (32, 1), (128, 1)):
+        n = B * T
+        proj = _bf(n, inner + C)
+        z, xbc = proj[:, :inner], proj[:, inner:]
+        step = torch.randn(n, H, **dev)
+        S = torch.zeros(B, H, N, P, **dev)
+        ring = torch.zeros(B, taps, C, dtype=bf, **dev)
+        conv = sv.ShortConv(w, ring, b)
+        ctx = 64 if T == 1 else 0
+        seg = _i32([(i, i * T, T, ctx) for i in range(B)])
+        rows, first = sv.chunk_table(seg.tolist())
+        tab = (_i32(rows), _i32(first)) if T > 1 else ()
+        x = sv.short_conv(xbc, conv, seg, _i32(rows), silu=True) \
+            if T > 1 else xbc
+        v, k, q = x.split((inner, gn, gn), 1)
+        gate = sv.TimeGate(step, *small, z, None if T > 1 else conv)
+        lp = _bf(n, 3 * LH * LD)
+        lq, lk, lv = lp.split(LH * LD, 1)
+        LS = torch.zeros(B, LH, LD, LD, **dev)
+        us, lus = _time([
+            _graphed(lambda: sv.memory_mix(q, k, v, gate, S, None, None, seg,
+                                           H, *tab)),
+            _graphed(lambda: sv.memory_mix(lq, lk, lv, like_gate, LS, None,
+                                           None, seg, LH, *tab))])
+        cs = 64 if T > 1 else 1
+        state = 8 if ctx else 4
+
+        def cost(h, g, d, e, extra):
+            return (2 * n * h * (cs / 2 * (d + e) + 2 * d * e),
+                    2 * n * (2 * g * d + (2 + extra) * h * e)
+                    + state * B * h * d * e)
+
+        fl, io = cost(H, G, N, P, 1)
+        io += 4 * n * H
+        f3 = 2 * n * H * (cs / 2 * (N + 3 * P) + 6 * N * P)
+        extra = {"roofline_32bit_us": round(
+            max(f3 / PEAK_FLOPS, io / PEAK_BYTES) * 1e6, 2)} if T > 1 else {}
+        if T == 1:
+            io += 2 * n * (taps + 1) * C
+        _report("memory_" + ("chunks" if T > 1 else "steps, convolution"), us,
+                fl, io, ("decayed memory", lus, *cost(LH, LH, LD, LD, 0)),
+                batch=B, tokens=T, heads=H, state=N, vdim=P, **extra)
+    # -- attention -------------------------------------------------------------
+    H, G, D = 32, 8, 128
+    sizes = (H * D, G * D, G * D, H)
+    slope = torch.tensor(alibi_slopes(H), **dev)
+    freq = sv.rotary_frequencies(5e5, D, "cuda")
+    nw, hw = _bf(D), _bf(H)
+    kinds = {
+        "bias, sink, gate": (
+            sv.QkvPrep(norm=True, q_norm=nw, k_norm=nw, eps=1e-5,
+                       temp_coef=0.1, temp_every=8192),
+            lambda g: sv.ScoreMod(slope=slope, sink=hw, gate=g)),
+        "rotation, cap, sink": (
+            sv.QkvPrep(freq=freq, norm=True, eps=1e-5),
+            lambda g: sv.ScoreMod(temp=hw, cap=50.0, sink=hw))}
+    for B, T, ctx in ((1, 4096, 0), (1, 8192, 0), (1, 1, 4096), (32, 1, 1024),
+                      (32, 1, 4096), (128, 1, 4096)):
+        p = _bf(B * T, sum(sizes))
+        q, k, v, g = p.split(sizes, 1)
+        n = -(-(ctx + T) // 64)
+        kc = torch.zeros(B * n, G, 64, D, dtype=bf, **dev)
+        vc = torch.zeros_like(kc)
+        batch = SimpleNamespace(
+            block_table=torch.randperm(B * n).int().cuda().view(B, n),
+            max_keys=ctx + T, pos=_i32(list(range(ctx, ctx + T)) * B),
+            seq=_i32([r for r in range(B) for _ in range(T)]),
+            portion_tokens=B * T if T > 1 else 0,
+            tiles=_i32([(r, r * T + s, 128, ctx + s) for r in range(B)
+                        for s in range(0, T, 128)] if T > 1 else []))
+        pairs = B * sum(ctx + i + 1 for i in range(T))
+        fl = 4 * pairs * H * D
+        io = 2 * B * T * (2 * H + 2 * G) * D + \
+            (4 * B * G * ctx * D if T == 1 else 0)
+        for name, (prep, mod) in kinds.items():
+            prep.first, prep.mix = v.clone(), nw[:1]
+            at = (batch.pos, batch.seq, batch.block_table)
+            us, pus, lus, aus = _time([
+                _graphed(lambda: sv.ragged_attention(
+                    q, k, v, batch, (kc, vc), H, D ** -0.5, prep=prep,
+                    mod=mod(g))),
+                _graphed(lambda: sv.qkv_append(q, k, v, kc, vc, *at, H, prep)),
+                _graphed(lambda: sv.ragged_attention(
+                    q, k, v, batch, (kc, vc), H, D ** -0.5)),
+                _graphed(lambda: sv.kv_append(k, v, kc, vc, *at))])
+            _report(f"attention ({name})", us, fl, io,
+                    ("plain attention", lus, fl, io), batch=B, tokens=T,
+                    context=ctx)
+            _report(f"qkv_append ({name})", pus, 0,
+                    2 * B * T * (2 * H + 5 * G) * D,
+                    ("kv_append", aus, 0, 8 * B * T * G * D), batch=B,
+                    tokens=T)
+    # -- norms, convolutions, routing -------------------------------------------
+    W = 4096
+    for B, T in ((32, 1), (1, 4096)):
+        n, top = B * T, 2
+        x, d, wn = torch.randn(n, W, **dev), _bf(n, W), _bf(W)
+        d2, coef = _bf(n * top, W), torch.rand(n, top, **dev)
+        cw = sv.ShortConv(_bf(4, W), torch.zeros(B, 4, W, dtype=bf, **dev))
+        seg = _i32([(i, i * T, T, 64 if T == 1 else 0) for i in range(B)])
+        rows, _ = sv.chunk_table(seg.tolist())
+        batch = SimpleNamespace(portion_tokens=n if T > 1 else 0,
+                                portions=seg, chunks=_i32(rows),
+                                singles=seg if T == 1 else seg[:0])
+        xi, xo = _bf(n, inner + C)[:, inner:], _bf(n, inner)
+        big = sv.ShortConv(w, torch.zeros(B, taps, C, dtype=bf, **dev), b)
+        gw = _bf(inner)
+        z, bias, table = torch.randn(n, 64, **dev), _bf(64), _bf(32000, 1024)
+        gx, tok = _bf(n, 256), torch.randint(0, 32000, (n,)).int().cuda()
+        y, u = _bf(n, W), _bf(n, 14336)
+        t = _time([
+            _graphed(lambda: sv.residual_norm(x, sv.Pending(d), 1e-5, wn)),
+            _graphed(lambda: sv.residual_norm(x, sv.Pending(d), 1e-5, wn,
+                                              groups=8)),
+            _graphed(lambda: sv.residual_norm(
+                x, sv.Pending(d, w1=wn), 1e-5, wn, groups=8, conv=cw,
+                batch=batch)),
+            _graphed(lambda: sv.residual_norm(
+                x, sv.Pending(d2, coef=coef), 1e-5, copy=True, dtype=bf)),
+            _graphed(lambda: sv.gated_norm(xo, gw, None, 1024, 1e-5)),
+            _graphed(lambda: sv.gated_norm(y, wn, d, 128, 1e-5)),
+            _graphed(lambda: sv.moe_plan(
+                z, bias, sv.Routing(6, True, 8, 4), 0)),
+            _graphed(lambda: sv.moe_plan(z, bias, 6, 0)),
+            _graphed(lambda: sv.gelu_rows_(gx, table, tok, 256)),
+            _graphed(lambda: sv.gelu_tanh_(gx)),
+            _graphed(lambda: sv.gelu_tanh_(u))])
+        like = ("residual_norm", t[0], 0, 12 * n * W)
+        _report("residual_norm (groups)", t[1], 0, 12 * n * W, like, rows=n)
+        _report("residual_norm (output norm, groups, convolution)", t[2], 0,
+                (16 if T > 1 else 12 + 10) * n * W, like, rows=n)
+        _report("residual_norm (experts' sum)", t[3], 0,
+                (10 + 2 * top) * n * W, like, rows=n)
+        _report("gated_norm (no gate)", t[4], 0, 4 * n * inner,
+                ("gated_norm", t[5], 0, 6 * n * W), rows=n)
+        if T > 1:
+            (us,) = _time([_graphed(lambda: sv.short_conv(
+                xi, big, seg, batch.chunks, silu=True))])
+            _report("short_conv", us, 0, 4 * n * C,
+                    ("gelu_tanh", t[10], 0, 4 * n * 14336), rows=n, channels=C)
+        io = 4 * n * 64 + 12 * n * 6
+        _report("moe_plan (sigmoid, groups)", t[6], 0, io,
+                ("moe_plan", t[7], 0, io), rows=n, experts=64, top=6)
+        _report("gelu_rows", t[8], 0, 6 * n * 256,
+                ("gelu_tanh", t[9], 0, 4 * n * 256), rows=n)
+
+
+def bench_state_models():
+    for size in ("bench", "bench-fine"):
+        _state_models(size)
+        torch.cuda.empty_cache()
+
+
+def _state_models(size):
+    from neuronx_distributed_amd.inference import (InferenceEngine, StepEntry,
+                                                   single_process_groups)
+    from neuronx_distributed_amd.models import (build_model,
+                                                get_nesilorn_config,
+                                                get_sutuvik_config)
+
+    single_process_groups()
+    torch.manual_seed(0)
+    cfgs = {"Sutuvik": get_sutuvik_config(f"sutuvik-{size}"),
+            "Nesilorn": get_nesilorn_config(f"nesilorn-{size}")}
+    models = {n: build_model(n, c, torch.bfloat16, "cuda")
+              for n, c in cfgs.items()}
+    out = {f"{n.lower()}_b_params": round(
+        sum(p.numel() for p in m.parameters()) / 1e9, 2)
+        for n, m in models.items()}
+    print(json.dumps({"size": size, **out,
+                      "width": cfgs["Sutuvik"].hidden_size,
+                      "layers": len(cfgs["Sutuvik"].layers),
+                      "data": "random weights"}), flush=True)
+
+    def turns(fns, reps):
+        best = [math.inf] * len(fns)
+        for _ in range(reps):
+            for i, f in enumerate(fns):
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                f()
+                torch.cuda.synchronize()
+                best[i] = min(best[i], time.perf_counter() - t0)
+        return best
+
+    for B, T in ((1, 2048), (1, 4096), (4, 4096)):
+        rows = torch.randint(0, 32000, (B, T)).tolist()
+
+        def run(eng):
+            eng.step([StepEntry(b, rows[b], [T - 1]) for b in range(B)])
+            for b in range(B):
+                eng.finish(b)
+
+        engs = [InferenceEngine(m, max_tokens=B * T, max_seqs=B)
+                for m in models.values()]
+        best = turns([lambda e=e: run(e) for e in engs], 4)
+        print(json.dumps({"prefill": {"batch": B, "tokens": T},
+                          **{f"{n.lower()}_tokens_per_s": round(B * T / s)
+                             for n, s in zip(models, best)}}), flush=True)
+        del engs
+        torch.cuda.empty_cache()
+    for B, ctx in ((1, 2048), (32, 2048), (128, 2048)):
+        steps = 8
+        rows = torch.randint(0, 32000, (B, ctx)).tolist()
+        engs = [InferenceEngine(m, max_tokens=B * (ctx + 64), max_seqs=B,
+                                max_context=ctx + 64)
+                for m in models.values()]
+        for eng in engs:
+            for b in range(B):
+                eng.step([StepEntry(b, rows[b])])
+
+        def decode(eng):
+            tok = [1] * B
+            for _ in range(steps):
+                tok = eng.step([StepEntry(b, [tok[b]], [0]) for b in
+                                range(B)]).argmax(-1).tolist()
+
+        best = turns([lambda e=e: decode(e) for e in engs], 4)
+        print(json.dumps({
+            "decode": {"batch": B, "context": ctx},
+            **{f"{n.lower()}_ms": round(s / steps * 1e3, 3)
+               for n, s in zip(models, best)},
+            **{f"{n.lower()}_tokens_per_s": round(B * steps / s)
+               for n, s in zip(models, best)}}), flush=True)
+        del engs
+        torch.cuda.empty_cache()
+
+
 DESIGNS = {"voletar": (bench_kernels, bench_models),
-           "nesilorn": (bench_latent_kernels, bench_latent_models)}
+           "nesilorn": (bench_latent_kernels, bench_latent_models),
+           "sutuvik": (bench_state_kernels, bench_state_models)}
 
 
 def main(what="all", design="all"):

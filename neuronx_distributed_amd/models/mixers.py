@@ -159,7 +159,8 @@ class ScoredAttention(Mixer):
                              f"{sv.MAX_HEAD_DIM}")
         self.heads, self.scale, self.eps = heads, scale, eps
         self.rot, self.qk_norm = rot, qk_norm
-        self.q_temp = (q_temp["coef"], q_temp["every"]) if q_temp else (0., 0)
+        self.q_temp = (q_temp["coef"], int(q_temp["every"])) if q_temp \
+            else (0.0, 0)
         self.slopes, self.softcap = slopes, softcap or 0.0
         self.v_mix, self.gated = v_mix, gate
         self.kv = PagedKV(kv_heads, dim, vdim)

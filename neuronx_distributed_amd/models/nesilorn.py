@@ -83,6 +83,12 @@ NESILORN_CONFIGS = {
         embedding_scale=2.0,
         layers=_bench_layers(4, 32, 128, 64, 128, 512, 4096, 14336, 8, 2,
                              14336, 0)),
+    # of many small experts
+    "nesilorn-bench-fine": NesilornConfig(
+        vocab_size=32000, hidden_size=2048, norm_eps=1e-5,
+        embedding_scale=2.0,
+        layers=_bench_layers(4, 16, 128, 64, 128, 512, 4096, 14336, 64, 6,
+                             1408, 0)),
     "nesilorn-tiny": NesilornConfig(
         vocab_size=320, hidden_size=128, norm_eps=1e-5, embedding_scale=2.0,
         layers=_bench_layers(3, 2, 24, 16, 40, 48, 50, 160, 6, 2, 72)),

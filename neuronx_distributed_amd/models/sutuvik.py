@@ -114,6 +114,12 @@ SUTUVIK_CONFIGS = {
         conv_taps=4, side_dim=256, logit_scale=0.5,
         layers=_bench_layers(_ORDER, 128, 64, 128, 8, 32, 8, 128, 8, 2, 4, 2,
                              14336)),
+    # of many small experts in groups
+    "sutuvik-bench-fine": SutuvikConfig(
+        vocab_size=32000, hidden_size=2048, norm_eps=1e-5, norm_groups=8,
+        conv_taps=4, side_dim=128, logit_scale=0.5,
+        layers=_bench_layers(_ORDER, 64, 64, 128, 4, 16, 4, 128, 64, 6, 8, 3,
+                             1408)),
     "sutuvik-tiny": SutuvikConfig(
         vocab_size=320, hidden_size=128, norm_eps=1e-5, norm_groups=2,
         conv_taps=3, side_dim=16, logit_scale=0.5,

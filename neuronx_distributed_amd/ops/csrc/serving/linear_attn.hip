@@ -75,7 +75,8 @@ __device__ __forceinline__ void log_gates(const MemoryArgs& a, long row,
 // ---------------------------------------------------------------------------
 // token after token: a workgroup owns 32 columns of one head's state
 // ---------------------------------------------------------------------------
-template <typename T, int NI, int GATE, bool VEC>
+// TAPS: 0 no convolution, 1 any number of taps, else this number
+template <typename T, int NI, int GATE, bool VEC, int TAPS>
 __global__ void __launch_bounds__(256)
 memory_steps_kernel(MemoryArgs a) {
   const int D = a.D, E = a.E;
@@ -126,18 +127,36 @@ memory_steps_kernel(MemoryArgs a) {
   }
   const float decay = GATE == DECAY ? a.decay[h] : 0.f;
   const int hk = GATE == TIMED ? h / (a.H / a.G) : h;   // head of q and k
-  const bool conv = GATE == TIMED && a.cw;
-  // channel c of a single token after its convolution; `keep` writes the
-  // token's own input into the ring
+  constexpr bool conv = TAPS > 0;
+  // The convolution of a single token: channel c's filter and earlier inputs,
+  // and its result; `keep` writes the token's own input into the ring.
+  constexpr int NT = TAPS > 1 ? TAPS : 1;
+  const int last = (TAPS > 1 ? TAPS : a.taps) - 1;
+  const int here = conv ? ctx % (last + 1) : 0;
+  auto place = [&](int k) {              // of the input last - k tokens ago
+    const int i = here - last + k;
+    return (long)(i < 0 ? i + last + 1 : i) * a.C;
+  };
   auto convolve = [&](float x, int c, bool keep) {
-    const int last = a.taps - 1;
-    T* ring = (T*)a.ring + slot * a.taps * a.C + c;
+    T* ring = (T*)a.ring + slot * (last + 1) * a.C + c;
     const T* w = (const T*)a.cw + c;
-    float y = to_f(((const T*)a.cb)[c]) + to_f(w[(long)last * a.C]) * x;
-    for (int k = max(0, last - ctx); k < last; ++k)
-      y += to_f(w[(long)k * a.C]) *
-           to_f(ring[(long)((ctx - last + k) % a.taps) * a.C]);
-    if (keep) from_f(ring[(long)(ctx % a.taps) * a.C], x);
+    float y = to_f(((const T*)a.cb)[c]);
+    if (TAPS > 1) {
+      float f[NT], in[NT];
+#pragma unroll
+      for (int k = 0; k < NT; ++k) {
+        f[k] = to_f(w[(long)k * a.C]);
+        in[k] = k < NT - 1 ? to_f(ring[place(k)]) : x;
+      }
+#pragma unroll
+      for (int k = 0; k < NT; ++k)
+        y += k >= last - ctx ? f[k] * in[k] : 0.f;
+    } else {
+      for (int k = max(0, last - ctx); k < last; ++k)
+        y += to_f(w[(long)k * a.C]) * to_f(ring[place(k)]);
+      y += to_f(w[(long)last * a.C]) * x;
+    }
+    if (keep) from_f(ring[(long)here * a.C], x);
     return silu_f(y);
   };
 
@@ -253,11 +272,11 @@ memory_steps_kernel(MemoryArgs a) {
   }
 }
 
-template <typename T, int GATE>
+template <typename T, int GATE, int TAPS>
 static int launch_steps(const MemoryArgs& a, int n_seg, hipStream_t stream) {
   const long grid = (long)n_seg * a.H * ((a.E + 31) / 32);
   const bool vec = a.E % 4 == 0;
-#define MS(N, V) memory_steps_kernel<T, N, GATE, V><<<grid, 256, 0, stream>>>(a)
+#define MS(N, V) memory_steps_kernel<T, N, GATE, V, TAPS><<<grid, 256, 0, stream>>>(a)
 #define MSV(N) do { if (vec) MS(N, true); else MS(N, false); } while (0)
   if (a.D <= 64) MSV(2);
   else if (a.D <= 128) MSV(4);
@@ -272,12 +291,14 @@ static int launch_steps(const MemoryArgs& a, int n_seg, hipStream_t stream) {
 extern "C" int sv_memory_steps(const MemoryArgs* a, int n_seg, int gating,
                                int f32, hipStream_t stream) {
   if (n_seg <= 0) return 0;
-#define MS(T)                                                          \
-  (gating == GATED   ? launch_steps<T, GATED>(*a, n_seg, stream)       \
-   : gating == TIMED ? launch_steps<T, TIMED>(*a, n_seg, stream)       \
-                     : launch_steps<T, DECAY>(*a, n_seg, stream))
+#define MST(T, K) launch_steps<T, TIMED, K>(*a, n_seg, stream)
+#define MS(T)                                                            \
+  (gating == GATED   ? launch_steps<T, GATED, 0>(*a, n_seg, stream)      \
+   : gating == DECAY ? launch_steps<T, DECAY, 0>(*a, n_seg, stream)      \
+   : !a->cw ? MST(T, 0) : a->taps == 4 ? MST(T, 4) : MST(T, 1))
   return f32 ? MS(float) : MS(short);
 #undef MS
+#undef MST
 }
 
 

@@ -231,6 +231,13 @@ struct RowsArgs {
   ScoreArgs mod;
 };
 
+// tanh, in the 32-bit mode to the last digits, else to 1e-7
+__device__ __forceinline__ float tanh_t(float x, float) { return tanhf(x); }
+__device__ __forceinline__ float tanh_t(float x, short) {
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(
+                         1.f + __builtin_amdgcn_exp2f(2.f * SV_LOG2E * x));
+}
+
 // LPR lanes own one key row (DPL dims each); RC query heads share the row.
 template <bool VEC, int DPL, typename T>
 __device__ __forceinline__ void load_dims(const T* p, int n, float* v) {
@@ -238,8 +245,9 @@ __device__ __forceinline__ void load_dims(const T* p, int n, float* v) {
   for (int j = 0; j < DPL; j += 8) load8<VEC>(p + j, n - j, v + j);
 }
 
-template <typename T, int LPR, int RC, bool VEC, int DPL = 8>
-__global__ void __launch_bounds__(256)
+// MOD: scores and softmax as ScoreArgs say; without it they are plain.
+template <bool MOD, typename T, int LPR, int RC, bool VEC, int DPL = 8>
+__global__ void __launch_bounds__(256, RC <= 4 && DPL == 8 ? 4 : 1)
 attn_rows_kernel(RowsArgs a) {
   constexpr int NR = 64 / LPR;     // key rows of one wave step
   constexpr int DV = LPR * DPL;
@@ -267,15 +275,20 @@ attn_rows_kernel(RowsArgs a) {
     const int h = g * rep + min(rc * RC + r, rep - 1);
     load_dims<VEC, DPL>((const T*)a.q + row * a.qst + (long)h * D + d0, nd, qv[r]);
   }
-  // scores in units of log 2, of the cap if there is one
-  const float cap = a.mod.cap;
+  // scores in units of log 2; of the cap, if there is one
+  const float cap = MOD ? a.mod.cap : 0.f;
   const float s2 = cap > 0.f ? a.scale / cap : a.scale * SV_LOG2E;
   float slope[RC];
 #pragma unroll
   for (int r = 0; r < RC; ++r) {
-    const int h = g * rep + min(rc * RC + r, rep - 1);
-    const float t = a.mod.temp ? s2 * to_f(((const T*)a.mod.temp)[h]) : s2;
-    slope[r] = a.mod.slope ? a.mod.slope[h] * SV_LOG2E : 0.f;
+    float t = s2;
+    if (MOD) {
+      const int h = g * rep + min(rc * RC + r, rep - 1);
+      if (a.mod.temp) t *= to_f(((const T*)a.mod.temp)[h]);
+      // the same for all lanes: not in a vector register
+      slope[r] = __uint_as_float(__builtin_amdgcn_readfirstlane(__float_as_uint(
+          a.mod.slope ? a.mod.slope[h] * SV_LOG2E : 0.f)));
+    }
 #pragma unroll
     for (int j = 0; j < DPL; ++j) qv[r][j] *= t;
   }
@@ -327,12 +340,15 @@ attn_rows_kernel(RowsArgs a) {
     for (int off = LPR / 2; off > 0; off >>= 1)
 #pragma unroll
       for (int r = 0; r < RC; ++r) s[r] += __shfl_xor(s[r], off, 64);
-    if (cap > 0.f)
+    if (MOD) {
+      if (cap > 0.f)
 #pragma unroll
-      for (int r = 0; r < RC; ++r) s[r] = cap * SV_LOG2E * tanhf(s[r]);
+        for (int r = 0; r < RC; ++r) s[r] = cap * SV_LOG2E * tanh_t(s[r], T());
+#pragma unroll
+      for (int r = 0; r < RC; ++r) s[r] -= slope[r] * away;
+    }
 #pragma unroll
     for (int r = 0; r < RC; ++r) {
-      s[r] -= slope[r] * away;
       const float mn = live ? fmaxf(m[r], s[r]) : m[r];
       const float al = __builtin_amdgcn_exp2f(m[r] - mn);
       const float p = live ? __builtin_amdgcn_exp2f(s[r] - mn) : 0.f;
@@ -353,7 +369,8 @@ attn_rows_kernel(RowsArgs a) {
 #pragma unroll
     for (int j = 0; j < DPL; ++j) kx[j] = vx[j] = 0.f;
     if (idx + 4 * NR < k1) fetch(idx + 4 * NR, kx, vx);
-    absorb(kf, vf, idx < k1, i_pos - (idx < nfirst ? idx : lo + idx - nfirst));
+    absorb(kf, vf, idx < k1,
+           MOD ? i_pos - (idx < nfirst ? idx : lo + idx - nfirst) : 0);
 #pragma unroll
     for (int j = 0; j < DPL; ++j) {
       kf[j] = kx[j];
@@ -410,7 +427,7 @@ attn_rows_kernel(RowsArgs a) {
       oo += so[w][r][e] * c;
     }
     const int h = g * rep + rc * RC + r;
-    if (a.mod.sink && split == 0) {      // once for all splits
+    if (MOD && a.mod.sink && split == 0) {   // once for all splits
       const float sink = to_f(((const T*)a.mod.sink)[h]) * SV_LOG2E;
       const float mn = fmaxf(mm, sink);
       const float c = __builtin_amdgcn_exp2f(mm - mn);
@@ -418,7 +435,7 @@ attn_rows_kernel(RowsArgs a) {
       oo *= c;
       mm = mn;
     }
-    if (a.mod.gate)
+    if (MOD && a.mod.gate)
       oo *= sigmoid_f(to_f(((const T*)a.mod.gate)[row * a.mod.gst + h]));
     if (a.splits == 1) {
       from_f(((T*)a.out)[((long)row * a.H + h) * E + e], oo / ll);
@@ -495,7 +512,7 @@ extern "C" int sv_attn_merge(const float* part, void* out, long rows,
   return (int)hipGetLastError();
 }
 
-template <typename T>
+template <bool MOD, typename T>
 static int launch_rows(const RowsArgs& a, int vec, hipStream_t stream) {
   const int rep = a.H / a.G;
   const int big = a.D > a.E ? a.D : a.E;
@@ -504,7 +521,7 @@ static int launch_rows(const RowsArgs& a, int vec, hipStream_t stream) {
   const int nrc = (rep + rcn - 1) / rcn;
   const long grid = (long)a.rows * a.G * nrc * a.splits;
 #define AR(L, ...) \
-  attn_rows_kernel<T, L, __VA_ARGS__><<<grid, 256, 0, stream>>>(a)
+  attn_rows_kernel<MOD, T, L, __VA_ARGS__><<<grid, 256, 0, stream>>>(a)
 #define ARV(L, R) do { if (vec) AR(L, R, true); else AR(L, R, false); } while (0)
 #define ARR(L)                                                         \
   do {                                                                 \
@@ -515,7 +532,7 @@ static int launch_rows(const RowsArgs& a, int vec, hipStream_t stream) {
   else if (big <= 128) ARR(16);
   else if (big <= 256) ARR(32);
   else if (big <= 512) ARR(64);
-  else if (big <= 1024) {
+  else if (big <= 1024 && !MOD) {
     if (rcn == 2) { if (vec) AR(64, 2, true, 16); else AR(64, 2, false, 16); }
     else { if (vec) AR(64, 1, true, 16); else AR(64, 1, false, 16); }
   } else return 1;
@@ -531,8 +548,13 @@ static int launch_rows(const RowsArgs& a, int vec, hipStream_t stream) {
 extern "C" int sv_attn_rows(const RowsArgs* a, int vec, int f32,
                             hipStream_t stream) {
   if (a->rows <= 0) return 0;
-  return f32 ? launch_rows<float>(*a, vec, stream)
-             : launch_rows<short>(*a, vec, stream);
+  const ScoreArgs& m = a->mod;
+  const bool mod = m.temp || m.sink || m.slope || m.gate || m.cap > 0.f;
+  if (f32)
+    return mod ? launch_rows<true, float>(*a, vec, stream)
+               : launch_rows<false, float>(*a, vec, stream);
+  return mod ? launch_rows<true, short>(*a, vec, stream)
+             : launch_rows<false, short>(*a, vec, stream);
 }
 
 // ---------------------------------------------------------------------------
