@@ -188,7 +188,7 @@ def _pages(lens, G, D, E, dtype, spare=2):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,G,D,E,dims,kind", [
-    (4, 2, 48, 32, 16, "weighted"), (3, 1, 11, 10, 10, "weighted"),
+    (4, 2, 56, 32, 16, "weighted"), (3, 1, 11, 10, 10, "weighted"),
     (2, 2, 128, 64, 128, "plain"), (2, 1, 200, 16, 64, "plain"),
     (5, 1, 40, 320, 0, None)])
 def test_prepared_queries_and_keys(dtype, H, G, D, E, dims, kind):
@@ -249,7 +249,7 @@ MODS = {
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("kind", list(MODS))
-@pytest.mark.parametrize("H,G,D,E", [(4, 2, 48, 32), (3, 1, 11, 10),
+@pytest.mark.parametrize("H,G,D,E", [(4, 2, 56, 32), (3, 1, 11, 10),
                                      (8, 1, 128, 48), (2, 2, 64, 200),
                                      (6, 2, 160, 96)])
 def test_modified_scores(dtype, kind, H, G, D, E):
@@ -369,7 +369,7 @@ def _ssm_want(case, params, H, G, N, P):
     return y.reshape(T, H * P) * so.silu(z), S
 
 
-SIZES = [(4, 2, 32, 48), (3, 1, 13, 7), (2, 1, 128, 64), (4, 1, 64, 136),
+SIZES = [(4, 2, 40, 56), (3, 1, 13, 7), (2, 1, 128, 64), (4, 1, 64, 136),
          (2, 2, 200, 16), (2, 1, 300, 40)]
 
 
@@ -448,7 +448,7 @@ def test_an_old_input_is_still_in_the_state(dtype):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("taps", [1, 2, 4, 9])
-@pytest.mark.parametrize("H,G,N,P", [(4, 2, 32, 48), (3, 1, 13, 7),
+@pytest.mark.parametrize("H,G,N,P", [(4, 2, 40, 56), (3, 1, 13, 7),
                                      (4, 4, 136, 40)])
 def test_convolution_fused_into_single_tokens(dtype, taps, H, G, N, P):
     """Decoding from the first token, and after a portion, with q, k and v
@@ -496,7 +496,7 @@ def test_convolution_fused_into_single_tokens(dtype, taps, H, G, N, P):
 
 @pytest.mark.parametrize("T", [1, 30, 200])
 @pytest.mark.parametrize("E,top,groups,keep", [
-    (12, 2, 2, 1), (12, 3, 4, 3), (7, 2, 7, 3), (9, 4, 1, 1), (64, 6, 8, 4),
+    (14, 2, 2, 1), (20, 3, 4, 3), (7, 2, 7, 3), (9, 4, 1, 1), (64, 6, 8, 4),
     (256, 8, 8, 4), (512, 10, 64, 5), (6, 6, 2, 2)])
 def test_group_limited_routing(T, E, top, groups, keep):
     """Chosen experts and weights; corrections push choice scores below zero,
