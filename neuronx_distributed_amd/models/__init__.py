@@ -9,5 +9,7 @@ from .nesilorn import (NesilornConfig, NesilornForCausalLM, NESILORN_CONFIGS,
                        get_nesilorn_config)
 from .sutuvik import (SutuvikConfig, SutuvikForCausalLM, SUTUVIK_CONFIGS,
                       get_sutuvik_config)
+from .pokepel import (PokepelConfig, PokepelForCausalLM, POKEPEL_CONFIGS,
+                      get_pokepel_config)
 from .registry import (ModelEntry, build_model, load_pretrained,
                        register_model, registered_models)

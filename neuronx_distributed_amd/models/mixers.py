@@ -66,22 +66,22 @@ class CheckpointReader:
                            f"{sorted(extra)[:5]}")
 
 
-class Mixer(nn.Module):
-    """``names`` are the checkpoint names of the projections in the order in
+class Projected(nn.Module):
+    """What reads projections of the layer's rows that one product makes.
+    ``names`` are the checkpoint names of the projections in the order in
     which they are stacked, ``sizes`` their widths."""
-    names: Sequence[str]
-    sizes: Sequence[int]
+    names: Sequence[str] = ()
+    sizes: Sequence[int] = ()
     padding = 0         # rows of zeros behind the projections
 
-    def cache_specs(self) -> list:
-        raise NotImplementedError
-
-    def stacked(self, get, prefix) -> torch.Tensor:
+    def stacked(self, get, prefix) -> Optional[torch.Tensor]:
         parts = [get(prefix + n) for n in self.names]
         for p, n, s in zip(parts, self.names, self.sizes):
             if p.shape[0] != s:
                 raise ValueError(f"{prefix}{n} has {p.shape[0]} rows, "
                                  f"expected {s}")
+        if not parts:
+            return None
         if self.padding:
             parts.append(parts[0].new_zeros(self.padding, parts[0].shape[1]))
         return torch.cat(parts)
@@ -92,6 +92,13 @@ class Mixer(nn.Module):
             out.append(proj[:, at:at + s])
             at += s
         return out
+
+
+class Mixer(Projected):
+    """Mixes the rows of a request; keeps something between steps."""
+
+    def cache_specs(self) -> list:
+        raise NotImplementedError
 
 
 class SlidingAttention(Mixer):
@@ -234,15 +241,28 @@ def alibi_slopes(heads: int) -> List[float]:
     return [2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)]
 
 
+def rotation(base, dims, scaling, device):
+    """Frequencies, scaled as YaRN does or plain, and their amplitude."""
+    if scaling:
+        return sv.yarn_frequencies(base, dims, device, scaling)
+    return sv.rotary_frequencies(base, dims, device), 1.0
+
+
 class LatentAttention(Mixer):
     """Softmax attention whose keys and values are projections of a small
     latent, which alone is cached beside one rotated key part that all heads
     share; a sliding window (0: plain causal) and a sigmoid gate on the
-    heads.  Every query head is [unrotated | rotated]."""
+    heads.  Every query head is [unrotated | rotated].
+
+    pairs      neighbours turn together, not element i and i + rot_dims / 2
+    scaling    of the rotation, see ``serving.yarn_frequencies``
+    sink       a learned score a head joins the denominator
+    """
     names = ("q", "dkv", "g")
 
     def __init__(self, width, heads, dim, rot_dim, vdim, rank, scale,
-                 rot_base, rot_dims, eps, window=0):
+                 rot_base, rot_dims, eps, window=0, pairs=False, scaling=None,
+                 sink=False):
         super().__init__()
         if rot_dims % 2 or not 0 <= rot_dims <= rot_dim:
             raise ValueError(f"{rot_dims} of {rot_dim} dimensions turn")
@@ -252,6 +272,7 @@ class LatentAttention(Mixer):
         self.heads, self.dim, self.vdim = heads, dim, vdim
         self.rank, self.scale, self.eps = rank, scale, eps
         self.rot_base, self.rot_dims = rot_base, rot_dims
+        self.pairs, self.scaling = pairs, scaling
         self.window = window
         self.latent = PagedLatent(rank, rot_dim, window)
         self.sizes = (heads * (dim + rot_dim), rank + rot_dim, heads * vdim)
@@ -261,7 +282,8 @@ class LatentAttention(Mixer):
             torch.randn(heads, rank, dim) * rank ** -0.5)
         self.expand = nn.Parameter(
             torch.randn(heads * (dim + vdim), rank) * rank ** -0.5)
-        self._freq = None
+        self.sink = nn.Parameter(torch.zeros(heads)) if sink else None
+        self._turn = None
         self.o = _row(heads * vdim, width)
 
     def cache_specs(self):
@@ -273,14 +295,17 @@ class LatentAttention(Mixer):
         copy_weight(self.expand, torch.cat([uk, get(prefix + "uv")]))
         copy_weight(self.absorb, uk.view(self.heads, self.dim, self.rank)
                     .transpose(1, 2))
+        if self.sink is not None:
+            copy_weight(self.sink, get(prefix + "sink"))
         copy_weight(self.o.weight, get(prefix + "o"))
 
     def forward(self, h, proj, batch, pools):
         q, kv, g = self.split(proj)
-        if self._freq is None or self._freq.device != h.device:
-            self._freq = sv.rotary_frequencies(self.rot_base, self.rot_dims,
-                                               h.device)
-        w = sv.LatentWeights(self.norm, self.absorb, self.expand, self._freq)
+        if self._turn is None or self._turn[0].device != h.device:
+            self._turn = rotation(self.rot_base, self.rot_dims, self.scaling,
+                                  h.device)
+        w = sv.LatentWeights(self.norm, self.absorb, self.expand, *self._turn,
+                             self.pairs, self.sink)
         return self.o(sv.latent_attention(
             q, kv, g, batch, pools[0], w, self.heads, self.dim, self.vdim,
             self.scale, self.eps, self.window))
@@ -290,6 +315,8 @@ class _MatrixMemory(Mixer):
     """A recurrent matrix state per head, a group-normed and gated output."""
     names = ("q", "k", "v", "g")
     normalized = False
+    weighted = True       # the norm
+    silu_gate = False     # instead of a sigmoid
 
     def __init__(self, width, heads, dim, vdim, eps, norm_group):
         super().__init__()
@@ -297,14 +324,15 @@ class _MatrixMemory(Mixer):
         self.norm_group = norm_group
         self.state = MatrixState(heads, dim, vdim, self.normalized)
         self.sizes = (heads * dim, heads * dim, heads * vdim, heads * vdim)
-        self.norm = _vector(heads * vdim)
+        self.norm = _vector(heads * vdim) if self.weighted else None
         self.o = _row(heads * vdim, width)
 
     def cache_specs(self):
         return [self.state]
 
     def load(self, get, prefix):
-        copy_weight(self.norm, get(prefix + "norm"))
+        if self.weighted:
+            copy_weight(self.norm, get(prefix + "norm"))
         copy_weight(self.o.weight, get(prefix + "o"))
 
     def gate(self, h):
@@ -323,7 +351,7 @@ class _MatrixMemory(Mixer):
             sv.memory_mix(q, k, v, gate, S, n, m, batch.singles, self.heads,
                           out=out)
         return self.o(sv.gated_norm(out, self.norm, g, self.norm_group,
-                                    self.eps))
+                                    self.eps, self.silu_gate))
 
 
 class DecayMemory(_MatrixMemory):
@@ -342,6 +370,55 @@ class DecayMemory(_MatrixMemory):
         if self._gate is None or self._gate.decay.device != h.device:
             self._gate = sv.decay_gate(self.decay, h.device)
         return self._gate
+
+
+class Retention(_MatrixMemory):
+    """Linear attention with a fixed decay per head on rotated queries and keys
+    (element i turns with i + dims / 2; keys times dim^-1/2); every head is
+    normed on its own, without a weight, and gated by silu."""
+    weighted, silu_gate = False, True
+
+    def __init__(self, width, heads, dim, vdim, decay, eps, rot_base,
+                 rot_dims, scaling=None):
+        super().__init__(width, heads, dim, vdim, eps, norm_group=vdim)
+        if len(decay) != heads:
+            raise ValueError("one decay per head")
+        if rot_dims % 2 or not 0 <= rot_dims <= dim:
+            raise ValueError(f"{rot_dims} of {dim} dimensions turn")
+        if dim > sv.MAX_HEAD_DIM:
+            raise ValueError(f"key size {dim} > {sv.MAX_HEAD_DIM}")
+        self.decay = [float(d) for d in decay]
+        self.rot = rot_base, rot_dims, scaling
+        self._gate = None
+
+    def gate(self, h):
+        if self._gate is None or self._gate.decay.device != h.device:
+            d = sv.decay_gate(self.decay, h.device)
+            self._gate = sv.TurnGate(d.decay, d.log2_decay, self.dim ** -0.5,
+                                     *rotation(*self.rot, h.device))
+        return self._gate
+
+    def forward(self, h, proj, batch, pools):
+        q, k, v, g = self.split(proj)
+        S, gate = pools[0][0], self.gate(h)
+        n, T = batch.portion_tokens, h.shape[0]
+        out = torch.empty(T, self.heads * self.vdim, dtype=h.dtype,
+                          device=h.device)
+        done = 0          # rows that are normed and gated
+        if n:
+            if gate.norm_fits(h.dtype, self.dim, self.vdim, q, k, v, g):
+                done = n
+            sv.memory_mix(q[:n], k[:n], v[:n], gate, S, None, None,
+                          batch.portions, self.heads, batch.chunks,
+                          batch.chunk_first, out=out[:n],
+                          silu_gate=g[:n] if done else None, eps=self.eps)
+        if n < T:
+            sv.memory_mix(q, k, v, gate, S, None, None, batch.singles,
+                          self.heads, out=out)
+        if done < T:
+            sv.gated_norm(out[done:], None, g[done:], self.vdim, self.eps,
+                          True, out=out[done:])
+        return self.o(out)
 
 
 class GatedMemory(_MatrixMemory):
@@ -505,6 +582,81 @@ class ParallelMixer(nn.Module):
             self.left_out, self.right_out, self.branch_scale)
 
 
+class GatedParallel(nn.Module):
+    """A mixer and a feed-forward (or none) side by side on the same rows h,
+    each result times sigmoid(W h + b) of its own.  One product makes the
+    projections of both and the gates; the results are left pending."""
+
+    def __init__(self, width, mixer: Mixer, mlp: Optional[Projected] = None):
+        super().__init__()
+        self.mixer, self.mlp = mixer, mlp
+        self.bias1 = nn.Parameter(torch.zeros(width))
+        if mlp is not None:
+            self.bias2 = nn.Parameter(torch.zeros(width))
+        sizes = [sum(mixer.sizes) + mixer.padding, width]
+        if mlp is not None:
+            sizes += [sum(mlp.sizes) + mlp.padding, width]
+        # every part starts at a 16-byte word
+        self.at, n = [], 0
+        for s in sizes:
+            self.at.append((n, n + s))
+            n += s + -s % 8
+        self.proj = _column(width, n)
+
+    def cache_specs(self) -> List:
+        return self.mixer.cache_specs()
+
+    def load(self, get, prefix):
+        w = torch.zeros_like(self.proj.weight)
+        parts = [self.mixer.stacked(get, prefix + "mix."),
+                 get(prefix + "rg1")]
+        copy_weight(self.bias1, get(prefix + "rg1.b"))
+        self.mixer.load(get, prefix + "mix.")
+        if self.mlp is not None:
+            parts += [self.mlp.stacked(get, prefix + "mlp."),
+                      get(prefix + "rg2")]
+            copy_weight(self.bias2, get(prefix + "rg2.b"))
+            self.mlp.load(get, prefix + "mlp.")
+        else:
+            get.skip(prefix + "rg2")
+            get.skip(prefix + "rg2.b")
+        for (a, b), part in zip(self.at, parts):
+            if part is not None:
+                copy_weight(w[a:b], part)
+        copy_weight(self.proj.weight, w)
+
+    def forward(self, h, batch, pools) -> sv.Pending:
+        proj = self.proj(h)
+        mix, gate1, *rest = [proj[:, a:b] for a, b in self.at]
+        branches = [sv.Branch(self.mixer(h, mix, batch, pools), gate=gate1,
+                              bias=self.bias1)]
+        if self.mlp is not None:
+            y = self.mlp(h, rest[0])
+            y.gate, y.bias = rest[1], self.bias2
+            branches.append(y)
+        return sv.Pending(branches=branches)
+
+
+class PolyNormMLP(Projected):
+    """down(a N(z) + b N(z^2) + c N(z^3) + e) of z = up h, where powers are
+    taken element by element and N divides a row by its root mean square."""
+    names = ("up",)
+
+    def __init__(self, width, ff, eps):
+        super().__init__()
+        self.sizes, self.eps = (ff,), eps
+        self.act = nn.Parameter(torch.tensor([1.0, 0.0, 0.0, 0.0]))
+        self.down = _row(ff, width)
+
+    def load(self, get, prefix):
+        copy_weight(self.act, get(prefix + "act"))
+        copy_weight(self.down.weight, get(prefix + "down"))
+
+    def forward(self, h, proj) -> sv.Branch:
+        return sv.Branch(self.down(sv.poly_norm(self.split(proj)[0], self.act,
+                                                self.eps)))
+
+
 class _PlainMLP(nn.Module):
     """down(act(up x))"""
     act = None
@@ -531,13 +683,14 @@ class GeluMLP(_PlainMLP):
 
 
 class ExpertsMLP(nn.Module):
-    """A router with a bias and gated experts: min(g, limit) sigmoid(alpha g)
-    (clamp(u, limit) + shift); the chosen experts are summed, weighted as
-    ``routing`` (or the plain routing, if it is a number of experts) says.  The
-    sum is left pending, so it fuses into the next residual norm."""
+    """A router with a bias (``bias_name`` None: without) and gated experts:
+    min(g, limit) sigmoid(alpha g) (clamp(u, limit) + shift); the chosen experts
+    are summed, weighted as ``routing`` (or the plain routing, if it is a number
+    of experts) says.  The sum is left pending, so it fuses into the next
+    residual norm."""
 
     def __init__(self, width, ff, experts, routing, limit=math.inf, alpha=1.0,
-                 shift=0.0, bias_name="router.b"):
+                 shift=0.0, bias_name: Optional[str] = "router.b"):
         super().__init__()
         self.routing = sv.Routing(routing) if isinstance(routing, int) \
             else routing
@@ -545,7 +698,7 @@ class ExpertsMLP(nn.Module):
         self.act, self.bias_name = (alpha, limit, shift), bias_name
         self.router = nn.Parameter(
             torch.randn(experts, width) * width ** -0.5)
-        self.bias = nn.Parameter(torch.zeros(experts))
+        self.bias = nn.Parameter(torch.zeros(experts)) if bias_name else None
         self.gate_up = nn.Parameter(torch.empty(experts, 2 * ff, width))
         self.down = nn.Parameter(torch.empty(experts, width, ff))
         nn.init.normal_(self.gate_up, std=width ** -0.5)
@@ -553,7 +706,8 @@ class ExpertsMLP(nn.Module):
 
     def load(self, get, prefix):
         copy_weight(self.router, get(prefix + "router"))
-        copy_weight(self.bias, get(prefix + self.bias_name))
+        if self.bias is not None:
+            copy_weight(self.bias, get(prefix + self.bias_name))
         for e, (gu, down) in enumerate(zip(self.gate_up, self.down)):
             p = f"{prefix}e{e}."
             copy_weight(gu, torch.cat([get(p + "gate"), get(p + "up")]))
@@ -562,6 +716,29 @@ class ExpertsMLP(nn.Module):
     def forward(self, h) -> sv.Pending:
         return sv.moe_mlp(h, sv.linear_f32(h, self.router), self.bias,
                           self.gate_up, self.down, self.routing, *self.act)
+
+
+class SharedExpertsMLP(Projected):
+    """Experts beside one (of ``shared_ff``, 0: none) that every row uses, whose
+    projections come with the layer's."""
+
+    def __init__(self, width, experts: ExpertsMLP, shared_ff=0):
+        super().__init__()
+        self.experts = experts
+        if shared_ff:
+            self.names = ("shared.gate", "shared.up")
+            self.sizes = (shared_ff, shared_ff)
+            self.down = _row(shared_ff, width)
+
+    def load(self, get, prefix):
+        self.experts.load(get, prefix)
+        if self.sizes:
+            copy_weight(self.down.weight, get(prefix + "shared.down"))
+
+    def forward(self, h, proj) -> sv.Branch:
+        y = self.experts(h)
+        plus = self.down(sv.silu_mul(proj)) if self.sizes else None
+        return sv.Branch(y.delta, y.coef, plus)
 
 
 class TokenSide(nn.Module):

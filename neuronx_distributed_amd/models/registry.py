@@ -176,3 +176,20 @@ def _sutuvik_build(config):
 register_model("Sutuvik", ModelEntry(
     _sutuvik_config, _sutuvik_build,
     lambda model, tensors: model.load_checkpoint(tensors)))
+
+
+def _pokepel_config(d: dict):
+    from .pokepel import PokepelConfig
+
+    return PokepelConfig.from_dict(d)
+
+
+def _pokepel_build(config):
+    from .pokepel import PokepelForCausalLM
+
+    return PokepelForCausalLM(config)
+
+
+register_model("Pokepel", ModelEntry(
+    _pokepel_config, _pokepel_build,
+    lambda model, tensors: model.load_checkpoint(tensors)))

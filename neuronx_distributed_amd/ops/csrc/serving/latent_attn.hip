@@ -14,6 +14,8 @@
 //   sv_head_linear    a small matrix per head (absorption, values), with an
 //                     optional sigmoid gate on the result
 //   sv_latent_rows    MFMA attention of one absorbed query row over its keys
+//
+// The denominator of the softmax may hold a sink, a number a head.
 
 #include "serving.h"
 
@@ -35,6 +37,8 @@ struct LatentAppendArgs {
   const int *pos, *seq, *bt;
   int MB, H, R, P, rot;     // rot <= P columns turn, the rest pass
   float eps;
+  float amp;                // multiplies cos and sin
+  int pairs;                // columns 2i and 2i + 1 turn, not i and i + rot / 2
 };
 
 template <typename T>
@@ -45,7 +49,12 @@ latent_append_kernel(LatentAppendArgs a) {
   const int t = blockIdx.x, tid = threadIdx.x;
   const int half = a.rot / 2, R = a.R, P = a.P;
   const int p = a.pos[t];
-  for (int i = tid; i < half; i += 256) turn(a.freq[i], p, cs + i, cs + half + i);
+  for (int i = tid; i < half; i += 256) {
+    float c, s;
+    turn(a.freq[i], p, &c, &s);
+    cs[i] = c * a.amp;
+    cs[half + i] = s * a.amp;
+  }
   const T* kv = (const T*)a.kv + t * a.kvst;
   float sq = 0.f;
   for (int i = tid; i < R; i += 256) {
@@ -62,9 +71,10 @@ latent_append_kernel(LatentAppendArgs a) {
   auto rotate = [&](const T* src, T* dst, int i) {   // i in [0, P - half)
     if (i < half) {
       const float c = cs[i], s = cs[half + i];
-      const float x = to_f(src[i]), y = to_f(src[i + half]);
-      from_f(dst[i], x * c - y * s);
-      from_f(dst[i + half], y * c + x * s);
+      const int u = a.pairs ? 2 * i : i, w = a.pairs ? u + 1 : i + half;
+      const float x = to_f(src[u]), y = to_f(src[w]);
+      from_f(dst[u], x * c - y * s);
+      from_f(dst[w], y * c + x * s);
     } else {
       dst[i + half] = src[i + half];
     }
@@ -241,6 +251,7 @@ struct LatentRowsArgs {
   short* out;               // [rows][H][R]
   int MB, rows, H, R, P, splits, window;
   float scale;
+  const short* sink;        // [H] or null
 };
 
 template <int EP>
@@ -308,6 +319,10 @@ latent_rows_kernel(LatentRowsArgs a) {
   f32x16 o[NB] = {};
   const int sh = tid >> 3, sk = tid & 7;   // softmax: head, 4-key group
   float m_run = NEG_BIG, l_run = 0.f;
+  if (a.sink && split == 0 && h0 + sh < a.H) {   // once for all splits
+    m_run = bits2f(a.sink[h0 + sh]) * SV_LOG2E;
+    l_run = 1.f;
+  }
   const float s2 = a.scale * SV_LOG2E;
   // transposing reads: a group of 16 lanes turns 4 keys x 16 columns
   const int tr_key = (lane & 15) >> 2, tr_col = ((lane >> 4) & 1) * 16 + (lane & 3) * 4;

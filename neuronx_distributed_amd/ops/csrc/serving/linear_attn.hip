@@ -3,7 +3,7 @@
 //   S_t = a_t S_(t-1) + b_t k_t v_t^T,    o_t = S_t^T q_t
 //
 // per head, with a 32-bit state S [D][E] per (slot, head) that lives across
-// steps.  Three gatings share the kernels:
+// steps.  Four gatings share the kernels:
 //
 //   decay  a_t = decay_h, b_t = 1; q, k and v pass through silu.
 //   gated  log gates i, f from a projection, soft-capped:
@@ -17,6 +17,8 @@
 //            b_t = softplus(x + bias), a_t = exp(-exp(A_log) b_t),
 //          heads share q and k in groups, o_t + skip v_t is multiplied by
 //          silu(z).
+//   turned a_t = decay_h, b_t = kscale; q and k are rotated at their position,
+//          in halves: elements i and i + rot / 2 turn together.
 //
 //   sv_memory_steps   token after token; single-token decoding, the 32-bit
 //                     mode and sizes the chunk kernels do not take
@@ -32,7 +34,7 @@
 
 #define GATED_EPS 1e-6f
 
-enum Gating { DECAY = 0, GATED = 1, TIMED = 2 };
+enum Gating { DECAY = 0, GATED = 1, TIMED = 2, TURNED = 3 };
 
 struct MemoryArgs {
   const void *q, *k, *v;    // first row of the step's projections
@@ -40,8 +42,8 @@ struct MemoryArgs {
   const float* gates;       // [T][2 H] raw i then f (gated); [T][H] (timed)
   const void *ib, *fb;      // [H] biases, T: of i and f (gated); of the time
                             //   step, and A_log (timed)
-  const float* decay;       // [H] (decay)
-  const float* log2_decay;  // [H] (decay)
+  const float* decay;       // [H] (decay, turned)
+  const float* log2_decay;  // [H] (decay, turned)
   float* S;                 // [slots][H][D][E]
   float* n;                 // [slots][H][ceil(E / 32)][D] (gated)
   float* m;                 // [slots][H][ceil(E / 32)] (gated)
@@ -58,6 +60,10 @@ struct MemoryArgs {
   const void *cw, *cb;      // [taps][C], [C]; cw null: they have passed it
   void* ring;               // [slots][taps][C]: position p in place p % taps
   int taps, C, kch, qch;    // channels of v, k, q start at 0, kch, qch
+  // turned only
+  const double* freq;       // [rot / 2] radians a position
+  int rot;
+  float amp, kscale;        // cos and sin are multiplied by amp
 };
 
 __device__ __forceinline__ float softplus_f(float x) {
@@ -121,11 +127,12 @@ memory_steps_kernel(MemoryArgs a) {
     }
     if (ctx > 0) m = a.m[(slot * a.H + h) * nt + vt];
   }
-  if (GATE != DECAY) {
+  constexpr bool fixed = GATE == DECAY || GATE == TURNED;
+  if (!fixed) {
     ib = to_f(((const T*)a.ib)[h]);
     fb = to_f(((const T*)a.fb)[h]);
   }
-  const float decay = GATE == DECAY ? a.decay[h] : 0.f;
+  const float decay = fixed ? a.decay[h] : 0.f;
   const int hk = GATE == TIMED ? h / (a.H / a.G) : h;   // head of q and k
   constexpr bool conv = TAPS > 0;
   // The convolution of a single token: channel c's filter and earlier inputs,
@@ -169,6 +176,19 @@ memory_steps_kernel(MemoryArgs a) {
         x = to_f(((const T*)a.q)[row * a.qst + (long)hk * D + d]);
         y = to_f(((const T*)a.k)[row * a.kst + (long)hk * D + d]);
         if (GATE == GATED) x *= a.qscale;
+        if (GATE == TURNED && d < a.rot) {
+          const int half = a.rot / 2;
+          const bool low = d < half;
+          const int i = low ? d : d - half;
+          const long o = (long)hk * D + (low ? d + half : i);
+          float c, s;
+          turn(a.freq[i], ctx + t, &c, &s);
+          c *= a.amp;
+          s *= low ? -a.amp : a.amp;
+          x = x * c + to_f(((const T*)a.q)[row * a.qst + o]) * s;
+          y = y * c + to_f(((const T*)a.k)[row * a.kst + o]) * s;
+        }
+        if (GATE == TURNED) y *= a.kscale;
         if (GATE == DECAY) { x = silu_f(x); y = silu_f(y); }
         if (conv) {
           const bool keep = vt == 0 && h % (a.H / a.G) == 0;
@@ -295,7 +315,9 @@ extern "C" int sv_memory_steps(const MemoryArgs* a, int n_seg, int gating,
 #define MS(T)                                                            \
   (gating == GATED   ? launch_steps<T, GATED, 0>(*a, n_seg, stream)      \
    : gating == DECAY ? launch_steps<T, DECAY, 0>(*a, n_seg, stream)      \
+   : gating == TURNED ? launch_steps<T, TURNED, 0>(*a, n_seg, stream)    \
    : !a->cw ? MST(T, 0) : a->taps == 4 ? MST(T, 4) : MST(T, 1))
+  if (gating == TURNED && (a->rot % 2 || a->rot > a->D)) return 1;
   return f32 ? MS(float) : MS(short);
 #undef MS
 #undef MST
@@ -319,12 +341,14 @@ extern "C" int sv_memory_steps(const MemoryArgs* a, int n_seg, int gating,
 //                  + sum_(s<=t) e^(b_t - b_s + i_s - m_t) (q_t . k_s) v_s
 //
 // every exponent is <= 0.  b is kept per 64 tokens (with the four totals of
-// a chunk), so near tokens never cancel large sums.  The plain decay has
+// a chunk), so near tokens never cancel large sums.  The fixed decays have
 // e^(b_t - b_s + i_s - m_t) = decay^(t-s) and no m; the timed gating has
 // e^(b_t - b_s) times the time step of s, and no m.
 //
 // 32-bit operands meet bf16 ones exactly: an f32 value is split into three
 // bf16 planes (8 + 8 + 8 bits) and each plane is multiplied on its own.
+// Rotated queries and keys are split into two planes (a rest below 2^-17);
+// where two split values meet, products below 2^-24 are left out.
 // Scores are produced transposed (lane = query), so they feed the next
 // product as its B operand from registers: the accumulator's row order is
 // the contraction order, and V^T is read from LDS in that same order.
@@ -345,8 +369,20 @@ struct ChunkArgs {
   short* P;                 // [n_chunks][H][3][E][D] state before the chunk
   float* mst;               // [n_chunks][H] m before the chunk (gated)
   short* VT;                // [n_chunks][H][E][256] V^T, activated
-  short* KA;                // [T][H][D] activated K (decay)
+  short* KA;                // [T][H][D] activated K (decay); two planes of
+                            //   rotated K (turned)
+  short* QA;                // two planes of rotated Q (turned)
+  float norm_eps;           // turned, with z: every head over its root mean
+                            //   square, times silu(z)
 };
+
+__host__ __device__ constexpr bool fixed_decay(int gate) {
+  return gate == DECAY || gate == TURNED;
+}
+// planes of queries and keys
+__host__ __device__ constexpr int qk_planes(int gate) {
+  return gate == TURNED ? 2 : 1;
+}
 
 // split a pair of floats into three planes of packed bf16
 __device__ __forceinline__ void split3(float x, float y, uint* w) {
@@ -425,10 +461,74 @@ memory_gates_kernel(ChunkArgs x) {
   if (GATE == GATED && t == MC_L - 1) x.cend[ci] = c;
 }
 
+// ---- rotation: one workgroup per token, q and k of all heads into planes ---
+template <bool VEC>
+__global__ void __launch_bounds__(256) memory_turn_kernel(ChunkArgs x) {
+  extern __shared__ float cs[];          // cos [rot / 2], sin [rot / 2]
+  const MemoryArgs& a = x.a;
+  const int ch = blockIdx.x / MC_L, t = blockIdx.x % MC_L;
+  if (t >= x.chunks[4 * ch + 2]) return;
+  const long row = x.chunks[4 * ch + 1] + t;
+  const int* sg = a.seg + 4L * x.chunks[4 * ch];
+  const int p = sg[3] + (int)row - sg[1];
+  const int half = a.rot / 2, D = a.D;
+  for (int i = threadIdx.x; i < half; i += 256) {
+    float c, s;
+    turn(a.freq[i], p, &c, &s);
+    cs[i] = c * a.amp;
+    cs[half + i] = s * a.amp;
+  }
+  __syncthreads();
+  const long HD = (long)a.H * D, plane = (long)x.T * HD;
+  constexpr int V = VEC ? 8 : 1;
+  const int items = (D - half) / V;      // of a head: pairs, then the rest
+  auto get = [&](const short* s, float* v) {
+    if (VEC) unpack8(*(const uint4v*)s, v); else v[0] = bits2f(s[0]);
+  };
+  auto put = [&](short* d, const float* v) {
+    if (VEC) {
+      uint4v w0, w1;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float u = v[2 * j % V], w = v[(2 * j + 1) % V];
+        w0[j] = pack_bf16x2(u, w);
+        w1[j] = pack_bf16x2(u - __uint_as_float(w0[j] << 16),
+                            w - __uint_as_float(w0[j] & 0xffff0000u));
+      }
+      *(uint4v*)d = w0;
+      *(uint4v*)(d + plane) = w1;
+    } else {
+      d[0] = f2bits(v[0]);
+      d[plane] = f2bits(v[0] - bits2f(d[0]));
+    }
+  };
+  for (int it = threadIdx.x; it < 2 * a.H * items; it += 256) {
+    const int h = it / items % a.H, i = it % items * V;
+    const bool key = it >= a.H * items;
+    const short* src = (key ? (const short*)a.k + row * a.kst
+                            : (const short*)a.q + row * a.qst) + (long)h * D;
+    short* dst = (key ? x.KA : x.QA) + row * HD + (long)h * D;
+    float u[V], w[V];
+    get(src + half + i, w);
+    if (i < half) {
+      get(src + i, u);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const float c = cs[i + j], s = cs[half + i + j], y = u[j];
+        u[j] = y * c - w[j] * s;
+        w[j] = w[j] * c + y * s;
+      }
+      put(dst + i, u);
+    }
+    put(dst + half + i, w);
+  }
+}
+
 // ---- states: U of a chunk, 64 columns per workgroup ------------------------
 template <int DP, int GATE>
 __global__ void __launch_bounds__(256)
 memory_states_kernel(ChunkArgs x) {
+  constexpr int KZ = qk_planes(GATE);
   constexpr int CPR = DP / 8, PAIRS = 32 * CPR / 256;
   constexpr int MT = DP / 32, NT = DP / 64;   // m tiles; tiles of a wave
   const MemoryArgs& a = x.a;
@@ -442,14 +542,14 @@ memory_states_kernel(ChunkArgs x) {
   const int col = lane & 31, hi = lane >> 5;
   const int e0 = et * 64;
   const long ci = (long)ch * a.H + h;
-  __shared__ __attribute__((aligned(16))) short kt[DP * 64];
+  __shared__ __attribute__((aligned(16))) short kt[KZ][DP * 64];
   __shared__ __attribute__((aligned(16))) short vw[3][64 * 64];
   __shared__ __attribute__((aligned(16))) short vu[64 * 64];  // V^T as it is
   __shared__ float s_w[MC_L];
   {
     float w = 0.f;
     if (tid < nrow) {
-      if (GATE != DECAY) {
+      if (!fixed_decay(GATE)) {
         const long o = (long)h * x.T + row0 + tid;
         float d = x.tot[ci * 4 + wid] - x.b[o];
         for (int j = wid + 1; j < 4; ++j) d += x.tot[ci * 4 + j];
@@ -457,15 +557,17 @@ memory_states_kernel(ChunkArgs x) {
                           : expf(d + (x.i[o] - x.cend[ci]));
       } else {
         w = __builtin_amdgcn_exp2f((nrow - 1 - tid) * a.log2_decay[h]);
+        if (GATE == TURNED) w *= a.kscale;
       }
     }
     s_w[tid] = w;
   }
   const int hk = GATE == TIMED ? h / (a.H / a.G) : h;
-  const short* kp = (const short*)a.k + (long)hk * D;
+  const short* kp = (GATE == TURNED ? x.KA : (const short*)a.k) + (long)hk * D;
+  const long kst = GATE == TURNED ? (long)a.H * D : a.kst;
   const short* vp = (const short*)a.v + (long)h * E + e0;
   const uint4v zero = {0, 0, 0, 0};
-  uint4v kreg[2 * PAIRS], vreg[2];
+  uint4v kreg[KZ][2 * PAIRS], vreg[2];
   const int v_r = tid >> 3 << 1, v_c = (tid & 7) * 8;
   const TileWrite vtw(v_c, v_r);
   const TileRead tr(col, 0);
@@ -476,9 +578,11 @@ memory_states_kernel(ChunkArgs x) {
       const int r = it / CPR * 2, c = it % CPR * 8;
 #pragma unroll
       for (int y = 0; y < 2; ++y)
-        kreg[2 * p + y] = c0 + r + y < nrow && c < D
-            ? *(const uint4v*)(kp + (long)(row0 + c0 + r + y) * a.kst + c)
-            : zero;
+#pragma unroll
+        for (int z = 0; z < KZ; ++z)
+          kreg[z][2 * p + y] = c0 + r + y < nrow && c < D
+              ? *(const uint4v*)(kp + ((long)z * x.T + row0 + c0 + r + y) * kst + c)
+              : zero;
     }
 #pragma unroll
     for (int y = 0; y < 2; ++y)
@@ -497,9 +601,17 @@ memory_states_kernel(ChunkArgs x) {
       const int it = p * 256 + tid;
       const int r = it / CPR * 2, c = it % CPR * 8;
       union { uint4v u; unsigned short s[8]; } y0, y1;
-      y0.u = silu8<GATE == DECAY>(kreg[2 * p]);
-      y1.u = silu8<GATE == DECAY>(kreg[2 * p + 1]);
       const TileWrite tw(c, r);
+#pragma unroll
+      for (int z = 1; z < KZ; ++z) {
+        y0.u = kreg[z][2 * p];
+        y1.u = kreg[z][2 * p + 1];
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          *(uint*)(&kt[z][tw.at(j)]) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
+      }
+      y0.u = silu8<GATE == DECAY>(kreg[0][2 * p]);
+      y1.u = silu8<GATE == DECAY>(kreg[0][2 * p + 1]);
       if (GATE == DECAY && et == 0 && c < D) {
         short* ka = x.KA + ((long)(row0 + c0 + r) * a.H + h) * D + c;
         if (c0 + r < nrow) *(uint4v*)ka = y0.u;
@@ -507,7 +619,7 @@ memory_states_kernel(ChunkArgs x) {
       }
 #pragma unroll
       for (int j = 0; j < 8; ++j)
-        *(uint*)(kt + tw.at(j)) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
+        *(uint*)(&kt[0][tw.at(j)]) = (uint)y0.s[j] | ((uint)y1.s[j] << 16);
     }
     {
       float f0[8], f1[8];
@@ -539,13 +651,17 @@ memory_states_kernel(ChunkArgs x) {
       for (int y = 0; y < NT; ++y) {
         const int tile = wid + 4 * y;
         const int m = tile % MT, n = tile / MT;
-        frag_u kf;
-        kf.u4 = *(const uint4v*)(kt + tr.at(m, 2 * kk + hi));
+        frag_u kf[KZ];
+#pragma unroll
+        for (int z = 0; z < KZ; ++z)
+          kf[z].u4 = *(const uint4v*)(&kt[z][tr.at(m, 2 * kk + hi)]);
 #pragma unroll
         for (int z = 0; z < 3; ++z) {
           frag_u vf;
           vf.u4 = *(const uint4v*)(&vw[z][tr.at(n, 2 * kk + hi)]);
-          acc[y] = mfma_bf16(kf.bf, vf.bf, acc[y]);
+#pragma unroll
+          for (int w = 0; w < KZ && w + z < 3; ++w)
+            acc[y] = mfma_bf16(kf[w].bf, vf.bf, acc[y]);
         }
       }
     }
@@ -553,7 +669,7 @@ memory_states_kernel(ChunkArgs x) {
 #pragma unroll
       for (int s = 0; s < 64; s += 8) {
         float kv[8];
-        unpack8(*(const uint4v*)(kt + tslot(tid, s)), kv);
+        unpack8(*(const uint4v*)(&kt[0][tslot(tid, s)]), kv);
 #pragma unroll
         for (int j = 0; j < 8; ++j) nacc += s_w[c0 + s + j] * kv[j];
       }
@@ -618,7 +734,7 @@ memory_scan_kernel(ChunkArgs x) {
   constexpr int PF = 4;
   __shared__ float s_b[64], s_c[64];
   const int c0 = x.first[sg], c1 = x.first[sg + 1];
-  const float l2d = GATE == DECAY ? a.log2_decay[h] : 0.f;
+  const float l2d = fixed_decay(GATE) ? a.log2_decay[h] : 0.f;
   const long at = (long)e * D + d, step = (long)a.H * E * D;
   const float* Up = x.U + ((long)c0 * a.H + h) * E * D + at;
   f32x4 Un[PF] = {};
@@ -629,7 +745,7 @@ memory_scan_kernel(ChunkArgs x) {
     __syncthreads();
     if (tid < 64 && cb + tid < c1) {
       const long ci = (long)(cb + tid) * a.H + h;
-      if (GATE != DECAY) {
+      if (!fixed_decay(GATE)) {
         const float* tt = x.tot + ci * 4;
         const float b = tt[0] + tt[1] + tt[2] + tt[3];
         s_b[tid] = GATE == TIMED ? expf(b) : b;
@@ -692,13 +808,15 @@ memory_scan_kernel(ChunkArgs x) {
 
 // ---- outputs: 128 queries x VT columns per workgroup -----------------------
 template <int DP, int VT, int GATE>
-__global__ void __launch_bounds__(256, DP <= 128 || VT <= 64 ? 2 : 1)
+__global__ void __launch_bounds__(
+    256, DP <= 128 || (VT <= 64 && GATE != TURNED) ? 2 : 1)
 memory_outputs_kernel(ChunkArgs x) {
+  constexpr int KZ = qk_planes(GATE);
   constexpr int NC = DP / 16, NB = VT / 32;
   constexpr int KP = DP * 2;             // K row pitch (bytes)
   constexpr int CPR = DP / 8, PAIRS = 32 * CPR / 256;
   constexpr int VN = VT / 32;            // 16-byte pieces of V^T a thread
-  constexpr int KV_B = 64 * KP + VT * 64 * 2;
+  constexpr int KV_B = KZ * 64 * KP + VT * 64 * 2;
   constexpr int ST_B = 3 * 32 * KP;
   const MemoryArgs& a = x.a;
   const int D = a.D, E = a.E;
@@ -731,7 +849,7 @@ memory_outputs_kernel(ChunkArgs x) {
   __shared__ __attribute__((aligned(16))) char
       buf[KV_B > ST_B ? KV_B : ST_B];
   char* kb = buf;
-  short* vb = (short*)(buf + 64 * KP);
+  short* vb = (short*)(buf + KZ * 64 * KP);
   __shared__ float s_col[64], s_step[GATE == TIMED ? 64 : 1];
   __shared__ float s_n[GATE == GATED ? DP : 1];
   auto kswz = [](int row, int byte) {
@@ -739,22 +857,25 @@ memory_outputs_kernel(ChunkArgs x) {
   };
 
   const int hk = GATE == TIMED ? h / (a.H / a.G) : h;
-  frag_u qf[NC];
-  {
-    const short* src = (const short*)a.q + (long)(row0 + min(t, nrow - 1)) *
-                       a.qst + (long)hk * D;
+  frag_u qf[KZ][NC];
+#pragma unroll
+  for (int z = 0; z < KZ; ++z) {
+    const long r = row0 + min(t, nrow - 1);
+    const short* src =
+        GATE == TURNED ? x.QA + (((long)z * x.T + r) * a.H + h) * D
+                       : (const short*)a.q + r * a.qst + (long)hk * D;
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       const int d = c * 16 + hi * 8;
-      qf[c].u4 = d < D ? silu8<GATE == DECAY>(*(const uint4v*)(src + d))
-                       : uint4v{0, 0, 0, 0};
+      qf[z][c].u4 = d < D ? silu8<GATE == DECAY>(*(const uint4v*)(src + d))
+                          : uint4v{0, 0, 0, 0};
     }
   }
   // row terms of the weights
   float row = 0.f, inter, em = 0.f, l2d = 0.f;
   const float qs = GATE == GATED ? a.qscale : 1.f;
   float tot[4];
-  if (GATE != DECAY) {
+  if (!fixed_decay(GATE)) {
     const long o = (long)h * x.T + row0 + min(t, nrow - 1);
     float before = GATE == GATED ? x.mst[ci] : 0.f;
 #pragma unroll
@@ -814,7 +935,9 @@ memory_outputs_kernel(ChunkArgs x) {
           frag_u sf;
           sf.u4 = *(const uint4v*)(buf + (z * 32 + col) * KP +
                                    kswz(col, (c * 16 + hi * 8) * 2));
-          ot[nb] = mfma_bf16(sf.bf, qf[c].bf, ot[nb]);
+#pragma unroll
+          for (int w = 0; w < KZ && w + z < 3; ++w)
+            ot[nb] = mfma_bf16(sf.bf, qf[w][c].bf, ot[nb]);
         }
       ot[nb] *= inter;
     }
@@ -822,7 +945,7 @@ memory_outputs_kernel(ChunkArgs x) {
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
         float qv[8];
-        unpack8(qf[c].u4, qv);
+        unpack8(qf[0][c].u4, qv);
 #pragma unroll
         for (int j = 0; j < 8; ++j) den += qv[j] * s_n[c * 16 + hi * 8 + j];
       }
@@ -831,11 +954,12 @@ memory_outputs_kernel(ChunkArgs x) {
   }
 
   // ---- keys of the chunk, 64 at a time, from the newest back ---------------
-  const short* kp = (GATE == DECAY ? x.KA : (const short*)a.k) + (long)hk * D;
-  const long kst = GATE == DECAY ? (long)a.H * D : a.kst;
+  const short* kp =
+      (fixed_decay(GATE) ? x.KA : (const short*)a.k) + (long)hk * D;
+  const long kst = fixed_decay(GATE) ? (long)a.H * D : a.kst;
   const short* vp = x.VT + (ci * E + e0) * MC_L;
   const uint4v zero = {0, 0, 0, 0};
-  uint4v kreg[2 * PAIRS], vreg[VN];
+  uint4v kreg[KZ][2 * PAIRS], vreg[VN];
   float colr = 0.f, stepr = 0.f;
   auto issue = [&](int J) {
     const int c0 = 64 * J;
@@ -843,8 +967,11 @@ memory_outputs_kernel(ChunkArgs x) {
     for (int p = 0; p < 2 * PAIRS; ++p) {
       const int it = p * 256 + tid;
       const int r = it / CPR, c = it % CPR * 8;
-      kreg[p] = c0 + r < nrow && c < D
-          ? *(const uint4v*)(kp + (long)(row0 + c0 + r) * kst + c) : zero;
+#pragma unroll
+      for (int z = 0; z < KZ; ++z)
+        kreg[z][p] = c0 + r < nrow && c < D
+            ? *(const uint4v*)(kp + ((long)z * x.T + row0 + c0 + r) * kst + c)
+            : zero;
     }
 #pragma unroll
     for (int p = 0; p < VN; ++p) {
@@ -852,7 +979,7 @@ memory_outputs_kernel(ChunkArgs x) {
       vreg[p] = e0 + e < E
           ? *(const uint4v*)(vp + (long)e * MC_L + c0 + 8 * (tid & 7)) : zero;
     }
-    if (GATE != DECAY && tid < 64) {
+    if (!fixed_decay(GATE) && tid < 64) {
       colr = -INFINITY;
       stepr = 0.f;
       if (c0 + tid < nrow) {
@@ -871,12 +998,14 @@ memory_outputs_kernel(ChunkArgs x) {
     for (int p = 0; p < 2 * PAIRS; ++p) {
       const int it = p * 256 + tid;
       const int r = it / CPR, c = it % CPR * 8;
-      *(uint4v*)(kb + r * KP + kswz(r, c * 2)) = kreg[p];
+#pragma unroll
+      for (int z = 0; z < KZ; ++z)
+        *(uint4v*)(kb + (z * 64 + r) * KP + kswz(r, c * 2)) = kreg[z][p];
     }
 #pragma unroll
     for (int p = 0; p < VN; ++p)
       *(uint4v*)(vb + tslot((p * 256 + tid) >> 3, 8 * (tid & 7))) = vreg[p];
-    if (GATE != DECAY && tid < 64) s_col[tid] = colr;
+    if (!fixed_decay(GATE) && tid < 64) s_col[tid] = colr;
     if (GATE == TIMED && tid < 64) s_step[tid] = stepr;
     __syncthreads();
     if (J > 0) issue(J - 1);
@@ -884,7 +1013,7 @@ memory_outputs_kernel(ChunkArgs x) {
 
     // row part of the exponent for keys of group J
     float base = row;
-    if (GATE != DECAY && J < jt) {
+    if (!fixed_decay(GATE) && J < jt) {
 #pragma unroll
       for (int j = 0; j < 4; ++j)
         if (j >= J && j < jt) base += tot[j];
@@ -896,10 +1025,15 @@ memory_outputs_kernel(ChunkArgs x) {
       f32x16 acc = {};
 #pragma unroll
       for (int c = 0; c < NC; ++c) {
-        frag_u kf;
-        kf.u4 =
-            *(const uint4v*)(kb + kr * KP + kswz(kr, (c * 16 + hi * 8) * 2));
-        acc = mfma_bf16(kf.bf, qf[c].bf, acc);
+#pragma unroll
+        for (int z = 0; z < KZ; ++z) {
+          frag_u kf;
+          kf.u4 = *(const uint4v*)(kb + (z * 64 + kr) * KP +
+                                   kswz(kr, (c * 16 + hi * 8) * 2));
+#pragma unroll
+          for (int w = 0; w < KZ && w + z < 2; ++w)
+            acc = mfma_bf16(kf.bf, qf[w][c].bf, acc);
+        }
       }
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
@@ -908,6 +1042,7 @@ memory_outputs_kernel(ChunkArgs x) {
         if (GATE == TIMED) w = __expf(base + s_col[s]) * s_step[s];
         else if (GATE == GATED) w = __expf(base + s_col[s]) * qs;
         else w = __builtin_amdgcn_exp2f((float)(t - 64 * J - s) * l2d);
+        if (GATE == TURNED) w *= a.kscale;
         if (J == jt && 64 * J + s > t) w = 0.f;
         acc[r] *= w;
         if (GATE == GATED) den += acc[r];
@@ -941,6 +1076,15 @@ memory_outputs_kernel(ChunkArgs x) {
     den += __shfl_xor(den, 32, 64);
     inv = 1.f / (fmaxf(fabsf(den), em) + GATED_EPS);
   }
+  if (GATE == TURNED && a.z) {           // the head's norm; e0 is 0
+    float sq = 0.f;
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) sq += ot[nb][r] * ot[nb][r];
+    sq += __shfl_xor(sq, 32, 64);
+    inv = 1.f / sqrtf(sq / E + x.norm_eps);
+  }
   if (t >= nrow) return;
   const float skip = GATE == TIMED ? bits2f(((const short*)a.skip)[h]) : 0.f;
   short* dst = (short*)a.out + ((long)(row0 + t) * a.H + h) * E + e0;
@@ -953,6 +1097,12 @@ memory_outputs_kernel(ChunkArgs x) {
       float o[4];
 #pragma unroll
       for (int j = 0; j < 4; ++j) o[j] = ot[nb][4 * rg + j] * inv;
+      if (GATE == TURNED && a.z) {
+        float z[4];
+        load4((const short*)a.z + (long)(row0 + t) * a.zst + (long)h * E + e, z);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) o[j] *= silu_f(z[j]);
+      }
       if (GATE == TIMED) {
         float v[4], z[4];
         const long at = (long)h * E + e0 + e;
@@ -972,7 +1122,13 @@ template <int DP, int GATE>
 static void launch_chunks(const ChunkArgs& x, hipStream_t stream) {
   const MemoryArgs& a = x.a;
   const long ch = (long)x.n_chunks * a.H;
-  if (GATE != DECAY) memory_gates_kernel<GATE><<<ch, MC_L, 0, stream>>>(x);
+  if (!fixed_decay(GATE)) memory_gates_kernel<GATE><<<ch, MC_L, 0, stream>>>(x);
+  if (GATE == TURNED) {
+    const size_t lds = a.rot * sizeof(float);
+    const long rows = (long)x.n_chunks * MC_L;
+    if (a.rot % 16 == 0) memory_turn_kernel<true><<<rows, 256, lds, stream>>>(x);
+    else memory_turn_kernel<false><<<rows, 256, lds, stream>>>(x);
+  }
   memory_states_kernel<DP, GATE>
       <<<ch * ((a.E + 63) / 64), 256, 0, stream>>>(x);
   memory_scan_kernel<GATE><<<(long)x.n_seg * a.H * ((a.D + 63) / 64) *
@@ -989,10 +1145,15 @@ static void launch_chunks(const ChunkArgs& x, hipStream_t stream) {
 extern "C" int sv_memory_chunks(const ChunkArgs* x, int gating,
                                 hipStream_t stream) {
   if (x->n_seg <= 0) return 0;
+  if (gating == TURNED &&
+      (x->a.rot % 2 || x->a.rot > x->a.D ||
+       (x->a.z && (x->a.E > 128 || (x->a.E > 64 && x->a.D > 128)))))
+    return 1;
 #define MC(P)                                                     \
   do {                                                            \
     if (gating == GATED) launch_chunks<P, GATED>(*x, stream);     \
     else if (gating == TIMED) launch_chunks<P, TIMED>(*x, stream); \
+    else if (gating == TURNED) launch_chunks<P, TURNED>(*x, stream); \
     else launch_chunks<P, DECAY>(*x, stream);                     \
   } while (0)
   if (x->a.D <= 64) MC(64);

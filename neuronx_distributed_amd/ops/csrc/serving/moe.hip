@@ -27,12 +27,14 @@ struct MoePlanArgs {
   int* order;               // [T * top] slot -> pair
   int* tiles;               // [max_tiles][4]: expert, first slot, slots, 0
   int T, E, top, tile_rows, max_tiles;
-  int sigmoid;              // scores sigmoid(z), chosen by score + bias
+  int kind;                 // 0: softmax over the chosen; 1: scores sigmoid(z), chosen by score + bias;
+                            // 2: weights are a softmax over all experts
   int groups, keep;         // experts of the best groups only (groups > 1)
+  int best;                 // a group counts the sum of its 1 or 2 largest
 };
 
-// Keep the choice scores v of the best groups, drop the others.  A group of
-// neighbours counts the sum of its two largest.  `mem` is the wave's own.
+// Keep the choice scores v of the best groups of neighbours, drop the others.
+// `mem` is the wave's own.
 template <int NV>
 __device__ __forceinline__ void best_groups(const MoePlanArgs& a, float* v,
                                             float* mem) {
@@ -49,7 +51,7 @@ __device__ __forceinline__ void best_groups(const MoePlanArgs& a, float* v,
       m2 = fmaxf(m2, fminf(m1, x));
       m1 = fmaxf(m1, x);
     }
-    score = size > 1 ? m1 + m2 : m1;
+    score = size > 1 && a.best > 1 ? m1 + m2 : m1;
   }
   __builtin_amdgcn_wave_barrier();
   unsigned long long kept = 0;
@@ -77,8 +79,9 @@ __device__ __forceinline__ void best_groups(const MoePlanArgs& a, float* v,
 
 // One wave, one row: the largest choice scores in descending order, the lower
 // index first among equals.  Choice scores are the logits with their bias, the
-// weights a softmax over the chosen; or sigmoids with a bias, the weights the
-// chosen sigmoids over their sum.
+// weights a softmax over the chosen, or over all (then they are not scaled to
+// a sum of one); or sigmoids with a bias, the weights the chosen sigmoids over
+// their sum.
 template <typename T>
 __device__ __forceinline__ void route_row(const MoePlanArgs& a, int t,
                                           float* mem) {
@@ -92,12 +95,22 @@ __device__ __forceinline__ void route_row(const MoePlanArgs& a, int t,
     v[i] = -INFINITY;
     if (e < a.E) {
       const float z = a.z[(long)t * a.E + e];
-      v[i] = (a.sigmoid ? 1.f / (1.f + expf(-z)) : z) +
+      v[i] = (a.kind == 1 ? 1.f / (1.f + expf(-z)) : z) +
              (bias ? to_f(bias[e]) : 0.f);
     }
   }
+  float first = 0.f, sum = 0.f;
+  if (a.kind == 2) {            // the softmax's denominator
+    first = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) first = fmaxf(first, v[i]);
+    first = wave_reduce(first, MaxOp());
+#pragma unroll
+    for (int i = 0; i < NV; ++i) sum += expf(v[i] - first);
+    sum = wave_reduce(sum, SumOp());
+  }
   if (a.groups > 1) best_groups<NV>(a, v, mem);
-  float mine = 0.f, first = 0.f, sum = 0.f;
+  float mine = 0.f;
   int mine_e = 0;
   for (int k = 0; k < a.top; ++k) {
     float best = -INFINITY;
@@ -121,16 +134,17 @@ __device__ __forceinline__ void route_row(const MoePlanArgs& a, int t,
 #pragma unroll
     for (int i = 0; i < NV; ++i)
       if (at == i * 64 + lane) v[i] = -INFINITY;
-    if (k == 0) first = best;
-    const float w = a.sigmoid ? 1.f / (1.f + expf(-a.z[(long)t * a.E + at]))
-                              : expf(best - first);
-    sum += w;
+    if (k == 0 && a.kind != 2) first = best;
+    const float w =
+        a.kind == 1 ? 1.f / (1.f + expf(-a.z[(long)t * a.E + at]))
+                       : expf(best - first);
+    if (a.kind != 2) sum += w;
     if (lane == k) {
       mine = w;
       mine_e = at;
     }
   }
-  if (a.sigmoid) sum += 1e-20f;
+  if (a.kind == 1) sum += 1e-20f;
   if (lane < a.top) {
     a.idx[(long)t * a.top + lane] = mine_e;
     a.coef[(long)t * a.top + lane] = mine / sum;
@@ -192,7 +206,8 @@ extern "C" int sv_moe_plan(const MoePlanArgs* a, int f32,
   if (a->T <= 0) return 0;
   if (a->E > MOE_MAX_EXPERTS || a->top > 64 || a->top > a->E) return 1;
   if (a->groups < 1 || a->groups > 64 || a->E % a->groups || a->keep < 1 ||
-      a->keep > a->groups || a->keep * (a->E / a->groups) < a->top)
+      a->keep > a->groups || a->keep * (a->E / a->groups) < a->top ||
+      a->best < 1 || a->best > 2)
     return 1;
   const bool fused = a->T <= 64;
   if (!fused) {

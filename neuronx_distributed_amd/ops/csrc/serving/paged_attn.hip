@@ -532,7 +532,7 @@ static int launch_rows(const RowsArgs& a, int vec, hipStream_t stream) {
   else if (big <= 128) ARR(16);
   else if (big <= 256) ARR(32);
   else if (big <= 512) ARR(64);
-  else if (big <= 1024 && !MOD) {
+  else if (big <= 1024) {
     if (rcn == 2) { if (vec) AR(64, 2, true, 16); else AR(64, 2, false, 16); }
     else { if (vec) AR(64, 1, true, 16); else AR(64, 1, false, 16); }
   } else return 1;

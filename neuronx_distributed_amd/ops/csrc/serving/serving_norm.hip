@@ -8,15 +8,29 @@
 // parallel branches.  One tensor or sum may be RMS-normed before it is added,
 // two branches always are; the result is scaled.  A norm may run in groups:
 // equal consecutive parts of the row, each over its own root mean square.
+// Instead of one result, up to two gated ones may be pending: each a tensor or
+// a weighted sum of rows, plus another tensor, times the sigmoid of a gate an
+// element.
 //
 // The normed rows of single tokens may pass a causal convolution over time on
 // their way out (h + conv(h)): the last inputs of their request come from a
 // ring, which takes the new one.
 //
-// gated_norm: RMS norm over groups of a row, times a weight, times
-// sigmoid(gate) if there is one — the output stage of the recurrent mixers.
+// gated_norm: RMS norm over groups of a row, times a weight if there is one,
+// times sigmoid(gate) or silu(gate) if there is one — the output stage of the
+// recurrent mixers.
 
 #include "serving.h"
+
+struct BranchArgs {
+  const void* delta;     // [rows, W], or [rows * parts, W] with coef
+  const float* coef;     // [rows, parts] or null
+  const void* plus;      // [rows, W] added to it, or null
+  const void* gate;      // [rows] rows of W; sigmoid(gate + bias) multiplies
+  long gst;              //   the sum; or null
+  const void* bias;      // [W] or null
+  long parts;
+};
 
 struct ResidualNormArgs {
   const float* x;        // [rows, W] residual, or null (starts from zero)
@@ -44,6 +58,8 @@ struct ResidualNormArgs {
   float eps, scale;
   float w_base, p_base;  // added to w, and to w1 and w2
   float h_scale;         // multiplies h
+  int branches;          // gated results that are pending
+  BranchArgs br[2];
 };
 
 template <typename T, int VEC>
@@ -55,7 +71,7 @@ __device__ __forceinline__ void st(T* p, const float* v) {
   if (VEC == 4) store4(p, v); else from_f(p[0], v[0]);
 }
 
-template <typename T, int VEC>
+template <typename T, int VEC, bool BRANCHES>
 __global__ void __launch_bounds__(256)
 residual_norm_kernel(ResidualNormArgs a) {
   extern __shared__ __attribute__((aligned(16))) float row[];  // [W]
@@ -163,6 +179,44 @@ residual_norm_kernel(ResidualNormArgs a) {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) v[j] += s1 * t[j];
     }
+    if (BRANCHES) {
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        if (b >= a.branches) break;
+        const BranchArgs& z = a.br[b];
+        float g[VEC];
+        if (z.gate) {
+          ld<T, VEC>((const T*)z.gate + r * z.gst + i, g);
+          if (z.bias) {
+            ld<T, VEC>((const T*)z.bias + i, u);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) g[j] += u[j];
+          }
+        }
+        if (z.coef) {
+          const T* d = (const T*)z.delta + r * z.parts * W + i;
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) t[j] = 0.f;
+#pragma unroll 2
+          for (int p = 0; p < z.parts; ++p) {
+            const float c = z.coef[r * z.parts + p];
+            ld<T, VEC>(d + (long)p * W, u);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) t[j] += c * u[j];
+          }
+        } else {
+          ld<T, VEC>((const T*)z.delta + r * W + i, t);
+        }
+        if (z.plus) {
+          ld<T, VEC>((const T*)z.plus + r * W + i, u);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) t[j] += u[j];
+        }
+#pragma unroll
+        for (int j = 0; j < VEC; ++j)
+          v[j] += z.gate ? t[j] * sigmoid_f(g[j]) : t[j];
+      }
+    }
     if (a.vec) {
       ld<T, VEC>((const T*)a.vec + i, t);
 #pragma unroll
@@ -240,27 +294,35 @@ extern "C" int sv_residual_norm(const ResidualNormArgs* a, int f32,
   if (a->W % a->groups || a->W % a->p_groups) return 1;
   if (a->conv && (!a->h || !a->w)) return 1;
   // four elements of a thread lie in one part
-  const bool vec = a->W % 4 == 0 && (a->W / a->groups) % 4 == 0 &&
-                   (a->W / a->p_groups) % 4 == 0;
+  bool vec = a->W % 4 == 0 && (a->W / a->groups) % 4 == 0 &&
+             (a->W / a->p_groups) % 4 == 0;
+  for (int b = 0; b < a->branches && b < 2; ++b)
+    vec = vec && (!a->br[b].gate ||
+                  (a->br[b].gst % 4 == 0 &&
+                   (size_t)a->br[b].gate % (f32 ? 16 : 8) == 0));
+  if (a->branches < 0 || a->branches > 2 || (a->branches && a->delta)) return 1;
+#define RNB(T, V, B)                                                       \
+  residual_norm_kernel<T, V, B><<<a->rows_out, 256, lds, stream>>>(*a)
 #define RN(T, V)                                                           \
-  residual_norm_kernel<T, V><<<a->rows_out, 256, lds, stream>>>(*a)
+  do { if (a->branches) RNB(T, V, true); else RNB(T, V, false); } while (0)
   if (f32) { if (vec) RN(float, 4); else RN(float, 1); }
   else     { if (vec) RN(short, 4); else RN(short, 1); }
 #undef RN
+#undef RNB
   return (int)hipGetLastError();
 }
 
 // ---------------------------------------------------------------------------
-// o [rows, groups * gs] -> o / rms(group) * w * sigmoid(gate)
+// o [rows, groups * gs] -> o / rms(group) * w * act(gate)
 // One wave per (row, group): NW waves of a block take neighbouring groups.
 // Long groups take the whole block.
 // ---------------------------------------------------------------------------
 template <typename T, int VEC, bool BLOCK>
 __global__ void __launch_bounds__(256)
-gated_norm_kernel(const T* __restrict__ o, const T* __restrict__ w,
+gated_norm_kernel(const T* o, const T* __restrict__ w,
                   const T* __restrict__ gate, long gate_stride,
-                  T* __restrict__ out, int rows, int groups, int gs,
-                  float eps) {
+                  T* out, int rows, int groups, int gs,
+                  float eps, int silu) {
   __shared__ float red[16];
   const int tid = BLOCK ? threadIdx.x : (threadIdx.x & 63);
   const int step = (BLOCK ? 256 : 64) * VEC;
@@ -281,14 +343,17 @@ gated_norm_kernel(const T* __restrict__ o, const T* __restrict__ w,
   const float rstd = 1.f / sqrtf(sq / gs + eps);
   for (int i = tid * VEC; i < gs; i += step) {
     ld<T, VEC>(src + i, v);
-    ld<T, VEC>(w + off + i, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) u[j] = 1.f;
+    if (w) ld<T, VEC>(w + off + i, u);
 #pragma unroll
     for (int j = 0; j < VEC; ++j) v[j] *= rstd * u[j];
     if (g) {
       float z[VEC];
       ld<T, VEC>(g + i, z);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) v[j] *= sigmoid_f(z[j]);
+      for (int j = 0; j < VEC; ++j)
+        v[j] *= silu ? z[j] * sigmoid_f(z[j]) : sigmoid_f(z[j]);
     }
     st<T, VEC>(out + item * gs + i, v);
   }
@@ -296,8 +361,8 @@ gated_norm_kernel(const T* __restrict__ o, const T* __restrict__ w,
 
 extern "C" int sv_gated_norm(const void* o, const void* w, const void* gate,
                              long gate_stride, void* out, int rows,
-                             int groups, int gs, float eps, int vec4, int f32,
-                             hipStream_t stream) {
+                             int groups, int gs, float eps, int silu,
+                             int vec4, int f32, hipStream_t stream) {
   if (rows <= 0) return 0;
   const bool block = gs > 1024;
   const long items = (long)rows * groups;
@@ -305,7 +370,7 @@ extern "C" int sv_gated_norm(const void* o, const void* w, const void* gate,
 #define GN(T, V, B)                                                         \
   gated_norm_kernel<T, V, B><<<grid, 256, 0, stream>>>(                     \
       (const T*)o, (const T*)w, (const T*)gate, gate_stride, (T*)out, rows, \
-      groups, gs, eps)
+      groups, gs, eps, silu)
 #define GNB(T, V) do { if (block) GN(T, V, true); else GN(T, V, false); } while (0)
   if (f32) { if (vec4) GNB(float, 4); else GNB(float, 1); }
   else     { if (vec4) GNB(short, 4); else GNB(short, 1); }
@@ -387,6 +452,123 @@ extern "C" int sv_gelu_rows(void* x, const void* table, long tst,
   else
     gelu_rows_kernel<short><<<blocks, 256, 0, stream>>>(
         (short*)x, (const short*)table, tst, tokens, rows, n, at);
+  return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// polynomial activation over a row z of n values: with N a division by the
+// root mean square of the row, out = a N(z) + b N(z^2) + c N(z^3) + e of
+// act [4].  One workgroup a row; up to 16384 values stay in registers.
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(512)
+poly_norm_kernel(const T* __restrict__ x, long xst, const T* __restrict__ act,
+                 T* __restrict__ out, int n, float eps) {
+  constexpr int KEEP = 32 / VEC;
+  __shared__ float red[3][8];
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const T* src = x + (long)blockIdx.x * xst;
+  T* dst = out + (long)blockIdx.x * n;
+  float kept[KEEP][VEC], s[3] = {0.f, 0.f, 0.f};
+  auto add = [&](const float* v) {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const float q = v[j] * v[j];
+      s[0] += q;
+      s[1] += q * q;
+      s[2] += q * q * q;
+    }
+  };
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int i = (k * 512 + tid) * VEC;
+    if (i < n) ld<T, VEC>(src + i, kept[k]);
+  }
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k)
+    if ((k * 512 + tid) * VEC < n) add(kept[k]);
+  for (int i = (KEEP * 512 + tid) * VEC; i < n; i += 512 * VEC) {
+    float v[VEC];
+    ld<T, VEC>(src + i, v);
+    add(v);
+  }
+#pragma unroll
+  for (int p = 0; p < 3; ++p) {
+    s[p] = wave_reduce(s[p], SumOp());
+    if (lane == 0) red[p][wid] = s[p];
+  }
+  __syncthreads();
+  float f[3];
+#pragma unroll
+  for (int p = 0; p < 3; ++p) {
+    float q = 0.f;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) q += red[p][w];
+    f[p] = to_f(act[p]) / sqrtf(q / n + eps);
+  }
+  const float e = to_f(act[3]);
+  auto put = [&](float* v, int i) {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j)
+      v[j] = e + v[j] * (f[0] + v[j] * (f[1] + v[j] * f[2]));
+    st<T, VEC>(dst + i, v);
+  };
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int i = (k * 512 + tid) * VEC;
+    if (i < n) put(kept[k], i);
+  }
+  for (int i = (KEEP * 512 + tid) * VEC; i < n; i += 512 * VEC) {
+    float v[VEC];
+    ld<T, VEC>(src + i, v);
+    put(v, i);
+  }
+}
+
+extern "C" int sv_poly_norm(const void* x, long xst, const void* act,
+                            void* out, int rows, int n, float eps, int vec4,
+                            int f32, hipStream_t stream) {
+  if (rows <= 0 || n <= 0) return 0;
+#define PN(T, V)                                                            \
+  poly_norm_kernel<T, V><<<rows, 512, 0, stream>>>((const T*)x, xst,        \
+                                                   (const T*)act, (T*)out, n, eps)
+  if (f32) { if (vec4) PN(float, 4); else PN(float, 1); }
+  else     { if (vec4) PN(short, 4); else PN(short, 1); }
+#undef PN
+  return (int)hipGetLastError();
+}
+
+// ---------------------------------------------------------------------------
+// x rows of 2 n: gate, then up -> out [rows][n] = silu(gate) up
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+silu_mul_kernel(const T* __restrict__ x, long xst, T* __restrict__ out,
+                int n) {
+  const int i = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (i >= n) return;
+  const T* src = x + (long)blockIdx.y * xst + i;
+  float g[VEC], u[VEC];
+  ld<T, VEC>(src, g);
+  ld<T, VEC>(src + n, u);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) u[j] *= silu_f(g[j]);
+  st<T, VEC>(out + (long)blockIdx.y * n + i, u);
+}
+
+extern "C" int sv_silu_mul(const void* x, long xst, void* out, int rows,
+                           int n, int vec4, int f32, hipStream_t stream) {
+  if (rows <= 0 || n <= 0) return 0;
+  for (int r0 = 0; r0 < rows; r0 += 65535) {
+    const int part = rows - r0 < 65535 ? rows - r0 : 65535;
+#define SM(T, V)                                                           \
+  silu_mul_kernel<T, V>                                                    \
+      <<<dim3((n / V + 255) / 256, part), 256, 0, stream>>>(               \
+          (const T*)x + r0 * xst, xst, (T*)out + (long)r0 * n, n)
+    if (f32) { if (vec4) SM(float, 4); else SM(float, 1); }
+    else     { if (vec4) SM(short, 4); else SM(short, 1); }
+#undef SM
+  }
   return (int)hipGetLastError();
 }
 

@@ -11,7 +11,7 @@ import ctypes
 import math
 import os
 from dataclasses import dataclass, replace
-from typing import Optional, Union
+from typing import Optional, Sequence, Union
 
 import torch
 
@@ -73,12 +73,21 @@ def _fields(names, ctype):
     return [(n, ctype) for n in names.split()]
 
 
+class _BranchArgs(ctypes.Structure):
+    _fields_ = (_fields("delta coef plus gate", ctypes.c_void_p)
+                + _fields("gst", ctypes.c_long)
+                + _fields("bias", ctypes.c_void_p)
+                + _fields("parts", ctypes.c_long))
+
+
 class _ResidualNormArgs(ctypes.Structure):
     _fields_ = (_fields("x delta delta2 w1 w2 coef vec x_out h w cat x0 "
                         "index conv ring singles hc", ctypes.c_void_p)
                 + _fields("rows_out W delta_f32 parts groups p_groups taps "
                           "conv_row", ctypes.c_int)
-                + _fields("eps scale w_base p_base h_scale", ctypes.c_float))
+                + _fields("eps scale w_base p_base h_scale", ctypes.c_float)
+                + _fields("branches", ctypes.c_int)
+                + [("br", _BranchArgs * 2)])
 
 
 class _ConvArgs(ctypes.Structure):
@@ -137,7 +146,8 @@ class _LatentAppendArgs(ctypes.Structure):
                 + _fields("kvst", ctypes.c_long)
                 + _fields("w freq cache pos seq bt", ctypes.c_void_p)
                 + _fields("MB H R P rot", ctypes.c_int)
-                + _fields("eps", ctypes.c_float))
+                + _fields("eps amp", ctypes.c_float)
+                + _fields("pairs", ctypes.c_int))
 
 
 class _HeadLinearArgs(ctypes.Structure):
@@ -153,12 +163,13 @@ class _HeadLinearArgs(ctypes.Structure):
 class _LatentRowsArgs(ctypes.Structure):
     _fields_ = (_fields("q cache pos seq bt part out", ctypes.c_void_p)
                 + _fields("MB rows H R P splits window", ctypes.c_int)
-                + _fields("scale", ctypes.c_float))
+                + _fields("scale", ctypes.c_float)
+                + _fields("sink", ctypes.c_void_p))
 
 
 class _MoePlanArgs(ctypes.Structure):
     _fields_ = (_fields("z bias idx coef order tiles", ctypes.c_void_p)
-                + _fields("T E top tile_rows max_tiles sigmoid groups keep",
+                + _fields("T E top tile_rows max_tiles kind groups keep best",
                           ctypes.c_int))
 
 
@@ -180,13 +191,17 @@ class _MemoryArgs(ctypes.Structure):
                 + _fields("skip z", ctypes.c_void_p)
                 + _fields("zst", ctypes.c_long)
                 + _fields("cw cb ring", ctypes.c_void_p)
-                + _fields("taps C kch qch", ctypes.c_int))
+                + _fields("taps C kch qch", ctypes.c_int)
+                + _fields("freq", ctypes.c_void_p)
+                + _fields("rot", ctypes.c_int)
+                + _fields("amp kscale", ctypes.c_float))
 
 
 class _ChunkArgs(ctypes.Structure):
     _fields_ = ([("a", _MemoryArgs)] + _fields("chunks first", ctypes.c_void_p)
                 + _fields("n_chunks n_seg T", ctypes.c_int)
-                + _fields("b i c tot cend U N P mst VT KA", ctypes.c_void_p))
+                + _fields("b i c tot cend U N P mst VT KA QA", ctypes.c_void_p)
+                + _fields("norm_eps", ctypes.c_float))
 
 
 # ---------------------------------------------------------------------------
@@ -212,8 +227,9 @@ class Pending:
     summed; ``scale`` times that.  One tensor is RMS-normed when ``w1`` is
     given, over ``groups`` equal parts each.  ``coef`` (rows, parts) makes a row the weighted sum of ``parts``
     rows of ``delta`` (rows * parts, W).  ``centred``: w1 and w2 are stored as
-    their distance from one.  ``vec`` is a row added to every token."""
-    delta: torch.Tensor
+    their distance from one.  ``vec`` is a row added to every token.  Instead
+    of ``delta``, up to two gated ``branches`` may be pending."""
+    delta: Optional[torch.Tensor] = None
     delta2: Optional[torch.Tensor] = None
     w1: Optional[torch.Tensor] = None
     w2: Optional[torch.Tensor] = None
@@ -222,6 +238,46 @@ class Pending:
     coef: Optional[torch.Tensor] = None
     centred: bool = False
     groups: int = 1
+    branches: Sequence["Branch"] = ()
+
+
+@dataclass
+class Branch:
+    """A gated sublayer result: the rows of ``delta``, or with ``coef`` (rows,
+    parts) their weighted sums; plus ``plus`` (rows, W); times sigmoid(gate +
+    bias) of ``gate`` (rows, W) and ``bias`` (W,)."""
+    delta: torch.Tensor
+    coef: Optional[torch.Tensor] = None
+    plus: Optional[torch.Tensor] = None
+    gate: Optional[torch.Tensor] = None
+    bias: Optional[torch.Tensor] = None
+
+    @property
+    def rows(self) -> int:
+        return (self.delta if self.coef is None else self.coef).shape[0]
+
+    def args(self, rows: int, W: int, dtype) -> _BranchArgs:
+        parts = 1 if self.coef is None else self.coef.shape[1]
+        assert self.delta.shape == (rows * parts, W)
+        assert self.delta.is_contiguous() and self.delta.dtype == dtype
+        a = _BranchArgs(delta=_p(self.delta), parts=parts)
+        if self.coef is not None:
+            assert self.coef.shape[0] == rows and self.coef.is_contiguous()
+            assert self.coef.dtype == torch.float32
+            a.coef = _p(self.coef)
+        if self.plus is not None:
+            assert self.plus.shape == (rows, W) and self.plus.dtype == dtype
+            assert self.plus.is_contiguous()
+            a.plus = _p(self.plus)
+        if self.gate is not None:
+            assert self.gate.shape == (rows, W) and self.gate.dtype == dtype
+            assert self.gate.stride(1) == 1
+            a.gate, a.gst = _p(self.gate), self.gate.stride(0)
+        if self.bias is not None:
+            assert self.bias.shape == (W,) and self.bias.dtype == dtype
+            assert self.gate is not None and self.bias.is_contiguous()
+            a.bias = _p(self.bias)
+        return a
 
 
 @dataclass
@@ -277,8 +333,15 @@ def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
     one of so many equal parts is normed on its own.  ``scale`` multiplies the
     second result.  ``conv``: the second result is h + conv(h) of the rows h of
     ``batch``."""
-    src = x if pending is None else pending.delta
+    branches = () if pending is None else pending.branches
+    src = x if pending is None else \
+        branches[0].delta if branches else pending.delta
     rows, W = src.shape
+    if branches:
+        assert pending.delta is None and pending.coef is None and \
+            pending.w1 is None and len(branches) <= 2
+        rows = branches[0].rows
+        assert x is None or x.shape == (rows, W)
     if pending is not None and pending.coef is not None:
         assert pending.coef.is_contiguous() and \
             pending.coef.dtype == torch.float32
@@ -300,14 +363,19 @@ def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
     a.x, a.x_out, a.h, a.w = _p(x), _p(x_new), _p(h), _p(weight)
     a.cat, a.x0, a.index = _p(cat), _p(x0), _p(index)
     a.w_base, a.scale = float(centred), 1.0
-    if pending is not None:
+    for i, b in enumerate(branches):
+        a.br[i] = b.args(rows, W, dtype)
+    a.branches = len(branches)
+    if pending is not None and pending.vec is not None:
+        a.vec = _p(pending.vec)
+    if pending is not None and not branches:
         d = pending.delta
         assert d.is_contiguous() and d.dtype in (dtype, torch.float32)
         assert pending.delta2 is None or (
             d.dtype == dtype and pending.delta2.is_contiguous()
             and pending.delta2.shape == d.shape)
         a.delta, a.delta2 = _p(d), _p(pending.delta2)
-        a.w1, a.w2, a.vec = _p(pending.w1), _p(pending.w2), _p(pending.vec)
+        a.w1, a.w2 = _p(pending.w1), _p(pending.w2)
         a.coef, a.scale = _p(pending.coef), pending.scale
         a.p_groups = pending.groups
         assert pending.groups == 1 or (pending.w1 is not None
@@ -337,14 +405,16 @@ def residual_norm(x: Optional[torch.Tensor], pending: Optional[Pending],
     return x_new, h, cat
 
 
-def gated_norm(o: torch.Tensor, weight: torch.Tensor,
+def gated_norm(o: torch.Tensor, weight: Optional[torch.Tensor],
                gate: Optional[torch.Tensor], group: int,
-               eps: float) -> torch.Tensor:
+               eps: float, silu: bool = False,
+               out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """o (T, N): every ``group`` elements divided by their root mean square,
-    times weight (N,), times sigmoid(gate (T, N)) if there is a gate."""
+    times weight (N,) if there is one, times sigmoid(gate (T, N)), or
+    silu(gate), if there is a gate.  ``out`` may be o."""
     T, N = o.shape
     assert N % group == 0 and o.is_contiguous()
-    out = torch.empty_like(o)
+    out = _out(out, T, N, o)
     vec4 = int(group % 4 == 0)
     if gate is not None:
         assert gate.shape == o.shape and gate.stride(1) == 1
@@ -355,7 +425,34 @@ def gated_norm(o: torch.Tensor, weight: torch.Tensor,
         ctypes.c_void_p(_p(gate)),
         ctypes.c_long(0 if gate is None else gate.stride(0)),
         ctypes.c_void_p(_p(out)), T, N // group, group, ctypes.c_float(eps),
-        vec4, _f32(o), _stream()), "gated_norm")
+        int(silu), vec4, _f32(o), _stream()), "gated_norm")
+    return out
+
+
+def poly_norm(x: torch.Tensor, act: torch.Tensor, eps: float) -> torch.Tensor:
+    """x (T, n) -> a N(x) + b N(x^2) + c N(x^3) + e of act = (a, b, c, e),
+    powers element by element; N divides a row by its root mean square."""
+    T, n = x.shape
+    assert x.stride(1) == 1 and act.shape == (4,) and act.is_contiguous()
+    assert act.dtype == x.dtype
+    out = torch.empty(T, n, dtype=x.dtype, device=x.device)
+    _check(library().sv_poly_norm(
+        ctypes.c_void_p(_p(x)), ctypes.c_long(x.stride(0)),
+        ctypes.c_void_p(_p(act)), ctypes.c_void_p(_p(out)), T, n,
+        ctypes.c_float(eps), _vec4((n,), x), _f32(x), _stream()),
+        "poly_norm")
+    return out
+
+
+def silu_mul(x: torch.Tensor) -> torch.Tensor:
+    """x (T, 2 n) = [gate | up] -> silu(gate) * up (T, n)."""
+    T, n = x.shape[0], x.shape[1] // 2
+    assert x.stride(1) == 1 and x.shape[1] == 2 * n
+    out = torch.empty(T, n, dtype=x.dtype, device=x.device)
+    _check(library().sv_silu_mul(
+        ctypes.c_void_p(_p(x)), ctypes.c_long(x.stride(0)),
+        ctypes.c_void_p(_p(out)), T, n, _vec4((n,), x), _f32(x),
+        _stream()), "silu_mul")
     return out
 
 
@@ -407,6 +504,12 @@ def _aligned(sizes, *tensors) -> bool:
     return all(s % 8 == 0 for s in sizes) and all(
         t.stride(0) % 8 == 0 and t.storage_offset() % 8 == 0
         for t in tensors)
+
+
+def _vec4(sizes, *tensors) -> int:
+    return int(all(s % 4 == 0 for s in sizes) and all(
+        t.stride(0) % 4 == 0 and t.storage_offset() % 4 == 0
+        for t in tensors))
 
 
 def _check_cache(q, k, v, kc, vc, H):
@@ -677,7 +780,25 @@ class TimeGate:
     conv: Optional[ShortConv] = None
 
 
-_GATINGS = {DecayGate: 0, ExpGate: 1, TimeGate: 2}
+@dataclass
+class TurnGate:
+    """S <- decay S + kscale k v^T, with q and k rotated at their position:
+    elements i and i + dims / 2 of a head turn together."""
+    decay: torch.Tensor        # (H,) float32
+    log2_decay: torch.Tensor   # (H,) float32
+    kscale: float
+    freq: torch.Tensor         # (dims / 2,) float64 rad a position
+    amplitude: float = 1.0     # of cos and sin
+
+    @staticmethod
+    def norm_fits(dtype, D: int, E: int, *tensors) -> bool:
+        """Can the chunk kernels norm and gate the heads as well?"""
+        return (dtype == torch.bfloat16 and D <= 256
+                and E <= (128 if D <= 128 else 64)
+                and _aligned((D, E), *tensors))
+
+
+_GATINGS = {DecayGate: 0, ExpGate: 1, TimeGate: 2, TurnGate: 3}
 
 
 def chunk_table(segments):
@@ -696,14 +817,18 @@ def chunk_table(segments):
 def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
                chunks: Optional[torch.Tensor] = None,
                chunk_first: Optional[torch.Tensor] = None,
-               out: Optional[torch.Tensor] = None) -> torch.Tensor:
+               out: Optional[torch.Tensor] = None,
+               silu_gate: Optional[torch.Tensor] = None,
+               eps: float = 0.0) -> torch.Tensor:
     """Run a matrix memory over segments of a ragged batch.  q, k (T, H*D),
     v (T, H*E) — q, k (T, G*D) for a TimeGate; S (slots, H, D, E) float32; n (slots, H, ceil(E/32), D) and
     m (slots, H, ceil(E/32)) float32 for an ExpGate.  ``seg`` (n, 4) int32
     lists (slot, first row, rows, context); rows count from the start of
     the tensors, so portions and single tokens of one batch can be run by
     two calls into one ``out``.  With the device form of
-    ``chunk_table`` the 256-token MFMA kernels run where they apply."""
+    ``chunk_table`` the 256-token MFMA kernels run where they apply; with a
+    TurnGate that ``norm_fits`` they also divide every head of the output by
+    its root mean square and multiply it by silu(``silu_gate`` (T, H*E))."""
     D, E = S.shape[2], S.shape[3]
     T = q.shape[0]
     assert q.shape[1] == k.shape[1] and v.shape[1] == heads * E
@@ -720,6 +845,7 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
     assert q.shape[1] == a.G * D and heads % a.G == 0
     gating = _GATINGS[type(gate)]
     gated, timed = isinstance(gate, ExpGate), isinstance(gate, TimeGate)
+    turned = isinstance(gate, TurnGate)
     assert timed or a.G == heads
     strided = [q, k, v]
     if timed:
@@ -751,6 +877,18 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
     else:
         assert gate.decay.shape == (heads,)
         a.decay, a.log2_decay = _p(gate.decay), _p(gate.log2_decay)
+    if turned:
+        assert gate.freq.dtype == torch.float64 and gate.freq.is_cuda
+        a.freq, a.rot = _p(gate.freq), 2 * gate.freq.shape[0]
+        a.amp, a.kscale = gate.amplitude, gate.kscale
+        if a.rot > D:
+            raise ValueError(f"{a.rot} of {D} elements turn")
+    if silu_gate is not None:
+        assert turned and chunks is not None
+        assert gate.norm_fits(q.dtype, D, E, q, k, v, silu_gate)
+        assert silu_gate.shape == v.shape and silu_gate.stride(1) == 1 \
+            and silu_gate.dtype == v.dtype
+        a.z, a.zst = _p(silu_gate), silu_gate.stride(0)
     lib = library()
     if (chunks is not None and q.dtype == torch.bfloat16 and D <= 256
             and _aligned((D, E), *strided)):
@@ -764,9 +902,14 @@ def memory_mix(q, k, v, gate, S, n, m, seg, heads: int,
                          device=q.device)
         KA = torch.empty(T, heads * D, dtype=q.dtype, device=q.device) \
             if isinstance(gate, DecayGate) else None
+        if turned:
+            KA, QA = torch.empty(2, 2, T, heads * D, dtype=q.dtype,
+                                 device=q.device)
         x = _ChunkArgs(a=a, chunks=_p(chunks), first=_p(chunk_first),
                        n_chunks=nc, n_seg=seg.shape[0], T=T, U=_p(U),
-                       P=_p(P), VT=_p(VT), KA=_p(KA))
+                       P=_p(P), VT=_p(VT), KA=_p(KA), norm_eps=eps)
+        if turned:
+            x.QA = _p(QA)
         if timed:
             bic = torch.empty(2, heads, T, **f32)
             small = torch.empty(nc, heads, 4, **f32)
@@ -837,12 +980,35 @@ def rotary_frequencies(base: float, dims: int, device,
     return f.to(device)
 
 
+def yarn_frequencies(base: float, dims: int, device, scaling: dict):
+    """Radians a position of every rotated pair, float64, and the amplitude
+    of cos and sin.  ``scaling`` (factor, original, fast, slow): pairs that turn
+    more than ``fast`` times in ``original`` positions are kept, those that turn
+    less than ``slow`` times are slowed by ``factor``; between them, pair by
+    pair, linearly from one to the other."""
+    f = rotary_frequencies(base, dims, "cpu")
+
+    def pair(turns):
+        return dims * math.log(scaling["original"] / (2 * math.pi * turns)) \
+            / (2 * math.log(base))
+
+    lo = max(math.floor(pair(scaling["fast"])), 0)
+    hi = min(math.ceil(pair(scaling["slow"])), dims - 1)
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    slow = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    f = f / scaling["factor"] * slow + f * (1.0 - slow)
+    return f.to(device), 0.1 * math.log(scaling["factor"]) + 1.0
+
+
 @dataclass
 class LatentWeights:
     norm: torch.Tensor         # (rank,) of the latents
     absorb: torch.Tensor       # (H, rank, dim): query -> latent space
     expand: torch.Tensor       # (H * dim + H * vdim, rank): keys, values
-    freq: torch.Tensor         # (rot / 2,) float64, from rotary_frequencies
+    freq: torch.Tensor         # (rot / 2,) float64 rad a position
+    amplitude: float = 1.0     # of cos and sin
+    pairs: bool = False        # neighbours turn together, not halves
+    sink: Optional[torch.Tensor] = None   # (H,) joins the denominator
 
 
 def latent_append(q, rot_at: int, q_step: int, qr, qr_at: int, qr_step: int,
@@ -868,7 +1034,8 @@ def latent_append(q, rot_at: int, q_step: int, qr, qr_at: int, qr_step: int,
         qr=_p(qr) + qr_at * size, qrst=qr.stride(0), qrh=qr_step, kv=_p(kv),
         kvst=kv.stride(0), w=_p(w.norm), freq=_p(w.freq), cache=_p(cache),
         pos=_p(pos), seq=_p(seq), bt=_p(block_table),
-        MB=block_table.shape[1], H=heads, R=R, P=P, rot=2 * half, eps=eps)
+        MB=block_table.shape[1], H=heads, R=R, P=P, rot=2 * half, eps=eps,
+        amp=w.amplitude, pairs=int(w.pairs))
     _check(library().sv_latent_append(ctypes.byref(a), T, _f32(q),
                                       _stream()), "latent_append")
 
@@ -904,15 +1071,18 @@ def latent_rows_supported(dtype, rank: int, shared: int) -> bool:
 
 
 def latent_rows(q, cache, rank: int, pos, seq, block_table, heads: int,
-                scale: float, window: int = 0, max_keys: int = 0):
+                scale: float, window: int = 0, max_keys: int = 0,
+                sink: Optional[torch.Tensor] = None):
     """Absorbed queries q (rows, H * (rank + P)) over the cached rows, which
-    hold the rows' own keys already -> (rows, H * rank) sums of latents."""
+    hold the rows' own keys already -> (rows, H * rank) sums of latents.
+    exp(sink[h]) joins the denominator."""
     rows, D = q.shape[0], cache.shape[2]
     assert q.is_contiguous() and q.shape[1] == heads * D
     assert cache.is_contiguous() and cache.shape[1] == PAGE_SIZE
     assert q.dtype == cache.dtype and pos.shape[0] == seq.shape[0] == rows
     if D > MAX_LATENT_ROW:
         raise ValueError(f"latent row of {D} > {MAX_LATENT_ROW}")
+    mod = _score_args(ScoreMod(sink=sink), q, heads)
     if window > 0:
         max_keys = min(max_keys, window) if max_keys else window
     out = torch.empty(rows, heads * rank, dtype=q.dtype, device=q.device)
@@ -927,7 +1097,7 @@ def latent_rows(q, cache, rank: int, pos, seq, block_table, heads: int,
             q=_p(q), cache=_p(cache), pos=_p(pos), seq=_p(seq),
             bt=_p(block_table), part=_p(part), out=_p(out),
             MB=block_table.shape[1], rows=rows, H=heads, R=rank, P=D - rank,
-            splits=splits, window=window, scale=scale)
+            splits=splits, window=window, scale=scale, sink=mod.sink)
         _check(library().sv_latent_rows(ctypes.byref(a), _stream()),
                "latent_rows")
         return out
@@ -938,7 +1108,7 @@ def latent_rows(q, cache, rank: int, pos, seq, block_table, heads: int,
                   bt=_p(block_table), part=_p(part), out=_p(out),
                   MB=block_table.shape[1], rows=rows, H=heads, G=1, D=D,
                   E=rank, splits=splits, append=0, window=window, keep=0,
-                  scale=scale)
+                  scale=scale, mod=mod)
     _check(library().sv_attn_rows(ctypes.byref(a),
                                   int(_aligned((D, rank), q)), _f32(q),
                                   _stream()), "attn_rows")
@@ -967,11 +1137,12 @@ def latent_portions(q, gate, cache, w: LatentWeights, batch,
         PAGE_SIZE * (R + P) * q.element_size(), _stream()), "latent_gather")
     kv = torch.mm(ws[:, :R], w.expand.t())
     return expanded_attention(q, gate, kv, ws, batch.tiles, spans, heads,
-                              dim, vdim, scale, window, out)
+                              dim, vdim, scale, window, out, w.sink)
 
 
 def expanded_attention(q, gate, kv, ws, tiles, spans: KeySpans, heads: int,
-                       dim: int, vdim: int, scale: float, window: int, out):
+                       dim: int, vdim: int, scale: float, window: int, out,
+                       sink: Optional[torch.Tensor] = None):
     """Query tiles over keys and values kv (rows, H * dim + H * vdim) of the
     workspace rows ws (rows, rank + P), whose last columns end every key."""
     P = q.shape[1] // heads - dim
@@ -988,7 +1159,8 @@ def expanded_attention(q, gate, kv, ws, tiles, spans: KeySpans, heads: int,
                    vpage=PAGE_SIZE * row, vhead=vdim, vrow=row, rrow=R + P,
                    tiles=_p(tiles), bt=_p(spans.table), out=_p(out),
                    MB=spans.table.shape[1], H=heads, G=heads, D=dim + P,
-                   E=vdim, DS=dim, window=window, keep=0, scale=scale)
+                   E=vdim, DS=dim, window=window, keep=0, scale=scale,
+                   mod=_score_args(ScoreMod(sink=sink), q, heads))
     if gate is not None:
         assert gate.shape == out.shape and gate.stride(1) == 1
         a.gate, a.gst = _p(gate), gate.stride(0)
@@ -1025,7 +1197,7 @@ def latent_attention(q, kv, gate, batch, cache, w: LatentWeights, heads: int,
                       heads, eps)
         head_linear(q[n:], dim + P, w.absorb, ql, D)
         lat = latent_rows(ql, cache, R, *at, heads, scale, window,
-                          batch.max_keys)
+                          batch.max_keys, w.sink)
         head_linear(lat, R, w.expand[heads * dim:].view(heads, vdim, R),
                     out[n:], vdim, None if gate is None else gate[n:])
     return out
@@ -1053,13 +1225,20 @@ def moe_kernel(pairs: int, experts: int) -> int:
 class Routing:
     """How logits choose experts.  Plain: the largest z + bias, weights a
     softmax over the chosen.  ``sigmoid``: the largest sigmoid(z) + bias,
-    weights the chosen sigmoids over their sum.  With several ``groups`` of
-    neighbours only the experts of the ``keep`` best can be chosen; a group
-    counts the sum of its two largest."""
+    weights the chosen sigmoids over their sum.  ``softmax``: the largest z +
+    bias, weights a softmax over all experts, not scaled to a sum of one.  With
+    several ``groups`` of neighbours only the experts of the ``keep`` best can
+    be chosen; a group counts the sum of its ``best`` (one or two) largest."""
     top: int
     sigmoid: bool = False
     groups: int = 1
     keep: int = 1
+    softmax: bool = False
+    best: int = 2
+
+    @property
+    def kind(self) -> int:
+        return 2 if self.softmax else int(self.sigmoid)
 
     def check(self, experts: int):
         g = self.groups
@@ -1069,6 +1248,8 @@ class Routing:
                 self.keep * (experts // g) < self.top:
             raise ValueError(f"{self.top} experts from {self.keep} of {g} "
                              f"groups of {experts}")
+        if self.best not in (1, 2) or (self.sigmoid and self.softmax):
+            raise ValueError(f"routing {self}")
 
 
 @dataclass
@@ -1099,8 +1280,8 @@ def moe_plan(z: torch.Tensor, bias: Optional[torch.Tensor],
     a = _MoePlanArgs(z=_p(z), bias=_p(bias), idx=_p(p.idx), coef=_p(p.coef),
                      order=_p(p.order), tiles=_p(p.tiles), T=T, E=E, top=top,
                      tile_rows=rows, max_tiles=n,
-                     sigmoid=int(routing.sigmoid), groups=routing.groups,
-                     keep=routing.keep)
+                     kind=routing.kind, groups=routing.groups,
+                     keep=routing.keep, best=routing.best)
     _check(library().sv_moe_plan(
         ctypes.byref(a), 0 if bias is None else _f32(bias), _stream()),
         "moe_plan")
