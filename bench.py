@@ -40,7 +40,8 @@ def parse_args():
                    help="instead: the serving benchmark of a design beside "
                         "its closest relative (bench_serving.py, 1 GPU)")
     p.add_argument("--design", default="all",
-                   choices=("all", "voletar", "nesilorn", "sutuvik"),
+                   choices=("all", "voletar", "nesilorn", "sutuvik",
+                            "pokepel"),
                    help="with --serving: Voletar beside Llama, Nesilorn "
                         "beside Mixtral, Sutuvik beside Nesilorn, or all")
     return p.parse_args()

@@ -1,8 +1,8 @@
 #!/usr/bin/env python3
 """Serving benchmark of a design beside its closest relative at equal layer
 sizes (random weights, one MI355X): Voletar beside Llama, Nesilorn beside
-Mixtral, Sutuvik beside Nesilorn (its kernels beside those of Voletar and
-Nesilorn).
+Mixtral, Sutuvik and Pokepel beside Nesilorn (their kernels beside those of
+Voletar and Nesilorn).
 
     python bench.py --serving                          all of it
     python bench.py --serving kernels                  (or: models)
@@ -788,30 +788,34 @@ def bench_state_kernels():
 
 
 def bench_state_models():
+    _engine_models("Sutuvik", "Nesilorn")
+
+
+def _engine_models(*names):
     for size in ("bench", "bench-fine"):
-        _state_models(size)
+        _side_by_side(size, names)
         torch.cuda.empty_cache()
 
 
-def _state_models(size):
+def _side_by_side(size, names):
+    """Models of the serving engine, each in its configuration ``size``."""
+    from neuronx_distributed_amd import models as zoo
     from neuronx_distributed_amd.inference import (InferenceEngine, StepEntry,
                                                    single_process_groups)
-    from neuronx_distributed_amd.models import (build_model,
-                                                get_nesilorn_config,
-                                                get_sutuvik_config)
+    from neuronx_distributed_amd.models import build_model
 
     single_process_groups()
     torch.manual_seed(0)
-    cfgs = {"Sutuvik": get_sutuvik_config(f"sutuvik-{size}"),
-            "Nesilorn": get_nesilorn_config(f"nesilorn-{size}")}
+    cfgs = {n: getattr(zoo, f"get_{n.lower()}_config")(f"{n.lower()}-{size}")
+            for n in names}
     models = {n: build_model(n, c, torch.bfloat16, "cuda")
               for n, c in cfgs.items()}
     out = {f"{n.lower()}_b_params": round(
         sum(p.numel() for p in m.parameters()) / 1e9, 2)
         for n, m in models.items()}
     print(json.dumps({"size": size, **out,
-                      "width": cfgs["Sutuvik"].hidden_size,
-                      "layers": len(cfgs["Sutuvik"].layers),
+                      "width": cfgs[names[0]].hidden_size,
+                      "layers": len(cfgs[names[0]].layers),
                       "data": "random weights"}), flush=True)
 
     def turns(fns, reps):
@@ -868,9 +872,157 @@ def _state_models(size):
         torch.cuda.empty_cache()
 
 
+# ---------------------------------------------------------------------------
+# Pokepel beside Nesilorn and Voletar
+# ---------------------------------------------------------------------------
+
+def bench_retention_kernels():
+    from dataclasses import replace
+
+    from neuronx_distributed_amd import ops
+    from neuronx_distributed_amd.ops import serving as sv
+
+    dev = dict(device="cuda")
+    # -- retention beside the decayed memory, each with its norm and gate ------
+    H, D, E, eps = 32, 128, 128, 1e-5
+    lgate = sv.decay_gate([0.99] * H, "cuda")
+    gate = sv.TurnGate(lgate.decay, lgate.log2_decay, D ** -0.5,
+                       sv.rotary_frequencies(1e4, D, "cuda"))
+    w = _bf(H * E)
+    for B, T in ((1, 4096), (4, 4096), (1, 1), (32, 1), (128, 1)):
+        n = B * T
+        q, k, v, g = _bf(n, 2 * H * (D + E)).split(
+            (H * D, H * D, H * E, H * E), 1)
+        S = torch.zeros(B, H, D, E, **dev)
+        ctx = 64 if T == 1 else 0
+        seg = _i32([(i, i * T, T, ctx) for i in range(B)])
+        rows, first = sv.chunk_table(seg.tolist())
+        tab = (_i32(rows), _i32(first)) if T > 1 else ()
+
+        def like():
+            o = sv.memory_mix(q, k, v, lgate, S, None, None, seg, H, *tab)
+            return sv.gated_norm(o, w, g, H * E, eps)
+
+        def mix():
+            if T > 1:
+                return sv.memory_mix(q, k, v, gate, S, None, None, seg, H,
+                                     *tab, silu_gate=g, eps=eps)
+            o = sv.memory_mix(q, k, v, gate, S, None, None, seg, H)
+            return sv.gated_norm(o, None, g, E, eps, True, out=o)
+
+        us, lus, mus, lmus = _time([
+            _graphed(mix), _graphed(like),
+            _graphed(lambda: sv.memory_mix(q, k, v, gate, S, None, None, seg,
+                                           H, *tab)),
+            _graphed(lambda: sv.memory_mix(q, k, v, lgate, S, None, None, seg,
+                                           H, *tab))])
+        cs = 64 if T > 1 else 1
+        fl = 2 * n * H * (cs / 2 * (D + E) + 2 * D * E)
+        io = 4 * n * H * (D + E) + (8 if ctx else 4) * B * H * D * E
+        # every product of split operands at its MFMA cost
+        f5 = 2 * n * H * (cs / 2 * (3 * D + 3 * E) + 10 * D * E)
+        extra = {"roofline_32bit_us": round(
+            max(f5 / PEAK_FLOPS, io / PEAK_BYTES) * 1e6, 2)} if T > 1 else {}
+        kw = dict(batch=B, tokens=T, heads=H, dim=D, vdim=E, **extra)
+        name = "chunks" if T > 1 else "steps"
+        _report(f"retention_{name} (rotation)", mus, fl, io,
+                ("decayed memory", lmus, fl, io), **kw)
+        _report(f"retention_{name} (rotation, norm, gate)", us, fl,
+                io + 2 * n * H * E, ("decayed memory, gated_norm", lus, fl,
+                                     io + 2 * n * H * E), **kw)
+    # -- latent attention with a sink and neighbouring pairs --------------------
+    H, D, P, E, R = 32, 128, 64, 128, 512
+    scale = (D + P) ** -0.5
+    sink = _bf(H)
+    for B, T, ctx in ((1, 4096, 0), (1, 8192, 0), (1, 1, 4096),
+                      (32, 1, 1024), (32, 1, 4096), (128, 1, 4096)):
+        b, lw, cache, q, kv, g = _latent_case(sv, B, T, ctx, H, D, P, E, R)
+        w = replace(lw, amplitude=1.14, pairs=True, sink=sink)
+        if T > 1:
+            pages, table = sv.key_spans([(0, 0, T, 0)],
+                                        b.block_table.tolist(), 0)
+            b.spans = {0: sv.KeySpans(_i32(pages), _i32(table))}
+        fns = [_graphed(lambda x=x: sv.latent_attention(
+            q, kv, g, b, cache, x, H, D, E, scale, 1e-5)) for x in (w, lw)]
+        pairs = B * sum(ctx + i + 1 for i in range(T))
+        if T > 1:
+            kve, ws = _bf(T, H * (D + E)), _bf(T, R + P)
+            out = torch.empty(T, H * E, dtype=torch.bfloat16, **dev)
+            fns += [_graphed(lambda s=s: sv.expanded_attention(
+                q, g, kve, ws, b.tiles, b.spans[0], H, D, E, scale, 0, out,
+                s)) for s in (sink, None)]
+            fl = 2 * pairs * H * (D + P + E)
+            io = 2 * T * (H * (D + P + 2 * E) + R + P) + \
+                2 * T * H * (D + E)
+            all_fl, all_io = fl + 2 * T * R * H * (D + E), io
+        else:
+            ql = _bf(B, H * (R + P))
+            fns += [_graphed(lambda s=s: sv.latent_rows(
+                ql, cache, R, b.pos, b.seq, b.block_table, H, scale, 0,
+                ctx + 1, s)) for s in (sink, None)]
+            fl = 2 * pairs * H * (2 * R + P)
+            io = 2 * B * (ctx + 1) * (R + P) + 2 * B * H * (2 * R + P)
+            all_fl = fl + 2 * B * H * R * (D + E)
+            all_io = io + 2 * H * (D + E) * R + 2 * B * H * (D + P + 2 * E)
+        t = _time(fns)
+        kw = dict(batch=B, tokens=T, context=ctx)
+        _report("latent_attention (sink, pairs)", t[0], all_fl, all_io,
+                ("latent_attention", t[1], all_fl, all_io), **kw)
+        name = "attn_tiles on expanded keys" if T > 1 else "latent_rows"
+        _report(name + " (sink)", t[2], fl, io, (name, t[3], fl, io), **kw)
+    # -- residual, activations, routing -----------------------------------------
+    for T in (32, 4096):
+        Wd, F, top = 4096, 14336, 2
+        x, d, d1, plus, wn = (torch.randn(T, Wd, **dev), _bf(T, Wd),
+                              _bf(T, Wd), _bf(T, Wd), _bf(Wd))
+        d2, coef = _bf(T * top, Wd), torch.rand(T, top, **dev)
+        gates = _bf(T, 2 * Wd)
+        A = sv.Branch(d1, gate=gates[:, :Wd], bias=wn)
+        dense = sv.Branch(plus, gate=gates[:, Wd:], bias=wn)
+        moe = sv.Branch(d2, coef, plus, gates[:, Wd:], wn)
+        u, gu, act = _bf(T, F + 64), _bf(T, 2 * F), _bf(4)
+        z = torch.randn(T, 64, **dev)
+        t = _time([
+            _graphed(lambda: sv.residual_norm(
+                x, sv.Pending(branches=[A, dense]), 1e-6, wn)),
+            _graphed(lambda: sv.residual_norm(
+                x, sv.Pending(branches=[A, moe]), 1e-6, wn)),
+            _graphed(lambda: sv.residual_norm(
+                x, sv.Pending(d, d1, wn, wn, 0.5), 1e-6, wn)),
+            _graphed(lambda: sv.poly_norm(u[:, :F], act, 1e-6)),
+            _graphed(lambda: sv.silu_mul(gu)),
+            _graphed(lambda: ops.swiglu(gu)),
+            _graphed(lambda: sv.gelu_tanh_(u)),
+            _graphed(lambda: sv.moe_plan(z, None, sv.Routing(
+                6, groups=8, keep=4, softmax=True, best=1), 0)),
+            _graphed(lambda: sv.moe_plan(z, None, 6, 0)),
+            _graphed(lambda: sv.gated_norm(d, None, d1, 128, 1e-5, True)),
+            _graphed(lambda: sv.gated_norm(d, wn, d1, 128, 1e-5))])
+        n = T * Wd
+        like = ("residual_norm (two branches)", t[2], 0, 14 * n)
+        _report("residual_norm (gated branches)", t[0], 0, 18 * n, like,
+                rows=T)
+        _report("residual_norm (gated branches, experts and a shared one)",
+                t[1], 0, (18 + 2 * top) * n, like, rows=T)
+        _report("poly_norm", t[3], 0, 4 * T * F,
+                ("gelu_tanh", t[6], 0, 4 * T * F), rows=T)
+        _report("silu_mul", t[4], 0, 6 * T * F,
+                ("swiglu", t[5], 0, 6 * T * F), rows=T)
+        io = 4 * T * 64 + 12 * T * 6
+        _report("moe_plan (softmax, groups)", t[7], 0, io,
+                ("moe_plan", t[8], 0, io), rows=T, experts=64, top=6)
+        _report("gated_norm (silu, no weight)", t[9], 0, 6 * n,
+                ("gated_norm", t[10], 0, 6 * n), rows=T)
+
+
+def bench_retention_models():
+    _engine_models("Pokepel", "Nesilorn")
+
+
 DESIGNS = {"voletar": (bench_kernels, bench_models),
            "nesilorn": (bench_latent_kernels, bench_latent_models),
-           "sutuvik": (bench_state_kernels, bench_state_models)}
+           "sutuvik": (bench_state_kernels, bench_state_models),
+           "pokepel": (bench_retention_kernels, bench_retention_models)}
 
 
 def main(what="all", design="all"):

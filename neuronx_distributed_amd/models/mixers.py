@@ -582,10 +582,24 @@ class ParallelMixer(nn.Module):
             self.left_out, self.right_out, self.branch_scale)
 
 
+_side_streams = {}
+
+
+def side_stream(device) -> torch.cuda.Stream:
+    """A second stream of the device, for work beside the current one's."""
+    if device not in _side_streams:
+        _side_streams[device] = torch.cuda.Stream(device)
+    return _side_streams[device]
+
+
 class GatedParallel(nn.Module):
     """A mixer and a feed-forward (or none) side by side on the same rows h,
     each result times sigmoid(W h + b) of its own.  One product makes the
-    projections of both and the gates; the results are left pending."""
+    projections of both and the gates; the results are left pending.
+
+    In steps of single tokens, what the feed-forward can do ``ahead`` of the
+    projections runs on a second stream (a second branch of a captured graph),
+    beside the mixer's small kernels."""
 
     def __init__(self, width, mixer: Mixer, mlp: Optional[Projected] = None):
         super().__init__()
@@ -626,14 +640,26 @@ class GatedParallel(nn.Module):
         copy_weight(self.proj.weight, w)
 
     def forward(self, h, batch, pools) -> sv.Pending:
+        ahead = None
+        beside = getattr(self.mlp, "ahead", None)
+        here = torch.cuda.current_stream(h.device)
+        if beside and not batch.portion_tokens:
+            # what is allocated on either stream is used on the other only
+            # between these two waits, or before the next layer's first
+            side = side_stream(h.device)
+            side.wait_stream(here)
+            with torch.cuda.stream(side):
+                ahead = beside(h)
         proj = self.proj(h)
         mix, gate1, *rest = [proj[:, a:b] for a, b in self.at]
         branches = [sv.Branch(self.mixer(h, mix, batch, pools), gate=gate1,
                               bias=self.bias1)]
         if self.mlp is not None:
-            y = self.mlp(h, rest[0])
+            y = self.mlp(h, rest[0], ahead)
             y.gate, y.bias = rest[1], self.bias2
             branches.append(y)
+        if ahead is not None:
+            here.wait_stream(side)
         return sv.Pending(branches=branches)
 
 
@@ -652,7 +678,7 @@ class PolyNormMLP(Projected):
         copy_weight(self.act, get(prefix + "act"))
         copy_weight(self.down.weight, get(prefix + "down"))
 
-    def forward(self, h, proj) -> sv.Branch:
+    def forward(self, h, proj, ahead=None) -> sv.Branch:
         return sv.Branch(self.down(sv.poly_norm(self.split(proj)[0], self.act,
                                                 self.eps)))
 
@@ -735,8 +761,11 @@ class SharedExpertsMLP(Projected):
         if self.sizes:
             copy_weight(self.down.weight, get(prefix + "shared.down"))
 
-    def forward(self, h, proj) -> sv.Branch:
-        y = self.experts(h)
+    def ahead(self, h) -> sv.Pending:
+        return self.experts(h)
+
+    def forward(self, h, proj, ahead=None) -> sv.Branch:
+        y = ahead or self.experts(h)
         plus = self.down(sv.silu_mul(proj)) if self.sizes else None
         return sv.Branch(y.delta, y.coef, plus)
 

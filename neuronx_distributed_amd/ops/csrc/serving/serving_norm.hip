@@ -71,8 +71,8 @@ __device__ __forceinline__ void st(T* p, const float* v) {
   if (VEC == 4) store4(p, v); else from_f(p[0], v[0]);
 }
 
-template <typename T, int VEC, bool BRANCHES>
-__global__ void __launch_bounds__(256)
+template <typename T, int VEC, bool BRANCHES, int NT>
+__global__ void __launch_bounds__(NT)
 residual_norm_kernel(ResidualNormArgs a) {
   extern __shared__ __attribute__((aligned(16))) float row[];  // [W]
   float* part_rstd = row + a.W;    // [groups], if a norm has several
@@ -108,7 +108,7 @@ residual_norm_kernel(ResidualNormArgs a) {
   auto norm_parts = [&](int n) {
     const int size = W / n, lane = tid & 63;
     __syncthreads();
-    for (int g = tid >> 6; g < n; g += 4) {
+    for (int g = tid >> 6; g < n; g += NT / 64) {
       float q = 0.f;
       for (int i = lane; i < size; i += 64) q += row[g * size + i] * row[g * size + i];
       q = wave_reduce(q, SumOp());
@@ -120,7 +120,7 @@ residual_norm_kernel(ResidualNormArgs a) {
   float s1 = a.scale, s2 = 0.f;
   if (a.delta2) {
     float q1 = 0.f, q2 = 0.f, v[VEC];
-    for (int i = tid * VEC; i < W; i += 256 * VEC) {
+    for (int i = tid * VEC; i < W; i += NT * VEC) {
       ld<T, VEC>(d1 + i, v);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) q1 += v[j] * v[j];
@@ -136,7 +136,7 @@ residual_norm_kernel(ResidualNormArgs a) {
     s2 = a.scale / sqrtf(q2 / W + a.eps);
   } else if (a.w1) {
     float q1 = 0.f, v[VEC];
-    for (int i = tid * VEC; i < W; i += 256 * VEC) {
+    for (int i = tid * VEC; i < W; i += NT * VEC) {
       single(i, v);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) q1 += v[j] * v[j];
@@ -153,7 +153,7 @@ residual_norm_kernel(ResidualNormArgs a) {
   const int p_size = a.p_groups > 1 ? W / a.p_groups : W;
 
   float sq = 0.f;
-  for (int i = tid * VEC; i < W; i += 256 * VEC) {
+  for (int i = tid * VEC; i < W; i += NT * VEC) {
     float v[VEC], t[VEC], u[VEC];
 #pragma unroll
     for (int j = 0; j < VEC; ++j) v[j] = 0.f;
@@ -180,42 +180,49 @@ residual_norm_kernel(ResidualNormArgs a) {
       for (int j = 0; j < VEC; ++j) v[j] += s1 * t[j];
     }
     if (BRANCHES) {
-#pragma unroll
-      for (int b = 0; b < 2; ++b) {
-        if (b >= a.branches) break;
+      // a long workgroup asks for all words first, so that their ways overlap
+      constexpr bool AHEAD = NT > 256;
+      constexpr int P = AHEAD ? 4 : 2;   // rows of a sum in flight
+      float g[2][VEC], e[2][VEC], d[2][P][VEC], q[2][VEC];
+      auto fetch = [&](int b) {
         const BranchArgs& z = a.br[b];
-        float g[VEC];
-        if (z.gate) {
-          ld<T, VEC>((const T*)z.gate + r * z.gst + i, g);
-          if (z.bias) {
-            ld<T, VEC>((const T*)z.bias + i, u);
+        if (z.gate) ld<T, VEC>((const T*)z.gate + r * z.gst + i, g[b]);
+        if (z.bias) ld<T, VEC>((const T*)z.bias + i, e[b]);
 #pragma unroll
-            for (int j = 0; j < VEC; ++j) g[j] += u[j];
-          }
+        for (int p = 0; p < P; ++p)
+          if (p < z.parts)
+            ld<T, VEC>((const T*)z.delta + (r * z.parts + p) * W + i, d[b][p]);
+        if (z.plus) ld<T, VEC>((const T*)z.plus + r * W + i, q[b]);
+      };
+      auto add = [&](int b) {
+        const BranchArgs& z = a.br[b];
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) t[j] = z.plus ? q[b][j] : 0.f;
+#pragma unroll
+        for (int p = 0; p < P; ++p) {
+          if (p >= z.parts) break;
+          const float c = z.coef ? z.coef[r * z.parts + p] : 1.f;
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) t[j] += c * d[b][p][j];
         }
-        if (z.coef) {
-          const T* d = (const T*)z.delta + r * z.parts * W + i;
-#pragma unroll
-          for (int j = 0; j < VEC; ++j) t[j] = 0.f;
 #pragma unroll 2
-          for (int p = 0; p < z.parts; ++p) {
-            const float c = z.coef[r * z.parts + p];
-            ld<T, VEC>(d + (long)p * W, u);
+        for (int p = P; p < z.parts; ++p) {
+          const float c = z.coef[r * z.parts + p];
+          ld<T, VEC>((const T*)z.delta + (r * z.parts + p) * W + i, u);
 #pragma unroll
-            for (int j = 0; j < VEC; ++j) t[j] += c * u[j];
-          }
-        } else {
-          ld<T, VEC>((const T*)z.delta + r * W + i, t);
-        }
-        if (z.plus) {
-          ld<T, VEC>((const T*)z.plus + r * W + i, u);
-#pragma unroll
-          for (int j = 0; j < VEC; ++j) t[j] += u[j];
+          for (int j = 0; j < VEC; ++j) t[j] += c * u[j];
         }
 #pragma unroll
         for (int j = 0; j < VEC; ++j)
-          v[j] += z.gate ? t[j] * sigmoid_f(g[j]) : t[j];
-      }
+          v[j] += !z.gate ? t[j]
+                          : t[j] * sigmoid_f(z.bias ? g[b][j] + e[b][j] : g[b][j]);
+      };
+      const bool two = a.branches > 1;
+      fetch(0);
+      if (AHEAD && two) fetch(1);
+      add(0);
+      if (!AHEAD && two) fetch(1);
+      if (two) add(1);
     }
     if (a.vec) {
       ld<T, VEC>((const T*)a.vec + i, t);
@@ -246,7 +253,7 @@ residual_norm_kernel(ResidualNormArgs a) {
   const int size = a.groups > 1 ? W / a.groups : W;
   const bool conv = a.conv && o >= a.conv_row;
   const int* sg = a.singles + 4L * (o - a.conv_row);
-  for (int i = tid * VEC; i < W; i += 256 * VEC) {
+  for (int i = tid * VEC; i < W; i += NT * VEC) {
     float v[VEC], u[VEC];
     ld<float, VEC>(row + i, v);  // written by this same thread
     ld<T, VEC>((const T*)a.w + i, u);
@@ -301,10 +308,16 @@ extern "C" int sv_residual_norm(const ResidualNormArgs* a, int f32,
                   (a->br[b].gst % 4 == 0 &&
                    (size_t)a->br[b].gate % (f32 ? 16 : 8) == 0));
   if (a->branches < 0 || a->branches > 2 || (a->branches && a->delta)) return 1;
-#define RNB(T, V, B)                                                       \
-  residual_norm_kernel<T, V, B><<<a->rows_out, 256, lds, stream>>>(*a)
+  // few rows: a longer workgroup hides the way to memory
+  const bool wide = a->rows_out <= 512 && a->W >= 2048;
+#define RNB(T, V, B, N)                                                    \
+  residual_norm_kernel<T, V, B, N><<<a->rows_out, N, lds, stream>>>(*a)
 #define RN(T, V)                                                           \
-  do { if (a->branches) RNB(T, V, true); else RNB(T, V, false); } while (0)
+  do {                                                                     \
+    if (a->branches && wide) RNB(T, V, true, 1024);                        \
+    else if (a->branches) RNB(T, V, true, 256);                            \
+    else RNB(T, V, false, 256);                                            \
+  } while (0)
   if (f32) { if (vec) RN(float, 4); else RN(float, 1); }
   else     { if (vec) RN(short, 4); else RN(short, 1); }
 #undef RN
