@@ -43,7 +43,8 @@ def parse_args():
                    choices=("all", "voletar", "nesilorn", "sutuvik",
                             "pokepel"),
                    help="with --serving: Voletar beside Llama, Nesilorn "
-                        "beside Mixtral, Sutuvik beside Nesilorn, or all")
+                        "beside Mixtral, Sutuvik and Pokepel beside Nesilorn, "
+                        "or all")
     return p.parse_args()
 
 
