@@ -27,7 +27,8 @@ struct MoePlanArgs {
   int* order;               // [T * top] slot -> pair
   int* tiles;               // [max_tiles][4]: expert, first slot, slots, 0
   int T, E, top, tile_rows, max_tiles;
-  int kind;                 // 0: softmax over the chosen; 1: scores sigmoid(z), chosen by score + bias;
+  int kind;                 // 0: weights are a softmax over the chosen;
+                            // 1: scores sigmoid(z), chosen by score + bias;
                             // 2: weights are a softmax over all experts
   int groups, keep;         // experts of the best groups only (groups > 1)
   int best;                 // a group counts the sum of its 1 or 2 largest
